@@ -463,6 +463,144 @@ uint64_t vx_scratch_generation(const vx_backend *be);
 /* The caller makes sure no replay of the graph is still running (vx_sync). */
 void vx_graph_destroy(vx_graph *g);
 
+/* ---- ragged mixed batches: layers of attention, selective scans and dense MLPs over bfloat16 weights ----------- */
+/* No counterpart in the reference. Every sequence of a step brings any number of new tokens (portions of prompts beside
+ * single decoded tokens); their rows are concatenated, sequence after sequence. Activations between the operations
+ * are bfloat16 (VX_ACT_BF16) or float32 (VX_ACT_F32: every product and sum in float32, no reduced-precision matrix
+ * mode); the residual stream, norms, attention scores and weights, and the scan are float32 in both. */
+enum { VX_ACT_F32 = 0, VX_ACT_BF16 = 1 };
+
+/* A step's rows and where their sequences live. The device arrays are what vx_pack_batch writes, from the same batch. */
+typedef struct vx_ragged {
+    int rows, n_seqs;
+    const int32_t *q_lens;       /* HOST int32[n_seqs], >= 1 each, or NULL: one row per sequence */
+    int max_kv_len;              /* >= every kv length after the step (bounds launches and scratch) */
+    const int32_t *cu_seqlens;   /* [n_seqs + 1] first row of every sequence */
+    const int32_t *token_pos;    /* [rows] position of every row in its sequence */
+    const int32_t *slot_mapping; /* [rows] physical block * block_size + offset */
+    const int32_t *table_rows;   /* [n_seqs] row of block_tables, and state slot, of every sequence */
+    const int32_t *kv_lens;      /* [n_seqs] tokens of the sequence, this step's included */
+    const int32_t *block_tables; /* [.., max_blocks] */
+    int max_blocks, block_size;
+} vx_ragged;
+
+/* Zeroes device memory with a kernel (may be captured into a graph). bytes a multiple of 4. */
+int vx_fill_zero(vx_backend *be, void *dst, size_t bytes);
+
+/* Weights of a linear map y = W x in the order the matrix cores take them: tiles of 16 output rows x 32 inputs, each 64
+ * lanes x 8 bfloat16. n_pad % 16 == 0, k_pad % 64 == 0; what no source covers is zero (vx_fill_zero first).
+ * vx_linear_pack puts the row-major bfloat16 matrix src [n, k] (device) at input column col0 of the packed matrix: source
+ * rows 16 i .. 16 i + 15 become its row tile tile0 + i * tile_step. */
+size_t vx_linear_bytes(int n_pad, int k_pad);
+int vx_linear_pack(vx_backend *be, const void *src, int n, int k, void *dst, int n_pad, int k_pad, int tile0, int tile_step,
+                   int col0);
+
+enum {
+    VX_LIN_PLAIN = 0,  /* out[r * ldo + c] for c < cols (out_f32: float32, else the activation type), or, with slices > 1,
+                          float32 partial sums over slices of the inputs, out[s][r * ldo + c], slice after slice */
+    VX_LIN_SWIGLU = 1, /* row tiles alternate gate, up: out = silu(gate) * up, 16 columns per pair of tiles */
+    VX_LIN_KV = 2,     /* PLAIN in the activation type, but columns [k_col, k_col + kv_heads * k_dim) and [v_col, ..) go
+                          to the paged pool at slot_mapping[r] (layout: vx_kv_block_elems) */
+    VX_LIN_SPLIT = 3,  /* columns < split to out (activation type), the others to out2[r * ldo2 + c - split] (float32) */
+    VX_LIN_SOFTPLUS = 4 /* float32 out = log(1 + exp(y + bias[c])) */
+};
+typedef struct vx_linear_out {
+    int kind, out_f32, ldo, cols, slices;
+    void *out;
+    float *out2;
+    int split, ldo2;
+    const float *bias;
+    int k_col, v_col, kv_heads, k_dim, v_dim, block_size;
+    void *pool;
+    const int32_t *slot_mapping;
+} vx_linear_out;
+/* out = a [rows, k] * W^T for a packed matrix [n, k] (padded sizes); a has lda >= k columns of the activation type, zero
+ * where k was padded, rows 16-byte aligned. vx_linear_slices: into how many slices a PLAIN float32 result is best cut
+ * (its consumer adds them: vx_residual_norm). */
+int vx_linear_slices(vx_backend *be, int n, int k, int rows);
+int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, int n, int k, int rows, const vx_linear_out *o);
+
+/* The seam between two sublayers, one row at a time, in float32:
+ *   x = x_in[r];  if y: x += mult * rmsnorm(sum over slices of y[s][r]) * w_post;  if add: x += add[r];  x_out[r] = x;
+ *   if w_pre: out[i] = rmsnorm(x) * w_pre in the activation type, columns cols .. ldo - 1 zero.
+ * r = row_idx ? row_idx[i] : i for i < rows. x_out may be x_in or NULL. rmsnorm(v) = v / sqrt(mean(v^2) + eps). */
+typedef struct vx_residual_norm_args {
+    int rows, cols;
+    const int32_t *row_idx;
+    const float *x_in, *add;
+    float *x_out;
+    const float *y, *w_post;
+    int y_slices, ldy;
+    int64_t y_stride;            /* floats from one slice to the next */
+    float mult, eps;
+    const float *w_pre;
+    void *out;
+    int ldo;
+} vx_residual_norm_args;
+int vx_residual_norm(vx_backend *be, int act, const vx_residual_norm_args *p);
+
+/* Causal grouped-query attention over the paged pool for every row of a mixed batch (the rows' K and V are in it already):
+ *   score(i, j) = (temp(i) * scale) * q_i . k_j + bias[h][min(i - j, bias_len - 1)],  softmax over j <= i,
+ *   out = out_scale * sigmoid(gate) * (weights . v)
+ * temp(i) = 1 + temp_coef * ln(floor((i + 1) / temp_every) + 1); temp_every 0: 1. bias NULL: none (float32
+ * [heads][bias_len] on the device). gate NULL: none. q, gate, out: activation type, head h at columns h * k_dim (q)
+ * and h * v_dim (gate, out).
+ * Pool of one layer: per physical block K [kv_heads][block_size][k_pad], then V transposed [kv_heads][v_dim][block_size],
+ * k_pad = k_dim up to a multiple of 8, elements of the activation type; it must have been zeroed once. */
+typedef struct vx_attn_args {
+    int heads, kv_heads, k_dim, v_dim;
+    float scale, temp_coef;
+    int temp_every;
+    const float *bias;
+    int bias_len;
+    const void *q, *gate;
+    int ldq, ldg;
+    const void *pool;
+    float out_scale;
+    void *out;
+    int ldo;
+} vx_attn_args;
+size_t vx_kv_block_elems(int block_size, int kv_heads, int k_dim, int v_dim);
+int vx_attn_ragged(vx_backend *be, int act, const vx_ragged *b, const vx_attn_args *p);
+/* 1 when the matrix-core kernels take the geometry, 0 when vx_attn_ragged uses the plain one. */
+int vx_attn_ragged_fast(int act, int block_size, int heads, int kv_heads, int k_dim, int v_dim);
+
+/* Causal depthwise convolution with SiLU over a mixed batch: out[r][c] = silu(b[c] + sum_t w[t][c] * x[position - (taps
+ * - 1 - t)][c]), positions before the sequence's start count as zero, positions before this step's rows come from
+ * the state [slots][taps - 1][channels] (activation type, the latest last), which is moved on. A sequence at position
+ * 0 takes nothing from its slot. out columns channels .. ldo - 1 become zero. */
+typedef struct vx_conv_args {
+    int channels, taps;
+    const void *x;
+    int ldx;
+    const float *w, *b;
+    void *state;
+    void *out;
+    int ldo;
+} vx_conv_args;
+int vx_conv_silu(vx_backend *be, int act, const vx_ragged *b, const vx_conv_args *p);
+
+/* Selective scan over a mixed batch, all in float32:
+ *   S[c][n] = exp(dt[c] * A[c][n]) * S[c][n] + dt[c] * x[c] * B[n];  y[c] = sum_n S[c][n] * C[n] + D[c] * x[c]
+ *   out[r][c] = out_scale * y[c] * silu(z[c])   (columns channels .. out_cols - 1 zero)
+ * states = n count padded with vx_scan_state_pad; a2 = A * log2(e) [channels][padded], zero where padded; bc [rows][2 * padded]
+ * float32 (B, then C; zero where padded); dt [rows][lddt] float32; x, z, out: activation type; state
+ * [slots][channels][padded] float32. A sequence at position 0 starts from zero. */
+typedef struct vx_scan_args {
+    int channels, states;
+    const float *a2, *d;
+    const void *x, *z;
+    int ldx, ldz;
+    const float *dt, *bc;
+    int lddt;
+    float *state;
+    float out_scale;
+    void *out;
+    int ldo, out_cols;
+} vx_scan_args;
+int vx_scan_state_pad(int states);  /* 16, 32, .. 256; -1 beyond 256 */
+int vx_selective_scan(vx_backend *be, int act, const vx_ragged *b, const vx_scan_args *p);
+
 /* Wall-clock helpers on the backend stream (HIP events), for benchmarks. */
 int vx_timer_start(vx_backend *be);
 int vx_timer_stop_ms(vx_backend *be, float *ms);

@@ -136,6 +136,16 @@ int vh_decode_batched(vh_model *m, const int32_t *tokens, const int64_t *seq_ids
  * temperature 0 is the greedy choice. tokens_out: host int32[rows]. */
 int vh_sample_last_logits(vh_model *m, int rows, const float *temperature, const int32_t *top_k, const float *top_p,
                           const float *uniform, int32_t *tokens_out);
+/* One step of n_seqs sequences that bring q_lens[i] >= 1 tokens each, concatenated in `tokens`: portions of prompts and
+ * single decoded tokens in one call, each appended to its sequence (an unknown id is a new sequence). Row numbers count
+ * over the concatenated tokens; want_rows[n_want] are the rows whose logits [n_want, vocab] and arg-max tokens are
+ * returned (either may be NULL). A mixer program runs the whole step as one batch (vh_model_mixed_batches is 1); models of
+ * the LLaMA family run each portion with vh_prefill and the single tokens with vh_decode_batched. With a mixer program
+ * vh_sample_last_logits afterwards samples the wanted rows, when there are at most max_batch of them. No counterpart in
+ * the reference, which prefills one sequence at a time. */
+int vh_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_lens, const int32_t *tokens, int n_want,
+            const int32_t *want_rows, float *logits_out, int32_t *argmax_out);
+int vh_model_mixed_batches(const vh_model *m);
 /* Speculative verification of a whole candidate tree for each of n_seqs sequences in one forward pass, greedy
  * acceptance and rollback. The reference's runTreeMedusaDecodeStep (scheduler/medusa_scheduler.go:733-861)
  * handles one sequence and verifies only the most confident path with VerifySpeculativeWithPagedKV
@@ -206,9 +216,12 @@ int vh_gguf_get_config(const vh_gguf *g, vh_gguf_config *out);
 /* gguf.GetLayerTensorName (pkg/gguf/loader.go:121-228), LLaMA-family names; others pass through. */
 int vh_gguf_tensor_name(const char *hf_name, char *out, size_t cap);
 
+enum { VH_DTYPE_DEFAULT = 0, VH_DTYPE_BF16 = 1, VH_DTYPE_F32 = 2 };
 typedef struct vh_load_options {  /* what the checkpoint does not say: the KV pool and batch geometry */
     int block_size;               /* 0 = 16 */
     int pool_blocks, max_seqs, max_blocks_per_seq, max_batch, kv_fp16;
+    int dtype;                    /* folders with a config.json: the activations' type (and the cache's), VH_DTYPE_*; the
+                                     default is bfloat16. GGUF models have one arithmetic of their own and ignore it. */
 } vh_load_options;
 /* ModelRuntime.LoadWeightsGGUF + CopyWeightsToDevice (runtime/loader.go:28-212, 560-700). general.architecture
  * selects the switches as ModelConfigFromGGUF does (runtime/config.go:388-470): llama / mistral; qwen2 (Q/K/V biases,
@@ -221,6 +234,17 @@ typedef struct vh_load_options {  /* what the checkpoint does not say: the KV po
  * dequantizes it to float32 at load (same values, float32 summation order aside). The model owns the device
  * copies; vh_model_destroy frees them. */
 int vh_model_load_gguf(vx_backend *be, const char *path, const vh_load_options *opt, vh_model **out);
+/* A model from `path`: a folder with config.json and model.safetensors, whose "architecture" is looked up in the
+ * registry of mixer programs (vh_architecture_name(0), (1), .. until NULL), or a GGUF file (vh_model_load_gguf). No
+ * counterpart in the reference, whose folders hold the GGUF architectures' tensors. */
+int vh_model_load(vx_backend *be, const char *path, const vh_load_options *opt, vh_model **out);
+const char *vh_architecture_name(int i);
+/* Parses and checks the config.json text of a mixer program without a device or weights: VH_OK, or what is wrong with it
+ * in vh_last_error(). */
+int vh_check_config(const char *json_text);
+/* Bucket of a key `distance` >= 0 back in a distance-bias table of `rows` rows: distances under rows/2 have a bucket each,
+ * larger ones share them logarithmically up to bias_max, from which on it is the last. -1: rows or bias_max out of range. */
+int vh_distance_bucket(int distance, int rows, int bias_max);
 /* Hands a vx_alloc_permanent buffer to the model, which frees it in vh_model_destroy. */
 void vh_model_adopt_buffer(vh_model *m, void *device_ptr);
 

@@ -18,6 +18,46 @@ class VxQWeight(C.Structure):
     _fields_ = [("fmt", C.c_int), ("data", C.c_void_p), ("n", C.c_int), ("k", C.c_int)]
 
 
+def _fields(spec):
+    """"int a b; ptr c" -> ctypes fields"""
+    kinds = {"int": C.c_int, "float": C.c_float, "ptr": C.c_void_p, "i64": C.c_int64}
+    out = []
+    for part in spec.split(";"):
+        kind, *names = part.split()
+        out += [(n, kinds[kind]) for n in names]
+    return out
+
+
+class VxRagged(C.Structure):
+    """vx_ragged: a mixed batch (q_lens is a host array)."""
+    _fields_ = _fields("int rows n_seqs; ptr q_lens; int max_kv_len; ptr cu_seqlens token_pos slot_mapping table_rows "
+                       "kv_lens block_tables; int max_blocks block_size")
+
+
+class VxLinearOut(C.Structure):
+    _fields_ = _fields("int kind out_f32 ldo cols slices; ptr out out2; int split ldo2; ptr bias; int k_col v_col kv_heads "
+                       "k_dim v_dim block_size; ptr pool slot_mapping")
+
+
+class VxResidualNormArgs(C.Structure):
+    _fields_ = _fields("int rows cols; ptr row_idx x_in add x_out y w_post; int y_slices ldy; i64 y_stride; float mult eps; "
+                       "ptr w_pre out; int ldo")
+
+
+class VxAttnArgs(C.Structure):
+    _fields_ = _fields("int heads kv_heads k_dim v_dim; float scale temp_coef; int temp_every; ptr bias; int bias_len; "
+                       "ptr q gate; int ldq ldg; ptr pool; float out_scale; ptr out; int ldo")
+
+
+class VxConvArgs(C.Structure):
+    _fields_ = _fields("int channels taps; ptr x; int ldx; ptr w b state out; int ldo")
+
+
+class VxScanArgs(C.Structure):
+    _fields_ = _fields("int channels states; ptr a2 d x z; int ldx ldz; ptr dt bc; int lddt; ptr state; float out_scale; "
+                       "ptr out; int ldo out_cols")
+
+
 class VexelError(RuntimeError):
     def __init__(self, code, msg):
         super().__init__("vexel_hip error %d: %s" % (code, msg))
@@ -388,6 +428,31 @@ class HipBackend:
         self.call("vx_pack_batch", seq_slots, positions, q_lens, batch, total_tokens, block_tables, max_blocks,
                   num_blocks, free_list, free_count, block_size, cu_seqlens, token_pos, slot_mapping, kv_lens,
                   status)
+
+    # ---- ragged mixed batches (structures: VxRagged and the Vx*Args above)
+    def fill_zero(self, dst, nbytes):
+        self.call("vx_fill_zero", dst, nbytes)
+
+    def linear_pack(self, src, n, k, dst, n_pad, k_pad, tile0=0, tile_step=1, col0=0):
+        self.call("vx_linear_pack", src, n, k, dst, n_pad, k_pad, tile0, tile_step, col0)
+
+    def linear_slices(self, n, k, rows):
+        return self._lib.vx_linear_slices(self._h, n, k, rows)
+
+    def linear(self, act, a, lda, w, n, k, rows, out):
+        self.call("vx_linear", act, a, lda, w, n, k, rows, C.byref(out))
+
+    def residual_norm(self, act, args):
+        self.call("vx_residual_norm", act, C.byref(args))
+
+    def attn_ragged(self, act, batch, args):
+        self.call("vx_attn_ragged", act, C.byref(batch), C.byref(args))
+
+    def conv_silu(self, act, batch, args):
+        self.call("vx_conv_silu", act, C.byref(batch), C.byref(args))
+
+    def selective_scan(self, act, batch, args):
+        self.call("vx_selective_scan", act, C.byref(batch), C.byref(args))
 
     # ---- graph capture / timing
     def graph_begin_capture(self):

@@ -12,7 +12,9 @@ HOST_LIB = os.path.join(HERE, "libvexel_host.so")
 SYNTH_LIB = os.path.join(HERE, "libvexel_synth.so")
 OBJ_DIR = os.path.join(HERE, "build")
 
-SOURCES = ["backend.hip", "elementwise.hip", "attention.hip", "qgemm.hip", "qstream.hip", "qmatvec.hip", "pack.hip", "sampler.hip", "medusa.hip"]
+SOURCES = ["backend.hip", "elementwise.hip", "attention.hip", "qgemm.hip", "qstream.hip", "qmatvec.hip", "pack.hip", "sampler.hip", "medusa.hip",
+           "linear.hip", "mixers.hip", "attn_ragged.hip"]
+HOST_SOURCES = ["runtime.cpp", "gguf.cpp", "scheduler.cpp", "layers.cpp", "checkpoint.cpp"]
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 FLAGS = ["-O3", "--offload-arch=gfx950", "-fPIC", "-std=c++17", "-fvisibility=default",
@@ -36,8 +38,14 @@ def _compile(src):
     return obj
 
 
-def build(verbose=True):
-    """Compiles every source and links the shared library. Always rebuilds."""
+def is_built():
+    """Whether the product's libraries are there."""
+    return os.path.exists(LIB) and os.path.exists(HOST_LIB)
+
+
+def build(verbose=True, bench_support=True):
+    """Compiles every source and links the shared libraries. Always rebuilds. bench_support: the synthetic-weight
+    generators of the benchmarks as well."""
     os.makedirs(OBJ_DIR, exist_ok=True)
     with ThreadPoolExecutor(max_workers=min(8, len(SOURCES))) as ex:
         objs = list(ex.map(_compile, SOURCES))
@@ -48,17 +56,17 @@ def build(verbose=True):
     if verbose:
         print("built", LIB)
     # benchmark support (synthetic weights / KV made on the device); not part of the C ABI
-    cmd = [HIPCC] + FLAGS + ["-shared", os.path.join(CSRC, "synth.hip"), "-o", SYNTH_LIB]
-    r = subprocess.run(cmd, capture_output=True, text=True)
-    if r.returncode != 0:
-        raise RuntimeError("synth build failed:\n" + r.stderr)
-    if verbose:
-        print("built", SYNTH_LIB)
+    if bench_support:
+        cmd = [HIPCC] + FLAGS + ["-shared", os.path.join(CSRC, "synth.hip"), "-o", SYNTH_LIB]
+        r = subprocess.run(cmd, capture_output=True, text=True)
+        if r.returncode != 0:
+            raise RuntimeError("synth build failed:\n" + r.stderr)
+        if verbose:
+            print("built", SYNTH_LIB)
     # host runtime: plain C++ above the C ABI (links the HIP library, finds it next to itself)
-    cmd = ["g++", "-O2", "-std=c++17", "-fPIC", "-shared", "-Wall", "-I" + os.path.join(ROOT, "include"),
-           os.path.join(HERE, "host", "runtime.cpp"), os.path.join(HERE, "host", "gguf.cpp"),
-           os.path.join(HERE, "host", "scheduler.cpp"), "-o", HOST_LIB, "-L" + HERE, "-lvexel_hip",
-           "-Wl,-rpath,$ORIGIN", "-pthread"]
+    cmd = ["g++", "-O2", "-std=c++17", "-fPIC", "-shared", "-Wall", "-I" + os.path.join(ROOT, "include")]
+    cmd += [os.path.join(HERE, "host", f) for f in HOST_SOURCES]
+    cmd += ["-o", HOST_LIB, "-L" + HERE, "-lvexel_hip", "-Wl,-rpath,$ORIGIN", "-pthread"]
     r = subprocess.run(cmd, capture_output=True, text=True)
     if r.returncode != 0:
         raise RuntimeError("host runtime build failed:\n" + r.stderr)

@@ -1,0 +1,597 @@
+// Causal grouped-query attention over a paged pool for mixed batches, with a per-head distance bias, a query temperature and
+// an output gate (vx_attn_ragged).
+//
+//  * prefill_kernel: sequences that bring several rows. A wave owns QT x 16 (row, head) pairs of one K/V head and walks
+//    the keys in groups of 32 (two 16-token blocks); the four waves of a workgroup walk the same keys.
+//  * decode_kernel + merge_kernel: sequences that bring one row. A workgroup takes a piece of one sequence's keys for all
+//    query heads of one K/V head, its waves every fourth group; the pieces' partial results are merged by a second
+//    launch, which also applies the gate.
+//  * plain_kernel: one workgroup per (row, head), any geometry, and everything in float32 batches.
+//
+// Matrix products of the first two: S^T = K Q^T and O^T = V^T P^T on the bfloat16 matrix cores. The keys of a group are
+// dealt to the two 16-row tiles of S^T so that a lane ends with eight consecutive keys of one query, which is the
+// operand layout of the second product; V lies transposed in the pool, so that its operand is eight consecutive keys
+// of one dimension as well, and nothing passes through LDS. The weights P are float32 and enter the second product as
+// two bfloat16 parts (16 bits of the 24). Scores, bias, softmax and sums are float32.
+#include <string.h>
+
+#include "ragged.h"
+
+using namespace vx;
+
+namespace {
+
+constexpr float kLog2e = 1.4426950408889634f;
+constexpr int BS = 16;               // tokens of a block (matrix-core kernels)
+constexpr int LUT_LDS = 12 * 1024;   // floats of bias tables kept in LDS
+
+struct Args {
+    vx_attn_args p;
+    const int32_t *cu, *pos, *rows, *kv_lens, *tables;
+    int n_seqs, max_blocks, block_size, one_token;
+    int kp;            // k_dim up to a multiple of 8
+    int group;         // query heads per K/V head
+    int vec_q, vec_o;  // vector access to q / gate and out
+    int lut_lds;
+    // prefill
+    int tile_rows, tiles;
+    // decode
+    const int32_t *items;
+    int piece, pieces;
+    float *partial;
+};
+
+__device__ __forceinline__ float temperature(const vx_attn_args &p, int pos) {
+    if (p.temp_every <= 0) return 1.0f;
+    return 1.0f + p.temp_coef * logf((float)((pos + 1) / p.temp_every) + 1.0f);
+}
+
+__device__ __forceinline__ bf16x8 zero8() {
+    bf16x8 z;
+#pragma unroll
+    for (int i = 0; i < 8; i++) z[i] = (bf16)0.f;
+    return z;
+}
+
+__device__ __forceinline__ bf16x8 load_q(const bf16 *q, int d, int dim, bool vec) {
+    if (vec) return d < dim ? *(const bf16x8 *)(q + d) : zero8();
+    bf16x8 v = zero8();
+#pragma unroll
+    for (int i = 0; i < 8; i++)
+        if (d + i < dim) v[i] = q[d + i];
+    return v;
+}
+
+template <bool NT> __device__ __forceinline__ bf16x8 ld8(const bf16 *p) {
+    return NT ? __builtin_nontemporal_load((const bf16x8 *)p) : *(const bf16x8 *)p;
+}
+
+// The keys of one group of 32 for a wave: K as two 16 x (32 KD) operands, V^T as VD 16 x 32 operands.
+template <int KD, int VD, bool NT> struct Keys {
+    bf16x8 k[2][KD];
+    bf16x8 v[VD];
+    // lane addresses inside a block
+    int ko[2], kd, vo, k_sel, v_sel, kp, v_rows;
+    const bf16 *pool;
+    size_t blk;
+    __device__ __forceinline__ void init(const Args &a, int g, int lane) {
+        const int i = lane & 15, q = lane >> 4;
+        pool = (const bf16 *)a.p.pool;
+        kp = a.kp, kd = q * 8, v_rows = a.p.v_dim;
+        blk = (size_t)a.p.kv_heads * BS * (kp + v_rows);
+        k_sel = i >> 3, v_sel = q >> 1;
+#pragma unroll
+        for (int t = 0; t < 2; t++) ko[t] = (g * BS + ((i >> 2) & 1) * 8 + t * 4 + (i & 3)) * kp;
+        vo = a.p.kv_heads * BS * kp + g * v_rows * BS + (q & 1) * 8;
+    }
+    __device__ __forceinline__ void load_k(int b0, int b1) {
+        const bf16 *base = pool + (size_t)(k_sel ? b1 : b0) * blk;
+#pragma unroll
+        for (int kk = 0; kk < KD; kk++) {
+            const int d = kk * 32 + kd;
+#pragma unroll
+            for (int t = 0; t < 2; t++) k[t][kk] = d < kp ? ld8<NT>(base + ko[t] + d) : zero8();
+        }
+    }
+    __device__ __forceinline__ void load_v(int b0, int b1, int lane) {
+        const bf16 *base = pool + (size_t)(v_sel ? b1 : b0) * blk + vo;
+#pragma unroll
+        for (int t = 0; t < VD; t++) v[t] = ld8<NT>(base + min(t * 16 + (lane & 15), v_rows - 1) * BS);
+    }
+};
+
+// The running softmax and output of QT x 16 queries of a wave.
+template <int KD, int VD, int QT> struct Queries {
+    bf16x8 q[QT][KD];
+    f32x4 o[QT][VD];
+    float m[QT], l[QT];       // l: this lane's share of the sum
+    float qs[QT], far[QT];    // score factor, bias of the last table entry (both for base-2 exponentials)
+    int pos[QT], lut[QT];     // position; the head's table
+    __device__ __forceinline__ void clear() {
+#pragma unroll
+        for (int t = 0; t < QT; t++) {
+            m[t] = -INFINITY, l[t] = 0.f;
+#pragma unroll
+            for (int v = 0; v < VD; v++) o[t][v] = f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+    }
+    // One group: keys k0 .. k0 + 31. Every key is visible to every query when `whole`; every distance is in the last
+    // bias entry when `distant`.
+    template <bool NT>
+    __device__ __forceinline__ void step(const Args &a, const Keys<KD, VD, NT> &ks, f32x4 st0, f32x4 st1, int t, int k0, int lane, bool whole, bool distant,
+                         const float *s_lut) {
+        const int key = k0 + (lane >> 4) * 8;
+        float s[8];
+        if (distant || !a.p.bias) {
+#pragma unroll
+            for (int j = 0; j < 8; j++) s[j] = fmaf((j < 4 ? st0[j & 3] : st1[j & 3]), qs[t], far[t]);
+        } else {
+            const int last = a.p.bias_len - 1, n0 = pos[t] - key;
+#pragma unroll
+            for (int j = 0; j < 8; j++) {
+                const int n = min(max(n0 - j, 0), last) + lut[t];
+                const float b = a.lut_lds ? s_lut[n] : a.p.bias[n] * kLog2e;
+                s[j] = fmaf((j < 4 ? st0[j & 3] : st1[j & 3]), qs[t], b);
+            }
+        }
+        if (!whole) {
+#pragma unroll
+            for (int j = 0; j < 8; j++)
+                if (key + j > pos[t]) s[j] = -INFINITY;
+        }
+        float mx = s[0];
+#pragma unroll
+        for (int j = 1; j < 8; j++) mx = fmaxf(mx, s[j]);
+        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        const float mn = fmaxf(m[t], mx);
+        if (__any(mn > m[t])) {
+            const float al = mn > -INFINITY ? __builtin_amdgcn_exp2f(m[t] - mn) : 1.0f;
+            l[t] *= al;
+#pragma unroll
+            for (int v = 0; v < VD; v++) o[t][v] *= al;
+            m[t] = mn;
+        }
+        const float ref = mn > -INFINITY ? mn : 0.f;
+        bf16x8 hi, lo;
+#pragma unroll
+        for (int j = 0; j < 8; j++) {
+            const float e = __builtin_amdgcn_exp2f(s[j] - ref);
+            l[t] += e;
+            hi[j] = (bf16)e;
+            lo[j] = (bf16)(e - (float)hi[j]);
+        }
+#pragma unroll
+        for (int v = 0; v < VD; v++) {
+            o[t][v] = mma(ks.v[v], hi, o[t][v]);
+            o[t][v] = mma(ks.v[v], lo, o[t][v]);
+        }
+    }
+};
+
+template <int KD, int VD, int QT, bool NT>
+__device__ __forceinline__ void group(const Args &a, Keys<KD, VD, NT> &ks, Queries<KD, VD, QT> &qs, int k0, int next_b0, int next_b1,
+                                      bool more, int lane, bool whole, bool distant, const float *s_lut) {
+    f32x4 st[QT][2];
+#pragma unroll
+    for (int t = 0; t < QT; t++)
+#pragma unroll
+        for (int h = 0; h < 2; h++) {
+            st[t][h] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kk = 0; kk < KD; kk++) st[t][h] = mma(ks.k[h][kk], qs.q[t][kk], st[t][h]);
+        }
+    if (more) ks.load_k(next_b0, next_b1);
+#pragma unroll
+    for (int t = 0; t < QT; t++) qs.step(a, ks, st[t][0], st[t][1], t, k0, lane, whole, distant, s_lut);
+}
+
+// bias tables of the workgroup's heads, times log2(e)
+__device__ __forceinline__ void load_lut(const Args &a, int g, float *s_lut) {
+    if (a.lut_lds) {
+        const float *src = a.p.bias + (size_t)g * a.group * a.p.bias_len;
+        for (int i = threadIdx.x; i < a.group * a.p.bias_len; i += blockDim.x) s_lut[i] = src[i] * kLog2e;
+        __syncthreads();
+    }
+}
+
+__device__ __forceinline__ void write4(const Args &a, int row, int h, int d, f32x4 v) {
+    const vx_attn_args &p = a.p;
+    const bf16 *gate = p.gate ? (const bf16 *)p.gate + (size_t)row * p.ldg + h * p.v_dim + d : nullptr;
+    bf16 *out = (bf16 *)p.out + (size_t)row * p.ldo + h * p.v_dim + d;
+    if (a.vec_o) {  // v_dim is a multiple of 4
+        if (d >= p.v_dim) return;
+        if (gate) {
+            const bf16x4 g4 = *(const bf16x4 *)gate;
+#pragma unroll
+            for (int r = 0; r < 4; r++) v[r] *= sigmoid_f((float)g4[r]);
+        }
+        store4(out, v * p.out_scale);
+    } else {
+#pragma unroll
+        for (int r = 0; r < 4; r++)
+            if (d + r < p.v_dim) out[r] = (bf16)(v[r] * (gate ? sigmoid_f((float)gate[r]) : 1.0f) * p.out_scale);
+    }
+}
+
+template <int KD, int VD, int QT>
+__global__ void __launch_bounds__(256) prefill_kernel(Args a) {
+    extern __shared__ float s_lut[];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int g = blockIdx.x % a.p.kv_heads, id = a.tiles - 1 - blockIdx.x / a.p.kv_heads;  // late tiles, the longest, first
+    int seq, ti, count;
+    if (!item_of_seq(a.cu, a.n_seqs, a.tile_rows, 2, id, &seq, &ti, &count)) return;
+    load_lut(a, g, s_lut);
+    const int row0 = a.cu[seq] + ti * a.tile_rows, ntok = min(a.tile_rows, a.cu[seq + 1] - row0);
+    const int pos0 = a.pos[row0];
+    const int m_first = wave * 16 * QT;
+    if (m_first >= ntok * a.group) return;  // (no barrier follows)
+    const int32_t *bt = a.tables + (size_t)a.rows[seq] * a.max_blocks;
+    const int t_lo = m_first / a.group, t_hi = min((m_first + 16 * QT - 1) / a.group, ntok - 1);
+    const int pos_lo = pos0 + t_lo, pos_hi = pos0 + t_hi, last_blk = pos_hi / BS, groups = pos_hi / 32 + 1;
+
+    Queries<KD, VD, QT> qs;
+    qs.clear();
+    int tok[QT], head[QT];
+#pragma unroll
+    for (int t = 0; t < QT; t++) {
+        const int m = m_first + t * 16 + (lane & 15);
+        tok[t] = m / a.group, head[t] = g * a.group + m % a.group;
+        const int tt = min(tok[t], ntok - 1);
+        qs.pos[t] = pos0 + tt;
+        qs.lut[t] = (a.lut_lds ? m % a.group : head[t]) * a.p.bias_len;
+        qs.qs[t] = a.p.scale * temperature(a.p, qs.pos[t]) * kLog2e;
+        qs.far[t] = a.p.bias ? a.p.bias[(size_t)head[t] * a.p.bias_len + a.p.bias_len - 1] * kLog2e : 0.f;
+        const bf16 *q = (const bf16 *)a.p.q + (size_t)(row0 + tt) * a.p.ldq + head[t] * a.p.k_dim;
+#pragma unroll
+        for (int kk = 0; kk < KD; kk++) qs.q[t][kk] = load_q(q, kk * 32 + (lane >> 4) * 8, a.p.k_dim, a.vec_q);
+    }
+    Keys<KD, VD, false> ks;
+    ks.init(a, g, lane);
+    int b0 = bt[0], b1 = bt[min(1, last_blk)];
+    ks.load_k(b0, b1);
+    for (int gi = 0; gi < groups; gi++) {
+        ks.load_v(b0, b1, lane);
+        const bool more = gi + 1 < groups;
+        if (more) b0 = bt[min(2 * gi + 2, last_blk)], b1 = bt[min(2 * gi + 3, last_blk)];
+        const int k0 = gi * 32;
+        group<KD, VD, QT, false>(a, ks, qs, k0, b0, b1, more, lane, k0 + 31 <= pos_lo, pos_lo - (k0 + 31) >= a.p.bias_len - 1, s_lut);
+    }
+#pragma unroll
+    for (int t = 0; t < QT; t++) {
+        float l = qs.l[t];
+        l += __shfl_xor(l, 16, 64);
+        l += __shfl_xor(l, 32, 64);
+        if (tok[t] >= ntok) continue;
+        const float inv = 1.0f / l;  // (a row sees itself: l > 0)
+#pragma unroll
+        for (int v = 0; v < VD; v++) write4(a, row0 + tok[t], head[t], v * 16 + (lane >> 4) * 4, qs.o[t][v] * inv);
+    }
+}
+
+template <int KD, int VD>
+__global__ void __launch_bounds__(256) decode_kernel(Args a) {
+    constexpr int QT = 1;
+    extern __shared__ float s_dyn[];
+    __shared__ float s_m[4][QT * 16], s_l[4][QT * 16];
+    float *s_lut = s_dyn;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int g = blockIdx.x % a.p.kv_heads, h0 = blockIdx.x / a.p.kv_heads * 16;  // 16 of the group's query heads
+    int seq, piece;
+    if (a.items) {
+        if ((int)blockIdx.y >= a.items[0]) return;
+        seq = a.items[4 + 4 * blockIdx.y], piece = a.items[5 + 4 * blockIdx.y];
+    } else {
+        piece = blockIdx.y, seq = blockIdx.z;
+    }
+    const int row = a.one_token ? seq : a.cu[seq];
+    if (!a.one_token && a.cu[seq + 1] - row != 1) return;
+    const int len = a.kv_lens[seq], k_lo = piece * a.piece, k_hi = min(len, k_lo + a.piece);
+    if (k_lo >= len) return;
+    load_lut(a, g, s_lut);
+    const int pos = len - 1, last_blk = pos / BS;
+    const int32_t *bt = a.tables + (size_t)a.rows[seq] * a.max_blocks;
+
+    Queries<KD, VD, QT> qs;
+    qs.clear();
+    const float temp = temperature(a.p, pos);
+#pragma unroll
+    for (int t = 0; t < QT; t++) {
+        const int hh = min(h0 + (lane & 15), a.group - 1), h = g * a.group + hh;
+        qs.pos[t] = pos;
+        qs.lut[t] = (a.lut_lds ? hh : h) * a.p.bias_len;
+        qs.qs[t] = a.p.scale * temp * kLog2e;
+        qs.far[t] = a.p.bias ? a.p.bias[(size_t)h * a.p.bias_len + a.p.bias_len - 1] * kLog2e : 0.f;
+        const bf16 *q = (const bf16 *)a.p.q + (size_t)row * a.p.ldq + h * a.p.k_dim;
+#pragma unroll
+        for (int kk = 0; kk < KD; kk++) qs.q[t][kk] = load_q(q, kk * 32 + (lane >> 4) * 8, a.p.k_dim, a.vec_q);
+    }
+    Keys<KD, VD, true> ks;
+    ks.init(a, g, lane);
+    const int g_hi = (k_hi + 31) / 32;
+    int gi = k_lo / 32 + wave;
+    if (gi < g_hi) {
+        int b0 = bt[min(2 * gi, last_blk)], b1 = bt[min(2 * gi + 1, last_blk)];
+        ks.load_k(b0, b1);
+        for (; gi < g_hi; gi += 4) {
+            ks.load_v(b0, b1, lane);
+            const bool more = gi + 4 < g_hi;
+            if (more) b0 = bt[min(2 * gi + 8, last_blk)], b1 = bt[min(2 * gi + 9, last_blk)];
+            const int k0 = gi * 32;
+            group<KD, VD, QT, true>(a, ks, qs, k0, b0, b1, more, lane, k0 + 31 <= pos, pos - (k0 + 31) >= a.p.bias_len - 1, s_lut);
+        }
+    }
+    // the four waves' results become one
+#pragma unroll
+    for (int t = 0; t < QT; t++) {
+        float l = qs.l[t];
+        l += __shfl_xor(l, 16, 64);
+        l += __shfl_xor(l, 32, 64);
+        if (lane < 16) s_m[wave][t * 16 + lane] = qs.m[t], s_l[wave][t * 16 + lane] = l;
+    }
+    __syncthreads();  // (the bias tables in s_dyn are done with as well)
+    float *s_o = s_dyn;  // [QT * 16][VD * 16 + 4]
+    constexpr int LDO = VD * 16 + 4;
+    for (int w = 0; w < 4; w++) {
+        if (wave == w) {
+#pragma unroll
+            for (int t = 0; t < QT; t++) {
+                const int c = t * 16 + (lane & 15);
+                const float mg = fmaxf(fmaxf(s_m[0][c], s_m[1][c]), fmaxf(s_m[2][c], s_m[3][c]));
+                const float f = qs.m[t] > -INFINITY ? __builtin_amdgcn_exp2f(qs.m[t] - mg) : 0.f;
+#pragma unroll
+                for (int v = 0; v < VD; v++) {
+                    f32x4 *dst = (f32x4 *)(s_o + c * LDO + v * 16 + (lane >> 4) * 4);
+                    const f32x4 x = qs.o[t][v] * f;
+                    *dst = w == 0 ? x : *dst + x;
+                }
+            }
+        }
+        __syncthreads();
+    }
+    const int vd = a.p.v_dim;
+    for (int hh = wave; hh < min(16, a.group - h0); hh += 4) {
+        float *dst = a.partial + (((size_t)seq * a.p.heads + g * a.group + h0 + hh) * a.pieces + piece) * (vd + 2);
+        float mg = -INFINITY, l = 0.f;
+        for (int w = 0; w < 4; w++) mg = fmaxf(mg, s_m[w][hh]);
+        for (int w = 0; w < 4; w++) l += s_m[w][hh] > -INFINITY ? s_l[w][hh] * __builtin_amdgcn_exp2f(s_m[w][hh] - mg) : 0.f;
+        if (lane == 0) dst[0] = mg, dst[1] = l;
+        for (int d = lane; d < vd; d += 64) dst[2 + d] = s_o[hh * LDO + d];
+    }
+}
+
+__global__ void __launch_bounds__(64) merge_kernel(Args a) {
+    const int h = blockIdx.x, seq = blockIdx.y, vd = a.p.v_dim;
+    const int row = a.one_token ? seq : a.cu[seq];
+    if (!a.one_token && a.cu[seq + 1] - row != 1) return;
+    const int n = (a.kv_lens[seq] + a.piece - 1) / a.piece;
+    const float *src = a.partial + ((size_t)seq * a.p.heads + h) * a.pieces * (vd + 2);
+    float m = -INFINITY;
+    for (int i = threadIdx.x; i < n; i += 64) m = fmaxf(m, src[(size_t)i * (vd + 2)]);
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
+    float l = 0.f;
+    for (int i = 0; i < n; i++) l += src[(size_t)i * (vd + 2) + 1] * __builtin_amdgcn_exp2f(src[(size_t)i * (vd + 2)] - m);
+    const float inv = a.p.out_scale / l;
+    for (int d = threadIdx.x; d < vd; d += 64) {
+        float o = 0.f;
+#pragma unroll 4
+        for (int i = 0; i < n; i++)
+            o = fmaf(src[(size_t)i * (vd + 2) + 2 + d], __builtin_amdgcn_exp2f(src[(size_t)i * (vd + 2)] - m), o);
+        o *= inv;
+        if (a.p.gate) o *= sigmoid_f((float)((const bf16 *)a.p.gate)[(size_t)row * a.p.ldg + h * vd + d]);
+        ((bf16 *)a.p.out)[(size_t)row * a.p.ldo + h * vd + d] = (bf16)o;
+    }
+}
+
+// ---------------------------------------------------------------- any geometry
+constexpr int PL_CHUNK = 1024;
+
+template <typename T>
+__global__ void __launch_bounds__(256) plain_kernel(Args a) {
+    extern __shared__ float s_q[];  // [k_dim]
+    __shared__ float s_s[PL_CHUNK], s_red[4];
+    const vx_attn_args &p = a.p;
+    const int h = blockIdx.x, row = blockIdx.y, g = h / a.group, tid = threadIdx.x;
+    const int seq = a.one_token ? row : seq_of_row(a.cu, a.n_seqs, row);
+    const int pos = a.pos[row], len = pos + 1;
+    const int32_t *bt = a.tables + (size_t)a.rows[seq] * a.max_blocks;
+    const T *pool = (const T *)p.pool;
+    const size_t blk = (size_t)p.kv_heads * a.block_size * (a.kp + p.v_dim), vpart = (size_t)p.kv_heads * a.block_size * a.kp;
+    const T *q = (const T *)p.q + (size_t)row * p.ldq + h * p.k_dim;
+    const float qf = p.scale * temperature(p, pos);
+    for (int d = tid; d < p.k_dim; d += 256) s_q[d] = (float)q[d];
+    // thread t accumulates dimension t % width over the keys t / width, t / width + groups, ..; wider heads: several each
+    const int width = p.v_dim < 256 ? p.v_dim : 256, kg = 256 / width, md = tid % width, mg = tid / width;
+    constexpr int MAXV = 8;  // dimensions of a thread: v_dim <= 2048
+    float acc[MAXV];
+#pragma unroll
+    for (int i = 0; i < MAXV; i++) acc[i] = 0.f;
+    float m = -INFINITY, l = 0.f;
+    for (int c0 = 0; c0 < len; c0 += PL_CHUNK) {
+        const int cn = min(PL_CHUNK, len - c0);
+        __syncthreads();
+        float mx = -INFINITY;
+        for (int i = tid; i < cn; i += 256) {
+            const int key = c0 + i;
+            const T *k = pool + (size_t)bt[key / a.block_size] * blk + ((size_t)g * a.block_size + key % a.block_size) * a.kp;
+            float dot = 0.f;
+            for (int d = 0; d < p.k_dim; d++) dot = fmaf(s_q[d], (float)k[d], dot);
+            float s = dot * qf;
+            if (p.bias) s += p.bias[(size_t)h * p.bias_len + min(pos - key, p.bias_len - 1)];
+            s_s[i] = s;
+            mx = fmaxf(mx, s);
+        }
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) mx = fmaxf(mx, __shfl_xor(mx, off, 64));
+        if ((tid & 63) == 0) s_red[tid >> 6] = mx;
+        __syncthreads();
+        mx = fmaxf(fmaxf(s_red[0], s_red[1]), fmaxf(s_red[2], s_red[3]));
+        const float mn = fmaxf(m, mx), al = expf(m - mn);
+        float sum = 0.f;
+        for (int i = tid; i < cn; i += 256) {
+            const float e = expf(s_s[i] - mn);
+            s_s[i] = e;
+            sum += e;
+        }
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) sum += __shfl_xor(sum, off, 64);
+        __syncthreads();
+        if ((tid & 63) == 0) s_red[tid >> 6] = sum;
+        __syncthreads();
+        l = l * al + (s_red[0] + s_red[1] + s_red[2] + s_red[3]);
+        m = mn;
+        if (mg < kg)
+            for (int v = 0; v < MAXV; v++) {
+                const int d = md + v * 256;
+                if (d >= p.v_dim) break;
+                float t = acc[v] * al;
+                for (int i = mg; i < cn; i += kg) {
+                    const int key = c0 + i;
+                    t = fmaf(s_s[i],
+                             (float)pool[(size_t)bt[key / a.block_size] * blk + vpart + ((size_t)g * p.v_dim + d) * a.block_size +
+                                         key % a.block_size],
+                             t);
+                }
+                acc[v] = t;
+            }
+    }
+    __syncthreads();
+    float *s_acc = s_s;  // [kg][width]
+    for (int v = 0; v < MAXV; v++) {
+        const int d = md + v * 256;
+        if (v * 256 >= p.v_dim) break;
+        if (mg < kg) s_acc[mg * width + md] = acc[v];
+        __syncthreads();
+        if (mg == 0 && d < p.v_dim) {
+            float t = 0.f;
+            for (int i = 0; i < kg; i++) t += s_acc[i * width + md];
+            t = t / l * p.out_scale;
+            if (p.gate) t *= sigmoid_f((float)((const T *)p.gate)[(size_t)row * p.ldg + h * p.v_dim + d]);
+            ((T *)p.out)[(size_t)row * p.ldo + h * p.v_dim + d] = (T)t;
+        }
+        __syncthreads();
+    }
+}
+
+template <int KD, int VD, int QT>
+void launch_prefill(vx_backend *be, Args a, const vx_ragged *b) {
+    a.tile_rows = 64 * QT / a.group;
+    a.tiles = count_items(b, a.tile_rows, 2);
+    const size_t lds = a.lut_lds ? (size_t)a.group * a.p.bias_len * 4 : 0;
+    if (a.tiles > 0) prefill_kernel<KD, VD, QT><<<a.tiles * a.p.kv_heads, 256, lds, be->stream>>>(a);
+}
+
+template <int KD, int VD>
+void launch_decode(vx_backend *be, const Args &a, dim3 grid) {
+    const size_t lut = a.lut_lds ? (size_t)a.group * a.p.bias_len * 4 : 0, o = (size_t)16 * (VD * 16 + 4) * 4;
+    decode_kernel<KD, VD><<<grid, 256, lut > o ? lut : o, be->stream>>>(a);
+}
+
+template <int KD, int VD>
+int run_fast(vx_backend *be, Args a, const vx_ragged *b) {
+    bool any_many = false, any_one = !b->q_lens;
+    int64_t many = 0;
+    if (b->q_lens)
+        for (int s = 0; s < b->n_seqs; s++) {
+            any_many |= b->q_lens[s] > 1, any_one |= b->q_lens[s] == 1;
+            if (b->q_lens[s] > 1) many += b->q_lens[s];
+        }
+    if (any_many) {
+        // two query tiles a wave where that still gives the chip enough workgroups
+        if (VD <= 8 && a.group <= 64 && many * a.p.heads / 128 >= 384) {
+            if constexpr (VD <= 8) launch_prefill<KD, VD, 2>(be, a, b);
+        } else {
+            launch_prefill<KD, VD, 1>(be, a, b);
+        }
+        VX_CHECK_LAUNCH();
+    }
+    if (any_one) {
+        int cu = 256;
+        a.piece = 256;
+        if ((int64_t)b->n_seqs * a.p.kv_heads * ceil_div(b->max_kv_len, 256) < 2 * cu) a.piece = 128;
+        a.pieces = ceil_div(b->max_kv_len, a.piece);
+        const size_t bytes = (size_t)b->n_seqs * a.p.heads * a.pieces * (a.p.v_dim + 2) * 4;
+        int rc = ensure_ws(be, &be->attn_ws, &be->attn_ws_bytes, bytes, "attention");
+        if (rc) return rc;
+        a.partial = (float *)be->attn_ws;
+        be->split.batch = 0;  // (whatever an earlier call left there is gone)
+        dim3 grid(a.p.kv_heads, a.pieces, b->n_seqs);
+        // vx_pack_batch's list of pieces of 256 tokens, when it was made for this batch
+        if (a.piece == ATTN_TPW / 2 && be->items.valid && be->items.kv_lens == b->kv_lens && be->items.table_rows == b->table_rows &&
+            be->items.batch == b->n_seqs && b->n_seqs * (int64_t)a.pieces <= 65535 &&
+            2 * be->items.cap >= (size_t)b->n_seqs * a.pieces) {
+            a.items = be->items.buf + (be->items.cap + 1) * 4;
+            grid = dim3(a.p.kv_heads, b->n_seqs * a.pieces, 1);
+        }
+        grid.x *= ceil_div(a.group, 16);
+        launch_decode<KD, VD>(be, a, grid);
+        VX_CHECK_LAUNCH();
+        merge_kernel<<<dim3(a.p.heads, b->n_seqs), 64, 0, be->stream>>>(a);
+        VX_CHECK_LAUNCH();
+    }
+    return VX_OK;
+}
+
+}  // namespace
+
+extern "C" {
+
+size_t vx_kv_block_elems(int block_size, int kv_heads, int k_dim, int v_dim) {
+    if (block_size < 1 || kv_heads < 1 || k_dim < 1 || v_dim < 1) return 0;
+    return (size_t)kv_heads * block_size * (((k_dim + 7) & ~7) + v_dim);
+}
+
+int vx_attn_ragged_fast(int act, int block_size, int heads, int kv_heads, int k_dim, int v_dim) {
+    if (heads < 1 || kv_heads < 1 || heads % kv_heads) return 0;
+    const int wide = k_dim > v_dim ? k_dim : v_dim, group = heads / kv_heads;
+    return act == VX_ACT_BF16 && block_size == BS && k_dim >= 1 && v_dim >= 1 && wide <= 256 && group <= (wide <= 128 ? 64 : 16);
+}
+
+int vx_attn_ragged(vx_backend *be, int act, const vx_ragged *b, const vx_attn_args *p) {
+    int rc = enter(be);
+    if (rc) return rc;
+    rc = check_ragged(b, "vx_attn_ragged");
+    if (rc) return rc;
+    VX_REQUIRE(act == VX_ACT_F32 || act == VX_ACT_BF16, "vx_attn_ragged: unknown activation type %d", act);
+    VX_REQUIRE(p && p->heads >= 1 && p->kv_heads >= 1 && p->heads % p->kv_heads == 0 && p->k_dim >= 1 && p->v_dim >= 1 && p->q &&
+                   p->pool && p->out,
+               "vx_attn_ragged: bad arguments");
+    VX_REQUIRE(p->k_dim <= 2048 && p->v_dim <= 2048, "vx_attn_ragged: heads of %d / %d (at most 2048)", p->k_dim, p->v_dim);
+    VX_REQUIRE(p->ldq >= p->heads * p->k_dim && p->ldo >= p->heads * p->v_dim && (!p->gate || p->ldg >= p->heads * p->v_dim),
+               "vx_attn_ragged: bad strides");
+    VX_REQUIRE(!p->bias || p->bias_len >= 1, "vx_attn_ragged: empty bias table");
+    VX_REQUIRE(b->rows <= 65535 || vx_attn_ragged_fast(act, b->block_size, p->heads, p->kv_heads, p->k_dim, p->v_dim),
+               "vx_attn_ragged: %d rows in one step (at most 65535)", b->rows);
+    VX_REQUIRE(b->n_seqs <= 65535, "vx_attn_ragged: %d sequences", b->n_seqs);
+    Args a;
+    memset(&a, 0, sizeof a);
+    a.p = *p;
+    if (!a.p.bias) a.p.bias_len = 1;
+    a.cu = b->cu_seqlens, a.pos = b->token_pos, a.rows = b->table_rows, a.kv_lens = b->kv_lens, a.tables = b->block_tables;
+    a.n_seqs = b->n_seqs, a.max_blocks = b->max_blocks, a.block_size = b->block_size, a.one_token = b->q_lens ? 0 : 1;
+    a.kp = (p->k_dim + 7) & ~7;
+    a.group = p->heads / p->kv_heads;
+    a.vec_q = p->k_dim % 8 == 0 && p->ldq % 8 == 0 && (uintptr_t)p->q % 16 == 0;
+    a.vec_o = p->v_dim % 4 == 0 && p->ldo % 4 == 0 && (uintptr_t)p->out % 8 == 0 &&
+              (!p->gate || (p->ldg % 4 == 0 && (uintptr_t)p->gate % 8 == 0));
+    a.lut_lds = p->bias && (int64_t)a.group * p->bias_len <= LUT_LDS ? 1 : 0;
+    if (vx_attn_ragged_fast(act, b->block_size, p->heads, p->kv_heads, p->k_dim, p->v_dim)) {
+        const int wide = p->k_dim > p->v_dim ? p->k_dim : p->v_dim;
+        if (wide <= 64) return run_fast<2, 4>(be, a, b);
+        if (wide <= 96) return run_fast<3, 6>(be, a, b);
+        if (wide <= 128) return run_fast<4, 8>(be, a, b);
+        if (wide <= 192) return run_fast<6, 12>(be, a, b);
+        return run_fast<8, 16>(be, a, b);
+    }
+    const dim3 grid(p->heads, b->rows);
+    const size_t lds = (size_t)p->k_dim * 4;
+    if (act == VX_ACT_BF16)
+        plain_kernel<bf16><<<grid, 256, lds, be->stream>>>(a);
+    else
+        plain_kernel<float><<<grid, 256, lds, be->stream>>>(a);
+    VX_CHECK_LAUNCH();
+    return VX_OK;
+}
+
+}  // extern "C"

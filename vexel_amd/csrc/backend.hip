@@ -120,6 +120,7 @@ void vx_backend_destroy(vx_backend *be) {
     if (be->part_ws) (void)hipFree(be->part_ws);
     if (be->part_ws2) (void)hipFree(be->part_ws2);
     if (be->attn_ws) (void)hipFree(be->attn_ws);
+    if (be->scan_ws) (void)hipFree(be->scan_ws);
     if (be->sample_ws) (void)hipFree(be->sample_ws);
     if (be->items.buf) (void)hipFree(be->items.buf);
     if (be->misc_ws) (void)hipFree(be->misc_ws);

@@ -122,6 +122,8 @@ struct vx_backend {
         bool valid = false;
     } items;
     float *ones = nullptr;       // 64 floats of 1.0 on the device (row factors of an unscaled activation)
+    void *scan_ws = nullptr;     // chunk states of vx_selective_scan
+    size_t scan_ws_bytes = 0;
     void *sample_ws = nullptr;   // probabilities and sort keys of vx_sample_rows
     size_t sample_ws_bytes = 0;
     void *misc_ws = nullptr;     // small device staging (pointer tables, argmax result)

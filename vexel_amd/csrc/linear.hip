@@ -1,0 +1,465 @@
+// Linear maps with bfloat16 weights for mixed batches (vx_linear_pack, vx_linear).
+//
+// The weights lie in tiles of 16 outputs x 32 inputs, each stored in the order in which the 64 lanes of a wave hold a
+// matrix-core operand: a wave reads a tile as one contiguous kilobyte. Both kernels compute W * a^T, so that a lane ends
+// with four consecutive output columns of one activation row and stores them together.
+//
+//  * linear_few_kernel (up to 64 rows: decode steps): bound by the weight stream. A workgroup owns one row tile (two for
+//    gate|up pairs), its waves take every WAVES-th step of 32 inputs for all activation rows and meet once, in LDS.
+//  * linear_many_kernel (more rows: prompts): tiles of BM rows x BN outputs, four waves in a 2 x 2 grid; the activations go
+//    through LDS, double-buffered, the weight operands come straight from memory a step ahead.
+//
+// Activations are bfloat16 or float32 (template parameter T); with float32 the weights are widened and the float32
+// matrix instruction multiplies them, so that nothing is rounded to fewer bits.
+#include <type_traits>
+
+#include "ragged.h"
+
+using namespace vx;
+
+namespace {
+
+struct LinArgs {
+    const void *a;
+    const void *w;
+    int lda, n, k, rows;
+    vx_linear_out o;
+};
+
+__device__ __forceinline__ size_t kv_elem_k(const vx_linear_out &o, int slot, int g, int d) {
+    const int kp = (o.k_dim + 7) & ~7;
+    const size_t blk = (size_t)o.kv_heads * o.block_size * (kp + o.v_dim);
+    return (size_t)(slot / o.block_size) * blk + ((size_t)g * o.block_size + slot % o.block_size) * kp + d;
+}
+__device__ __forceinline__ size_t kv_elem_v(const vx_linear_out &o, int slot, int g, int d) {
+    const int kp = (o.k_dim + 7) & ~7;
+    const size_t blk = (size_t)o.kv_heads * o.block_size * (kp + o.v_dim);
+    return (size_t)(slot / o.block_size) * blk + (size_t)o.kv_heads * o.block_size * kp +
+           ((size_t)g * o.v_dim + d) * o.block_size + slot % o.block_size;
+}
+
+template <typename P>
+__device__ __forceinline__ void put4(P *row, int c, int cols, int ld, f32x4 v) {
+    if (c + 4 <= cols && (ld & 3) == 0) {
+        store4(row + c, v);
+    } else {
+#pragma unroll
+        for (int r = 0; r < 4; r++)
+            if (c + r < cols) row[c + r] = (P)v[r];
+    }
+}
+
+// Columns c .. c + 3 of activation row `row`.
+template <typename T, int KIND>
+__device__ __forceinline__ void emit(const LinArgs &p, int slice, int row, int c, f32x4 v) {
+    const vx_linear_out &o = p.o;
+    if (row >= p.rows) return;
+    if constexpr (KIND == VX_LIN_PLAIN) {
+        if (o.out_f32)
+            put4((float *)o.out + ((size_t)slice * p.rows + row) * o.ldo, c, o.cols, o.ldo, v);
+        else
+            put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
+    } else if constexpr (KIND == VX_LIN_SWIGLU) {
+        put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
+    } else if constexpr (KIND == VX_LIN_SPLIT) {
+        if (c < o.split)
+            put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
+        else
+            put4(o.out2 + (size_t)row * o.ldo2, c - o.split, o.ldo2, o.ldo2, v);
+    } else if constexpr (KIND == VX_LIN_SOFTPLUS) {
+        f32x4 u;
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            const float z = v[r] + (c + r < o.cols ? o.bias[c + r] : 0.f);
+            u[r] = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
+        }
+        put4((float *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, u);
+    } else {  // VX_LIN_KV: K and V columns leave for the pool (segments start at multiples of 16 columns)
+        const int kw = o.kv_heads * o.k_dim, vw = o.kv_heads * o.v_dim;
+        const int ck = c - o.k_col, cv = c - o.v_col;
+        if (ck >= 0 && ck < kw) {
+            const int slot = o.slot_mapping[row];
+            T *pool = (T *)o.pool;
+            if ((o.k_dim & 3) == 0) {
+                store4(pool + kv_elem_k(o, slot, ck / o.k_dim, ck % o.k_dim), v);
+            } else {
+#pragma unroll
+                for (int r = 0; r < 4; r++)
+                    if (ck + r < kw) pool[kv_elem_k(o, slot, (ck + r) / o.k_dim, (ck + r) % o.k_dim)] = (T)v[r];
+            }
+        } else if (cv >= 0 && cv < vw) {
+            const int slot = o.slot_mapping[row];
+            T *pool = (T *)o.pool;
+#pragma unroll
+            for (int r = 0; r < 4; r++)
+                if (cv + r < vw) pool[kv_elem_v(o, slot, (cv + r) / o.v_dim, (cv + r) % o.v_dim)] = (T)v[r];
+        } else {
+            put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
+        }
+    }
+}
+
+// ---------------------------------------------------------------- up to 64 rows
+template <typename T, int MT, int NT, int WAVES, int KIND>
+__global__ void __launch_bounds__(64 * WAVES) linear_few_kernel(LinArgs p) {
+    typedef typename Vec8<T>::type A8;
+    __shared__ f32x4 red[WAVES][NT * MT][64];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int steps = p.k >> 5, slices = gridDim.y, slice = blockIdx.y;
+    const int s0 = (int)((int64_t)steps * slice / slices), s1 = (int)((int64_t)steps * (slice + 1) / slices);
+    const int tile = blockIdx.x * NT;
+    const bf16 *w = (const bf16 *)p.w + ((size_t)tile * steps) * 512 + lane * 8;
+    const T *a[MT];
+#pragma unroll
+    for (int m = 0; m < MT; m++) a[m] = (const T *)p.a + (size_t)min(m * 16 + (lane & 15), p.rows - 1) * p.lda + (lane >> 4) * 8;
+    f32x4 acc[NT][MT];
+#pragma unroll
+    for (int t = 0; t < NT; t++)
+#pragma unroll
+        for (int m = 0; m < MT; m++) acc[t][m] = f32x4{0.f, 0.f, 0.f, 0.f};
+    constexpr int U = sizeof(T) == 4 ? 2 : 4;
+    int s = s0 + wave;
+    for (; s + (U - 1) * WAVES < s1; s += U * WAVES) {
+        bf16x8 wf[U][NT];
+        A8 af[U][MT];
+#pragma unroll
+        for (int u = 0; u < U; u++) {
+#pragma unroll
+            for (int t = 0; t < NT; t++)
+                wf[u][t] = __builtin_nontemporal_load((const bf16x8 *)(w + ((size_t)t * steps + s + u * WAVES) * 512));
+#pragma unroll
+            for (int m = 0; m < MT; m++) af[u][m] = *(const A8 *)(a[m] + (size_t)(s + u * WAVES) * 32);
+        }
+#pragma unroll
+        for (int u = 0; u < U; u++)
+#pragma unroll
+            for (int t = 0; t < NT; t++)
+#pragma unroll
+                for (int m = 0; m < MT; m++) acc[t][m] = mma(wf[u][t], af[u][m], acc[t][m]);
+    }
+    for (; s < s1; s += WAVES) {
+        bf16x8 wf[NT];
+#pragma unroll
+        for (int t = 0; t < NT; t++) wf[t] = __builtin_nontemporal_load((const bf16x8 *)(w + ((size_t)t * steps + s) * 512));
+#pragma unroll
+        for (int m = 0; m < MT; m++) {
+            const A8 af = *(const A8 *)(a[m] + (size_t)s * 32);
+#pragma unroll
+            for (int t = 0; t < NT; t++) acc[t][m] = mma(wf[t], af, acc[t][m]);
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < NT; t++)
+#pragma unroll
+        for (int m = 0; m < MT; m++) red[wave][t * MT + m][lane] = acc[t][m];
+    __syncthreads();
+    constexpr int ITEMS = (KIND == VX_LIN_SWIGLU ? 1 : NT) * MT * 64;
+    for (int i = threadIdx.x; i < ITEMS; i += 64 * WAVES) {
+        const int l = i & 63, tm = i >> 6, t = tm / MT, m = tm % MT;
+        f32x4 v = red[0][tm][l];
+#pragma unroll
+        for (int x = 1; x < WAVES; x++) v += red[x][tm][l];
+        const int row = m * 16 + (l & 15);
+        if constexpr (KIND == VX_LIN_SWIGLU) {
+            f32x4 u = red[0][MT + m][l];
+#pragma unroll
+            for (int x = 1; x < WAVES; x++) u += red[x][MT + m][l];
+#pragma unroll
+            for (int r = 0; r < 4; r++) v[r] = silu_f(v[r]) * u[r];
+            emit<T, KIND>(p, slice, row, (tile / 2) * 16 + (l >> 4) * 4, v);
+        } else {
+            emit<T, KIND>(p, slice, row, (tile + t) * 16 + (l >> 4) * 4, v);
+        }
+    }
+}
+
+// ---------------------------------------------------------------- more rows
+template <typename T, int BM, int BN, int KIND>
+__global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_tiles) {
+    typedef typename Vec8<T>::type A8;
+    constexpr int EPC = 16 / (int)sizeof(T);           // elements of a 16-byte piece
+    constexpr int CPR = 64 / EPC;                      // pieces of a 64-element row
+    constexpr int LOADS = BM * CPR / 256;              // pieces per thread and step
+    constexpr int MI = BM / 32, NI = BN / 32;          // 16-wide tiles per wave in each direction
+    typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+    extern __shared__ u32x4 lds[];                     // [2][BM][CPR], pieces of a row permuted by the row's low bits
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int wm = (wave & 1) * (BM / 2), wn = (wave >> 1) * NI;
+    const int rt = blockIdx.x % row_tiles, nt = blockIdx.x / row_tiles;  // the row tiles of one weight tile run together
+    const int m0 = rt * BM, tile0 = nt * (BN / 16);
+    const int n_tiles = p.n >> 4;
+    const int ktiles = p.k >> 6, slices = gridDim.y, slice = blockIdx.y;
+    const int k0 = (int)((int64_t)ktiles * slice / slices), k1 = (int)((int64_t)ktiles * (slice + 1) / slices);
+    const size_t steps = p.k >> 5;
+    auto piece = [](int row, int c) { return row * CPR + (c ^ ((row & 7) * (sizeof(T) == 4 ? 2 : 1))); };
+
+    const bf16 *w[NI];
+#pragma unroll
+    for (int t = 0; t < NI; t++) w[t] = (const bf16 *)p.w + (size_t)min(tile0 + wn + t, n_tiles - 1) * steps * 512 + lane * 8;
+    const u32x4 *ap[LOADS];
+    int dst[LOADS];
+#pragma unroll
+    for (int i = 0; i < LOADS; i++) {
+        const int idx = tid + i * 256, row = idx / CPR, c = idx % CPR;
+        ap[i] = (const u32x4 *)((const T *)p.a + (size_t)min(m0 + row, p.rows - 1) * p.lda) + c;
+        dst[i] = piece(row, c);
+    }
+    u32x4 ar[LOADS];
+    bf16x8 wf[2][NI];
+    auto fetch = [&](int kt) {
+#pragma unroll
+        for (int i = 0; i < LOADS; i++) ar[i] = ap[i][(size_t)kt * CPR];
+    };
+    auto fetch_w = [&](int kt) {
+#pragma unroll
+        for (int h = 0; h < 2; h++)
+#pragma unroll
+            for (int t = 0; t < NI; t++) wf[h][t] = *(const bf16x8 *)(w[t] + (size_t)(kt * 2 + h) * 512);
+    };
+    f32x4 acc[NI][MI];
+#pragma unroll
+    for (int t = 0; t < NI; t++)
+#pragma unroll
+        for (int m = 0; m < MI; m++) acc[t][m] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (k0 < k1) {
+        fetch(k0);
+        fetch_w(k0);
+    }
+    for (int kt = k0; kt < k1; kt++) {
+        u32x4 *buf = lds + ((kt - k0) & 1) * BM * CPR;
+#pragma unroll
+        for (int i = 0; i < LOADS; i++) buf[dst[i]] = ar[i];
+        bf16x8 cur[2][NI];
+#pragma unroll
+        for (int h = 0; h < 2; h++)
+#pragma unroll
+            for (int t = 0; t < NI; t++) cur[h][t] = wf[h][t];
+        __syncthreads();  // (the buffer written now was last read two steps ago, before the barrier of the step between)
+        if (kt + 1 < k1) {
+            fetch(kt + 1);
+            fetch_w(kt + 1);
+        }
+#pragma unroll
+        for (int h = 0; h < 2; h++) {
+            A8 af[MI];
+#pragma unroll
+            for (int m = 0; m < MI; m++) {
+                const int row = wm + m * 16 + (lane & 15), q = lane >> 4;
+                if constexpr (sizeof(T) == 2) {
+                    af[m] = *(const A8 *)(buf + piece(row, h * 4 + q));
+                } else {  // (the two pieces of eight floats stay neighbours)
+                    af[m] = *(const A8 *)(buf + piece(row, h * 8 + q * 2));
+                }
+            }
+#pragma unroll
+            for (int t = 0; t < NI; t++)
+#pragma unroll
+                for (int m = 0; m < MI; m++) acc[t][m] = mma(cur[h][t], af[m], acc[t][m]);
+        }
+    }
+    const int q4 = (lane >> 4) * 4;
+#pragma unroll
+    for (int m = 0; m < MI; m++) {
+        const int row = m0 + wm + m * 16 + (lane & 15);
+        if constexpr (KIND == VX_LIN_SWIGLU) {
+#pragma unroll
+            for (int t = 0; t < NI; t += 2) {
+                if (tile0 + wn + t >= n_tiles) continue;
+                f32x4 v;
+#pragma unroll
+                for (int r = 0; r < 4; r++) v[r] = silu_f(acc[t][m][r]) * acc[t + 1][m][r];
+                emit<T, KIND>(p, slice, row, (tile0 + wn + t) / 2 * 16 + q4, v);
+            }
+        } else {
+#pragma unroll
+            for (int t = 0; t < NI; t++)
+                if (tile0 + wn + t < n_tiles) emit<T, KIND>(p, slice, row, (tile0 + wn + t) * 16 + q4, acc[t][m]);
+        }
+    }
+}
+
+// ---------------------------------------------------------------- packing
+__global__ void linear_pack_kernel(const uint16_t *src, int n, int k, uint16_t *dst, int k_pad, int tile0, int tile_step, int col0) {
+    const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= (int64_t)n * k) return;
+    const int r = (int)(i / k), c = (int)(i % k) + col0;
+    const int tile = tile0 + (r >> 4) * tile_step, step = c >> 5, lane = (r & 15) + 16 * ((c & 31) >> 3);
+    dst[((size_t)tile * (k_pad >> 5) + step) * 512 + lane * 8 + (c & 7)] = src[i];
+}
+
+__global__ void fill_zero_kernel(uint32_t *p, size_t n) {
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) p[i] = 0;
+}
+
+// ---------------------------------------------------------------- launches
+template <typename T, int MT, int KIND>
+void launch_few(vx_backend *be, const LinArgs &p, int slices) {
+    constexpr int NT = KIND == VX_LIN_SWIGLU ? 2 : 1;
+    const int groups = (p.n >> 4) / NT;
+    // a narrow map gives the chip few workgroups: more waves each
+    if (groups * slices < 256)
+        linear_few_kernel<T, MT, NT, 16 / NT / (MT == 4 ? 2 : 1), KIND><<<dim3(groups, slices), 64 * (16 / NT / (MT == 4 ? 2 : 1)), 0, be->stream>>>(p);
+    else
+        linear_few_kernel<T, MT, NT, 8 / (MT == 4 && NT == 2 ? 2 : 1), KIND><<<dim3(groups, slices), 64 * (8 / (MT == 4 && NT == 2 ? 2 : 1)), 0, be->stream>>>(p);
+}
+
+template <typename T, int BM, int BN, int KIND>
+void launch_many(vx_backend *be, const LinArgs &p, int slices) {
+    const int rt = ceil_div(p.rows, BM), nt = ceil_div(p.n, BN);
+    linear_many_kernel<T, BM, BN, KIND><<<dim3(rt * nt, slices), 256, 2 * BM * 64 * sizeof(T), be->stream>>>(p, rt);
+}
+
+// The widest tiles that still give every compute unit a workgroup.
+void many_tile(int n, int rows, int slices, int *bm, int *bn) {
+    auto wgs = [&](int m, int nn) { return (int64_t)ceil_div(rows, m) * ceil_div(n, nn) * slices; };
+    *bm = 128, *bn = 128;
+    if (wgs(128, 128) >= 256) return;
+    *bm = 64;
+    if (wgs(64, 128) >= 256) return;
+    *bn = 64;
+}
+
+template <typename T, int KIND>
+int launch(vx_backend *be, const LinArgs &p, int slices) {
+    if (p.rows <= 64) {
+        if (p.rows <= 16)
+            launch_few<T, 1, KIND>(be, p, slices);
+        else if (p.rows <= 32)
+            launch_few<T, 2, KIND>(be, p, slices);
+        else
+            launch_few<T, 4, KIND>(be, p, slices);
+    } else {
+        int bm, bn;
+        many_tile(p.n, p.rows, slices, &bm, &bn);
+        if constexpr (sizeof(T) == 4) {
+            launch_many<T, 64, 64, KIND>(be, p, slices);
+        } else if (bn == 64) {
+            launch_many<T, 64, 64, KIND>(be, p, slices);
+        } else if (bm == 64) {
+            launch_many<T, 64, 128, KIND>(be, p, slices);
+        } else {
+            launch_many<T, 128, 128, KIND>(be, p, slices);
+        }
+    }
+    VX_CHECK_LAUNCH();
+    return VX_OK;
+}
+
+template <typename T>
+int dispatch(vx_backend *be, const LinArgs &p, int slices) {
+    switch (p.o.kind) {
+        case VX_LIN_PLAIN: return launch<T, VX_LIN_PLAIN>(be, p, slices);
+        case VX_LIN_SWIGLU: return launch<T, VX_LIN_SWIGLU>(be, p, slices);
+        case VX_LIN_KV: return launch<T, VX_LIN_KV>(be, p, slices);
+        case VX_LIN_SPLIT: return launch<T, VX_LIN_SPLIT>(be, p, slices);
+        default: return launch<T, VX_LIN_SOFTPLUS>(be, p, slices);
+    }
+}
+
+}  // namespace
+
+namespace vx {
+int check_ragged(const vx_ragged *b, const char *who) {
+    VX_REQUIRE(b != nullptr, "%s: null batch", who);
+    VX_REQUIRE(b->cu_seqlens && b->token_pos && b->slot_mapping && b->table_rows && b->kv_lens && b->block_tables,
+               "%s: null batch array", who);
+    VX_REQUIRE(b->rows >= 1 && b->n_seqs >= 1 && b->max_blocks >= 1 && b->block_size >= 1 && b->max_kv_len >= 1 &&
+                   b->max_kv_len <= (int64_t)b->max_blocks * b->block_size,
+               "%s: bad batch sizes", who);
+    if (b->q_lens) {
+        int64_t t = 0;
+        for (int s = 0; s < b->n_seqs; s++) {
+            VX_REQUIRE(b->q_lens[s] >= 1, "%s: sequence %d brings no rows", who, s);
+            t += b->q_lens[s];
+        }
+        VX_REQUIRE(t == b->rows, "%s: the sequences bring %lld rows, the batch has %d", who, (long long)t, b->rows);
+    } else {
+        VX_REQUIRE(b->rows == b->n_seqs, "%s: %d rows for %d sequences of one row", who, b->rows, b->n_seqs);
+    }
+    return VX_OK;
+}
+}  // namespace vx
+
+extern "C" {
+
+int vx_fill_zero(vx_backend *be, void *dst, size_t bytes) {
+    int rc = enter(be);
+    if (rc) return rc;
+    if (bytes == 0) return VX_OK;
+    VX_REQUIRE(dst && bytes % 4 == 0 && (uintptr_t)dst % 4 == 0, "vx_fill_zero: bad arguments");
+    items_written(be, dst, bytes);
+    const size_t n = bytes / 4;
+    const int grid = (int)(n / 256 + 1 < 4096 ? n / 256 + 1 : 4096);
+    fill_zero_kernel<<<grid, 256, 0, be->stream>>>((uint32_t *)dst, n);
+    VX_CHECK_LAUNCH();
+    return VX_OK;
+}
+
+size_t vx_linear_bytes(int n_pad, int k_pad) { return n_pad > 0 && k_pad > 0 ? (size_t)n_pad * k_pad * 2 : 0; }
+
+int vx_linear_pack(vx_backend *be, const void *src, int n, int k, void *dst, int n_pad, int k_pad, int tile0, int tile_step,
+                   int col0) {
+    int rc = enter(be);
+    if (rc) return rc;
+    VX_REQUIRE(src && dst && n > 0 && k > 0 && tile0 >= 0 && tile_step >= 1 && col0 >= 0, "vx_linear_pack: bad arguments");
+    VX_REQUIRE(n_pad % 16 == 0 && k_pad % 64 == 0 && col0 + k <= k_pad && tile0 + (int64_t)((n - 1) / 16) * tile_step < n_pad / 16,
+               "vx_linear_pack: [%d, %d] at tile %d (step %d), column %d does not fit [%d, %d]", n, k, tile0, tile_step, col0, n_pad,
+               k_pad);
+    linear_pack_kernel<<<(unsigned)ceil_div64((int64_t)n * k, 256), 256, 0, be->stream>>>((const uint16_t *)src, n, k, (uint16_t *)dst,
+                                                                                         k_pad, tile0, tile_step, col0);
+    VX_CHECK_LAUNCH();
+    return VX_OK;
+}
+
+int vx_linear_slices(vx_backend *be, int n, int k, int rows) {
+    (void)be;
+    if (n <= 0 || k <= 0 || rows <= 0) return 1;
+    const int most = k / 64 / 8 > 1 ? k / 64 / 8 : 1;  // at least 512 inputs a slice
+    int64_t wgs;
+    if (rows <= 64) {
+        wgs = n / 16;
+        if (wgs >= 192) return 1;
+    } else {
+        int bm, bn;
+        many_tile(n, rows, 1, &bm, &bn);
+        wgs = (int64_t)ceil_div(rows, bm) * ceil_div(n, bn);
+        if (wgs >= 192) return 1;
+    }
+    int s = (int)(256 / (wgs > 0 ? wgs : 1));
+    if (s > 8) s = 8;
+    if (s > most) s = most;
+    return s < 1 ? 1 : s;
+}
+
+int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, int n, int k, int rows, const vx_linear_out *o) {
+    int rc = enter(be);
+    if (rc) return rc;
+    VX_REQUIRE(a && w && o && o->out && rows >= 1, "vx_linear: bad arguments");
+    VX_REQUIRE(act == VX_ACT_F32 || act == VX_ACT_BF16, "vx_linear: unknown activation type %d", act);
+    VX_REQUIRE(n >= 16 && n % 16 == 0 && k >= 64 && k % 64 == 0 && lda >= k && lda % 8 == 0 && (uintptr_t)a % 16 == 0 &&
+                   (uintptr_t)w % 16 == 0 && (uintptr_t)o->out % 16 == 0,
+               "vx_linear: sizes or alignment (n %d, k %d, lda %d)", n, k, lda);
+    VX_REQUIRE(o->kind >= VX_LIN_PLAIN && o->kind <= VX_LIN_SOFTPLUS, "vx_linear: unknown kind %d", o->kind);
+    VX_REQUIRE(o->cols >= 1 && o->ldo >= o->cols, "vx_linear: %d columns in rows of %d", o->cols, o->ldo);
+    const int slices = o->slices > 1 ? o->slices : 1;
+    VX_REQUIRE(slices == 1 || (o->kind == VX_LIN_PLAIN && o->out_f32 && slices <= 64), "vx_linear: slices need a plain float32 result");
+    if (o->kind == VX_LIN_SWIGLU) {
+        VX_REQUIRE(n % 32 == 0 && o->cols <= n / 2, "vx_linear: gate|up pairs of %d rows for %d columns", n, o->cols);
+    } else if (o->kind == VX_LIN_SPLIT) {
+        VX_REQUIRE(o->out2 && o->split % 16 == 0 && o->split > 0 && o->split < n && o->cols == o->split && o->ldo2 >= n - o->split &&
+                       (uintptr_t)o->out2 % 16 == 0,
+                   "vx_linear: bad split");
+    } else {
+        VX_REQUIRE(o->cols <= n, "vx_linear: %d columns of %d", o->cols, n);
+    }
+    if (o->kind == VX_LIN_SOFTPLUS) VX_REQUIRE(o->bias != nullptr, "vx_linear: null bias");
+    if (o->kind == VX_LIN_KV)
+        VX_REQUIRE(o->pool && o->slot_mapping && o->kv_heads >= 1 && o->k_dim >= 1 && o->v_dim >= 1 && o->block_size >= 1 &&
+                       o->k_col % 16 == 0 && o->v_col % 16 == 0 && o->k_col >= 0 && o->v_col >= 0 &&
+                       o->k_col + o->kv_heads * o->k_dim <= n && o->v_col + o->kv_heads * o->v_dim <= n,
+                   "vx_linear: bad K/V columns");
+    LinArgs p{a, w, lda, n, k, rows, *o};
+    return act == VX_ACT_BF16 ? dispatch<bf16>(be, p, slices) : dispatch<float>(be, p, slices);
+}
+
+}  // extern "C"

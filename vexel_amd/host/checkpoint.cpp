@@ -1,0 +1,609 @@
+// Folders with config.json and model.safetensors: the readers of both, the registry of architectures and the builder that
+// turns a configuration and its tensors into a mixer program (model.h).
+//
+// A safetensors file is an 8-byte little-endian length, that many bytes of JSON (name -> dtype, shape, data_offsets) and
+// the data; it is mapped read-only. Matrices go to the device as they are and are packed there (vx_linear_pack); vectors and
+// small tables become float32 on the host.
+#include <errno.h>
+#include <fcntl.h>
+#include <math.h>
+#include <stdio.h>
+#include <stdlib.h>
+#include <string.h>
+#include <sys/mman.h>
+#include <sys/stat.h>
+#include <unistd.h>
+
+#include <utility>
+
+#include "model.h"
+
+namespace vh {
+namespace {
+
+// ---------------------------------------------------------------- JSON
+struct Json {
+    enum Type { NIL, BOOL, NUM, STR, ARR, OBJ } type = NIL;
+    bool b = false;
+    double num = 0;
+    std::string str;
+    std::vector<Json> arr;
+    std::vector<std::pair<std::string, Json>> obj;
+    const Json *get(const char *key) const {
+        for (const auto &kv : obj)
+            if (kv.first == key) return &kv.second;
+        return nullptr;
+    }
+    bool absent() const { return type == NIL; }
+};
+
+struct JsonReader {
+    const char *p, *end;
+    int depth = 0;
+    void space() {
+        while (p < end && (*p == ' ' || *p == '\t' || *p == '\n' || *p == '\r')) p++;
+    }
+    bool word(const char *w) {
+        const size_t n = strlen(w);
+        if ((size_t)(end - p) < n || memcmp(p, w, n)) return false;
+        p += n;
+        return true;
+    }
+    bool hex4(unsigned *u) {
+        if (end - p < 4) return false;
+        *u = 0;
+        for (int i = 0; i < 4; i++, p++) {
+            const char c = *p;
+            const int v = c >= '0' && c <= '9' ? c - '0' : c >= 'a' && c <= 'f' ? c - 'a' + 10 : c >= 'A' && c <= 'F' ? c - 'A' + 10 : -1;
+            if (v < 0) return false;
+            *u = *u * 16 + v;
+        }
+        return true;
+    }
+    bool string(std::string *out) {
+        if (p >= end || *p != '"') return false;
+        for (p++; p < end && *p != '"';) {
+            if (*p != '\\') {
+                out->push_back(*p++);
+                continue;
+            }
+            if (++p >= end) return false;
+            const char c = *p++;
+            switch (c) {
+                case 'n': out->push_back('\n'); break;
+                case 't': out->push_back('\t'); break;
+                case 'r': out->push_back('\r'); break;
+                case 'b': out->push_back('\b'); break;
+                case 'f': out->push_back('\f'); break;
+                case 'u': {  // as UTF-8; a surrogate pair makes one character
+                    unsigned u, lo;
+                    if (!hex4(&u)) return false;
+                    if (u >= 0xD800 && u < 0xDC00) {
+                        if (!word("\\u") || !hex4(&lo) || lo < 0xDC00 || lo > 0xDFFF) return false;
+                        u = 0x10000 + ((u - 0xD800) << 10) + (lo - 0xDC00);
+                    }
+                    if (u < 0x80) {
+                        out->push_back((char)u);
+                    } else {
+                        const int more = u < 0x800 ? 1 : u < 0x10000 ? 2 : 3;
+                        out->push_back((char)((more == 1 ? 0xC0 : more == 2 ? 0xE0 : 0xF0) | (u >> (6 * more))));
+                        for (int i = more - 1; i >= 0; i--) out->push_back((char)(0x80 | ((u >> (6 * i)) & 0x3F)));
+                    }
+                    break;
+                }
+                default: out->push_back(c);  // quote, backslash, slash
+            }
+        }
+        if (p >= end) return false;
+        p++;
+        return true;
+    }
+    bool value(Json *v) {
+        space();
+        if (p >= end || depth > 64) return false;
+        if (*p == '{' || *p == '[') {
+            const bool is_obj = *p++ == '{';
+            const char close = is_obj ? '}' : ']';
+            v->type = is_obj ? Json::OBJ : Json::ARR;
+            depth++;
+            space();
+            if (p < end && *p == close) {
+                p++, depth--;
+                return true;
+            }
+            for (;;) {
+                std::string key;
+                if (is_obj) {
+                    space();
+                    if (!string(&key)) return false;
+                    space();
+                    if (p >= end || *p++ != ':') return false;
+                }
+                Json e;
+                if (!value(&e)) return false;
+                if (is_obj)
+                    v->obj.emplace_back(std::move(key), std::move(e));
+                else
+                    v->arr.push_back(std::move(e));
+                space();
+                if (p >= end) return false;
+                const char c = *p++;
+                if (c == close) break;
+                if (c != ',') return false;
+            }
+            depth--;
+            return true;
+        }
+        if (*p == '"') {
+            v->type = Json::STR;
+            return string(&v->str);
+        }
+        if (word("null")) return true;
+        if (word("true") || word("false")) {
+            v->type = Json::BOOL;
+            v->b = p[-1] == 'e' && p[-2] == 'u';
+            return true;
+        }
+        std::string n;
+        while (p < end && (strchr("+-.eE", *p) || (*p >= '0' && *p <= '9'))) n.push_back(*p++);
+        char *stop = nullptr;
+        v->type = Json::NUM;
+        v->num = n.empty() ? 0 : strtod(n.c_str(), &stop);
+        return !n.empty() && stop && *stop == 0;
+    }
+};
+
+bool parse_json(const char *text, size_t n, Json *out) {
+    JsonReader r{text, text + n};
+    if (!r.value(out)) return false;
+    r.space();
+    return r.p == r.end;
+}
+
+// ---------------------------------------------------------------- safetensors
+struct Mapped {
+    const uint8_t *base = nullptr;
+    size_t size = 0;
+    ~Mapped() {
+        if (base) munmap((void *)base, size);
+    }
+    int open(const std::string &path) {
+        const int fd = ::open(path.c_str(), O_RDONLY | O_CLOEXEC);
+        if (fd < 0) return fail("%s: %s", path.c_str(), strerror(errno));
+        struct stat st;
+        void *p = MAP_FAILED;
+        if (fstat(fd, &st) == 0 && st.st_size > 0) p = mmap(nullptr, (size_t)st.st_size, PROT_READ, MAP_PRIVATE, fd, 0);
+        ::close(fd);
+        if (p == MAP_FAILED) return fail("%s: cannot be mapped", path.c_str());
+        base = (const uint8_t *)p, size = (size_t)st.st_size;
+        return VH_OK;
+    }
+};
+
+struct TensorView {
+    std::string dtype;
+    std::vector<int64_t> shape;
+    const uint8_t *data = nullptr;
+};
+
+struct SafeTensors {
+    Mapped file;
+    std::unordered_map<std::string, TensorView> tensors;
+    int open(const std::string &path) {
+        VHC(file.open(path));
+        uint64_t n = 0;
+        if (file.size < 8) return fail("%s: too short", path.c_str());
+        for (int i = 0; i < 8; i++) n |= (uint64_t)file.base[i] << (8 * i);
+        Json head;
+        if (n > file.size - 8 || !parse_json((const char *)file.base + 8, (size_t)n, &head) || head.type != Json::OBJ)
+            return fail("%s: no safetensors header", path.c_str());
+        const uint8_t *data = file.base + 8 + n;
+        const uint64_t room = file.size - 8 - n;
+        for (const auto &kv : head.obj) {
+            if (kv.first == "__metadata__") continue;
+            const Json *dt = kv.second.get("dtype"), *sh = kv.second.get("shape"), *off = kv.second.get("data_offsets");
+            if (!dt || dt->type != Json::STR || !sh || sh->type != Json::ARR || !off || off->type != Json::ARR || off->arr.size() != 2)
+                return fail("%s: %s: incomplete entry", path.c_str(), kv.first.c_str());
+            TensorView t;
+            t.dtype = dt->str;
+            uint64_t elems = 1;
+            for (const Json &d : sh->arr) {
+                if (d.type != Json::NUM || d.num < 0 || d.num > 1e12) return fail("%s: %s: bad shape", path.c_str(), kv.first.c_str());
+                t.shape.push_back((int64_t)d.num);
+                elems *= (uint64_t)d.num;
+            }
+            const int es = t.dtype == "BF16" || t.dtype == "F16" || t.dtype == "I16" ? 2 : t.dtype == "F32" || t.dtype == "I32" ? 4 : t.dtype == "I64" || t.dtype == "F64" ? 8 : 1;
+            const double lo = off->arr[0].num, hi = off->arr[1].num;
+            if (lo < 0 || hi < lo || hi > (double)room || (uint64_t)(hi - lo) != elems * es)
+                return fail("%s: %s: its bytes do not fit its shape or the file", path.c_str(), kv.first.c_str());
+            t.data = data + (uint64_t)lo;
+            tensors[kv.first] = std::move(t);
+        }
+        return VH_OK;
+    }
+};
+
+float bf16_to_f32(const uint8_t *p) {
+    const uint32_t u = ((uint32_t)p[0] | (uint32_t)p[1] << 8) << 16;
+    float f;
+    memcpy(&f, &u, 4);
+    return f;
+}
+
+// ---------------------------------------------------------------- configuration
+// Reads numbers out of nested objects; the first thing missing or out of range is kept as the error.
+struct Fields {
+    std::string where;
+    const Json *o;
+    int *rc;
+    Fields(const std::string &w, const Json *obj, int *r) : where(w), o(obj), rc(r) {
+        if ((!o || o->type != Json::OBJ) && *rc == VH_OK) *rc = fail("config.json: %s is not an object", where.c_str());
+    }
+    const Json *need(const char *key, Json::Type t) const {
+        const Json *v = o && o->type == Json::OBJ ? o->get(key) : nullptr;
+        if (v && v->type == t) return v;
+        if (*rc == VH_OK) *rc = fail("config.json: %s.%s is missing or of another type", where.c_str(), key);
+        return nullptr;
+    }
+    double num(const char *key) const {
+        const Json *v = need(key, Json::NUM);
+        return v ? v->num : 0;
+    }
+    int count(const char *key, int lo = 1, int hi = 1 << 24) const {
+        const double d = num(key);
+        if (*rc == VH_OK && (d != floor(d) || d < lo || d > hi)) *rc = fail("config.json: %s.%s = %g is not a whole number in %d..%d", where.c_str(), key, d, lo, hi);
+        return *rc == VH_OK ? (int)d : lo;
+    }
+    Fields sub(const char *key) const { return Fields(where + "." + key, o && o->type == Json::OBJ ? o->get(key) : nullptr, rc); }
+    bool has(const char *key) const {
+        const Json *v = o && o->type == Json::OBJ ? o->get(key) : nullptr;
+        return v && !v->absent();
+    }
+};
+
+// What a Lozedra config.json says, layer by layer.
+struct LozedraLayer {
+    int heads = 1, kv_heads = 1, dim = 1, vdim = 1, bias_max = 1, temp_every = 0;
+    float scale = 1.f, temp_coef = 0.f, left_scale = 1.f, right_scale = 1.f;
+    int inner = 1, state = 1, dt_rank = 1, conv = 1;
+    int ff = 0;  // 0: no feed-forward
+};
+struct LozedraConfig {
+    std::vector<LozedraLayer> layers;
+    int loop_start = 0, loop_stop = 0, loop_times = 1;
+    float eps = 1e-5f, mult = 1.f;
+    int vocab = 1, width = 1;
+};
+
+int parse_lozedra(const Json &j, LozedraConfig *c) {
+    int rc = VH_OK;
+    const Fields root("config", &j, &rc);
+    c->vocab = root.count("vocab");
+    c->width = root.count("width", 1, 1 << 20);
+    c->mult = (float)root.num("residual_mult");
+    c->eps = (float)root.sub("norm").num("eps");
+    const Json *layers = root.need("layers", Json::ARR);
+    if (rc != VH_OK) return rc;
+    if (layers->arr.empty()) return fail("config.json: no layers");
+    for (size_t i = 0; i < layers->arr.size(); i++) {
+        const Fields l("layers[" + std::to_string(i) + "]", &layers->arr[i], &rc);
+        const Json *type = l.need("type", Json::STR);
+        if (rc != VH_OK) return rc;
+        if (type->str != "parallel") return fail("config.json: layer %zu has the unknown mixer type '%s'", i, type->str.c_str());
+        LozedraLayer o;
+        const Fields mx = l.sub("mixer"), left = mx.sub("left"), right = mx.sub("right");
+        o.left_scale = (float)mx.num("left_scale"), o.right_scale = (float)mx.num("right_scale");
+        o.heads = left.count("heads", 1, 4096), o.kv_heads = left.count("kv_heads", 1, 4096);
+        o.dim = left.count("dim", 1, 2048), o.vdim = left.count("vdim", 1, 2048);
+        o.scale = (float)left.num("scale");
+        o.bias_max = left.count("bias_max");
+        if (left.has("q_temp")) {
+            const Fields q = left.sub("q_temp");
+            o.temp_coef = (float)q.num("coef"), o.temp_every = q.count("every");
+        }
+        o.inner = right.count("inner", 1, 1 << 20), o.state = right.count("state", 1, 256);
+        o.dt_rank = right.count("dt_rank", 1, 1 << 16), o.conv = right.count("conv", 1, 64);
+        if (l.has("mlp")) {
+            const Fields mlp = l.sub("mlp");
+            const Json *kind = mlp.need("kind", Json::STR);
+            if (rc == VH_OK && kind->str != "dense") return fail("config.json: layer %zu has the unknown feed-forward '%s'", i, kind->str.c_str());
+            o.ff = mlp.count("ff", 1, 1 << 20);
+        }
+        if (rc != VH_OK) return rc;
+        if (o.heads % o.kv_heads) return fail("config.json: layer %zu: %d heads are no multiple of %d", i, o.heads, o.kv_heads);
+        c->layers.push_back(o);
+    }
+    if (root.has("loop")) {
+        const Fields lp = root.sub("loop");
+        const int n = (int)c->layers.size();
+        c->loop_start = lp.count("start", 0, n), c->loop_stop = lp.count("stop", 0, n), c->loop_times = lp.count("times", 1, 4096);
+        if (rc == VH_OK && c->loop_stop < c->loop_start) return fail("config.json: loop of layers %d .. %d", c->loop_start, c->loop_stop);
+    }
+    return rc;
+}
+
+// ---------------------------------------------------------------- weights
+struct Builder {
+    vx_backend *be;
+    const SafeTensors *st;
+    vh_model *m;
+    void *stage = nullptr;       // device copy of the matrix being packed
+    size_t stage_bytes = 0;
+    int pad(int n, int to) const { return (n + to - 1) / to * to; }
+
+    ~Builder() {
+        if (stage) vx_free(be, stage);
+    }
+    int view(const std::string &name, std::vector<int64_t> shape, const TensorView **out) const {
+        const auto it = st->tensors.find(name);
+        if (it == st->tensors.end()) return fail("tensor %s is missing", name.c_str());
+        if (it->second.shape != shape) {
+            std::string want, have;
+            for (int64_t d : shape) want += " " + std::to_string(d);
+            for (int64_t d : it->second.shape) have += " " + std::to_string(d);
+            return fail("tensor %s: shape [%s ], the configuration needs [%s ]", name.c_str(), have.c_str(), want.c_str());
+        }
+        if (it->second.dtype != "BF16") return fail("tensor %s: type %s, not BF16", name.c_str(), it->second.dtype.c_str());
+        *out = &it->second;
+        return VH_OK;
+    }
+    int floats(const std::string &name, std::vector<int64_t> shape, std::vector<float> *out) const {
+        const TensorView *t;
+        VHC(view(name, shape, &t));
+        size_t n = 1;
+        for (int64_t d : shape) n *= (size_t)d;
+        out->resize(n);
+        for (size_t i = 0; i < n; i++) (*out)[i] = bf16_to_f32(t->data + 2 * i);
+        return VH_OK;
+    }
+    int upload(const std::vector<float> &v, const float **out) {
+        void *p = vx_alloc_permanent(be, (v.size() * 4 + 15) / 16 * 16 + 16);
+        if (!p) return fail("device memory: %s", vx_last_error());
+        m->adopted.push_back(p);
+        VXC(vx_to_device(be, p, v.data(), v.size() * 4));
+        *out = (const float *)p;
+        return VH_OK;
+    }
+    int vec(const std::string &name, int n, const float **out) {
+        std::vector<float> v;
+        VHC(floats(name, {n}, &v));
+        return upload(v, out);
+    }
+    int packed(Linear *w, int n, int k) {
+        w->n = pad(n, 16), w->k = pad(k, 64);
+        w->w = vx_alloc_permanent(be, vx_linear_bytes(w->n, w->k));
+        if (!w->w) return fail("device memory: %s", vx_last_error());
+        m->adopted.push_back(w->w);
+        VXC(vx_fill_zero(be, w->w, vx_linear_bytes(w->n, w->k)));
+        return VH_OK;
+    }
+    // rows first .. first + n - 1 of the matrix [total, k] -> rows row0 .. (tile step `step`), columns col0 ..
+    int pack(const std::string &name, int total, int k, int first, int n, const Linear &w, int row0, int step, int col0) {
+        const TensorView *t;
+        VHC(view(name, {total, k}, &t));
+        const size_t bytes = (size_t)n * k * 2;
+        if (bytes > stage_bytes) {
+            if (stage) vx_free(be, stage);
+            stage = vx_alloc_permanent(be, bytes);
+            stage_bytes = stage ? bytes : 0;
+            if (!stage) return fail("device memory: %s", vx_last_error());
+        }
+        VXC(vx_to_device(be, stage, t->data + (size_t)first * k * 2, bytes));
+        VXC(vx_linear_pack(be, stage, n, k, w.w, w.n, w.k, row0 / 16, step, col0));
+        return VH_OK;
+    }
+};
+
+int distance_bucket(int n, int rows, int bias_max) {
+    const int half = rows / 2;
+    if (rows < 2 || bias_max <= half || n < 0) return -1;
+    if (n < half) return n;
+    if (n >= bias_max) return rows - 1;
+    // a distance at which the logarithm reaches a whole number has reached it, whatever the last bit of the quotient says
+    const double v = log((double)n / half) / log((double)bias_max / half) * (rows - half), near = round(v);
+    const int b = half + (int)(fabs(v - near) < 1e-9 ? near : floor(v));
+    return b < rows - 1 ? b : rows - 1;
+}
+
+int build_lozedra(Builder &b, const Json &config, MixModel *x, vh_config *cfg) {
+    LozedraConfig c;
+    VHC(parse_lozedra(config, &c));
+    cfg->hidden = c.width, cfg->vocab = c.vocab, cfg->eps = c.eps;
+    x->eps = c.eps, x->mult = c.mult;
+    for (size_t i = 0; i < c.layers.size(); i++) {
+        const LozedraLayer &s = c.layers[i];
+        const std::string l = "l" + std::to_string(i) + ".", left = l + "mix.left.", right = l + "mix.right.", mlp = l + "mlp.";
+        const int W = c.width, qd = s.heads * s.dim, kd = s.kv_heads * s.dim, vd = s.kv_heads * s.vdim, od = s.heads * s.vdim;
+        MixLayer o;
+        VHC(b.vec(l + "norm1", W, &o.norm1));
+        VHC(b.vec(l + "norm1b", W, &o.norm1b));
+        // one input projection for both mixers, its parts at whole tiles
+        AttnMixer &a = o.attn;
+        ScanMixer &n = o.scan;
+        o.has_attn = o.has_scan = true;
+        a.heads = s.heads, a.kv_heads = s.kv_heads, a.k_dim = s.dim, a.v_dim = s.vdim;
+        a.scale = s.scale, a.temp_coef = s.temp_coef, a.temp_every = s.temp_every, a.gate = true, a.out_scale = s.left_scale;
+        n.channels = s.inner, n.states = s.state, n.pad = vx_scan_state_pad(s.state), n.taps = s.conv, n.dt_rank = s.dt_rank;
+        n.dt_pad = b.pad(s.dt_rank, 64), n.out_scale = s.right_scale;
+        a.q_col = 0;
+        a.k_col = b.pad(qd, 16);
+        a.v_col = a.k_col + b.pad(kd, 16);
+        a.g_col = a.v_col + b.pad(vd, 16);
+        n.x_col = a.g_col + b.pad(od, 16);
+        n.z_col = n.x_col + b.pad(s.inner, 16);
+        VHC(b.packed(&o.in, n.z_col + s.inner, W));
+        VHC(b.pack(left + "q", qd, W, 0, qd, o.in, a.q_col, 1, 0));
+        VHC(b.pack(left + "k", kd, W, 0, kd, o.in, a.k_col, 1, 0));
+        VHC(b.pack(left + "v", vd, W, 0, vd, o.in, a.v_col, 1, 0));
+        VHC(b.pack(left + "g", od, W, 0, od, o.in, a.g_col, 1, 0));
+        VHC(b.pack(right + "in", 2 * s.inner, W, 0, s.inner, o.in, n.x_col, 1, 0));
+        VHC(b.pack(right + "in", 2 * s.inner, W, s.inner, s.inner, o.in, n.z_col, 1, 0));
+        // one output projection: its inputs are the heads, then the channels
+        VHC(b.packed(&o.out, W, od + s.inner));
+        VHC(b.pack(left + "o", W, od, 0, W, o.out, 0, 1, 0));
+        VHC(b.pack(right + "o", W, s.inner, 0, W, o.out, 0, 1, od));
+        // the distance bias, spread out to one value per distance
+        std::vector<float> rel;
+        const auto it = b.st->tensors.find(left + "rel");
+        if (it == b.st->tensors.end() || it->second.shape.size() != 2) return fail("tensor %srel is missing or no table", left.c_str());
+        const int rows = (int)it->second.shape[0];
+        VHC(b.floats(left + "rel", {rows, s.heads}, &rel));
+        if (distance_bucket(0, rows, s.bias_max) < 0)
+            return fail("layer %zu: a bias table of %d rows with bias_max %d", i, rows, s.bias_max);
+        a.bias_len = s.bias_max + 1;
+        std::vector<float> bias((size_t)s.heads * a.bias_len);
+        for (int h = 0; h < s.heads; h++)
+            for (int d = 0; d < a.bias_len; d++)
+                bias[(size_t)h * a.bias_len + d] = rel[(size_t)distance_bucket(d, rows, s.bias_max) * s.heads + h];
+        VHC(b.upload(bias, &a.bias));
+        // the scan's own weights
+        std::vector<float> cw, t, tr;
+        VHC(b.floats(right + "conv", {s.inner, s.conv}, &cw));
+        tr.resize(cw.size());
+        for (int ch = 0; ch < s.inner; ch++)
+            for (int k = 0; k < s.conv; k++) tr[(size_t)k * s.inner + ch] = cw[(size_t)ch * s.conv + k];
+        VHC(b.upload(tr, &n.conv_w));
+        VHC(b.vec(right + "conv.b", s.inner, &n.conv_b));
+        VHC(b.packed(&n.x, n.dt_pad + 2 * n.pad, s.inner));
+        const int xr = s.dt_rank + 2 * s.state;
+        VHC(b.pack(right + "x", xr, s.inner, 0, s.dt_rank, n.x, 0, 1, 0));
+        VHC(b.pack(right + "x", xr, s.inner, s.dt_rank, s.state, n.x, n.dt_pad, 1, 0));
+        VHC(b.pack(right + "x", xr, s.inner, s.dt_rank + s.state, s.state, n.x, n.dt_pad + n.pad, 1, 0));
+        VHC(b.packed(&n.dt, s.inner, s.dt_rank));
+        VHC(b.pack(right + "dt", s.inner, s.dt_rank, 0, s.inner, n.dt, 0, 1, 0));
+        VHC(b.vec(right + "dt.b", s.inner, &n.dt_bias));
+        VHC(b.floats(right + "A_log", {s.inner, s.state}, &t));
+        std::vector<float> a2((size_t)s.inner * n.pad, 0.f);
+        for (int ch = 0; ch < s.inner; ch++)
+            for (int k = 0; k < s.state; k++)
+                a2[(size_t)ch * n.pad + k] = (float)(-exp((double)t[(size_t)ch * s.state + k]) * 1.4426950408889634);
+        VHC(b.upload(a2, &n.a2));
+        VHC(b.vec(right + "D", s.inner, &n.d));
+        if (s.ff > 0) {
+            o.has_mlp = true;
+            o.ff_pad = b.pad(s.ff, 64);
+            VHC(b.vec(l + "norm2", W, &o.norm2));
+            VHC(b.vec(l + "norm2b", W, &o.norm2b));
+            VHC(b.packed(&o.gate_up, 2 * o.ff_pad, W));
+            VHC(b.pack(mlp + "gate", s.ff, W, 0, s.ff, o.gate_up, 0, 2, 0));
+            VHC(b.pack(mlp + "up", s.ff, W, 0, s.ff, o.gate_up, 16, 2, 0));
+            VHC(b.packed(&o.down, W, s.ff));
+            VHC(b.pack(mlp + "down", W, s.ff, 0, W, o.down, 0, 1, 0));
+        }
+        x->layers.push_back(o);
+    }
+    auto run = [&](int layer, bool again) {
+        LayerRun r;
+        r.layer = layer, r.add_embedding = again;
+        x->runs.push_back(r);
+    };
+    const int n = (int)c.layers.size();
+    for (int i = 0; i < c.loop_start; i++) run(i, false);
+    for (int pass = 0; pass < c.loop_times; pass++)
+        for (int i = c.loop_start; i < c.loop_stop; i++) run(i, pass > 0 && i == c.loop_start);
+    for (int i = c.loop_stop; i < n; i++) run(i, false);
+    std::vector<float> emb;
+    VHC(b.floats("embed", {c.vocab, c.width}, &emb));
+    VHC(b.upload(emb, &b.m->embedding));
+    VHC(b.vec("final.norm", c.width, &b.m->final_norm));
+    VHC(b.packed(&x->head, c.vocab, c.width));
+    return b.pack("head", c.vocab, c.width, 0, c.vocab, x->head, 0, 1, 0);
+}
+
+int check_lozedra(const Json &config) {
+    LozedraConfig c;
+    return parse_lozedra(config, &c);
+}
+
+// ---------------------------------------------------------------- registry
+struct Architecture {
+    const char *name;                                                    // config.json "architecture"
+    int (*check)(const Json &);
+    int (*build)(Builder &, const Json &, MixModel *, vh_config *);      // fills program, weights, and width / vocab / eps
+};
+const Architecture kArchitectures[] = {
+    {"Lozedra", check_lozedra, build_lozedra},
+};
+
+const Architecture *find_architecture(const Json &config) {
+    const Json *name = config.type == Json::OBJ ? config.get("architecture") : nullptr;
+    if (!name || name->type != Json::STR) {
+        fail("config.json names no architecture");
+        return nullptr;
+    }
+    for (const Architecture &a : kArchitectures)
+        if (name->str == a.name) return &a;
+    std::string known;
+    for (const Architecture &a : kArchitectures) known += std::string(known.empty() ? "" : ", ") + a.name;
+    fail("config.json: unknown architecture '%s' (known: %s)", name->str.c_str(), known.c_str());
+    return nullptr;
+}
+
+}  // namespace
+}  // namespace vh
+
+using namespace vh;
+
+extern "C" {
+
+const char *vh_architecture_name(int i) {
+    return i >= 0 && i < (int)(sizeof kArchitectures / sizeof kArchitectures[0]) ? kArchitectures[i].name : nullptr;
+}
+
+int vh_distance_bucket(int distance, int rows, int bias_max) { return distance_bucket(distance, rows, bias_max); }
+
+int vh_check_config(const char *json_text) {
+    Json config;
+    if (!json_text || !parse_json(json_text, strlen(json_text), &config)) return fail("config.json is not JSON");
+    const Architecture *arch = find_architecture(config);
+    return arch ? arch->check(config) : (int)VH_ERR;
+}
+
+int vh_model_load(vx_backend *be, const char *path, const vh_load_options *opt, vh_model **out) {
+    if (!be || !path || !opt || !out) return fail("vh_model_load: null argument");
+    *out = nullptr;
+    struct stat sb;
+    if (stat(path, &sb) != 0) return fail("%s: %s", path, strerror(errno));
+    if (!S_ISDIR(sb.st_mode)) return vh_model_load_gguf(be, path, opt, out);
+    const std::string dir = path;
+    Json config;
+    {
+        Mapped text;
+        VHC(text.open(dir + "/config.json"));
+        if (!parse_json((const char *)text.base, text.size, &config)) return fail("%s/config.json is not JSON", path);
+    }
+    const Architecture *arch = find_architecture(config);
+    if (!arch) return VH_ERR;
+    VHC(arch->check(config));
+    SafeTensors st;
+    VHC(st.open(dir + "/model.safetensors"));
+    vh_config c;
+    memset(&c, 0, sizeof c);
+    c.block_size = opt->block_size > 0 ? opt->block_size : 16;
+    c.pool_blocks = opt->pool_blocks, c.max_seqs = opt->max_seqs, c.max_blocks_per_seq = opt->max_blocks_per_seq, c.max_batch = opt->max_batch;
+    if (c.block_size % 8 || c.pool_blocks <= 0 || c.max_seqs <= 0 || c.max_blocks_per_seq <= 0 || c.max_batch <= 0 || c.max_batch > 1024)
+        return fail("bad pool or batch sizes");
+    if (opt->dtype < VH_DTYPE_DEFAULT || opt->dtype > VH_DTYPE_F32) return fail("unknown dtype %d", opt->dtype);
+    vh_model *m = new vh_model();
+    m->be = be;
+    m->mix.reset(new MixModel());
+    m->mix->act = opt->dtype == VH_DTYPE_F32 ? VX_ACT_F32 : VX_ACT_BF16;
+    int rc;
+    {
+        Builder b{be, &st, m};
+        rc = arch->build(b, config, m->mix.get(), &c);
+    }
+    c.num_layers = (int)m->mix->runs.size();  // (the layers that hold a cache: every pass has its own)
+    m->cfg = c;
+    if (rc == VH_OK) rc = mix_finish(m);
+    if (rc != VH_OK) {
+        const std::string keep = vh_last_error();
+        vh_model_destroy(m);
+        vh_set_error(keep.c_str());
+        return VH_ERR;
+    }
+    *out = m;
+    return VH_OK;
+}
+
+}  // extern "C"

@@ -28,12 +28,13 @@
 #include <unordered_map>
 #include <vector>
 
-#include "vexel_host.h"
+#include "model.h"
 
 namespace {
-
 thread_local char g_err[512] = "";
+}
 
+namespace vh {
 int fail(const char *fmt, ...) {
     va_list ap;
     va_start(ap, fmt);
@@ -41,121 +42,6 @@ int fail(const char *fmt, ...) {
     va_end(ap);
     return VH_ERR;
 }
-
-#define VXC(expr)                                                         \
-    do {                                                                  \
-        int _rc = (expr);                                                 \
-        if (_rc != VX_OK) return fail("%s: %s", #expr, vx_last_error());  \
-    } while (0)
-#define VHC(expr)                      \
-    do {                               \
-        if ((expr) != VH_OK) return VH_ERR; \
-    } while (0)
-
-struct SeqState {
-    std::vector<int32_t> table;  // logical block -> physical block (same for every layer)
-    int seq_len = 0;
-    int slot = -1;               // row in the device block-table matrix
-    bool dirty = true;           // device row differs from `table`
-};
-
-struct Fragment {                 // kv/fragment.go:9-16
-    int num_tokens = 0;
-    std::vector<int32_t> blocks;  // the cached sequence's table (the same for every layer), one reference each
-};
-
-struct BlockPool {
-    int block_size = 16, max_blocks = 0;
-    std::map<std::string, Fragment> fragments;    // kv/fragment.go:19-23
-    std::vector<int32_t> free_list;               // gpu_block_pool.go:110-116
-    std::unordered_map<int32_t, int> ref_counts;  // gpu_block_pool.go:42-43
-    std::map<int64_t, SeqState> seqs;
-    std::mutex mu;                                // gpu_block_pool.go:46
-    std::vector<int> free_slots;
-    bool free_dirty = true;
-
-    int alloc_block(int32_t *out) {               // gpu_block_pool.go:200-209
-        if (free_list.empty()) return fail("no free blocks (max=%d)", max_blocks);
-        *out = free_list.back();
-        free_list.pop_back();
-        ref_counts[*out] = 1;
-        free_dirty = true;
-        return VH_OK;
-    }
-    void release_block(int32_t b) {               // gpu_block_pool.go:211-219
-        auto it = ref_counts.find(b);
-        int rc = it == ref_counts.end() ? 0 : it->second;
-        if (rc <= 1) {
-            if (it != ref_counts.end()) ref_counts.erase(it);
-            free_list.push_back(b);
-            free_dirty = true;
-        } else {
-            it->second = rc - 1;
-        }
-    }
-    int ensure_blocks(SeqState &s, int end_pos) {  // gpu_block_pool.go:234-245
-        if (end_pos <= 0) return VH_OK;
-        int last = (end_pos - 1) / block_size;
-        while ((int)s.table.size() <= last) {
-            int32_t b;
-            VHC(alloc_block(&b));
-            s.table.push_back(b);
-            s.dirty = true;
-        }
-        return VH_OK;
-    }
-};
-
-}  // namespace
-
-struct vh_model {
-    vx_backend *be = nullptr;
-    vh_config cfg{};
-    std::vector<vh_layer_weights> layers;
-    const float *embedding = nullptr;
-    const float *final_norm = nullptr;
-    vh_qweight lm_head{};
-    std::vector<void *> adopted;  // device buffers a loader handed over (vh_model_adopt_buffer)
-    BlockPool pool;
-    std::vector<void *> kv;
-
-    int32_t *d_tables = nullptr, *d_num_blocks = nullptr, *d_free = nullptr, *d_free_count = nullptr;
-    int32_t *d_slots = nullptr, *d_positions = nullptr, *d_tokens = nullptr, *d_next = nullptr;
-    int32_t *d_cu = nullptr, *d_token_pos = nullptr, *d_slot_map = nullptr, *d_kv_lens = nullptr;
-    int32_t *d_pos_in = nullptr;  // positions of a host-driven step, input of the packing kernel
-    int32_t *d_status = nullptr, *d_step = nullptr, *d_log = nullptr;
-    int log_cap = 0;  // steps the log can hold
-
-    float *x = nullptr, *norm = nullptr, *q = nullptr, *k = nullptr, *v = nullptr, *attn = nullptr;
-    float *gate = nullptr, *up = nullptr, *logits = nullptr;
-
-    bool fused = true;  // take the fused decode entry points where the weights allow it
-
-    vh_arch arch{};                       // all zero: the LLaMA arm
-    std::vector<vh_layer_extras> extras;  // per layer, all NULL by default
-    const float *final_norm_bias = nullptr;
-    float *zeros = nullptr;               // [hidden] zeros: the bias of a LayerNorm whose bias tensor is absent
-    bool general = false;                 // some switch or extra tensor is set: the one-call-per-operation sequence
-    bool fused_ok = true;                 // the layer differs from LLaMA's at most by Q/K/V biases and the RoPE form
-    bool attn_fused_ok = true;            // the attention half does (RMSNorm without a bias in front of Q|K|V): its fused block serves it
-                                          // (Qwen 2): decode may still take the fused entry points
-
-    vx_graph *graph = nullptr;
-    int graph_batch = 0;
-    uint64_t graph_scratch_gen = 0;  // vx_scratch_generation() when the graph was captured
-    std::vector<int64_t> dev_seq_ids;  // batch currently loaded in d_slots (device-driven mode)
-    std::vector<int32_t> dev_positions;
-};
-
-namespace {
-
-template <class T>
-int dev_alloc(vh_model *m, T **p, size_t count) {
-    *p = (T *)vx_alloc_permanent(m->be, (count ? count : 1) * sizeof(T));
-    if (!*p) return fail("vx_alloc_permanent(%zu): %s", count * sizeof(T), vx_last_error());
-    return VH_OK;
-}
-
 SeqState *find_seq(vh_model *m, int64_t id) {
     auto it = m->pool.seqs.find(id);
     return it == m->pool.seqs.end() ? nullptr : &it->second;
@@ -198,6 +84,19 @@ int sync_pool_to_device(vh_model *m) {
         VXC(vx_to_device(m->be, m->d_free_count, &fc, 4));
         p.free_dirty = false;
     }
+    return VH_OK;
+}
+
+}  // namespace vh
+
+using namespace vh;
+
+namespace {
+
+template <class T>
+int dev_alloc(vh_model *m, T **p, size_t count) {
+    *p = (T *)vx_alloc_permanent(m->be, (count ? count : 1) * sizeof(T));
+    if (!*p) return fail("vx_alloc_permanent(%zu): %s", count * sizeof(T), vx_last_error());
     return VH_OK;
 }
 
@@ -443,6 +342,13 @@ int execute_layer_decode(vh_model *m, int layer, int rows, int max_kv_len, const
 // embedding -> layers -> final norm -> lm_head -> argmax for a decode batch (decode.go:404-452)
 int forward_decode(vh_model *m, int rows, int max_kv_len) {
     const vh_config &c = m->cfg;
+    if (m->mix) {
+        const vx_ragged b{rows, rows, nullptr, max_kv_len, m->d_cu, m->d_token_pos, m->d_slot_map, m->d_slots, m->d_kv_lens, m->d_tables,
+                          c.max_blocks_per_seq, c.block_size};
+        VHC(mix_forward(m, b, m->d_tokens, m->mix->perm, nullptr, rows, m->logits));
+        VXC(vx_argmax_rows(m->be, m->logits, rows, c.vocab, m->d_next));
+        return VH_OK;
+    }
     VXC(vx_embedding(m->be, m->d_tokens, rows, m->embedding, m->x, c.vocab, c.hidden));
     VHC(g_scale_embedding(m, m->x, rows));
     const bool head_prepared = rows > 1 && m->fused && (!m->general || m->fused_ok) && fast(m->lm_head) && c.hidden % 256 == 0;
@@ -469,7 +375,46 @@ int forward_decode(vh_model *m, int rows, int max_kv_len) {
     return VH_OK;
 }
 
+}  // namespace
+
+namespace vh {
+int init_common(vh_model *m) {
+    const vh_config &c = m->cfg;
+    const size_t mb = c.max_batch;
+    m->pool.block_size = c.block_size;
+    m->pool.max_blocks = c.pool_blocks;
+    m->pool.free_list.resize(c.pool_blocks);
+    for (int i = 0; i < c.pool_blocks; i++) m->pool.free_list[i] = i;
+    for (int i = c.max_seqs - 1; i >= 0; i--) m->pool.free_slots.push_back(i);
+    int rc = VH_OK;
+    rc |= dev_alloc(m, &m->d_tables, (size_t)c.max_seqs * c.max_blocks_per_seq);
+    rc |= dev_alloc(m, &m->d_num_blocks, c.max_seqs);
+    rc |= dev_alloc(m, &m->d_free, c.pool_blocks);
+    rc |= dev_alloc(m, &m->d_free_count, 1);
+    rc |= dev_alloc(m, &m->d_slots, mb);
+    rc |= dev_alloc(m, &m->d_positions, mb);
+    rc |= dev_alloc(m, &m->d_tokens, mb);
+    rc |= dev_alloc(m, &m->d_next, mb);
+    rc |= dev_alloc(m, &m->d_cu, mb + 1);
+    rc |= dev_alloc(m, &m->d_token_pos, mb);
+    rc |= dev_alloc(m, &m->d_slot_map, mb);
+    rc |= dev_alloc(m, &m->d_kv_lens, mb);
+    rc |= dev_alloc(m, &m->d_pos_in, mb);
+    rc |= dev_alloc(m, &m->d_status, 1);
+    rc |= dev_alloc(m, &m->d_step, 1);
+    rc |= dev_alloc(m, &m->logits, mb * c.vocab);
+    if (rc) return VH_ERR;
+    std::vector<int32_t> zeros((size_t)c.max_seqs * c.max_blocks_per_seq, 0);
+    VXC(vx_to_device(m->be, m->d_tables, zeros.data(), zeros.size() * 4));
+    VXC(vx_to_device(m->be, m->d_num_blocks, zeros.data(), (size_t)c.max_seqs * 4));
+    return VH_OK;
+}
+}  // namespace vh
+
+namespace {
+
 int check_ready(vh_model *m) {
+    if (m->mix) return VH_OK;  // (complete once it exists)
     if (!m->embedding || !m->final_norm || !m->lm_head.data) return fail("model head / embedding not set");
     for (auto &l : m->layers)
         if (!l.attn_norm || !l.wq.data) return fail("a layer's weights are not set");
@@ -507,11 +452,6 @@ int vh_model_create(vx_backend *be, const vh_config *cfg, vh_model **out) {
     m->cfg = c;
     m->layers.resize(c.num_layers);
     m->extras.resize(c.num_layers);
-    m->pool.block_size = c.block_size;
-    m->pool.max_blocks = c.pool_blocks;
-    m->pool.free_list.resize(c.pool_blocks);
-    for (int i = 0; i < c.pool_blocks; i++) m->pool.free_list[i] = i;
-    for (int i = c.max_seqs - 1; i >= 0; i--) m->pool.free_slots.push_back(i);
     const size_t kv_bytes = (size_t)c.pool_blocks * 2 * c.block_size * c.num_kv_heads * c.head_dim * (c.kv_fp16 ? 2 : 4);
     m->kv.resize(c.num_layers, nullptr);
     for (int l = 0; l < c.num_layers; l++) {
@@ -523,22 +463,7 @@ int vh_model_create(vx_backend *be, const vh_config *cfg, vh_model **out) {
         }
     }
     const size_t mb = c.max_batch;
-    int rc = VH_OK;
-    rc |= dev_alloc(m, &m->d_tables, (size_t)c.max_seqs * c.max_blocks_per_seq);
-    rc |= dev_alloc(m, &m->d_num_blocks, c.max_seqs);
-    rc |= dev_alloc(m, &m->d_free, c.pool_blocks);
-    rc |= dev_alloc(m, &m->d_free_count, 1);
-    rc |= dev_alloc(m, &m->d_slots, mb);
-    rc |= dev_alloc(m, &m->d_positions, mb);
-    rc |= dev_alloc(m, &m->d_tokens, mb);
-    rc |= dev_alloc(m, &m->d_next, mb);
-    rc |= dev_alloc(m, &m->d_cu, mb + 1);
-    rc |= dev_alloc(m, &m->d_token_pos, mb);
-    rc |= dev_alloc(m, &m->d_slot_map, mb);
-    rc |= dev_alloc(m, &m->d_kv_lens, mb);
-    rc |= dev_alloc(m, &m->d_pos_in, mb);
-    rc |= dev_alloc(m, &m->d_status, 1);
-    rc |= dev_alloc(m, &m->d_step, 1);
+    int rc = init_common(m);
     rc |= dev_alloc(m, &m->x, mb * c.hidden);
     rc |= dev_alloc(m, &m->norm, mb * c.hidden);
     rc |= dev_alloc(m, &m->q, mb * c.num_heads * c.head_dim);
@@ -547,15 +472,7 @@ int vh_model_create(vx_backend *be, const vh_config *cfg, vh_model **out) {
     rc |= dev_alloc(m, &m->attn, mb * c.num_heads * c.head_dim);
     rc |= dev_alloc(m, &m->gate, mb * c.ffn);
     rc |= dev_alloc(m, &m->up, mb * c.ffn);
-    rc |= dev_alloc(m, &m->logits, mb * c.vocab);
     if (rc) {
-        vh_model_destroy(m);
-        return VH_ERR;
-    }
-    std::vector<int32_t> zeros((size_t)c.max_seqs * c.max_blocks_per_seq, 0);
-    if (vx_to_device(be, m->d_tables, zeros.data(), zeros.size() * 4) ||
-        vx_to_device(be, m->d_num_blocks, zeros.data(), (size_t)c.max_seqs * 4)) {
-        fail("init: %s", vx_last_error());
         vh_model_destroy(m);
         return VH_ERR;
     }
@@ -579,6 +496,7 @@ void vh_model_destroy(vh_model *m) {
 
 int vh_model_set_layer(vh_model *m, int layer, const vh_layer_weights *w) {
     if (!m || !w || layer < 0 || layer >= m->cfg.num_layers) return fail("bad layer index");
+    if (m->mix) return fail("the layers of a loaded mixer program cannot be replaced");
     const vh_config &c = m->cfg;
     const int qd = c.num_heads * c.head_dim, kvd = c.num_kv_heads * c.head_dim;
     if (w->wq.n != qd || w->wq.k != c.hidden || w->wk.n != kvd || w->wv.n != kvd || w->wo.n != c.hidden ||
@@ -602,6 +520,7 @@ int vh_model_set_layer(vh_model *m, int layer, const vh_layer_weights *w) {
 
 int vh_model_set_head(vh_model *m, const float *embedding, const float *final_norm, const vh_qweight *lm_head) {
     if (!m || !embedding || !final_norm || !lm_head) return fail("null argument");
+    if (m->mix) return fail("the head of a loaded mixer program cannot be replaced");
     if (lm_head->n != m->cfg.vocab || lm_head->k != m->cfg.hidden) return fail("lm_head shape mismatch");
     drop_graph(m);
     m->embedding = embedding;
@@ -647,6 +566,7 @@ static void refresh_general(vh_model *m) {
 
 int vh_model_set_architecture(vh_model *m, const vh_arch *arch) {
     if (!m || !arch) return fail("null argument");
+    if (m->mix) return fail("a mixer program has no architecture switches");
     const vh_arch &a = *arch;
     if (a.norm_type < 0 || a.norm_type > VH_NORM_LAYER || a.mlp_type < 0 || a.mlp_type > VH_MLP_GEGLU)
         return fail("unknown norm type %d / MLP type %d", a.norm_type, a.mlp_type);
@@ -676,6 +596,7 @@ void vh_model_get_architecture(const vh_model *m, vh_arch *out) {
 
 int vh_model_set_layer_extras(vh_model *m, int layer, const vh_layer_extras *extras) {
     if (!m || !extras || layer < 0 || layer >= m->cfg.num_layers) return fail("bad layer index");
+    if (m->mix) return fail("the layers of a loaded mixer program cannot be replaced");
     m->extras[layer] = *extras;
     drop_graph(m);
     refresh_general(m);
@@ -684,6 +605,7 @@ int vh_model_set_layer_extras(vh_model *m, int layer, const vh_layer_extras *ext
 
 int vh_model_set_final_norm_bias(vh_model *m, const float *bias) {
     if (!m) return fail("null argument");
+    if (m->mix) return fail("a mixer program has no final norm bias");
     m->final_norm_bias = bias;
     refresh_general(m);
     return VH_OK;
@@ -725,6 +647,7 @@ int vh_pool_truncate_sequence(vh_model *m, int64_t seq_id, int new_len) {  // gp
     std::lock_guard<std::mutex> g(m->pool.mu);
     SeqState *s = find_seq(m, seq_id);
     if (!s || new_len >= s->seq_len) return VH_OK;
+    if (m->mix && new_len > 0) return fail("sequence %lld: its recurrent state cannot go back to length %d", (long long)seq_id, new_len);
     int keep = 0;
     if (new_len > 0) keep = (new_len - 1) / m->pool.block_size + 1;
     for (int i = keep; i < (int)s->table.size(); i++) m->pool.release_block(s->table[i]);
@@ -742,6 +665,7 @@ int vh_pool_has_sequence(vh_model *m, int64_t seq_id) {
 }
 
 int vh_pool_share_blocks(vh_model *m, int64_t src_id, int64_t dst_id, int num_tokens) {  // gpu_block_pool.go:572-607
+    if (m->mix) return fail("vh_pool_share_blocks: a sequence of this model is more than its blocks (recurrent state)");
     std::lock_guard<std::mutex> g(m->pool.mu);
     SeqState *src = find_seq(m, src_id);
     if (!src) return fail("source sequence %lld not found", (long long)src_id);
@@ -766,6 +690,7 @@ static void release_fragment(vh_model *m, const Fragment &f) {  // fragment.go:8
 
 int vh_fragment_cache(vh_model *m, const char *name, int64_t seq_id) {  // paged_cache.go:324-343, fragment.go:36-60
     if (!m || !name) return fail("bad arguments");
+    if (m->mix) return fail("vh_fragment_cache: a sequence of this model is more than its blocks (recurrent state)");
     std::lock_guard<std::mutex> g(m->pool.mu);
     SeqState *s = find_seq(m, seq_id);
     if (!s) return VH_OK;  // paged_cache.go:331-333: an unknown sequence caches nothing
@@ -812,6 +737,7 @@ int vh_fragment_delete(vh_model *m, const char *name) {  // fragment.go:71-79
 int vh_fragment_insert(vh_model *m, int64_t seq_id, const char *name, int insert_pos, int *num_tokens) {
     if (num_tokens) *num_tokens = 0;
     if (!m || !name || insert_pos < 0) return fail("bad arguments");
+    if (m->mix) return fail("vh_fragment_insert: a sequence of this model is more than its blocks (recurrent state)");
     const vh_config &c = m->cfg;
     if (m->arch.rope_neox || (m->arch.rope_dim != 0 && m->arch.rope_dim != c.head_dim))
         return fail("fragments are rotated as RoPEShift rotates (whole head, pairs 2j and 2j+1): not this model's RoPE");
@@ -902,6 +828,7 @@ int vh_pool_block_table(vh_model *m, int64_t seq_id, int32_t *out, int cap) {
 }
 
 int vh_pool_adopt_blocks(vh_model *m, int64_t seq_id, const int32_t *blocks, int num_blocks, int seq_len) {
+    if (m->mix) return fail("vh_pool_adopt_blocks: a sequence of this model is more than its blocks (recurrent state)");
     std::lock_guard<std::mutex> g(m->pool.mu);
     SeqState *s = find_seq(m, seq_id);
     if (!s) return fail("sequence %lld not found", (long long)seq_id);
@@ -957,6 +884,17 @@ int vh_decode_batched(vh_model *m, const int32_t *tokens, const int64_t *seq_ids
     if (batch < 0 || batch > m->cfg.max_batch) return fail("batch %d exceeds max_batch %d", batch, m->cfg.max_batch);
     VHC(check_ready(m));
     const vh_config &c = m->cfg;
+    if (m->mix) {
+        for (int i = 0; i < batch; i++) {
+            const int len = std::max(0, vh_pool_seq_len(m, seq_ids[i]));
+            if (positions[i] != len)
+                return fail("sequence %lld: position %d is not its length %d", (long long)seq_ids[i], positions[i], len);
+        }
+        const std::vector<int32_t> ones(batch, 1);
+        std::vector<int32_t> want(batch);
+        for (int i = 0; i < batch; i++) want[i] = i;
+        return mix_step(m, batch, seq_ids, ones.data(), tokens, batch, want.data(), logits_out, argmax_out);
+    }
     std::vector<int32_t> slots(batch), slot_map(batch), kv_lens(batch);
     int max_kv = 1;
     {
@@ -1030,6 +968,14 @@ int vh_prefill(vh_model *m, const int32_t *tokens, int n, int64_t seq_id, int st
     if (!m || !tokens || n <= 0 || start_pos < 0) return fail("bad arguments");
     VHC(check_ready(m));
     const vh_config &c = m->cfg;
+    if (m->mix) {
+        const int len = std::max(0, vh_pool_seq_len(m, seq_id));
+        if (start_pos != len) return fail("sequence %lld: position %d is not its length %d", (long long)seq_id, start_pos, len);
+        std::vector<int32_t> want(all_logits ? n : 1, n - 1);
+        if (all_logits)
+            for (int i = 0; i < n; i++) want[i] = i;
+        return mix_step(m, 1, &seq_id, &n, tokens, (int)want.size(), want.data(), logits_out, nullptr);
+    }
     std::vector<int32_t> page(n), offs(n), kvl(n), table;
     int seq_len;
     {
@@ -1189,6 +1135,62 @@ int vh_prefill(vh_model *m, const int32_t *tokens, int n, int64_t seq_id, int st
     return VH_OK;
 }
 
+// ------------------------------------------------------------------ a step of portions and single tokens
+int vh_model_mixed_batches(const vh_model *m) { return m && m->mix ? 1 : 0; }
+
+int vh_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_lens, const int32_t *tokens, int n_want,
+            const int32_t *want_rows, float *logits_out, int32_t *argmax_out) {
+    if (!m || n_seqs < 0 || n_want < 0 || (n_seqs > 0 && (!seq_ids || !q_lens || !tokens)) || (n_want > 0 && !want_rows))
+        return fail("vh_step: bad arguments");
+    if (n_seqs == 0) return n_want == 0 ? (int)VH_OK : fail("vh_step: rows wanted of an empty step");
+    VHC(check_ready(m));
+    if (m->mix) return mix_step(m, n_seqs, seq_ids, q_lens, tokens, n_want, want_rows, logits_out, argmax_out);
+    // the LLaMA family: every portion by itself, then the single tokens as one batch
+    const int V = m->cfg.vocab;
+    std::vector<int> row0(n_seqs + 1, 0), one;
+    for (int i = 0; i < n_seqs; i++) {
+        if (q_lens[i] < 1) return fail("vh_step: sequence %lld brings no tokens", (long long)seq_ids[i]);
+        row0[i + 1] = row0[i] + q_lens[i];
+    }
+    for (int w = 0; w < n_want; w++)
+        if (want_rows[w] < 0 || want_rows[w] >= row0[n_seqs]) return fail("vh_step: wanted row %d of %d", want_rows[w], row0[n_seqs]);
+    auto deliver = [&](int row, const float *logits) {
+        for (int w = 0; w < n_want; w++) {
+            if (want_rows[w] != row) continue;
+            if (logits_out) memcpy(logits_out + (size_t)w * V, logits, (size_t)V * 4);
+            if (argmax_out) argmax_out[w] = vh_argmax(logits, V);
+        }
+    };
+    std::vector<float> lg;
+    for (int i = 0; i < n_seqs; i++) {
+        if (q_lens[i] == 1) {
+            one.push_back(i);
+            continue;
+        }
+        bool all = false;
+        for (int w = 0; w < n_want; w++) all = all || (want_rows[w] >= row0[i] && want_rows[w] < row0[i + 1] - 1);
+        lg.resize((size_t)(all ? q_lens[i] : 1) * V);
+        VHC(vh_prefill(m, tokens + row0[i], q_lens[i], seq_ids[i], std::max(0, vh_pool_seq_len(m, seq_ids[i])), all ? 1 : 0, lg.data()));
+        if (!all)
+            deliver(row0[i + 1] - 1, lg.data());
+        else
+            for (int r = 0; r < q_lens[i]; r++) deliver(row0[i] + r, lg.data() + (size_t)r * V);
+    }
+    for (size_t o = 0; o < one.size(); o += m->cfg.max_batch) {
+        const int b = (int)std::min(one.size() - o, (size_t)m->cfg.max_batch);
+        std::vector<int32_t> tok(b), pos(b);
+        std::vector<int64_t> ids(b);
+        for (int i = 0; i < b; i++) {
+            const int s = one[o + i];
+            tok[i] = tokens[row0[s]], ids[i] = seq_ids[s], pos[i] = std::max(0, vh_pool_seq_len(m, seq_ids[s]));
+        }
+        lg.resize((size_t)b * V);
+        VHC(vh_decode_batched(m, tok.data(), ids.data(), pos.data(), b, lg.data(), nullptr));
+        for (int i = 0; i < b; i++) deliver(row0[one[o + i]], lg.data() + (size_t)i * V);
+    }
+    return VH_OK;
+}
+
 // ------------------------------------------------------------------ tree verification of a batch of sequences
 int vh_verify_tree(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *input_tokens, const int32_t *start_pos,
                    const int32_t *n_nodes, const int32_t *node_tokens, const int32_t *parent_idx, int32_t *num_accepted,
@@ -1196,6 +1198,7 @@ int vh_verify_tree(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_
     if (!m || n_seqs < 0 || !seq_ids || !input_tokens || !start_pos || !n_nodes || !num_accepted || !final_tokens)
         return fail("bad arguments");
     if (n_seqs == 0) return VH_OK;
+    if (m->mix) return fail("vh_verify_tree: the recurrent state of a mixer program cannot follow several branches");
     VHC(check_ready(m));
     const vh_config &c = m->cfg;
     struct SeqRows { int row0, rows, node0, start, slot, pad; };

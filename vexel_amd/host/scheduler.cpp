@@ -15,6 +15,9 @@
 //    math/rand (whose generator table is no part of the reference's tree). Greedy requests (temperature 0) use the
 //    device argmax; in decode steps sampled requests are sampled on the device too (vh_sample_last_logits, the
 //    same sums in the same order), so logits move to the host only for the token that follows a prompt.
+//  * Models that run mixed batches (vh_model_mixed_batches) get one vh_step per scheduler step: the next piece of every
+//    prompt beside the decoding sequences' tokens. A prompt that ends in a step yields its first token there and decodes
+//    from the next step on.
 #include <math.h>
 #include <stdarg.h>
 #include <stdio.h>
@@ -268,6 +271,56 @@ int vh_sched_step(vh_scheduler *s, int *tokens_out) {
         return vh_sample(row, V, q.temperature, q.top_k, q.top_p, next_uniform(&q.rng));
     };
     int produced = 0;
+    if (vh_model_mixed_batches(s->m)) {
+        // one batch: the next piece of every prompt and the next token of every decoding sequence
+        std::vector<int64_t> ids;
+        std::vector<int32_t> tokens, lens, want;
+        std::vector<char> ends;  // whether the sequence's last row of this step is sampled
+        for (int64_t id : batch) {
+            Seq &q = s->seqs[id];
+            int n = 1;
+            bool last = true;
+            if (!q.prefill_complete()) {
+                const int left = (int)q.prompt.size() - q.prompt_pos;
+                n = s->cfg.prefill_chunk > 0 ? std::min(left, s->cfg.prefill_chunk) : left;
+                last = n == left;
+                tokens.insert(tokens.end(), q.prompt.begin() + q.prompt_pos, q.prompt.begin() + q.prompt_pos + n);
+            } else {
+                tokens.push_back(q.generated.empty() ? 1 : q.generated.back());  // (BOS for an empty prompt, as below)
+            }
+            ids.push_back(id), lens.push_back(n), ends.push_back(last);
+            if (last) want.push_back((int32_t)tokens.size() - 1);
+        }
+        std::vector<int32_t> am(want.size());
+        if (vh_step(s->m, (int)ids.size(), ids.data(), lens.data(), tokens.data(), (int)want.size(), want.data(), nullptr,
+                    am.data()) != VH_OK)
+            return VH_ERR;
+        std::vector<float> temp(want.size(), 0.f), tp(want.size(), 0.f), uni(want.size(), 0.f);
+        std::vector<int32_t> tk(want.size(), 0);
+        bool sampled = false;
+        for (size_t i = 0, w = 0; i < ids.size(); i++) {
+            if (!ends[i]) continue;
+            Seq &q = s->seqs[ids[i]];
+            if (q.sampled) temp[w] = q.temperature, tk[w] = q.top_k, tp[w] = q.top_p, uni[w] = next_uniform(&q.rng), sampled = true;
+            w++;
+        }
+        if (sampled && vh_sample_last_logits(s->m, (int)want.size(), temp.data(), tk.data(), tp.data(), uni.data(), am.data()) != VH_OK)
+            return VH_ERR;
+        for (size_t i = 0, w = 0; i < ids.size(); i++) {
+            Seq &q = s->seqs[ids[i]];
+            const bool prompt = !q.prefill_complete();
+            if (prompt) q.prompt_pos += lens[i];
+            q.position += lens[i];
+            q.state = ends[i] ? VH_SEQ_DECODING : VH_SEQ_PREFILL;
+            if (!ends[i]) continue;
+            const int tok = am[w++];
+            q.generated.push_back(tok);
+            produced++;
+            if (is_stop(tok) || q.reached_max(s->cfg.max_tokens)) q.state = VH_SEQ_FINISHED;
+        }
+        if (tokens_out) *tokens_out = produced;
+        return VH_OK;
+    }
     // prefill (scheduler.go:255-274, 483-552): a pending sequence with prompt left is fed before any decode
     for (int64_t id : batch) {
         Seq &q = s->seqs[id];

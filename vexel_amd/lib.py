@@ -9,6 +9,8 @@ LIB_PATH = os.path.join(HERE, "libvexel_hip.so")
 
 VX_OK, VX_ERR_INVALID, VX_ERR_OOM, VX_ERR_HIP, VX_ERR_UNSUPPORTED = 0, 1, 2, 3, 4
 VX_Q4_0, VX_Q8_0, VX_Q4_K, VX_Q6_K = 1, 2, 3, 4
+VX_ACT_F32, VX_ACT_BF16 = 0, 1
+VX_LIN_PLAIN, VX_LIN_SWIGLU, VX_LIN_KV, VX_LIN_SPLIT, VX_LIN_SOFTPLUS = 0, 1, 2, 3, 4
 
 _vp, _i, _f, _sz, _i64 = C.c_void_p, C.c_int, C.c_float, C.c_size_t, C.c_int64
 
@@ -111,6 +113,18 @@ SIGNATURES = {
     "vx_graph_end_capture": (_i, [_vp, C.POINTER(_vp)]),
     "vx_graph_launch": (_i, [_vp, _vp]),
     "vx_graph_destroy": (None, [_vp]),
+    "vx_fill_zero": (_i, [_vp, _vp, _sz]),
+    "vx_linear_bytes": (_sz, [_i, _i]),
+    "vx_linear_pack": (_i, [_vp, _vp, _i, _i, _vp, _i, _i, _i, _i, _i]),
+    "vx_linear_slices": (_i, [_vp, _i, _i, _i]),
+    "vx_linear": (_i, [_vp, _i, _vp, _i, _vp, _i, _i, _i, _vp]),
+    "vx_residual_norm": (_i, [_vp, _i, _vp]),
+    "vx_kv_block_elems": (_sz, [_i, _i, _i, _i]),
+    "vx_attn_ragged": (_i, [_vp, _i, _vp, _vp]),
+    "vx_attn_ragged_fast": (_i, [_i, _i, _i, _i, _i, _i]),
+    "vx_conv_silu": (_i, [_vp, _i, _vp, _vp]),
+    "vx_scan_state_pad": (_i, [_i]),
+    "vx_selective_scan": (_i, [_vp, _i, _vp, _vp]),
     "vx_timer_start": (_i, [_vp]),
     "vx_timer_stop_ms": (_i, [_vp, C.POINTER(_f)]),
 }

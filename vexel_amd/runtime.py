@@ -27,7 +27,10 @@ VH_F32 = 0             # vh_qweight.fmt of a float32 output head
 
 class VhLoadOptions(C.Structure):
     _fields_ = [(n, C.c_int) for n in ("block_size", "pool_blocks", "max_seqs", "max_blocks_per_seq", "max_batch",
-                                        "kv_fp16")]
+                                        "kv_fp16", "dtype")]
+
+
+DTYPES = {None: 0, "bfloat16": 1, "float32": 2}  # VH_DTYPE_*
 
 
 class VhLayerWeights(C.Structure):
@@ -73,6 +76,13 @@ def load_host():
         h.vh_model_get_config.argtypes = [C.c_void_p, C.POINTER(VhConfig)]
         h.vh_model_get_config.restype = None
         h.vh_model_load_gguf.argtypes = [C.c_void_p, C.c_char_p, C.POINTER(VhLoadOptions), C.POINTER(C.c_void_p)]
+        h.vh_model_load.argtypes = [C.c_void_p, C.c_char_p, C.POINTER(VhLoadOptions), C.POINTER(C.c_void_p)]
+        h.vh_architecture_name.argtypes = [C.c_int]
+        h.vh_architecture_name.restype = C.c_char_p
+        h.vh_check_config.argtypes = [C.c_char_p]
+        h.vh_distance_bucket.argtypes = [C.c_int, C.c_int, C.c_int]
+        h.vh_step.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p]
+        h.vh_model_mixed_batches.argtypes = [C.c_void_p]
         h.vh_model_set_fused.argtypes = [C.c_void_p, C.c_int]
         h.vh_model_set_fused.restype = None
         h.vh_model_set_layer.argtypes = [C.c_void_p, C.c_int, C.POINTER(VhLayerWeights)]
@@ -101,6 +111,21 @@ def load_host():
                                       C.c_void_p, C.POINTER(C.c_float)]
         _host = h
     return _host
+
+
+def architectures():
+    """The architectures a folder's config.json may name."""
+    h, out = load_host(), []
+    while (name := h.vh_architecture_name(len(out))) is not None:
+        out.append(name.decode())
+    return out
+
+
+def check_config(text):
+    """Raises VexelError when a config.json text is not a known architecture's or something in it is wrong."""
+    h = load_host()
+    if h.vh_check_config(text.encode()) != 0:
+        raise VexelError(1, h.vh_last_error().decode())
 
 
 class VhSchedConfig(C.Structure):
@@ -201,15 +226,26 @@ class ModelRuntime:
                   max_batch=64, kv_fp16=True):
         """ModelRuntime.LoadWeightsGGUF + CopyWeightsToDevice (runtime/loader.go): a LLaMA-family checkpoint read
         by the C++ loader; the model owns the device copies of the weights."""
+        return cls._load(be, "vh_model_load_gguf", path, VhLoadOptions(
+            block_size, pool_blocks, max_seqs, max_blocks_per_seq or pool_blocks, max_batch, int(bool(kv_fp16)), 0))
+
+    @classmethod
+    def load(cls, be: HipBackend, path, dtype=None, block_size=16, pool_blocks=256, max_seqs=64, max_blocks_per_seq=None,
+             max_batch=64):
+        """A model from a folder with config.json and model.safetensors (the architectures of `architectures()`), or from
+        a GGUF file. dtype: "bfloat16" (default) or "float32" activations, for folders."""
+        return cls._load(be, "vh_model_load", path, VhLoadOptions(
+            block_size, pool_blocks, max_seqs, max_blocks_per_seq or pool_blocks, max_batch, 1, DTYPES[dtype]))
+
+    @classmethod
+    def _load(cls, be, entry, path, opt):
         self = cls.__new__(cls)
         self._h = load_host()
         self.be = be
-        opt = VhLoadOptions(block_size, pool_blocks, max_seqs, max_blocks_per_seq or pool_blocks, max_batch,
-                            int(bool(kv_fp16)))
         m = C.c_void_p()
         self._m = None
         self._keep = []
-        self._ck(self._h.vh_model_load_gguf(be._h, os.fsencode(path), C.byref(opt), C.byref(m)))
+        self._ck(getattr(self._h, entry)(be._h, os.fsencode(path), C.byref(opt), C.byref(m)))
         self._m = m
         self.cfg = VhConfig()
         self._h.vh_model_get_config(m, C.byref(self.cfg))
@@ -391,6 +427,25 @@ class ModelRuntime:
         self._ck(self._h.vh_prefill(self._m, t.ctypes.data, t.size, seq_id, start_pos, int(all_logits),
                                     logits.ctypes.data))
         return logits if all_logits else logits[0]
+
+    def step(self, entries, want, want_logits=True):
+        """One mixed step (vh_step). entries: [(sequence id, its next tokens)]; want: row numbers over the concatenated
+        tokens -> (logits [len(want), vocab] or None, arg-max tokens)"""
+        ids = np.array([e[0] for e in entries], dtype=np.int64)
+        lens = np.array([len(e[1]) for e in entries], dtype=np.int32)
+        toks = np.array([t for e in entries for t in e[1]], dtype=np.int32)
+        w = np.array(want, dtype=np.int32)
+        logits = np.empty((w.size, self.cfg.vocab), dtype=np.float32) if want_logits else None
+        am = np.empty(max(1, w.size), dtype=np.int32)
+        self._ck(self._h.vh_step(self._m, ids.size, ids.ctypes.data, lens.ctypes.data, toks.ctypes.data, w.size,
+                                 w.ctypes.data, logits.ctypes.data if want_logits and w.size else None,
+                                 am.ctypes.data if w.size else None))
+        return logits, am[:w.size]
+
+    @property
+    def mixed_batches(self):
+        """Whether a step of this model is one batch of portions and single tokens (a mixer program)."""
+        return bool(self._h.vh_model_mixed_batches(self._m))
 
     def verify_tree(self, seq_ids, input_tokens, start_pos, trees, want_logits=True):
         """One verification pass over a candidate tree per sequence (vh_verify_tree). trees: one
