@@ -773,6 +773,124 @@ def arch_report(be):
         mr.close()
 
 
+# Shapes of --lozedra-report: layers like those of models of about 1.5 and 8 billion parameters, a few of them.
+LOZEDRA_SHAPES = {
+    "2048": dict(width=2048, heads=16, kv_heads=4, dim=128, inner=4096, dt_rank=128, ff=5632, layers=6),
+    "4096": dict(width=4096, heads=32, kv_heads=8, dim=128, inner=8192, dt_rank=256, ff=14336, layers=4),
+}
+LOZEDRA_VOCAB = 32000
+
+
+def write_lozedra(folder, width, heads, kv_heads, dim, inner, dt_rank, ff, layers, state=16, conv=4, bias_rows=32,
+                  bias_max=512, vocab=LOZEDRA_VOCAB):
+    """A Lozedra model of that shape with random weights (one random megaword repeated) as config.json + model.safetensors."""
+    mixer = {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "bias_max": bias_max,
+                      "q_temp": {"coef": 0.1, "every": 128}},
+             "right": {"inner": inner, "state": state, "dt_rank": dt_rank, "conv": conv}, "left_scale": 0.7, "right_scale": 0.6}
+    cfg = {"architecture": "Lozedra", "layers": [{"type": "parallel", "mixer": mixer, "mlp": {"kind": "dense", "ff": ff}}] * layers,
+           "loop": None, "norm": {"eps": 1e-5}, "residual_mult": 0.5, "vocab": vocab, "width": width}
+    shapes = {"embed": (vocab, width), "final.norm": (width,), "head": (vocab, width)}
+    for i in range(layers):
+        l = "l%d." % i
+        for n in ("norm1", "norm1b", "norm2", "norm2b"):
+            shapes[l + n] = (width,)
+        left, right = l + "mix.left.", l + "mix.right."
+        shapes.update({left + "q": (heads * dim, width), left + "k": (kv_heads * dim, width), left + "v": (kv_heads * dim, width),
+                       left + "g": (heads * dim, width), left + "o": (width, heads * dim), left + "rel": (bias_rows, heads),
+                       right + "in": (2 * inner, width), right + "conv": (inner, conv), right + "conv.b": (inner,),
+                       right + "x": (dt_rank + 2 * state, inner), right + "dt": (inner, dt_rank), right + "dt.b": (inner,),
+                       right + "A_log": (inner, state), right + "D": (inner,), right + "o": (width, inner),
+                       l + "mlp.gate": (ff, width), l + "mlp.up": (ff, width), l + "mlp.down": (width, ff)})
+    rng = np.random.default_rng(11)
+    noise = rng.standard_normal(1 << 20).astype(np.float32)
+
+    def bf16(a):
+        return ((np.ascontiguousarray(a, dtype=np.float32).view(np.uint32) + 0x8000) >> 16).astype("<u2")
+
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    head, at = {}, 0
+    for name, shape in shapes.items():
+        size = 2 * int(np.prod(shape))
+        head[name] = {"dtype": "BF16", "shape": list(shape), "data_offsets": [at, at + size]}
+        at += size
+    js = json.dumps(head).encode()
+    js += b" " * (-len(js) % 8)
+    small, ones = bf16(0.02 * noise), bf16(1.0 + 0.05 * noise)
+    with open(os.path.join(folder, "model.safetensors"), "wb") as f:
+        f.write(len(js).to_bytes(8, "little") + js)
+        for name, shape in shapes.items():
+            n = int(np.prod(shape))
+            if name.endswith("A_log"):
+                f.write(bf16(np.tile(np.log(np.arange(1, state + 1)), shape[0])).tobytes())
+                continue
+            src = ones if "norm" in name or name.endswith(".D") else small
+            left = n
+            while left > 0:
+                f.write(src[:min(left, src.size)].tobytes())
+                left -= src.size
+
+
+def lozedra_report(be, only=None, use_graph=True):
+    """Decode and prefill rates of Lozedra layers at real sizes (random weights) beside the closest model the engine had
+    before, a LLaMA layer graph with Q8_0 weights of the same width, heads and feed-forward. Decode: 32 sequences at the
+    end of a real 1000-token prompt each, greedy, replayed from a hipGraph. Prefill: one portion of a prompt."""
+    import shutil
+    import tempfile
+    from vexel_amd import lib
+    from vexel_amd.runtime import ModelRuntime
+    nseq, ctx, steps = 32, 1000, 32
+    portions = ((512, 0), (512, 3584), (2048, 0))
+    rng = np.random.default_rng(2)
+    for name, c in LOZEDRA_SHAPES.items():
+        if only not in (None, name):
+            continue
+        folder = tempfile.mkdtemp()
+        try:
+            write_lozedra(folder, **c)
+            mr = ModelRuntime.load(be, folder, pool_blocks=(nseq * (ctx + 200) + 8192) // BLOCK, max_seqs=nseq + 1,
+                                   max_blocks_per_seq=8192 // BLOCK, max_batch=64)
+        finally:
+            shutil.rmtree(folder)
+        llama = dict(num_layers=c["layers"], hidden=c["width"], num_heads=c["heads"], num_kv_heads=c["kv_heads"],
+                     head_dim=c["dim"], ffn=c["ff"], vocab=LOZEDRA_VOCAB)
+        lr, lids = build_model(be, [ctx] * nseq, 200, c["layers"], llama, {"*": lib.VX_Q8_0}, spare_tokens=8192)
+        tok = lambda n: rng.integers(0, LOZEDRA_VOCAB, n).tolist()
+        for lo in range(0, nseq, 4):
+            mr.step([(s, tok(ctx)) for s in range(lo, lo + 4)], [])
+        first = np.array(tok(nseq), dtype=np.int32)
+        print("layers of width %s, %d of each model" % (name, c["layers"]))
+        for label, r, ids in (("Lozedra bf16", mr, list(range(nseq))), ("LLaMA Q8_0", lr, lids)):
+            r.decode_graph(first, ids, [ctx] * nseq, 4, use_graph=use_graph)
+            be.sync()
+            t0 = time.perf_counter()
+            r.decode_graph(None, None, None, steps, use_graph=use_graph, batch=nseq)
+            be.sync()
+            dt = (time.perf_counter() - t0) / steps
+            print("  %-13s decode  %d x ctx %d: %8.0f tok/s  %7.3f ms/step  %6.1f us/layer" %
+                  (label, nseq, ctx, nseq / dt, dt * 1e3, dt * 1e6 / c["layers"]), flush=True)
+            for n, start in portions:
+                best = 1e9
+                for rep in range(4):
+                    sid = 5000
+                    at = 0
+                    while at < start:
+                        m = min(512, start - at)
+                        r.step([(sid, tok(m))], [])
+                        at += m
+                    body = tok(n)
+                    be.sync()
+                    t0 = time.perf_counter()
+                    r.step([(sid, body)], [n - 1])
+                    best = min(best, time.perf_counter() - t0) if rep else best   # (the first sizes the workspaces)
+                    r.delete_sequence(sid)
+                print("  %-13s prefill %4d tokens at %4d: %8.0f tok/s  %7.3f ms      %6.1f us/layer" %
+                      (label, n, start, n / best, best * 1e3, best * 1e6 / c["layers"]), flush=True)
+        mr.close()
+        lr.close()
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -799,6 +917,9 @@ def main():
                     help="batched decode rates of the Qwen 2 / Phi-2 / Gemma 2 layer graphs at published shapes, then exit")
     ap.add_argument("--medusa-report", action="store_true",
                     help="time the Medusa heads' forward pass and top-k at the 7B shape, then exit")
+    ap.add_argument("--lozedra-report", nargs="?", const="all", choices=["all"] + list(LOZEDRA_SHAPES),
+                    help="decode and prefill rates of Lozedra layers at real sizes beside LLaMA Q8_0 layers of the same "
+                         "sizes, then exit")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU: this build has no multi-GPU path (run with --gpus 1)", file=sys.stderr)
@@ -819,6 +940,9 @@ def main():
         return
     if args.arch_report:
         arch_report(be)
+        return
+    if args.lozedra_report:
+        lozedra_report(be, None if args.lozedra_report == "all" else args.lozedra_report, use_graph=not args.no_graph)
         return
     ctx = ragged_contexts(n=args.seqs) if args.seqs != BATCH else ragged_contexts()
     nseq = len(ctx)

@@ -31,9 +31,14 @@ def softplus(z):
     return np.logaddexp(0.0, z)
 
 
+# What an implementation with 16-bit activations rounds: the inputs of linear maps and the operands of attention. The
+# default keeps everything as it is; forward(.., rounded=True) uses bfloat16, to measure what that rounding alone does.
+_round = lambda a: a
+
+
 def linear(w, h):
     """w [out, in], h [tokens, in]"""
-    return h @ w.T
+    return _round(h) @ w.T
 
 
 def distance_bucket(n, rows, bias_max):
@@ -62,8 +67,9 @@ def attention(h, t, cfg):
     """t: tensors q, k, v, g, o, rel of one layer; positions 0 .. len(h) - 1"""
     T, H, G, D, V = len(h), cfg["heads"], cfg["kv_heads"], cfg["dim"], cfg["vdim"]
     q = linear(t["q"], h).reshape(T, H, D)
-    k = linear(t["k"], h).reshape(T, G, D)
-    v = linear(t["v"], h).reshape(T, G, V)
+    k = _round(linear(t["k"], h)).reshape(T, G, D)
+    v = _round(linear(t["v"], h)).reshape(T, G, V)
+    q = _round(q)
     pos = np.arange(T)
     qt = cfg.get("q_temp")
     if qt:
@@ -141,8 +147,15 @@ def layer_order(cfg):
     return runs + [(i, False) for i in range(lp["stop"], n)]
 
 
-def forward(cfg, tensors, tokens, residuals=None):
+def forward(cfg, tensors, tokens, residuals=None, rounded=False):
     """-> logits [tokens, vocab]; residuals: a list that receives the stream after every layer run"""
+    global _round
+    if rounded:
+        _round = lambda a: bf16_round(a).astype(F)
+        try:
+            return forward(cfg, tensors, tokens, residuals)
+        finally:
+            _round = lambda a: a
     T = {k: np.asarray(v, dtype=F) for k, v in tensors.items()}
     eps, mult = cfg["norm"]["eps"], cfg["residual_mult"]
     emb = T["embed"][np.asarray(tokens)]

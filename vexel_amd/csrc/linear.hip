@@ -278,6 +278,21 @@ __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_til
     }
 }
 
+// Adds up the slices of a VX_LIN_SPLIT map and deals the columns to its two results.
+template <typename T>
+__global__ void __launch_bounds__(256) split_sum_kernel(const float *part, int slices, int rows, int n, vx_linear_out o) {
+    const int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    const int per = n / 4, row = (int)(id / per), c = (int)(id % per) * 4;
+    if (row >= rows) return;
+    const float *src = part + (size_t)row * n + c;
+    f32x4 v = *(const f32x4 *)src;
+    for (int s = 1; s < slices; s++) v += *(const f32x4 *)(src + (size_t)s * rows * n);
+    if (c < o.split)
+        put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
+    else
+        put4(o.out2 + (size_t)row * o.ldo2, c - o.split, o.ldo2, o.ldo2, v);
+}
+
 // ---------------------------------------------------------------- packing
 __global__ void linear_pack_kernel(const uint16_t *src, int n, int k, uint16_t *dst, int k_pad, int tile0, int tile_step, int col0) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -292,15 +307,24 @@ __global__ void fill_zero_kernel(uint32_t *p, size_t n) {
 }
 
 // ---------------------------------------------------------------- launches
+template <typename T, int MT, int NT, int WAVES, int KIND>
+void launch_few_as(vx_backend *be, const LinArgs &p, int slices) {
+    linear_few_kernel<T, MT, NT, WAVES, KIND><<<dim3((p.n >> 4) / NT, slices), 64 * WAVES, 0, be->stream>>>(p);
+}
 template <typename T, int MT, int KIND>
 void launch_few(vx_backend *be, const LinArgs &p, int slices) {
-    constexpr int NT = KIND == VX_LIN_SWIGLU ? 2 : 1;
-    const int groups = (p.n >> 4) / NT;
-    // a narrow map gives the chip few workgroups: more waves each
-    if (groups * slices < 256)
-        linear_few_kernel<T, MT, NT, 16 / NT / (MT == 4 ? 2 : 1), KIND><<<dim3(groups, slices), 64 * (16 / NT / (MT == 4 ? 2 : 1)), 0, be->stream>>>(p);
-    else
-        linear_few_kernel<T, MT, NT, 8 / (MT == 4 && NT == 2 ? 2 : 1), KIND><<<dim3(groups, slices), 64 * (8 / (MT == 4 && NT == 2 ? 2 : 1)), 0, be->stream>>>(p);
+    const int tiles = p.n >> 4;
+    // two row tiles to a workgroup (an activation operand serves both) where that leaves enough workgroups
+    if constexpr (KIND == VX_LIN_SWIGLU) {
+        launch_few_as<T, MT, 2, MT == 4 ? 4 : 8, KIND>(be, p, slices);
+    } else if constexpr (MT < 4) {
+        if (tiles % 2 == 0 && tiles / 2 * slices >= 512)
+            launch_few_as<T, MT, 2, 8, KIND>(be, p, slices);
+        else
+            launch_few_as<T, MT, 1, 8, KIND>(be, p, slices);
+    } else {
+        launch_few_as<T, MT, 1, 8, KIND>(be, p, slices);
+    }
 }
 
 template <typename T, int BM, int BN, int KIND>
@@ -317,6 +341,24 @@ void many_tile(int n, int rows, int slices, int *bm, int *bn) {
     *bm = 64;
     if (wgs(64, 128) >= 256) return;
     *bn = 64;
+}
+
+// In how many slices of its inputs a map is best computed, when something adds the slices up afterwards.
+int pick_slices(int n, int k, int rows) {
+    const int ktiles = k / 64;
+    int64_t wgs;
+    int want, least;
+    if (rows <= 64) {
+        wgs = n / 16, want = wgs >= 192 ? 512 : 192, least = 16;  // (a wave's four steps of 32 inputs, eight waves)
+        if (wgs >= want) return 1;
+    } else {
+        wgs = (int64_t)ceil_div(rows, 128) * ceil_div(n, 128), want = 512, least = 12;
+        if (wgs >= 384) return 1;
+    }
+    int s = (int)((want + wgs - 1) / wgs);
+    if (s > 8) s = 8;
+    if (s > ktiles / least) s = ktiles / least;
+    return s < 1 ? 1 : s;
 }
 
 template <typename T, int KIND>
@@ -414,21 +456,7 @@ int vx_linear_pack(vx_backend *be, const void *src, int n, int k, void *dst, int
 int vx_linear_slices(vx_backend *be, int n, int k, int rows) {
     (void)be;
     if (n <= 0 || k <= 0 || rows <= 0) return 1;
-    const int most = k / 64 / 8 > 1 ? k / 64 / 8 : 1;  // at least 512 inputs a slice
-    int64_t wgs;
-    if (rows <= 64) {
-        wgs = n / 16;
-        if (wgs >= 192) return 1;
-    } else {
-        int bm, bn;
-        many_tile(n, rows, 1, &bm, &bn);
-        wgs = (int64_t)ceil_div(rows, bm) * ceil_div(n, bn);
-        if (wgs >= 192) return 1;
-    }
-    int s = (int)(256 / (wgs > 0 ? wgs : 1));
-    if (s > 8) s = 8;
-    if (s > most) s = most;
-    return s < 1 ? 1 : s;
+    return pick_slices(n, k, rows);
 }
 
 int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, int n, int k, int rows, const vx_linear_out *o) {
@@ -459,6 +487,24 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
                        o->k_col + o->kv_heads * o->k_dim <= n && o->v_col + o->kv_heads * o->v_dim <= n,
                    "vx_linear: bad K/V columns");
     LinArgs p{a, w, lda, n, k, rows, *o};
+    if (o->kind == VX_LIN_SPLIT) {  // (narrow and deep as a rule) in slices, added up by a kernel of their own
+        const int cut = pick_slices(n, k, rows);
+        if (cut > 1) {
+            const size_t bytes = (size_t)cut * rows * n * 4;
+            rc = ensure_ws(be, &be->part_ws, &be->part_ws_bytes, bytes, "partial sums");
+            if (rc) return rc;
+            p.o.kind = VX_LIN_PLAIN, p.o.out_f32 = 1, p.o.out = be->part_ws, p.o.ldo = p.o.cols = n;
+            rc = act == VX_ACT_BF16 ? dispatch<bf16>(be, p, cut) : dispatch<float>(be, p, cut);
+            if (rc) return rc;
+            const unsigned grid = (unsigned)ceil_div64((int64_t)rows * (n / 4), 256);
+            if (act == VX_ACT_BF16)
+                split_sum_kernel<bf16><<<grid, 256, 0, be->stream>>>((const float *)be->part_ws, cut, rows, n, *o);
+            else
+                split_sum_kernel<float><<<grid, 256, 0, be->stream>>>((const float *)be->part_ws, cut, rows, n, *o);
+            VX_CHECK_LAUNCH();
+            return VX_OK;
+        }
+    }
     return act == VX_ACT_BF16 ? dispatch<bf16>(be, p, slices) : dispatch<float>(be, p, slices);
 }
 

@@ -133,35 +133,45 @@ struct ConvArgs {
     int n_seqs, one_token;
 };
 
-template <typename T>
-__global__ void __launch_bounds__(256) conv_silu_kernel(ConvArgs a) {
+// A thread takes VEC neighbouring channels of one row.
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256) conv_silu_kernel(ConvArgs a, int rows) {
+    typedef T V __attribute__((ext_vector_type(VEC)));
+    typedef float F __attribute__((ext_vector_type(VEC)));
     const vx_conv_args &p = a.p;
-    const int row = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x;
-    if (c >= p.ldo) return;
-    T *out = (T *)p.out + (size_t)row * p.ldo + c;
+    const int per = p.ldo / VEC;
+    const int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    const int row = (int)(id / per), c = (int)(id % per) * VEC;
+    if (row >= rows) return;
+    V *out = (V *)((T *)p.out + (size_t)row * p.ldo + c);
     if (c >= p.channels) {
-        *out = (T)0.f;
+        *out = (V)(T)0.f;
         return;
     }
     const int seq = a.one_token ? row : seq_of_row(a.cu, a.n_seqs, row);
     const int local = a.one_token ? 0 : row - a.cu[seq], pos = a.pos[row], hist = p.taps - 1;
     T *st = (T *)p.state + (size_t)a.slots[seq] * hist * p.channels + c;
     const T *x = (const T *)p.x + (size_t)row * p.ldx + c;
-    float acc = p.b[c];
+    F acc = *(const F *)(p.b + c);
     for (int t = 0; t < p.taps; t++) {
         const int d = hist - t;  // tokens back
-        float v = 0.f;
+        V v = (V)(T)0.f;
         if (d <= local)
-            v = (float)*(x - (ptrdiff_t)d * p.ldx);
+            v = *(const V *)(x - (ptrdiff_t)d * p.ldx);
         else if (d <= pos)
-            v = (float)st[(size_t)(hist - (d - local)) * p.channels];
-        acc = fmaf(p.w[(size_t)t * p.channels + c], v, acc);
+            v = *(const V *)(st + (size_t)(hist - (d - local)) * p.channels);
+        const F w = *(const F *)(p.w + (size_t)t * p.channels + c);
+#pragma unroll
+        for (int e = 0; e < VEC; e++) acc[e] = fmaf(w[e], (float)v[e], acc[e]);
     }
-    *out = (T)silu_f(acc);
-    if (a.one_token) {  // this thread alone reads and moves the channel's history
+    V o;
+#pragma unroll
+    for (int e = 0; e < VEC; e++) o[e] = (T)silu_f(acc[e]);
+    *out = o;
+    if (a.one_token) {  // this thread alone reads and moves the channels' history
         for (int k = 0; k + 1 < hist; k++)
-            st[(size_t)k * p.channels] = pos - (hist - 1 - k) >= 0 ? st[(size_t)(k + 1) * p.channels] : (T)0.f;
-        if (hist > 0) st[(size_t)(hist - 1) * p.channels] = *x;
+            *(V *)(st + (size_t)k * p.channels) = pos - (hist - 1 - k) >= 0 ? *(const V *)(st + (size_t)(k + 1) * p.channels) : (V)(T)0.f;
+        if (hist > 0) *(V *)(st + (size_t)(hist - 1) * p.channels) = *(const V *)x;
     }
 }
 
@@ -405,13 +415,22 @@ int vx_conv_silu(vx_backend *be, int act, const vx_ragged *b, const vx_conv_args
                    p->ldx >= p->channels && p->ldo >= p->channels,
                "vx_conv_silu: bad arguments");
     ConvArgs a{*p, b->cu_seqlens, b->token_pos, b->table_rows, b->n_seqs, b->q_lens ? 0 : 1};
-    const dim3 grid(b->rows, ceil_div(p->ldo, 256)), sgrid(b->n_seqs, ceil_div(p->channels, 256));
-    if (act == VX_ACT_BF16) {
-        conv_silu_kernel<bf16><<<grid, 256, 0, be->stream>>>(a);
-        if (b->q_lens && p->taps > 1) conv_state_kernel<bf16><<<sgrid, 256, 0, be->stream>>>(a);
-    } else {
-        conv_silu_kernel<float><<<grid, 256, 0, be->stream>>>(a);
-        if (b->q_lens && p->taps > 1) conv_state_kernel<float><<<sgrid, 256, 0, be->stream>>>(a);
+    const auto al = [](const void *q) { return (uintptr_t)q % 32 == 0; };
+    const bool vec = p->channels % 8 == 0 && p->ldx % 8 == 0 && p->ldo % 8 == 0 && al(p->w) && al(p->b) && (uintptr_t)p->x % 16 == 0 &&
+                     (uintptr_t)p->out % 16 == 0 && (uintptr_t)p->state % 16 == 0 && act == VX_ACT_BF16;
+    const unsigned grid = (unsigned)ceil_div64((int64_t)b->rows * (p->ldo / (vec ? 8 : 1)), 256);
+    const dim3 sgrid(b->n_seqs, ceil_div(p->channels, 256));
+    if (vec)
+        conv_silu_kernel<bf16, 8><<<grid, 256, 0, be->stream>>>(a, b->rows);
+    else if (act == VX_ACT_BF16)
+        conv_silu_kernel<bf16, 1><<<grid, 256, 0, be->stream>>>(a, b->rows);
+    else
+        conv_silu_kernel<float, 1><<<grid, 256, 0, be->stream>>>(a, b->rows);
+    if (b->q_lens && p->taps > 1) {
+        if (act == VX_ACT_BF16)
+            conv_state_kernel<bf16><<<sgrid, 256, 0, be->stream>>>(a);
+        else
+            conv_state_kernel<float><<<sgrid, 256, 0, be->stream>>>(a);
     }
     VX_CHECK_LAUNCH();
     return VX_OK;

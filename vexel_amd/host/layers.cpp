@@ -271,8 +271,10 @@ int mix_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_l
     {
         std::lock_guard<std::mutex> g(m->pool.mu);
         int64_t need = 0;
+        size_t fresh = 0;
         for (int i = 0; i < n_seqs; i++) {  // nothing changes unless the whole step has room
             const SeqState *s = find_seq(m, seq_ids[i]);
+            fresh += s == nullptr;
             const int have = s ? (int)s->table.size() : 0, len = (s ? s->seq_len : 0) + q_lens[i];
             const int blocks = (len - 1) / c.block_size + 1;
             if (blocks > c.max_blocks_per_seq)
@@ -280,6 +282,7 @@ int mix_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_l
                             c.max_blocks_per_seq);
             need += std::max(0, blocks - have);
         }
+        if (fresh > m->pool.free_slots.size()) return fail("more than %d live sequences", c.max_seqs);
         if (need > (int64_t)m->pool.free_list.size())
             return fail("no free blocks: the step needs %lld, the pool has %zu", (long long)need, m->pool.free_list.size());
         for (int i = 0; i < n_seqs; i++) {
