@@ -780,6 +780,20 @@ def test_loader_errors(be, tmp_path):
         ModelRuntime.load(be, str(tmp_path / "nothing"))
 
 
+def test_generation_from_the_command_line(be, tmp_path, capsys):
+    from vexel_amd.__main__ import main
+    cfg = SMALL
+    t = tensors(cfg, 2)
+    lz.write_model(str(tmp_path / "m"), cfg, t)
+    prompts = [prompt(cfg, 9, 1), prompt(cfg, 30, 2)]
+    args = ["generate", "--model", str(tmp_path / "m"), "--dtype", "float32", "--max-new", "5", "--prefill-chunk", "8"]
+    for p in prompts:
+        args += ["--tokens", ",".join(map(str, p))]
+    assert main(args) == 0
+    got = [[int(x) for x in line.split()] for line in capsys.readouterr().out.splitlines()]
+    assert got == [greedy(cfg, t, p, 5) for p in prompts]
+
+
 def test_trace_replay(be, tmp_path):
     """bin/trace_run in a process of its own: steps in, logits out, blocks and slots given back at the end of requests."""
     cfg = SMALL

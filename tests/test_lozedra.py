@@ -140,3 +140,9 @@ def test_written_tensors_come_back(tmp_path):
     lz.write_model(str(tmp_path), SMALL, t)
     back = lz.read_tensors(str(tmp_path / "model.safetensors"))
     assert set(back) == set(t) and all(np.array_equal(back[n], t[n]) for n in t)
+
+
+def test_command_line_lists_architectures(capsys):
+    from vexel_amd.__main__ import main
+    assert main(["architectures"]) == 0
+    assert "Lozedra" in capsys.readouterr().out.split()
