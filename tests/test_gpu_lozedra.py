@@ -466,9 +466,11 @@ def test_attention_options(be, act):
             run_attention(be, act, Batch(be, *batch, seed=3), 4, 2, 32, 48, seed=5, **kw)
 
 
-def test_attention_many_query_tiles(be):
-    """Enough rows for the kernel with two query tiles a wave."""
-    run_attention(be, BF16, Batch(be, [0, 33], [210, 170], seed=4), 128, 64, 16, 16, seed=1)
+@pytest.mark.parametrize("heads,start,lens", [(128, 33, 400), (128, 0, 180), (16, 1000, 515), (64, 5, 402), (64, 0, 263)])
+def test_attention_many_rows(be, heads, start, lens):
+    """Enough rows for each way of dealing queries and keys to a workgroup's waves: one or two query tiles a wave, one, two or
+    four waves to the same queries."""
+    run_attention(be, BF16, Batch(be, [start, 40, 0], [lens, 1, 3], seed=4), heads, heads // 4, 16, 16, seed=1)
 
 
 @pytest.mark.parametrize("act", ACTS)

@@ -214,21 +214,26 @@ __device__ __forceinline__ void write4(const Args &a, int row, int h, int d, f32
     }
 }
 
-template <int KD, int VD, int QT>
+// The four waves of a workgroup: 4 / KS groups of QT x 16 queries, KS waves to a group that take turns at the key groups.
+template <int KD, int VD, int QT, int KS>
 __global__ void __launch_bounds__(256) prefill_kernel(Args a) {
-    extern __shared__ float s_lut[];
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    extern __shared__ float s_dyn[];
+    constexpr int RG = 4 / KS, LDO = VD * 16 + 4;
+    __shared__ float s_m[RG][KS][QT * 16], s_l[RG][KS][QT * 16];
+    float *s_lut = s_dyn;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, rg = wave / KS, ks_id = wave % KS;
     const int g = blockIdx.x % a.p.kv_heads, id = a.tiles - 1 - blockIdx.x / a.p.kv_heads;  // late tiles, the longest, first
     int seq, ti, count;
     if (!item_of_seq(a.cu, a.n_seqs, a.tile_rows, 2, id, &seq, &ti, &count)) return;
     load_lut(a, g, s_lut);
     const int row0 = a.cu[seq] + ti * a.tile_rows, ntok = min(a.tile_rows, a.cu[seq + 1] - row0);
     const int pos0 = a.pos[row0];
-    const int m_first = wave * 16 * QT;
-    if (m_first >= ntok * a.group) return;  // (no barrier follows)
+    const int m_first = rg * 16 * QT;
+    const bool any = m_first < ntok * a.group;  // the group has queries (the last tile of a sequence may be short)
+    if (KS == 1 && !any) return;                // (no barrier follows)
     const int32_t *bt = a.tables + (size_t)a.rows[seq] * a.max_blocks;
-    const int t_lo = m_first / a.group, t_hi = min((m_first + 16 * QT - 1) / a.group, ntok - 1);
-    const int pos_lo = pos0 + t_lo, pos_hi = pos0 + t_hi, last_blk = pos_hi / BS, groups = pos_hi / 32 + 1;
+    const int t_lo = min(m_first / a.group, ntok - 1), t_hi = min((m_first + 16 * QT - 1) / a.group, ntok - 1);
+    const int pos_lo = pos0 + t_lo, pos_hi = pos0 + t_hi, last_blk = pos_hi / BS, groups = any ? pos_hi / 32 + 1 : 0;
 
     Queries<KD, VD, QT> qs;
     qs.clear();
@@ -248,24 +253,77 @@ __global__ void __launch_bounds__(256) prefill_kernel(Args a) {
     }
     Keys<KD, VD, false> ks;
     ks.init(a, g, lane);
-    int b0 = bt[0], b1 = bt[min(1, last_blk)];
-    ks.load_k(b0, b1);
-    for (int gi = 0; gi < groups; gi++) {
-        ks.load_v(b0, b1, lane);
-        const bool more = gi + 1 < groups;
-        if (more) b0 = bt[min(2 * gi + 2, last_blk)], b1 = bt[min(2 * gi + 3, last_blk)];
-        const int k0 = gi * 32;
-        group<KD, VD, QT, false>(a, ks, qs, k0, b0, b1, more, lane, k0 + 31 <= pos_lo, pos_lo - (k0 + 31) >= a.p.bias_len - 1, s_lut);
+    int gi = ks_id;
+    if (gi < groups) {
+        int b0 = bt[min(2 * gi, last_blk)], b1 = bt[min(2 * gi + 1, last_blk)];
+        ks.load_k(b0, b1);
+        for (; gi < groups; gi += KS) {
+            ks.load_v(b0, b1, lane);
+            const bool more = gi + KS < groups;
+            if (more) b0 = bt[min(2 * (gi + KS), last_blk)], b1 = bt[min(2 * (gi + KS) + 1, last_blk)];
+            const int k0 = gi * 32;
+            group<KD, VD, QT, false>(a, ks, qs, k0, b0, b1, more, lane, k0 + 31 <= pos_lo, pos_lo - (k0 + 31) >= a.p.bias_len - 1, s_lut);
+        }
     }
+    float l[QT];
 #pragma unroll
     for (int t = 0; t < QT; t++) {
-        float l = qs.l[t];
-        l += __shfl_xor(l, 16, 64);
-        l += __shfl_xor(l, 32, 64);
-        if (tok[t] >= ntok) continue;
-        const float inv = 1.0f / l;  // (a row sees itself: l > 0)
+        l[t] = qs.l[t];
+        l[t] += __shfl_xor(l[t], 16, 64);
+        l[t] += __shfl_xor(l[t], 32, 64);
+    }
+    if constexpr (KS == 1) {
 #pragma unroll
-        for (int v = 0; v < VD; v++) write4(a, row0 + tok[t], head[t], v * 16 + (lane >> 4) * 4, qs.o[t][v] * inv);
+        for (int t = 0; t < QT; t++) {
+            if (tok[t] >= ntok) continue;
+            const float inv = 1.0f / l[t];  // (a row sees itself: l > 0)
+#pragma unroll
+            for (int v = 0; v < VD; v++) write4(a, row0 + tok[t], head[t], v * 16 + (lane >> 4) * 4, qs.o[t][v] * inv);
+        }
+    } else {
+        // the results of a group's waves become one
+#pragma unroll
+        for (int t = 0; t < QT; t++)
+            if (lane < 16) s_m[rg][ks_id][t * 16 + lane] = qs.m[t], s_l[rg][ks_id][t * 16 + lane] = l[t];
+        __syncthreads();  // (the bias tables in s_dyn are done with as well)
+        float *s_o = s_dyn + rg * QT * 16 * LDO;
+        float mg[QT];
+#pragma unroll
+        for (int t = 0; t < QT; t++) {
+            mg[t] = -INFINITY;
+#pragma unroll
+            for (int w = 0; w < KS; w++) mg[t] = fmaxf(mg[t], s_m[rg][w][t * 16 + (lane & 15)]);
+        }
+        for (int w = 0; w < KS; w++) {
+            if (ks_id == w) {
+#pragma unroll
+                for (int t = 0; t < QT; t++) {
+                    const float f = qs.m[t] > -INFINITY ? __builtin_amdgcn_exp2f(qs.m[t] - mg[t]) : 0.f;
+#pragma unroll
+                    for (int v = 0; v < VD; v++) {
+                        f32x4 *dst = (f32x4 *)(s_o + (t * 16 + (lane & 15)) * LDO + v * 16 + (lane >> 4) * 4);
+                        const f32x4 x = qs.o[t][v] * f;
+                        *dst = w == 0 ? x : *dst + x;
+                    }
+                }
+            }
+            __syncthreads();
+        }
+        if (!any) return;
+#pragma unroll
+        for (int t = 0; t < QT; t++) {
+            if (tok[t] >= ntok) continue;
+            float sum = 0.f;
+#pragma unroll
+            for (int w = 0; w < KS; w++) {
+                const float mw = s_m[rg][w][t * 16 + (lane & 15)];
+                if (mw > -INFINITY) sum += s_l[rg][w][t * 16 + (lane & 15)] * __builtin_amdgcn_exp2f(mw - mg[t]);
+            }
+            const float inv = 1.0f / sum;
+            for (int v = ks_id; v < VD; v += KS)
+                write4(a, row0 + tok[t], head[t], v * 16 + (lane >> 4) * 4,
+                       *(const f32x4 *)(s_o + (t * 16 + (lane & 15)) * LDO + v * 16 + (lane >> 4) * 4) * inv);
+        }
     }
 }
 
@@ -474,12 +532,13 @@ __global__ void __launch_bounds__(256) plain_kernel(Args a) {
     }
 }
 
-template <int KD, int VD, int QT>
+template <int KD, int VD, int QT, int KS>
 void launch_prefill(vx_backend *be, Args a, const vx_ragged *b) {
-    a.tile_rows = 64 * QT / a.group;
+    a.tile_rows = 64 / KS * QT / a.group;
     a.tiles = count_items(b, a.tile_rows, 2);
-    const size_t lds = a.lut_lds ? (size_t)a.group * a.p.bias_len * 4 : 0;
-    if (a.tiles > 0) prefill_kernel<KD, VD, QT><<<a.tiles * a.p.kv_heads, 256, lds, be->stream>>>(a);
+    const size_t lut = a.lut_lds ? (size_t)a.group * a.p.bias_len * 4 : 0;
+    const size_t o = KS > 1 ? (size_t)4 / KS * QT * 16 * (VD * 16 + 4) * 4 : 0;
+    if (a.tiles > 0) prefill_kernel<KD, VD, QT, KS><<<a.tiles * a.p.kv_heads, 256, lut > o ? lut : o, be->stream>>>(a);
 }
 
 template <int KD, int VD>
@@ -498,11 +557,30 @@ int run_fast(vx_backend *be, Args a, const vx_ragged *b) {
             if (b->q_lens[s] > 1) many += b->q_lens[s];
         }
     if (any_many) {
-        // two query tiles a wave where that still gives the chip enough workgroups
-        if (VD <= 8 && a.group <= 64 && many * a.p.heads / 128 >= 384) {
-            if constexpr (VD <= 8) launch_prefill<KD, VD, 2>(be, a, b);
-        } else {
-            launch_prefill<KD, VD, 1>(be, a, b);
+        // Two query tiles a wave halve the keys' traffic; waves that share queries make more workgroups of few rows (the
+        // limits are measured).
+        const int64_t tiles16 = many * a.p.heads / 16;  // query tiles of the step
+        const int qt = VD <= 8 && (tiles16 >= 2048 || (tiles16 >= 512 && b->max_kv_len > 1024)) ? 2 : 1;
+        const int64_t wgs = tiles16 / (4 * qt);
+        int ks = wgs >= 384 ? 1 : wgs >= (qt == 2 ? 128 : 256) ? 2 : 4;
+        while (ks > 1 && 64 / ks * qt < a.group) ks /= 2;
+        if constexpr (VD <= 8) {
+            if (qt == 2) {
+                if (ks == 1)
+                    launch_prefill<KD, VD, 2, 1>(be, a, b);
+                else if (ks == 2)
+                    launch_prefill<KD, VD, 2, 2>(be, a, b);
+                else
+                    launch_prefill<KD, VD, 2, 4>(be, a, b);
+            }
+        }
+        if (qt == 1) {
+            if (ks == 1)
+                launch_prefill<KD, VD, 1, 1>(be, a, b);
+            else if (ks == 2)
+                launch_prefill<KD, VD, 1, 2>(be, a, b);
+            else
+                launch_prefill<KD, VD, 1, 4>(be, a, b);
         }
         VX_CHECK_LAUNCH();
     }

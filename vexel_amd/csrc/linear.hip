@@ -70,8 +70,7 @@ __device__ __forceinline__ void emit(const LinArgs &p, int slice, int row, int c
         f32x4 u;
 #pragma unroll
         for (int r = 0; r < 4; r++) {
-            const float z = v[r] + (c + r < o.cols ? o.bias[c + r] : 0.f);
-            u[r] = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
+            u[r] = softplus_f(v[r] + (c + r < o.cols ? o.bias[c + r] : 0.f));
         }
         put4((float *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, u);
     } else {  // VX_LIN_KV: K and V columns leave for the pool (segments start at multiples of 16 columns)

@@ -30,8 +30,25 @@ __device__ __forceinline__ f32x4 mma(bf16x8 a, f32x8 b, f32x4 acc) {  // bfloat1
     return acc;
 }
 
-__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+// The hardware's exponential and reciprocal are good to a unit in the last place; the exponent's own rounding adds |z| times
+// that.
+__device__ __forceinline__ float sigmoid_f(float z) {
+    return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z * -1.4426950408889634f));
+}
+__device__ __forceinline__ float silu_f(float z) { return z * sigmoid_f(z); }
+
+// log(1 + exp(z)) = max(z, 0) + log(1 + e), e = exp(-|z|); log(1 + e) = 2 artanh(s), s = e / (2 + e) <= 1/3, by its series
+// (the first term left out is below 2e-8 of the sum), which keeps the relative precision of small results.
+__device__ __forceinline__ float softplus_f(float z) {
+    const float e = expf(-fabsf(z)), s = e / (2.0f + e), q = s * s;
+    float t = 1.0f / 13.0f;
+    t = fmaf(t, q, 1.0f / 11.0f);
+    t = fmaf(t, q, 1.0f / 9.0f);
+    t = fmaf(t, q, 1.0f / 7.0f);
+    t = fmaf(t, q, 1.0f / 5.0f);
+    t = fmaf(t, q, 1.0f / 3.0f);
+    return fmaxf(z, 0.f) + 2.0f * fmaf(s * q, t, s);
+}
 
 __device__ __forceinline__ void store4(float *p, f32x4 v) { *(f32x4 *)p = v; }
 __device__ __forceinline__ void store4(bf16 *p, f32x4 v) {
