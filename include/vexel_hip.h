@@ -502,7 +502,10 @@ enum {
     VX_LIN_KV = 2,     /* PLAIN in the activation type, but columns [k_col, k_col + kv_heads * k_dim) and [v_col, ..) go
                           to the paged pool at slot_mapping[r] (layout: vx_kv_block_elems) */
     VX_LIN_SPLIT = 3,  /* columns < split to out (activation type), the others to out2[r * ldo2 + c - split] (float32) */
-    VX_LIN_SOFTPLUS = 4 /* float32 out = log(1 + exp(y + bias[c])) */
+    VX_LIN_SOFTPLUS = 4, /* float32 out = log(1 + exp(y + bias[c])) */
+    VX_LIN_ROTARY = 5  /* columns < split to out (activation type) in heads of rot_stride columns, whose columns rot_first ..
+                          rot_first + 2 * rot_pairs - 1 are turned in neighbouring pairs by rot_tab (vx_rotary_table); the
+                          others (split = n: none) to out2 as with SPLIT */
 };
 typedef struct vx_linear_out {
     int kind, out_f32, ldo, cols, slices;
@@ -512,7 +515,13 @@ typedef struct vx_linear_out {
     const float *bias;
     int k_col, v_col, kv_heads, k_dim, v_dim, block_size;
     void *pool;
-    const int32_t *slot_mapping;
+    const int32_t *slot_mapping; /* NULL: row r's slot is r */
+    const int32_t *a_rows;       /* activation row r is row a_rows[r] of a; NULL: row r */
+    float softcap;               /* > 0 (PLAIN, one slice): softcap * tanh(y / softcap) */
+    int groups, a_group, out_group; /* groups > 1 (PLAIN, one slice): that many maps [n, k] one behind the other in w; map g takes
+                                    the activations from column g * a_group on and writes from column g * out_group on */
+    int rot_stride, rot_first, rot_pairs;
+    const float *rot_tab;
 } vx_linear_out;
 /* out = a [rows, k] * W^T for a packed matrix [n, k] (padded sizes); a has lda >= k columns of the activation type, zero
  * where k was padded, rows 16-byte aligned. vx_linear_slices: into how many slices a PLAIN float32 result is best cut
@@ -541,7 +550,7 @@ int vx_residual_norm(vx_backend *be, int act, const vx_residual_norm_args *p);
 
 /* Causal grouped-query attention over the paged pool for every row of a mixed batch (the rows' K and V are in it already):
  *   score(i, j) = (temp(i) * scale) * q_i . k_j + bias[h][min(i - j, bias_len - 1)],  softmax over j <= i,
- *   out = out_scale * sigmoid(gate) * (weights . v)
+ *   out = out_scale * sigmoid(gate) * (weights . v);  with sink, exp(sink[h]) counts once more in the weights' denominator
  * temp(i) = 1 + temp_coef * ln(floor((i + 1) / temp_every) + 1); temp_every 0: 1. bias NULL: none (float32
  * [heads][bias_len] on the device). gate NULL: none. q, gate, out: activation type, head h at columns h * k_dim (q)
  * and h * v_dim (gate, out).
@@ -559,11 +568,89 @@ typedef struct vx_attn_args {
     float out_scale;
     void *out;
     int ldo;
+    const float *sink;           /* [heads]: the softmax's denominator also holds exp(sink[h]); NULL: none */
+    int min_rows;                /* > 1: only the rows of sequences that bring at least so many */
 } vx_attn_args;
 size_t vx_kv_block_elems(int block_size, int kv_heads, int k_dim, int v_dim);
 int vx_attn_ragged(vx_backend *be, int act, const vx_ragged *b, const vx_attn_args *p);
 /* 1 when the matrix-core kernels take the geometry, 0 when vx_attn_ragged uses the plain one. */
 int vx_attn_ragged_fast(int act, int block_size, int heads, int kv_heads, int k_dim, int v_dim);
+
+/* ---- latent attention: a token is kept as one normed vector c [rank] and one rotated key part kr [rot_dim] for all heads.
+ * Pool of one layer: one row per slot (block * block_size + offset), c at column 0 and kr at column vx_latent_pad(rank), of
+ * vx_latent_row(rank, rot_dim) columns of the activation type; it must have been zeroed once (the columns between stay
+ * zero). */
+int vx_latent_pad(int rank);
+int vx_latent_row(int rank, int rot_dim);
+/* cos and sin of position * freqs[i], times factor, for every row and pair: out [rows][pairs][2]. freqs: device double. */
+int vx_rotary_table(vx_backend *be, const int32_t *token_pos, int rows, int pairs, const double *freqs, float factor, float *out);
+/* From a float32 projection y (slices added up): c = rmsnorm(y[c_col ..]) * w_c and kr = y[kr_col ..] turned in neighbouring
+ * pairs go to the pool at slot_mapping[r] (rank 0: neither); rmsnorm(y[q_col ..]) * w_q goes to q_out (q_rank 0: not), its
+ * columns q_rank .. ldq - 1 zero. */
+typedef struct vx_latent_store_args {
+    int rank, rot_dim, q_rank;
+    const float *y;
+    int y_slices, ldy;
+    int64_t y_stride;
+    int c_col, kr_col, q_col;
+    float eps;
+    const float *w_c, *w_q, *rot_tab;
+    void *pool, *q_out;
+    int ldq;
+} vx_latent_store_args;
+int vx_latent_store(vx_backend *be, int act, const vx_ragged *b, const vx_latent_store_args *p);
+/* Causal attention over the latents as they are kept, for queries that were carried into the latents' space:
+ *   score(i, j, h) = scale * (q_i[h] . c_j + qr_i[h] . kr_j),  weights over j <= i with exp(sink[h]) in the denominator,
+ *   out_i[h] = weights . c
+ * q and out: activation type, head h at columns h * vx_latent_pad(rank) (columns beyond rank: zero in q, written in out); qr: head
+ * h at columns h * qr_stride, columns rot_dim .. rot_dim rounded up to 16 zero. max_rows > 0: only the rows of sequences that bring at most
+ * so many. */
+typedef struct vx_latent_attn_args {
+    int heads, rank, rot_dim;
+    float scale;
+    const float *sink;
+    const void *q, *qr;
+    int ldq, ldqr, qr_stride;
+    const void *pool;
+    void *out;
+    int ldo, max_rows;
+} vx_latent_attn_args;
+int vx_attn_latent(vx_backend *be, int act, const vx_ragged *b, const vx_latent_attn_args *p);
+/* 1 when the matrix-core kernel takes the geometry, 0 when vx_attn_latent uses the plain one. */
+int vx_attn_latent_fast(int act, int block_size, int rank, int rot_dim);
+/* The rotated key part of row a_rows[r] of a latent pool into columns first .. of every head of row r of a K pool (layout:
+ * vx_kv_block_elems; the slot of row r is r). */
+int vx_latent_spread(vx_backend *be, int act, const void *latent_pool, int rank, int rot_dim, const int32_t *a_rows, int rows, void *pool,
+                     int kv_heads, int k_dim, int v_dim, int block_size, int first);
+
+/* The seam behind a sublayer whose norm follows the residual sum, one row at a time, in float32:
+ *   v = alpha * x_in[r] + sum over slices of y[s][r], normed and multiplied by w   (w NULL: v = x_in[r], y unused)
+ *   n_avg > 0: hist[n_avg - 1][r] = v (keep), v = sum over j < n_avg of avg[j] * hist[j][r]
+ *   x_out[r] = v (NULL: not);  out[i] = v, or rmsnorm(v) * w_pre, in the activation type, columns cols .. ldo - 1 zero
+ * r = row_idx ? row_idx[i] : i for i < rows. x_out may be x_in. w, w_pre, avg: device float32. */
+typedef struct vx_post_norm_args {
+    int rows, cols;
+    const int32_t *row_idx;
+    const float *x_in, *y;
+    int y_slices, ldy;
+    int64_t y_stride;
+    float alpha, eps;
+    const float *w;
+    float *hist;
+    int64_t hist_stride;         /* floats from one result to the next */
+    const float *avg;
+    int n_avg, keep;
+    float *x_out;
+    const float *w_pre;
+    void *out;
+    int ldo;
+} vx_post_norm_args;
+int vx_post_norm(vx_backend *be, int act, const vx_post_norm_args *p);
+
+/* Polynomial activation normed over the row, in float32: out = coef[0] * N(z) + coef[1] * N(z^2) + coef[2] * N(z^3) + coef[3] with
+ * N(u) = u / sqrt(mean over the row's cols columns of u^2 + eps), powers element by element. z, out: activation type;
+ * columns cols .. ldo - 1 of out become zero. coef: device float32[4]. */
+int vx_poly_norm(vx_backend *be, int act, const void *z, int ldz, int rows, int cols, const float *coef, float eps, void *out, int ldo);
 
 /* Causal depthwise convolution with SiLU over a mixed batch: out[r][c] = silu(b[c] + sum_t w[t][c] * x[position - (taps
  * - 1 - t)][c]), positions before the sequence's start count as zero, positions before this step's rows come from

@@ -36,7 +36,8 @@ class VxRagged(C.Structure):
 
 class VxLinearOut(C.Structure):
     _fields_ = _fields("int kind out_f32 ldo cols slices; ptr out out2; int split ldo2; ptr bias; int k_col v_col kv_heads "
-                       "k_dim v_dim block_size; ptr pool slot_mapping")
+                       "k_dim v_dim block_size; ptr pool slot_mapping a_rows; float softcap; int groups a_group out_group "
+                       "rot_stride rot_first rot_pairs; ptr rot_tab")
 
 
 class VxResidualNormArgs(C.Structure):
@@ -46,7 +47,21 @@ class VxResidualNormArgs(C.Structure):
 
 class VxAttnArgs(C.Structure):
     _fields_ = _fields("int heads kv_heads k_dim v_dim; float scale temp_coef; int temp_every; ptr bias; int bias_len; "
-                       "ptr q gate; int ldq ldg; ptr pool; float out_scale; ptr out; int ldo")
+                       "ptr q gate; int ldq ldg; ptr pool; float out_scale; ptr out; int ldo; ptr sink; int min_rows")
+
+
+class VxLatentStoreArgs(C.Structure):
+    _fields_ = _fields("int rank rot_dim q_rank; ptr y; int y_slices ldy; i64 y_stride; int c_col kr_col q_col; float eps; "
+                       "ptr w_c w_q rot_tab pool q_out; int ldq")
+
+
+class VxLatentAttnArgs(C.Structure):
+    _fields_ = _fields("int heads rank rot_dim; float scale; ptr sink q qr; int ldq ldqr qr_stride; ptr pool out; int ldo max_rows")
+
+
+class VxPostNormArgs(C.Structure):
+    _fields_ = _fields("int rows cols; ptr row_idx x_in y; int y_slices ldy; i64 y_stride; float alpha eps; ptr w hist; "
+                       "i64 hist_stride; ptr avg; int n_avg keep; ptr x_out w_pre out; int ldo")
 
 
 class VxConvArgs(C.Structure):
@@ -447,6 +462,24 @@ class HipBackend:
 
     def attn_ragged(self, act, batch, args):
         self.call("vx_attn_ragged", act, C.byref(batch), C.byref(args))
+
+    def rotary_table(self, token_pos, rows, pairs, freqs, factor, out):
+        self.call("vx_rotary_table", token_pos, rows, pairs, freqs, factor, out)
+
+    def latent_store(self, act, batch, args):
+        self.call("vx_latent_store", act, C.byref(batch), C.byref(args))
+
+    def attn_latent(self, act, batch, args):
+        self.call("vx_attn_latent", act, C.byref(batch), C.byref(args))
+
+    def latent_spread(self, act, latent_pool, rank, rot_dim, a_rows, rows, pool, kv_heads, k_dim, v_dim, block_size, first):
+        self.call("vx_latent_spread", act, latent_pool, rank, rot_dim, a_rows, rows, pool, kv_heads, k_dim, v_dim, block_size, first)
+
+    def post_norm(self, act, args):
+        self.call("vx_post_norm", act, C.byref(args))
+
+    def poly_norm(self, act, z, ldz, rows, cols, coef, eps, out, ldo):
+        self.call("vx_poly_norm", act, z, ldz, rows, cols, coef, eps, out, ldo)
 
     def conv_silu(self, act, batch, args):
         self.call("vx_conv_silu", act, C.byref(batch), C.byref(args))

@@ -1,12 +1,12 @@
-// Causal grouped-query attention over a paged pool for mixed batches, with a per-head distance bias, a query temperature and
-// an output gate (vx_attn_ragged).
+// Causal grouped-query attention over a paged pool for mixed batches, with a per-head distance bias, a query temperature, a
+// softmax sink per head and an output gate (vx_attn_ragged).
 //
 //  * prefill_kernel: sequences that bring several rows. A wave owns QT x 16 (row, head) pairs of one K/V head and walks
 //    the keys in groups of 32 (two 16-token blocks); the four waves of a workgroup walk the same keys.
 //  * decode_kernel + merge_kernel: sequences that bring one row. A workgroup takes a piece of one sequence's keys for all
 //    query heads of one K/V head, its waves every fourth group; the pieces' partial results are merged by a second
 //    launch, which also applies the gate.
-//  * plain_kernel: one workgroup per (row, head), any geometry, and everything in float32 batches.
+//  * attn_plain_kernel (attn_plain.h): one workgroup per (row, head), any geometry, and everything in float32 batches.
 //
 // Matrix products of the first two: S^T = K Q^T and O^T = V^T P^T on the bfloat16 matrix cores. The keys of a group are
 // dealt to the two 16-row tiles of S^T so that a lane ends with eight consecutive keys of one query, which is the
@@ -15,13 +15,12 @@
 // two bfloat16 parts (16 bits of the 24). Scores, bias, softmax and sums are float32.
 #include <string.h>
 
-#include "ragged.h"
+#include "attn_plain.h"
 
 using namespace vx;
 
 namespace {
 
-constexpr float kLog2e = 1.4426950408889634f;
 constexpr int BS = 16;               // tokens of a block (matrix-core kernels)
 constexpr int LUT_LDS = 12 * 1024;   // floats of bias tables kept in LDS
 
@@ -34,7 +33,7 @@ struct Args {
     int vec_q, vec_o;  // vector access to q / gate and out
     int lut_lds;
     // prefill
-    int tile_rows, tiles;
+    int tile_rows, tiles, min_rows;
     // decode
     const int32_t *items;
     int piece, pieces;
@@ -42,8 +41,11 @@ struct Args {
 };
 
 __device__ __forceinline__ float temperature(const vx_attn_args &p, int pos) {
-    if (p.temp_every <= 0) return 1.0f;
-    return 1.0f + p.temp_coef * logf((float)((pos + 1) / p.temp_every) + 1.0f);
+    return query_temperature(p.temp_coef, p.temp_every, pos);
+}
+// What the sink adds to a denominator whose terms are relative to m (base-2 exponents).
+__device__ __forceinline__ float sink_term(const vx_attn_args &p, int h, float m) {
+    return p.sink ? __builtin_amdgcn_exp2f(p.sink[h] * kLog2e - m) : 0.f;
 }
 
 __device__ __forceinline__ bf16x8 zero8() {
@@ -224,7 +226,7 @@ __global__ void __launch_bounds__(256) prefill_kernel(Args a) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, rg = wave / KS, ks_id = wave % KS;
     const int g = blockIdx.x % a.p.kv_heads, id = a.tiles - 1 - blockIdx.x / a.p.kv_heads;  // late tiles, the longest, first
     int seq, ti, count;
-    if (!item_of_seq(a.cu, a.n_seqs, a.tile_rows, 2, id, &seq, &ti, &count)) return;
+    if (!item_of_seq(a.cu, a.n_seqs, a.tile_rows, a.min_rows, id, &seq, &ti, &count)) return;
     load_lut(a, g, s_lut);
     const int row0 = a.cu[seq] + ti * a.tile_rows, ntok = min(a.tile_rows, a.cu[seq + 1] - row0);
     const int pos0 = a.pos[row0];
@@ -276,7 +278,7 @@ __global__ void __launch_bounds__(256) prefill_kernel(Args a) {
 #pragma unroll
         for (int t = 0; t < QT; t++) {
             if (tok[t] >= ntok) continue;
-            const float inv = 1.0f / l[t];  // (a row sees itself: l > 0)
+            const float inv = 1.0f / (l[t] + sink_term(a.p, head[t], qs.m[t]));  // (a row sees itself: l > 0)
 #pragma unroll
             for (int v = 0; v < VD; v++) write4(a, row0 + tok[t], head[t], v * 16 + (lane >> 4) * 4, qs.o[t][v] * inv);
         }
@@ -319,7 +321,7 @@ __global__ void __launch_bounds__(256) prefill_kernel(Args a) {
                 const float mw = s_m[rg][w][t * 16 + (lane & 15)];
                 if (mw > -INFINITY) sum += s_l[rg][w][t * 16 + (lane & 15)] * __builtin_amdgcn_exp2f(mw - mg[t]);
             }
-            const float inv = 1.0f / sum;
+            const float inv = 1.0f / (sum + sink_term(a.p, head[t], mg[t]));
             for (int v = ks_id; v < VD; v += KS)
                 write4(a, row0 + tok[t], head[t], v * 16 + (lane >> 4) * 4,
                        *(const f32x4 *)(s_o + (t * 16 + (lane & 15)) * LDO + v * 16 + (lane >> 4) * 4) * inv);
@@ -430,7 +432,7 @@ __global__ void __launch_bounds__(64) merge_kernel(Args a) {
     for (int off = 32; off > 0; off >>= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
     float l = 0.f;
     for (int i = 0; i < n; i++) l += src[(size_t)i * (vd + 2) + 1] * __builtin_amdgcn_exp2f(src[(size_t)i * (vd + 2)] - m);
-    const float inv = a.p.out_scale / l;
+    const float inv = a.p.out_scale / (l + sink_term(a.p, h, m));
     for (int d = threadIdx.x; d < vd; d += 64) {
         float o = 0.f;
 #pragma unroll 4
@@ -442,100 +444,10 @@ __global__ void __launch_bounds__(64) merge_kernel(Args a) {
     }
 }
 
-// ---------------------------------------------------------------- any geometry
-constexpr int PL_CHUNK = 1024;
-
-template <typename T>
-__global__ void __launch_bounds__(256) plain_kernel(Args a) {
-    extern __shared__ float s_q[];  // [k_dim]
-    __shared__ float s_s[PL_CHUNK], s_red[4];
-    const vx_attn_args &p = a.p;
-    const int h = blockIdx.x, row = blockIdx.y, g = h / a.group, tid = threadIdx.x;
-    const int seq = a.one_token ? row : seq_of_row(a.cu, a.n_seqs, row);
-    const int pos = a.pos[row], len = pos + 1;
-    const int32_t *bt = a.tables + (size_t)a.rows[seq] * a.max_blocks;
-    const T *pool = (const T *)p.pool;
-    const size_t blk = (size_t)p.kv_heads * a.block_size * (a.kp + p.v_dim), vpart = (size_t)p.kv_heads * a.block_size * a.kp;
-    const T *q = (const T *)p.q + (size_t)row * p.ldq + h * p.k_dim;
-    const float qf = p.scale * temperature(p, pos);
-    for (int d = tid; d < p.k_dim; d += 256) s_q[d] = (float)q[d];
-    // thread t accumulates dimension t % width over the keys t / width, t / width + groups, ..; wider heads: several each
-    const int width = p.v_dim < 256 ? p.v_dim : 256, kg = 256 / width, md = tid % width, mg = tid / width;
-    constexpr int MAXV = 8;  // dimensions of a thread: v_dim <= 2048
-    float acc[MAXV];
-#pragma unroll
-    for (int i = 0; i < MAXV; i++) acc[i] = 0.f;
-    float m = -INFINITY, l = 0.f;
-    for (int c0 = 0; c0 < len; c0 += PL_CHUNK) {
-        const int cn = min(PL_CHUNK, len - c0);
-        __syncthreads();
-        float mx = -INFINITY;
-        for (int i = tid; i < cn; i += 256) {
-            const int key = c0 + i;
-            const T *k = pool + (size_t)bt[key / a.block_size] * blk + ((size_t)g * a.block_size + key % a.block_size) * a.kp;
-            float dot = 0.f;
-            for (int d = 0; d < p.k_dim; d++) dot = fmaf(s_q[d], (float)k[d], dot);
-            float s = dot * qf;
-            if (p.bias) s += p.bias[(size_t)h * p.bias_len + min(pos - key, p.bias_len - 1)];
-            s_s[i] = s;
-            mx = fmaxf(mx, s);
-        }
-#pragma unroll
-        for (int off = 32; off > 0; off >>= 1) mx = fmaxf(mx, __shfl_xor(mx, off, 64));
-        if ((tid & 63) == 0) s_red[tid >> 6] = mx;
-        __syncthreads();
-        mx = fmaxf(fmaxf(s_red[0], s_red[1]), fmaxf(s_red[2], s_red[3]));
-        const float mn = fmaxf(m, mx), al = expf(m - mn);
-        float sum = 0.f;
-        for (int i = tid; i < cn; i += 256) {
-            const float e = expf(s_s[i] - mn);
-            s_s[i] = e;
-            sum += e;
-        }
-#pragma unroll
-        for (int off = 32; off > 0; off >>= 1) sum += __shfl_xor(sum, off, 64);
-        __syncthreads();
-        if ((tid & 63) == 0) s_red[tid >> 6] = sum;
-        __syncthreads();
-        l = l * al + (s_red[0] + s_red[1] + s_red[2] + s_red[3]);
-        m = mn;
-        if (mg < kg)
-            for (int v = 0; v < MAXV; v++) {
-                const int d = md + v * 256;
-                if (d >= p.v_dim) break;
-                float t = acc[v] * al;
-                for (int i = mg; i < cn; i += kg) {
-                    const int key = c0 + i;
-                    t = fmaf(s_s[i],
-                             (float)pool[(size_t)bt[key / a.block_size] * blk + vpart + ((size_t)g * p.v_dim + d) * a.block_size +
-                                         key % a.block_size],
-                             t);
-                }
-                acc[v] = t;
-            }
-    }
-    __syncthreads();
-    float *s_acc = s_s;  // [kg][width]
-    for (int v = 0; v < MAXV; v++) {
-        const int d = md + v * 256;
-        if (v * 256 >= p.v_dim) break;
-        if (mg < kg) s_acc[mg * width + md] = acc[v];
-        __syncthreads();
-        if (mg == 0 && d < p.v_dim) {
-            float t = 0.f;
-            for (int i = 0; i < kg; i++) t += s_acc[i * width + md];
-            t = t / l * p.out_scale;
-            if (p.gate) t *= sigmoid_f((float)((const T *)p.gate)[(size_t)row * p.ldg + h * p.v_dim + d]);
-            ((T *)p.out)[(size_t)row * p.ldo + h * p.v_dim + d] = (T)t;
-        }
-        __syncthreads();
-    }
-}
-
 template <int KD, int VD, int QT, int KS>
 void launch_prefill(vx_backend *be, Args a, const vx_ragged *b) {
     a.tile_rows = 64 / KS * QT / a.group;
-    a.tiles = count_items(b, a.tile_rows, 2);
+    a.tiles = count_items(b, a.tile_rows, a.min_rows);
     const size_t lut = a.lut_lds ? (size_t)a.group * a.p.bias_len * 4 : 0;
     const size_t o = KS > 1 ? (size_t)4 / KS * QT * 16 * (VD * 16 + 4) * 4 : 0;
     if (a.tiles > 0) prefill_kernel<KD, VD, QT, KS><<<a.tiles * a.p.kv_heads, 256, lut > o ? lut : o, be->stream>>>(a);
@@ -549,12 +461,13 @@ void launch_decode(vx_backend *be, const Args &a, dim3 grid) {
 
 template <int KD, int VD>
 int run_fast(vx_backend *be, Args a, const vx_ragged *b) {
-    bool any_many = false, any_one = !b->q_lens;
+    bool any_many = false, any_one = !b->q_lens && a.p.min_rows <= 1;
     int64_t many = 0;
+    a.min_rows = a.p.min_rows > 2 ? a.p.min_rows : 2;
     if (b->q_lens)
         for (int s = 0; s < b->n_seqs; s++) {
-            any_many |= b->q_lens[s] > 1, any_one |= b->q_lens[s] == 1;
-            if (b->q_lens[s] > 1) many += b->q_lens[s];
+            any_many |= b->q_lens[s] >= a.min_rows, any_one |= b->q_lens[s] == 1 && a.p.min_rows <= 1;
+            if (b->q_lens[s] >= a.min_rows) many += b->q_lens[s];
         }
     if (any_many) {
         // Two query tiles a wave halve the keys' traffic; waves that share queries make more workgroups of few rows (the
@@ -659,15 +572,23 @@ int vx_attn_ragged(vx_backend *be, int act, const vx_ragged *b, const vx_attn_ar
         if (wide <= 64) return run_fast<2, 4>(be, a, b);
         if (wide <= 96) return run_fast<3, 6>(be, a, b);
         if (wide <= 128) return run_fast<4, 8>(be, a, b);
+        if (p->k_dim <= 192 && p->v_dim <= 128) return run_fast<6, 8>(be, a, b);
         if (wide <= 192) return run_fast<6, 12>(be, a, b);
         return run_fast<8, 16>(be, a, b);
     }
-    const dim3 grid(p->heads, b->rows);
-    const size_t lds = (size_t)p->k_dim * 4;
-    if (act == VX_ACT_BF16)
-        plain_kernel<bf16><<<grid, 256, lds, be->stream>>>(a);
-    else
-        plain_kernel<float><<<grid, 256, lds, be->stream>>>(a);
+    PlainAttn t;
+    memset(&t, 0, sizeof t);
+    t.heads = p->heads, t.group = a.group;
+    t.q[0] = {p->q, p->ldq, p->k_dim, 0, p->k_dim, p->k_dim};  // (elements, first, room, stride)
+    t.row = p->k_dim, t.v_dim = p->v_dim;
+    t.pool = p->pool, t.block = (int64_t)vx_kv_block_elems(b->block_size, p->kv_heads, p->k_dim, p->v_dim);
+    t.k_head = (int64_t)b->block_size * a.kp, t.k_tok = a.kp;
+    t.v_first = p->kv_heads * t.k_head, t.v_head = (int64_t)b->block_size * p->v_dim, t.v_tok = 1, t.v_elem = b->block_size;
+    t.scale = p->scale, t.temp_coef = p->temp_coef, t.temp_every = p->temp_every;
+    t.bias = p->bias, t.bias_len = p->bias_len, t.sink = p->sink;
+    t.gate = p->gate, t.ldg = p->ldg, t.out_scale = p->out_scale, t.out = p->out, t.ldo = p->ldo, t.out_head = p->v_dim, t.out_cols = p->v_dim;
+    t.min_rows = p->min_rows;
+    launch_plain(be, act, b, t);
     VX_CHECK_LAUNCH();
     return VX_OK;
 }

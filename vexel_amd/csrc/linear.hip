@@ -38,6 +38,9 @@ __device__ __forceinline__ size_t kv_elem_v(const vx_linear_out &o, int slot, in
            ((size_t)g * o.v_dim + d) * o.block_size + slot % o.block_size;
 }
 
+// Where row r of the activations lies.
+__device__ __forceinline__ size_t a_row(const LinArgs &p, int r) { return p.o.a_rows ? (size_t)p.o.a_rows[r] : (size_t)r; }
+
 template <typename P>
 __device__ __forceinline__ void put4(P *row, int c, int cols, int ld, f32x4 v) {
     if (c + 4 <= cols && (ld & 3) == 0) {
@@ -49,12 +52,41 @@ __device__ __forceinline__ void put4(P *row, int c, int cols, int ld, f32x4 v) {
     }
 }
 
+// Columns c .. c + 3 of a row, those in the rotated part of their head turned by the row's angles.
+__device__ __forceinline__ f32x4 turned(const vx_linear_out &o, int row, int c, f32x4 v) {
+    const int pair = (c % o.rot_stride - o.rot_first) >> 1;
+    if (c % o.rot_stride < o.rot_first) return v;
+    const float *cs = o.rot_tab + ((size_t)row * o.rot_pairs + pair) * 2;
+#pragma unroll
+    for (int i = 0; i < 2; i++)
+        if (pair + i < o.rot_pairs) {
+            const float u = v[2 * i], w = v[2 * i + 1], co = cs[2 * i], si = cs[2 * i + 1];
+            v[2 * i] = u * co - w * si;
+            v[2 * i + 1] = w * co + u * si;
+        }
+    return v;
+}
+
+// The launch's group of independent maps: its weights, its columns of the activations and of the result.
+template <typename T>
+__device__ __forceinline__ void take_group(LinArgs &p) {
+    if (gridDim.z == 1) return;
+    const size_t g = blockIdx.z;
+    p.w = (const bf16 *)p.w + g * p.n * p.k;
+    p.a = (const T *)p.a + g * p.o.a_group;
+    p.o.out = p.o.out_f32 ? (void *)((float *)p.o.out + g * p.o.out_group) : (void *)((T *)p.o.out + g * p.o.out_group);
+}
+
 // Columns c .. c + 3 of activation row `row`.
 template <typename T, int KIND>
 __device__ __forceinline__ void emit(const LinArgs &p, int slice, int row, int c, f32x4 v) {
     const vx_linear_out &o = p.o;
     if (row >= p.rows) return;
     if constexpr (KIND == VX_LIN_PLAIN) {
+        if (o.softcap > 0.f) {
+#pragma unroll
+            for (int r = 0; r < 4; r++) v[r] = o.softcap * tanhf(v[r] / o.softcap);
+        }
         if (o.out_f32)
             put4((float *)o.out + ((size_t)slice * p.rows + row) * o.ldo, c, o.cols, o.ldo, v);
         else
@@ -66,6 +98,11 @@ __device__ __forceinline__ void emit(const LinArgs &p, int slice, int row, int c
             put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
         else
             put4(o.out2 + (size_t)row * o.ldo2, c - o.split, o.ldo2, o.ldo2, v);
+    } else if constexpr (KIND == VX_LIN_ROTARY) {
+        if (c < o.split)
+            put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, turned(o, row, c, v));
+        else
+            put4(o.out2 + (size_t)row * o.ldo2, c - o.split, o.ldo2, o.ldo2, v);
     } else if constexpr (KIND == VX_LIN_SOFTPLUS) {
         f32x4 u;
 #pragma unroll
@@ -74,10 +111,11 @@ __device__ __forceinline__ void emit(const LinArgs &p, int slice, int row, int c
         }
         put4((float *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, u);
     } else {  // VX_LIN_KV: K and V columns leave for the pool (segments start at multiples of 16 columns)
+        const auto slot_of = [&](int r) { return o.slot_mapping ? o.slot_mapping[r] : r; };
         const int kw = o.kv_heads * o.k_dim, vw = o.kv_heads * o.v_dim;
         const int ck = c - o.k_col, cv = c - o.v_col;
         if (ck >= 0 && ck < kw) {
-            const int slot = o.slot_mapping[row];
+            const int slot = slot_of(row);
             T *pool = (T *)o.pool;
             if ((o.k_dim & 3) == 0) {
                 store4(pool + kv_elem_k(o, slot, ck / o.k_dim, ck % o.k_dim), v);
@@ -87,7 +125,7 @@ __device__ __forceinline__ void emit(const LinArgs &p, int slice, int row, int c
                     if (ck + r < kw) pool[kv_elem_k(o, slot, (ck + r) / o.k_dim, (ck + r) % o.k_dim)] = (T)v[r];
             }
         } else if (cv >= 0 && cv < vw) {
-            const int slot = o.slot_mapping[row];
+            const int slot = slot_of(row);
             T *pool = (T *)o.pool;
 #pragma unroll
             for (int r = 0; r < 4; r++)
@@ -103,6 +141,7 @@ template <typename T, int MT, int NT, int WAVES, int KIND>
 __global__ void __launch_bounds__(64 * WAVES) linear_few_kernel(LinArgs p) {
     typedef typename Vec8<T>::type A8;
     __shared__ f32x4 red[WAVES][NT * MT][64];
+    if constexpr (KIND == VX_LIN_PLAIN) take_group<T>(p);
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int steps = p.k >> 5, slices = gridDim.y, slice = blockIdx.y;
     const int s0 = (int)((int64_t)steps * slice / slices), s1 = (int)((int64_t)steps * (slice + 1) / slices);
@@ -110,7 +149,7 @@ __global__ void __launch_bounds__(64 * WAVES) linear_few_kernel(LinArgs p) {
     const bf16 *w = (const bf16 *)p.w + ((size_t)tile * steps) * 512 + lane * 8;
     const T *a[MT];
 #pragma unroll
-    for (int m = 0; m < MT; m++) a[m] = (const T *)p.a + (size_t)min(m * 16 + (lane & 15), p.rows - 1) * p.lda + (lane >> 4) * 8;
+    for (int m = 0; m < MT; m++) a[m] = (const T *)p.a + a_row(p, min(m * 16 + (lane & 15), p.rows - 1)) * p.lda + (lane >> 4) * 8;
     f32x4 acc[NT][MT];
 #pragma unroll
     for (int t = 0; t < NT; t++)
@@ -182,6 +221,7 @@ __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_til
     constexpr int MI = BM / 32, NI = BN / 32;          // 16-wide tiles per wave in each direction
     typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
     extern __shared__ u32x4 lds[];                     // [2][BM][CPR], pieces of a row permuted by the row's low bits
+    if constexpr (KIND == VX_LIN_PLAIN) take_group<T>(p);
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int wm = (wave & 1) * (BM / 2), wn = (wave >> 1) * NI;
     const int rt = blockIdx.x % row_tiles, nt = blockIdx.x / row_tiles;  // the row tiles of one weight tile run together
@@ -200,7 +240,7 @@ __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_til
 #pragma unroll
     for (int i = 0; i < LOADS; i++) {
         const int idx = tid + i * 256, row = idx / CPR, c = idx % CPR;
-        ap[i] = (const u32x4 *)((const T *)p.a + (size_t)min(m0 + row, p.rows - 1) * p.lda) + c;
+        ap[i] = (const u32x4 *)((const T *)p.a + a_row(p, min(m0 + row, p.rows - 1)) * p.lda) + c;
         dst[i] = piece(row, c);
     }
     u32x4 ar[LOADS];
@@ -277,7 +317,7 @@ __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_til
     }
 }
 
-// Adds up the slices of a VX_LIN_SPLIT map and deals the columns to its two results.
+// Adds up the slices of a VX_LIN_SPLIT or VX_LIN_ROTARY map and deals the columns to its two results.
 template <typename T>
 __global__ void __launch_bounds__(256) split_sum_kernel(const float *part, int slices, int rows, int n, vx_linear_out o) {
     const int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x;
@@ -287,7 +327,7 @@ __global__ void __launch_bounds__(256) split_sum_kernel(const float *part, int s
     f32x4 v = *(const f32x4 *)src;
     for (int s = 1; s < slices; s++) v += *(const f32x4 *)(src + (size_t)s * rows * n);
     if (c < o.split)
-        put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
+        put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, o.rot_tab ? turned(o, row, c, v) : v);
     else
         put4(o.out2 + (size_t)row * o.ldo2, c - o.split, o.ldo2, o.ldo2, v);
 }
@@ -308,7 +348,7 @@ __global__ void fill_zero_kernel(uint32_t *p, size_t n) {
 // ---------------------------------------------------------------- launches
 template <typename T, int MT, int NT, int WAVES, int KIND>
 void launch_few_as(vx_backend *be, const LinArgs &p, int slices) {
-    linear_few_kernel<T, MT, NT, WAVES, KIND><<<dim3((p.n >> 4) / NT, slices), 64 * WAVES, 0, be->stream>>>(p);
+    linear_few_kernel<T, MT, NT, WAVES, KIND><<<dim3((p.n >> 4) / NT, slices, p.o.groups), 64 * WAVES, 0, be->stream>>>(p);
 }
 template <typename T, int MT, int KIND>
 void launch_few(vx_backend *be, const LinArgs &p, int slices) {
@@ -317,7 +357,7 @@ void launch_few(vx_backend *be, const LinArgs &p, int slices) {
     if constexpr (KIND == VX_LIN_SWIGLU) {
         launch_few_as<T, MT, 2, MT == 4 ? 4 : 8, KIND>(be, p, slices);
     } else if constexpr (MT < 4) {
-        if (tiles % 2 == 0 && tiles / 2 * slices >= 512)
+        if (tiles % 2 == 0 && (int64_t)tiles / 2 * slices * p.o.groups >= 512)
             launch_few_as<T, MT, 2, 8, KIND>(be, p, slices);
         else
             launch_few_as<T, MT, 1, 8, KIND>(be, p, slices);
@@ -329,7 +369,7 @@ void launch_few(vx_backend *be, const LinArgs &p, int slices) {
 template <typename T, int BM, int BN, int KIND>
 void launch_many(vx_backend *be, const LinArgs &p, int slices) {
     const int rt = ceil_div(p.rows, BM), nt = ceil_div(p.n, BN);
-    linear_many_kernel<T, BM, BN, KIND><<<dim3(rt * nt, slices), 256, 2 * BM * 64 * sizeof(T), be->stream>>>(p, rt);
+    linear_many_kernel<T, BM, BN, KIND><<<dim3(rt * nt, slices, p.o.groups), 256, 2 * BM * 64 * sizeof(T), be->stream>>>(p, rt);
 }
 
 // The widest tiles that still give every compute unit a workgroup.
@@ -371,7 +411,7 @@ int launch(vx_backend *be, const LinArgs &p, int slices) {
             launch_few<T, 4, KIND>(be, p, slices);
     } else {
         int bm, bn;
-        many_tile(p.n, p.rows, slices, &bm, &bn);
+        many_tile(p.n, p.rows, slices * p.o.groups, &bm, &bn);
         if constexpr (sizeof(T) == 4) {
             launch_many<T, 64, 64, KIND>(be, p, slices);
         } else if (bn == 64) {
@@ -393,6 +433,7 @@ int dispatch(vx_backend *be, const LinArgs &p, int slices) {
         case VX_LIN_SWIGLU: return launch<T, VX_LIN_SWIGLU>(be, p, slices);
         case VX_LIN_KV: return launch<T, VX_LIN_KV>(be, p, slices);
         case VX_LIN_SPLIT: return launch<T, VX_LIN_SPLIT>(be, p, slices);
+        case VX_LIN_ROTARY: return launch<T, VX_LIN_ROTARY>(be, p, slices);
         default: return launch<T, VX_LIN_SOFTPLUS>(be, p, slices);
     }
 }
@@ -466,7 +507,7 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
     VX_REQUIRE(n >= 16 && n % 16 == 0 && k >= 64 && k % 64 == 0 && lda >= k && lda % 8 == 0 && (uintptr_t)a % 16 == 0 &&
                    (uintptr_t)w % 16 == 0 && (uintptr_t)o->out % 16 == 0,
                "vx_linear: sizes or alignment (n %d, k %d, lda %d)", n, k, lda);
-    VX_REQUIRE(o->kind >= VX_LIN_PLAIN && o->kind <= VX_LIN_SOFTPLUS, "vx_linear: unknown kind %d", o->kind);
+    VX_REQUIRE(o->kind >= VX_LIN_PLAIN && o->kind <= VX_LIN_ROTARY, "vx_linear: unknown kind %d", o->kind);
     VX_REQUIRE(o->cols >= 1 && o->ldo >= o->cols, "vx_linear: %d columns in rows of %d", o->cols, o->ldo);
     const int slices = o->slices > 1 ? o->slices : 1;
     VX_REQUIRE(slices == 1 || (o->kind == VX_LIN_PLAIN && o->out_f32 && slices <= 64), "vx_linear: slices need a plain float32 result");
@@ -476,17 +517,34 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
         VX_REQUIRE(o->out2 && o->split % 16 == 0 && o->split > 0 && o->split < n && o->cols == o->split && o->ldo2 >= n - o->split &&
                        (uintptr_t)o->out2 % 16 == 0,
                    "vx_linear: bad split");
+    } else if (o->kind == VX_LIN_ROTARY) {
+        VX_REQUIRE(o->split % 16 == 0 && o->split > 0 && o->split <= n && o->cols == o->split &&
+                       (o->split == n || (o->out2 && o->ldo2 >= n - o->split && (uintptr_t)o->out2 % 16 == 0)),
+                   "vx_linear: bad split");
+        VX_REQUIRE(o->rot_tab && o->rot_pairs >= 1 && o->rot_first >= 0 && o->rot_first % 4 == 0 && o->rot_stride % 4 == 0 &&
+                       o->rot_first + 2 * o->rot_pairs <= o->rot_stride,
+                   "vx_linear: %d rotated pairs at %d in heads of %d columns", o->rot_pairs, o->rot_first, o->rot_stride);
     } else {
         VX_REQUIRE(o->cols <= n, "vx_linear: %d columns of %d", o->cols, n);
     }
     if (o->kind == VX_LIN_SOFTPLUS) VX_REQUIRE(o->bias != nullptr, "vx_linear: null bias");
     if (o->kind == VX_LIN_KV)
-        VX_REQUIRE(o->pool && o->slot_mapping && o->kv_heads >= 1 && o->k_dim >= 1 && o->v_dim >= 1 && o->block_size >= 1 &&
+        VX_REQUIRE(o->pool && o->kv_heads >= 1 && o->k_dim >= 1 && o->v_dim >= 1 && o->block_size >= 1 &&
                        o->k_col % 16 == 0 && o->v_col % 16 == 0 && o->k_col >= 0 && o->v_col >= 0 &&
                        o->k_col + o->kv_heads * o->k_dim <= n && o->v_col + o->kv_heads * o->v_dim <= n,
                    "vx_linear: bad K/V columns");
+    VX_REQUIRE(o->softcap == 0.f || (o->softcap > 0.f && o->kind == VX_LIN_PLAIN && slices == 1), "vx_linear: a cap needs a plain whole result");
     LinArgs p{a, w, lda, n, k, rows, *o};
-    if (o->kind == VX_LIN_SPLIT) {  // (narrow and deep as a rule) in slices, added up by a kernel of their own
+    if (o->groups > 1) {
+        VX_REQUIRE(o->kind == VX_LIN_PLAIN && slices == 1 && o->groups <= 65535 && o->a_group >= 0 && o->out_group >= o->cols &&
+                       o->a_group % 8 == 0 && o->out_group % 4 == 0 && lda >= (o->groups - 1) * (int64_t)o->a_group + k &&
+                       o->ldo >= (o->groups - 1) * (int64_t)o->out_group + o->cols,
+                   "vx_linear: bad groups");
+    } else {
+        p.o.groups = 1;
+    }
+    if (o->kind != VX_LIN_ROTARY) p.o.rot_tab = nullptr;
+    if (o->kind == VX_LIN_SPLIT || o->kind == VX_LIN_ROTARY) {  // (narrow and deep as a rule) in slices, added up by a kernel of their own
         const int cut = pick_slices(n, k, rows);
         if (cut > 1) {
             const size_t bytes = (size_t)cut * rows * n * 4;

@@ -1,5 +1,5 @@
-// The pieces of mixed-batch layers beside linear maps and attention: the norm | residual | norm seam, the causal depthwise
-// convolution and the selective scan. All of them in float32 on activations that are bfloat16 or float32 (T).
+// The pieces of mixed-batch layers beside linear maps and attention: the norm | residual | norm seam, the residual | norm |
+// average over the depth seam, the normed polynomial activation, the causal depthwise convolution and the selective scan. All of them in float32 on activations that are bfloat16 or float32 (T).
 //
 // Scan: a lane keeps 8 states of one channel in registers, LP = padded / 8 neighbouring lanes make up the channel. A
 // sequence's rows are cut into chunks of CHUNK; where a sequence has several, a first pass finds what every chunk adds to
@@ -124,6 +124,190 @@ __global__ void __launch_bounds__(1024) residual_norm_kernel(vx_residual_norm_ar
     }
     if (out)
         for (int c = p.cols + tid; c < p.ldo; c += nt) out[c] = (T)0.f;
+}
+
+// NV as above. The earlier results of a row are read only where it is averaged.
+template <typename T, int NV>
+__global__ void __launch_bounds__(1024) post_norm_kernel(vx_post_norm_args p) {
+    __shared__ float sm[16];
+    const int i = blockIdx.x, r = p.row_idx ? p.row_idx[i] : i, tid = threadIdx.x, nt = blockDim.x;
+    const float *xr = p.x_in + (size_t)r * p.cols;
+    float *xo = p.x_out ? p.x_out + (size_t)r * p.cols : nullptr;
+    float *hr = p.n_avg > 0 ? p.hist + (size_t)r * p.cols : nullptr;
+    T *out = p.out ? (T *)p.out + (size_t)i * p.ldo : nullptr;
+    const float n = (float)p.cols;
+    if constexpr (NV > 0) {
+        f32x4 x[NV];
+        const int n4 = p.cols >> 2;
+        float ss = 0.f;
+#pragma unroll
+        for (int v = 0; v < NV; v++) {
+            const int c = tid + v * nt;
+            x[v] = c < n4 ? ((const f32x4 *)xr)[c] : f32x4{0.f, 0.f, 0.f, 0.f};
+            if (p.w && c < n4) {
+                const float *yr = p.y + (size_t)r * p.ldy + c * 4;
+                f32x4 y = *(const f32x4 *)yr;
+                for (int s = 1; s < p.y_slices; s++) y += *(const f32x4 *)(yr + (size_t)s * p.y_stride);
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    x[v][e] = fmaf(p.alpha, x[v][e], y[e]);
+                    ss = fmaf(x[v][e], x[v][e], ss);
+                }
+            }
+        }
+        if (p.w) {
+            const float inv = 1.0f / sqrtf(block_sum(ss, sm) / n + p.eps);
+#pragma unroll
+            for (int v = 0; v < NV; v++) {
+                const int c = tid + v * nt;
+                if (c < n4) x[v] = x[v] * inv * ((const f32x4 *)p.w)[c];
+            }
+        }
+        if (hr) {
+            if (p.keep)
+#pragma unroll
+                for (int v = 0; v < NV; v++) {
+                    const int c = tid + v * nt;
+                    if (c < n4) ((f32x4 *)(hr + (size_t)(p.n_avg - 1) * p.hist_stride))[c] = x[v];
+                }
+            const float own = p.avg[p.n_avg - 1];
+#pragma unroll
+            for (int v = 0; v < NV; v++) x[v] *= own;
+            for (int j = 0; j + 1 < p.n_avg; j++) {
+                const float w = p.avg[j];
+#pragma unroll
+                for (int v = 0; v < NV; v++) {
+                    const int c = tid + v * nt;
+                    if (c < n4) x[v] += w * ((const f32x4 *)(hr + (size_t)j * p.hist_stride))[c];
+                }
+            }
+        }
+        if (xo)
+#pragma unroll
+            for (int v = 0; v < NV; v++) {
+                const int c = tid + v * nt;
+                if (c < n4) ((f32x4 *)xo)[c] = x[v];
+            }
+        if (!out) return;
+        float inv = 1.0f;
+        if (p.w_pre) {
+            ss = 0.f;
+#pragma unroll
+            for (int v = 0; v < NV; v++)
+#pragma unroll
+                for (int e = 0; e < 4; e++) ss = fmaf(x[v][e], x[v][e], ss);
+            inv = 1.0f / sqrtf(block_sum(ss, sm) / n + p.eps);
+        }
+#pragma unroll
+        for (int v = 0; v < NV; v++) {
+            const int c = tid + v * nt;
+            if (c < n4) store4(out + c * 4, p.w_pre ? x[v] * inv * ((const f32x4 *)p.w_pre)[c] : x[v]);
+        }
+    } else {
+        // any width: the row is worked out again for every pass; a thread reads and writes its own columns only
+        auto sum = [&](int c) {
+            if (!p.w) return xr[c];
+            float t = p.y[(size_t)r * p.ldy + c];
+            for (int s = 1; s < p.y_slices; s++) t += p.y[(size_t)s * p.y_stride + (size_t)r * p.ldy + c];
+            return fmaf(p.alpha, xr[c], t);
+        };
+        float inv = 1.0f;
+        if (p.w) {
+            float ss = 0.f;
+            for (int c = tid; c < p.cols; c += nt) {
+                const float t = sum(c);
+                ss = fmaf(t, t, ss);
+            }
+            inv = 1.0f / sqrtf(block_sum(ss, sm) / n + p.eps);
+        }
+        auto result = [&](int c, bool keep) {
+            float t = p.w ? sum(c) * inv * p.w[c] : xr[c];
+            if (!hr) return t;
+            if (keep) hr[(size_t)(p.n_avg - 1) * p.hist_stride + c] = t;
+            t *= p.avg[p.n_avg - 1];
+            for (int j = 0; j + 1 < p.n_avg; j++) t += p.avg[j] * hr[(size_t)j * p.hist_stride + c];
+            return t;
+        };
+        float inv_o = 1.0f;
+        if (out && p.w_pre) {
+            float ss = 0.f;
+            for (int c = tid; c < p.cols; c += nt) {
+                const float t = result(c, false);
+                ss = fmaf(t, t, ss);
+            }
+            inv_o = 1.0f / sqrtf(block_sum(ss, sm) / n + p.eps);
+        }
+        for (int c = tid; c < p.cols; c += nt) {
+            const float t = result(c, p.keep);
+            if (xo) xo[c] = t;
+            if (out) out[c] = (T)(p.w_pre ? t * inv_o * p.w_pre[c] : t);
+        }
+    }
+    if (out)
+        for (int c = p.cols + tid; c < p.ldo; c += nt) out[c] = (T)0.f;
+}
+
+// A row per workgroup; NV > 0: cols is a multiple of 8 and at most 8 * NV * blockDim.x, rows aligned: they live in registers.
+template <typename T, int NV>
+__global__ void __launch_bounds__(1024) poly_norm_kernel(const T *z, int ldz, int cols, const float *coef, float eps, T *out, int ldo) {
+    typedef typename Vec8<T>::type V8;
+    __shared__ float sm[3][16];
+    const int tid = threadIdx.x, nt = blockDim.x, waves = nt >> 6;
+    const T *zr = z + (size_t)blockIdx.x * ldz;
+    T *o = out + (size_t)blockIdx.x * ldo;
+    float s[3] = {0.f, 0.f, 0.f};
+    const auto add = [&](float t) {
+        const float q = t * t;
+        s[0] += q;
+        s[1] = fmaf(q, q, s[1]);
+        s[2] = fmaf(q * q, q, s[2]);
+    };
+    V8 v[NV > 0 ? NV : 1];
+    if constexpr (NV > 0) {
+#pragma unroll
+        for (int i = 0; i < NV; i++) {
+            const int c = (tid + i * nt) * 8;
+            if (c < cols) v[i] = *(const V8 *)(zr + c);
+        }
+#pragma unroll
+        for (int i = 0; i < NV; i++)
+            if ((tid + i * nt) * 8 < cols)
+#pragma unroll
+                for (int e = 0; e < 8; e++) add((float)v[i][e]);
+    } else {
+        for (int c = tid; c < cols; c += nt) add((float)zr[c]);
+    }
+    float f[3];
+#pragma unroll
+    for (int k = 0; k < 3; k++) {
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) s[k] += __shfl_xor(s[k], off, 64);
+        if ((tid & 63) == 0) sm[k][tid >> 6] = s[k];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < 3; k++) {
+        float t = 0.f;
+        for (int w = 0; w < waves; w++) t += sm[k][w];
+        f[k] = coef[k] / sqrtf(t / (float)cols + eps);
+    }
+    const float e0 = coef[3];
+    const auto value = [&](float t) { return fmaf(fmaf(fmaf(f[2], t, f[1]), t, f[0]), t, e0); };
+    if constexpr (NV > 0) {
+#pragma unroll
+        for (int i = 0; i < NV; i++) {
+            const int c = (tid + i * nt) * 8;
+            if (c < cols) {
+                V8 w;
+#pragma unroll
+                for (int e = 0; e < 8; e++) w[e] = (T)value((float)v[i][e]);
+                *(V8 *)(o + c) = w;
+            }
+        }
+    } else {
+        for (int c = tid; c < cols; c += nt) o[c] = (T)value((float)zr[c]);
+    }
+    for (int c = cols + tid; c < ldo; c += nt) o[c] = (T)0.f;
 }
 
 // ---------------------------------------------------------------- convolution
@@ -385,9 +569,78 @@ void launch_norm(vx_backend *be, const vx_residual_norm_args &p) {
         residual_norm_kernel<T, 8><<<p.rows, threads, 0, be->stream>>>(p);
 }
 
+template <typename T>
+void launch_post_norm(vx_backend *be, const vx_post_norm_args &p) {
+    const auto al = [](const void *q) { return (uintptr_t)q % 16 == 0; };
+    const bool vec = p.cols % 4 == 0 && al(p.x_in) && al(p.x_out) && al(p.y) && al(p.w) && al(p.w_pre) && al(p.out) && al(p.hist) &&
+                     p.hist_stride % 4 == 0 && (!p.w || (p.ldy % 4 == 0 && p.y_stride % 4 == 0)) && p.ldo % 4 == 0;
+    const int n4 = p.cols / 4;
+    int threads = p.rows <= 256 ? 1024 : 256;
+    while (threads > 64 && threads / 2 >= n4) threads /= 2;
+    const int nv = ceil_div(n4, threads);
+    if (!vec || nv > 8)
+        post_norm_kernel<T, 0><<<p.rows, 256, 0, be->stream>>>(p);
+    else if (nv <= 1)
+        post_norm_kernel<T, 1><<<p.rows, threads, 0, be->stream>>>(p);
+    else if (nv <= 2)
+        post_norm_kernel<T, 2><<<p.rows, threads, 0, be->stream>>>(p);
+    else if (nv <= 4)
+        post_norm_kernel<T, 4><<<p.rows, threads, 0, be->stream>>>(p);
+    else
+        post_norm_kernel<T, 8><<<p.rows, threads, 0, be->stream>>>(p);
+}
+
+template <typename T>
+void launch_poly_norm(vx_backend *be, const T *z, int ldz, int rows, int cols, const float *coef, float eps, T *out, int ldo) {
+    const bool vec = cols % 8 == 0 && ldz % 8 == 0 && ldo % 8 == 0 && (uintptr_t)z % 16 == 0 && (uintptr_t)out % 16 == 0;
+    const int n8 = cols / 8;
+    int threads = rows <= 256 ? 1024 : 256;
+    while (threads > 64 && threads / 2 >= n8) threads /= 2;
+    while (threads < 1024 && n8 > 4 * threads) threads *= 2;
+    const int nv = ceil_div(n8, threads);
+    if (!vec || nv > 4)
+        poly_norm_kernel<T, 0><<<rows, 1024, 0, be->stream>>>(z, ldz, cols, coef, eps, out, ldo);
+    else if (nv <= 1)
+        poly_norm_kernel<T, 1><<<rows, threads, 0, be->stream>>>(z, ldz, cols, coef, eps, out, ldo);
+    else if (nv <= 2)
+        poly_norm_kernel<T, 2><<<rows, threads, 0, be->stream>>>(z, ldz, cols, coef, eps, out, ldo);
+    else
+        poly_norm_kernel<T, 4><<<rows, threads, 0, be->stream>>>(z, ldz, cols, coef, eps, out, ldo);
+}
+
 }  // namespace
 
 extern "C" {
+
+int vx_post_norm(vx_backend *be, int act, const vx_post_norm_args *a) {
+    int rc = enter(be);
+    if (rc) return rc;
+    VX_REQUIRE(a && a->rows >= 1 && a->cols >= 1 && a->x_in, "vx_post_norm: bad arguments");
+    VX_REQUIRE(act == VX_ACT_F32 || act == VX_ACT_BF16, "vx_post_norm: unknown activation type %d", act);
+    VX_REQUIRE(!a->w || (a->y && a->y_slices >= 1 && a->ldy >= a->cols), "vx_post_norm: incomplete sublayer output");
+    VX_REQUIRE(a->n_avg == 0 || (a->n_avg > 0 && a->hist && a->avg && a->hist_stride >= 0), "vx_post_norm: incomplete average");
+    VX_REQUIRE(!a->out || a->ldo >= a->cols, "vx_post_norm: rows of %d for %d columns", a->ldo, a->cols);
+    VX_REQUIRE(a->out || a->x_out, "vx_post_norm: nothing to write");
+    if (act == VX_ACT_BF16)
+        launch_post_norm<bf16>(be, *a);
+    else
+        launch_post_norm<float>(be, *a);
+    VX_CHECK_LAUNCH();
+    return VX_OK;
+}
+
+int vx_poly_norm(vx_backend *be, int act, const void *z, int ldz, int rows, int cols, const float *coef, float eps, void *out, int ldo) {
+    int rc = enter(be);
+    if (rc) return rc;
+    VX_REQUIRE(act == VX_ACT_F32 || act == VX_ACT_BF16, "vx_poly_norm: unknown activation type %d", act);
+    VX_REQUIRE(z && coef && out && z != out && rows >= 1 && cols >= 1 && ldz >= cols && ldo >= cols, "vx_poly_norm: bad arguments");
+    if (act == VX_ACT_BF16)
+        launch_poly_norm<bf16>(be, (const bf16 *)z, ldz, rows, cols, coef, eps, (bf16 *)out, ldo);
+    else
+        launch_poly_norm<float>(be, (const float *)z, ldz, rows, cols, coef, eps, (float *)out, ldo);
+    VX_CHECK_LAUNCH();
+    return VX_OK;
+}
 
 int vx_residual_norm(vx_backend *be, int act, const vx_residual_norm_args *a) {
     int rc = enter(be);

@@ -1,4 +1,4 @@
-// Shared pieces of the mixed-batch kernels (linear.hip, mixers.hip, attn_ragged.hip): activation types, eight-element
+// Shared pieces of the mixed-batch kernels (linear.hip, mixers.hip, attn_ragged.hip, attn_latent.hip): activation types, eight-element
 // vectors of them, the matrix-core product of one 16 x 16 x 32 tile, and the map from work items to sequences.
 #pragma once
 
@@ -72,13 +72,14 @@ __device__ __forceinline__ int seq_of_row(const int32_t *cu, int n_seqs, int row
 }
 
 // Work item `id` of a launch that gives every sequence with at least `min_rows` rows ceil(rows / per_item) items, in
-// batch order: its sequence, its index in the sequence and the sequence's item count. False beyond the last.
+// batch order: its sequence, its index in the sequence and the sequence's item count. False beyond the last. A row may be `each`
+// units of which an item takes per_item; max_rows > 0 leaves out sequences with more.
 __device__ __forceinline__ bool item_of_seq(const int32_t *cu, int n_seqs, int per_item, int min_rows, int id, int *seq, int *index,
-                                            int *count) {
+                                            int *count, int each = 1, int max_rows = 0) {
     int c0 = cu[0];
     for (int s = 0; s < n_seqs; s++) {
         const int c1 = cu[s + 1], n = c1 - c0;
-        const int items = n < min_rows ? 0 : (n + per_item - 1) / per_item;
+        const int items = n < min_rows || (max_rows > 0 && n > max_rows) ? 0 : (n * each + per_item - 1) / per_item;
         if (id < items) {
             *seq = s, *index = id, *count = items;
             return true;

@@ -327,6 +327,7 @@ struct Builder {
     vx_backend *be;
     const SafeTensors *st;
     vh_model *m;
+    int block_size;
     void *stage = nullptr;       // device copy of the matrix being packed
     size_t stage_bytes = 0;
     int pad(int n, int to) const { return (n + to - 1) / to * to; }
@@ -392,6 +393,42 @@ struct Builder {
         VXC(vx_linear_pack(be, stage, n, k, w.w, w.n, w.k, row0 / 16, step, col0));
         return VH_OK;
     }
+    int pack_host(const std::vector<uint16_t> &h, int n, int k, const Linear &w, int row0) {
+        const size_t bytes = h.size() * 2;
+        if (bytes > stage_bytes) {
+            if (stage) vx_free(be, stage);
+            stage = vx_alloc_permanent(be, bytes);
+            stage_bytes = stage ? bytes : 0;
+            if (!stage) return fail("device memory: %s", vx_last_error());
+        }
+        VXC(vx_to_device(be, stage, h.data(), bytes));
+        VXC(vx_linear_pack(be, stage, n, k, w.w, w.n, w.k, row0 / 16, 1, 0));
+        return VH_OK;
+    }
+    // A matrix [n, k] put together on the host from the elements of that tensor [total, from]: place(row, col) says which element
+    // (row * from + col) goes there, -1 none.
+    template <class Place>
+    int pack_placed(const std::string &name, int total, int from, int n, int k, const Linear &w, int row0, Place &&place) {
+        const TensorView *t;
+        VHC(view(name, {total, from}, &t));
+        std::vector<uint16_t> h((size_t)n * k, 0);
+        for (int r = 0; r < n; r++)
+            for (int c = 0; c < k; c++) {
+                const int64_t e = place(r, c);
+                if (e >= 0) memcpy(&h[(size_t)r * k + c], t->data + 2 * e, 2);
+            }
+        return pack_host(h, n, k, w, row0);
+    }
+    // The same in whole rows: row r is row src(r) of the tensor, -1 none.
+    template <class Row>
+    int pack_rows(const std::string &name, int total, int k, int n, const Linear &w, int row0, Row &&src) {
+        const TensorView *t;
+        VHC(view(name, {total, k}, &t));
+        std::vector<uint16_t> h((size_t)n * k, 0);
+        for (int r = 0; r < n; r++)
+            if (const int s = src(r); s >= 0) memcpy(&h[(size_t)r * k], t->data + (size_t)s * k * 2, (size_t)k * 2);
+        return pack_host(h, n, k, w, row0);
+    }
 };
 
 int distance_bucket(int n, int rows, int bias_max) {
@@ -409,7 +446,7 @@ int build_lozedra(Builder &b, const Json &config, MixModel *x, vh_config *cfg) {
     LozedraConfig c;
     VHC(parse_lozedra(config, &c));
     cfg->hidden = c.width, cfg->vocab = c.vocab, cfg->eps = c.eps;
-    x->eps = c.eps, x->mult = c.mult;
+    x->eps = c.eps, x->mult = c.mult, x->recurrent = true;
     for (size_t i = 0; i < c.layers.size(); i++) {
         const LozedraLayer &s = c.layers[i];
         const std::string l = "l" + std::to_string(i) + ".", left = l + "mix.left.", right = l + "mix.right.", mlp = l + "mlp.";
@@ -515,6 +552,225 @@ int check_lozedra(const Json &config) {
     return parse_lozedra(config, &c);
 }
 
+// ---------------------------------------------------------------- Tulipel
+struct TulipelLayer {
+    int heads = 1, dim = 1, rot_dim = 2, vdim = 1, rank = 1, q_rank = 0;  // q_rank 0: queries straight from the stream
+    float scale = 1.f;
+    bool halves = false;          // rotated pairs are (i, i + n / 2) in the tensors; packed as neighbours
+    double base = 1.0;
+    bool yarn = false;
+    double factor = 1.0, original = 1.0, fast = 1.0, slow = 1.0;
+    int kv_from = -1, ff = 0;     // ff 0: no feed-forward
+    bool same_rotation(const TulipelLayer &o) const {
+        return rot_dim == o.rot_dim && halves == o.halves && base == o.base && yarn == o.yarn &&
+               (!yarn || (factor == o.factor && original == o.original && fast == o.fast && slow == o.slow));
+    }
+};
+struct TulipelConfig {
+    std::vector<TulipelLayer> layers;
+    float eps = 1e-5f, alpha = 1.f, softcap = 0.f;
+    int vocab = 1, width = 1;
+};
+
+int parse_tulipel(const Json &j, TulipelConfig *c) {
+    int rc = VH_OK;
+    const Fields root("config", &j, &rc);
+    c->vocab = root.count("vocab");
+    c->width = root.count("width", 1, 1 << 20);
+    c->alpha = (float)root.num("postln_alpha");
+    c->eps = (float)root.sub("norm").num("eps");
+    if (root.has("logit_softcap")) {
+        c->softcap = (float)root.num("logit_softcap");
+        if (rc == VH_OK && !(c->softcap > 0.f)) return fail("config.json: logit_softcap is not above 0");
+    }
+    const Json *layers = root.need("layers", Json::ARR);
+    if (rc != VH_OK) return rc;
+    if (layers->arr.empty()) return fail("config.json: no layers");
+    for (size_t i = 0; i < layers->arr.size(); i++) {
+        const Fields l("layers[" + std::to_string(i) + "]", &layers->arr[i], &rc);
+        const Json *type = l.need("type", Json::STR);
+        if (rc != VH_OK) return rc;
+        TulipelLayer o;
+        const Fields mx = l.sub("mixer"), rot = mx.sub("rot");
+        if (type->str == "latent_attention")
+            o.q_rank = mx.count("q_rank", 1, 1 << 16);
+        else if (type->str == "latent_attention_2")
+            o.halves = true;
+        else
+            return fail("config.json: layer %zu has the unknown mixer type '%s'", i, type->str.c_str());
+        o.heads = mx.count("heads", 1, 4096), o.dim = mx.count("dim", 1, 2048), o.vdim = mx.count("vdim", 1, 2048);
+        o.rank = mx.count("kv_rank", 1, 2048), o.rot_dim = mx.count("rot_dim", 2, 1024);
+        o.scale = (float)mx.num("scale");
+        o.base = rot.num("base");
+        const int dims = rot.count("dims", 2, 1024);
+        if (rot.has("scaling")) {
+            const Fields y = rot.sub("scaling");
+            o.yarn = true;
+            o.factor = y.num("factor"), o.original = y.num("original"), o.fast = y.num("fast"), o.slow = y.num("slow");
+            if (rc == VH_OK && !(o.factor > 0 && o.original > 0 && o.fast > 0 && o.slow > 0)) return fail("config.json: layer %zu: rot.scaling is not above 0", i);
+        }
+        if (mx.has("kv_from")) o.kv_from = mx.count("kv_from", 0, 1 << 16);
+        if (l.has("mlp")) {
+            const Fields mlp = l.sub("mlp");
+            const Json *kind = mlp.need("kind", Json::STR);
+            if (rc == VH_OK && kind->str != "dense") return fail("config.json: layer %zu has the unknown feed-forward '%s'", i, kind->str.c_str());
+            o.ff = mlp.count("ff", 1, 1 << 20);
+        }
+        if (rc != VH_OK) return rc;
+        if (o.rot_dim % 2 || dims != o.rot_dim) return fail("config.json: layer %zu turns %d of %d dimensions", i, dims, o.rot_dim);
+        if (!(o.base > 1.0)) return fail("config.json: layer %zu: rot.base is not above 1", i);
+        if (o.kv_from >= 0) {
+            if (o.kv_from >= (int)i || c->layers[o.kv_from].kv_from >= 0)
+                return fail("config.json: layer %zu: layer %d holds no latents for it", i, o.kv_from);
+            const TulipelLayer &f = c->layers[o.kv_from];
+            if (f.rank != o.rank || !f.same_rotation(o)) return fail("config.json: layer %zu: the latents of layer %d are of another kind", i, o.kv_from);
+        }
+        c->layers.push_back(o);
+    }
+    return rc;
+}
+
+// Radians per position of every pair, and the factor of cosine and sine.
+void rotary_frequencies(int dims, double base, bool yarn, double factor, double original, double fast, double slow, std::vector<double> *f, double *both) {
+    f->resize(dims / 2);
+    for (int i = 0; i < dims / 2; i++) (*f)[i] = pow(base, -2.0 * i / dims);
+    *both = 1.0;
+    if (!yarn) return;
+    // the (fractional) dimension whose pair makes that many turns over the original length
+    const auto dim_of = [&](double turns) { return dims * log(original / (2 * M_PI * turns)) / (2 * log(base)); };
+    const double lo = fmax(floor(dim_of(fast)), 0.0), hi = fmin(ceil(dim_of(slow)), dims - 1.0);
+    for (int i = 0; i < dims / 2; i++) {
+        const double ramp = fmin(fmax((i - lo) / fmax(hi - lo, 0.001), 0.0), 1.0);
+        (*f)[i] = (*f)[i] / factor * ramp + (*f)[i] * (1.0 - ramp);
+    }
+    *both = 0.1 * log(factor) + 1.0;
+}
+
+// From how many rows of a sequence on it pays to spell its keys and values out: per (row, key, head) that takes 2 rank - dim - vdim
+// products less, and rank (dim + vdim) per (key, head) once. Half as many rows again, since the keys before the sequence's
+// new rows count in full and the spelled-out ones have to be written and read.
+int spell_out_rows(const LatentMixer &t, int dim, int vdim) {
+    const int64_t less = 2 * (int64_t)t.rank - dim - vdim;
+    if (less <= 0) return 0;
+    const int64_t rows = (3 * (int64_t)t.rank * (dim + vdim) / 2 + less - 1) / less;
+    return rows < (1 << 20) ? (int)(rows < 2 ? 2 : rows) : 0;
+}
+
+int build_tulipel(Builder &b, const Json &config, MixModel *x, vh_config *cfg) {
+    TulipelConfig c;
+    VHC(parse_tulipel(config, &c));
+    cfg->hidden = c.width, cfg->vocab = c.vocab, cfg->eps = c.eps;
+    x->eps = c.eps, x->post_norm = true, x->alpha = c.alpha, x->softcap = c.softcap;
+    const int W = c.width;
+    std::vector<int> rotation_layer;  // a layer that has rotation 0, 1, ..
+    const auto around_zero = [&](const std::string &name, const float **out) -> int {
+        std::vector<float> v;
+        VHC(b.floats(name, {W}, &v));
+        for (float &f : v) f += 1.0f;
+        return b.upload(v, out);
+    };
+    for (size_t i = 0; i < c.layers.size(); i++) {
+        const TulipelLayer &s = c.layers[i];
+        const std::string l = "l" + std::to_string(i) + ".", mix = l + "mix.", mlp = l + "mlp.";
+        MixLayer o;
+        o.has_latent = true;
+        LatentMixer &t = o.latent;
+        VHC(around_zero(l + "norm1", &o.norm1));
+        t.heads = s.heads, t.rank = s.rank, t.rot_dim = s.rot_dim, t.q_rank = s.q_rank, t.scale = s.scale, t.kv_from = s.kv_from;
+        t.dim_pad = b.pad(s.dim, 64), t.head_cols = t.dim_pad + b.pad(s.rot_dim, 16), t.v_pad = b.pad(s.vdim, 16);
+        t.rank_pad = vx_latent_pad(s.rank), t.row = vx_latent_row(s.rank, s.rot_dim);
+        for (size_t k = 0; k < rotation_layer.size(); k++)
+            if (s.same_rotation(c.layers[rotation_layer[k]])) t.rotation = (int)k;
+        if (t.rotation < 0) {
+            t.rotation = (int)rotation_layer.size();
+            rotation_layer.push_back((int)i);
+            Rotation r;
+            double both;
+            rotary_frequencies(s.rot_dim, s.base, s.yarn, s.factor, s.original, s.fast, s.slow, &r.freqs, &both);
+            r.factor = (float)both;
+            x->rotations.push_back(r);
+        }
+        // columns: heads, each its plain part, then its rotated part with the pairs as neighbours
+        const int half = s.rot_dim / 2, q_cols = s.heads * t.head_cols, qd = s.heads * (s.dim + s.rot_dim);
+        const auto pair_place = [&](int d) { return s.halves ? d / 2 + d % 2 * half : d; };  // packed rotated column -> stored one
+        const auto q_row = [&](int r) {
+            const int h = r / t.head_cols, d = r % t.head_cols, rd = d - t.dim_pad;
+            if (rd >= 0) return rd < s.rot_dim ? h * (s.dim + s.rot_dim) + s.dim + pair_place(rd) : -1;
+            return d < s.dim ? h * (s.dim + s.rot_dim) + d : -1;
+        };
+        const bool own = s.kv_from < 0;
+        const int first = s.q_rank > 0 ? b.pad(s.q_rank, 16) : q_cols;
+        const int kv_cols = own ? b.pad(s.rank, 16) + b.pad(s.rot_dim, 16) : 0;
+        t.c_col = s.q_rank > 0 ? first : 0, t.kr_col = t.c_col + b.pad(s.rank, 16), t.kv_cols = kv_cols;
+        VHC(b.packed(&o.in, first + kv_cols, W));
+        if (s.q_rank > 0) {
+            VHC(b.pack(mix + "dq", s.q_rank, W, 0, s.q_rank, o.in, 0, 1, 0));
+            VHC(b.vec(mix + "dq.norm", s.q_rank, &t.norm_q));
+            VHC(b.packed(&t.q_up, q_cols, s.q_rank));
+            VHC(b.pack_rows(mix + "uq", qd, s.q_rank, q_cols, t.q_up, 0, q_row));
+        } else {
+            VHC(b.pack_rows(mix + "q", qd, W, q_cols, o.in, 0, q_row));
+        }
+        if (own) {
+            VHC(b.pack(mix + "dkv", s.rank + s.rot_dim, W, 0, s.rank, o.in, first, 1, 0));
+            VHC(b.pack_rows(mix + "dkv", s.rank + s.rot_dim, W, s.rot_dim, o.in, first + b.pad(s.rank, 16), [&](int r) { return s.rank + pair_place(r); }));
+            VHC(b.vec(mix + "dkv.norm", s.rank, &t.norm_c));
+        }
+        VHC(b.vec(mix + "sink", s.heads, &t.sink));
+        // out of the latents: keys of all heads, then values; into them: per head, the keys' matrix transposed
+        VHC(b.packed(&t.expand, q_cols + s.heads * t.v_pad, t.rank_pad));
+        VHC(b.pack_rows(mix + "uk", s.heads * s.dim, s.rank, q_cols, t.expand, 0, [&](int r) {
+            const int h = r / t.head_cols, d = r % t.head_cols;
+            return d < s.dim ? h * s.dim + d : -1;
+        }));
+        VHC(b.pack_rows(mix + "uv", s.heads * s.vdim, s.rank, s.heads * t.v_pad, t.expand, q_cols, [&](int r) {
+            const int h = r / t.v_pad, d = r % t.v_pad;
+            return d < s.vdim ? h * s.vdim + d : -1;
+        }));
+        VHC(b.packed(&t.absorb, s.heads * t.rank_pad, t.dim_pad));
+        VHC(b.pack_placed(mix + "uk", s.heads * s.dim, s.rank, s.heads * t.rank_pad, s.dim, t.absorb, 0, [&](int r, int d) -> int64_t {
+            const int h = r / t.rank_pad, e = r % t.rank_pad;
+            return e < s.rank ? ((int64_t)h * s.dim + d) * s.rank + e : -1;
+        }));
+        VHC(b.packed(&o.out, W, s.heads * t.v_pad));
+        VHC(b.pack_placed(mix + "o", W, s.heads * s.vdim, W, s.heads * t.v_pad, o.out, 0, [&](int r, int k) -> int64_t {
+            const int h = k / t.v_pad, d = k % t.v_pad;
+            return d < s.vdim ? (int64_t)r * s.heads * s.vdim + h * s.vdim + d : -1;
+        }));
+        if (x->act == VX_ACT_BF16 && vx_attn_latent_fast(x->act, b.block_size, s.rank, s.rot_dim) &&
+            vx_attn_ragged_fast(x->act, b.block_size, s.heads, s.heads, t.head_cols, t.v_pad)) {
+            t.expand_rows = spell_out_rows(t, s.dim + b.pad(s.rot_dim, 16) - s.rot_dim, s.vdim);
+            if (t.expand_rows > 0 && (x->expand_rows == 0 || t.expand_rows < x->expand_rows)) x->expand_rows = t.expand_rows;
+        }
+        if (s.ff > 0) {
+            o.has_mlp = true;
+            o.ff = s.ff, o.ff_pad = b.pad(s.ff, 64);
+            VHC(around_zero(l + "norm2", &o.norm2));
+            VHC(b.packed(&o.gate_up, o.ff_pad, W));
+            VHC(b.pack(mlp + "up", s.ff, W, 0, s.ff, o.gate_up, 0, 1, 0));
+            VHC(b.packed(&o.down, W, s.ff));
+            VHC(b.pack(mlp + "down", W, s.ff, 0, W, o.down, 0, 1, 0));
+            VHC(b.vec(mlp + "act", 4, &o.poly));
+        }
+        VHC(b.vec(l + "dwa", (int)i + 2, &o.depth_avg));
+        x->layers.push_back(o);
+        LayerRun r;
+        r.layer = (int)i;
+        x->runs.push_back(r);
+    }
+    std::vector<float> emb;
+    VHC(b.floats("embed", {c.vocab, W}, &emb));
+    VHC(b.upload(emb, &b.m->embedding));
+    VHC(around_zero("final.norm", &b.m->final_norm));
+    VHC(b.packed(&x->head, c.vocab, W));
+    return b.pack("head", c.vocab, W, 0, c.vocab, x->head, 0, 1, 0);
+}
+
+int check_tulipel(const Json &config) {
+    TulipelConfig c;
+    return parse_tulipel(config, &c);
+}
+
 // ---------------------------------------------------------------- registry
 struct Architecture {
     const char *name;                                                    // config.json "architecture"
@@ -523,6 +779,7 @@ struct Architecture {
 };
 const Architecture kArchitectures[] = {
     {"Lozedra", check_lozedra, build_lozedra},
+    {"Tulipel", check_tulipel, build_tulipel},
 };
 
 const Architecture *find_architecture(const Json &config) {
@@ -590,7 +847,7 @@ int vh_model_load(vx_backend *be, const char *path, const vh_load_options *opt, 
     m->mix->act = opt->dtype == VH_DTYPE_F32 ? VX_ACT_F32 : VX_ACT_BF16;
     int rc;
     {
-        Builder b{be, &st, m};
+        Builder b{be, &st, m, c.block_size};
         rc = arch->build(b, config, m->mix.get(), &c);
     }
     c.num_layers = (int)m->mix->runs.size();  // (the layers that hold a cache: every pass has its own)

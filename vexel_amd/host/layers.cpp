@@ -3,6 +3,9 @@
 // A step is a set of sequences with any number of new tokens each. Its rows run through every layer together:
 //   norm | input projection (K and V leave for the paged pool on the way) | attention and / or convolution + scan | output
 //   projection | norm, residual, norm | gate|up with SiLU | down | norm, residual, and the next layer's norm
+// or, with the norm behind the residual sum and latent attention,
+//   input projection (queries turned on the way) | norms, latents to the paged pool | queries into the latents' space |
+//   attention | results out of it | output projection | residual, norm | up | activation | down | residual, norm, average
 // The block tables, the pool's bookkeeping and the sequence slots are the runtime's own; recurrent state lies in one slot
 // per sequence (the row of its block table), and a sequence at position 0 starts from nothing whatever the slot holds.
 #include <math.h>
@@ -22,13 +25,14 @@ size_t esize(const MixModel &x) { return x.act == VX_ACT_F32 ? 4 : 2; }
 
 struct Widths {
     int width_pad = 0, in = 0, out = 0, xc = 0, dtr = 0, bc = 0, dt = 0, act = 0;
+    int qc = 0, qa = 0, z = 0, rot = 0;
 };
 
 Widths widths(const vh_model *m) {
     Widths w;
     w.width_pad = pad_to(m->cfg.hidden, 64);
     for (const MixLayer &l : m->mix->layers) {
-        w.in = std::max(w.in, l.in.n);
+        w.in = std::max(w.in, l.has_latent ? l.latent.heads * l.latent.head_cols : l.in.n);
         w.out = std::max(w.out, l.out.k);
         w.act = std::max(w.act, l.ff_pad);
         if (l.has_scan) {
@@ -37,18 +41,33 @@ Widths widths(const vh_model *m) {
             w.bc = std::max(w.bc, 2 * l.scan.pad);
             w.dt = std::max(w.dt, l.scan.dt.n);
         }
+        if (l.has_latent) {
+            w.qc = std::max(w.qc, l.latent.q_up.k);
+            w.qa = std::max(w.qa, l.latent.heads * l.latent.rank_pad);
+        }
+        if (l.poly) w.z = std::max(w.z, l.ff_pad);
     }
+    for (const Rotation &r : m->mix->rotations) w.rot += 2 * (int)r.freqs.size();
     return w;
 }
 
-// slices x rows of float32 sublayer outputs that a step of up to `rows` rows may need
-size_t slice_rows(const vh_model *m, int rows, bool up_to) {
+// floats of sliced sublayer outputs, and of latent projections, that a step of up to `rows` rows may need
+size_t slice_floats(const vh_model *m, int rows, bool up_to) {
     size_t most = 1;
-    for (const MixLayer &l : m->mix->layers)
-        for (const Linear *w : {&l.out, &l.down}) {
-            if (!w->w) continue;
-            for (int r = up_to ? 1 : rows; r <= rows; r++) most = std::max(most, (size_t)r * vx_linear_slices(m->be, w->n, w->k, r));
-        }
+    const auto sliced = [&](const Linear &w, int cols) {
+        if (!w.w) return;
+        for (int r = up_to ? 1 : rows; r <= rows; r++) most = std::max(most, (size_t)r * vx_linear_slices(m->be, w.n, w.k, r) * cols);
+    };
+    const int cols = pad_to(m->cfg.hidden, 16);
+    for (const MixLayer &l : m->mix->layers) {
+        sliced(l.out, cols);
+        sliced(l.down, cols);
+        if (!l.has_latent) continue;
+        if (l.latent.q_rank > 0)
+            sliced(l.in, l.in.n);
+        else
+            most = std::max(most, (size_t)rows * l.latent.kv_cols);
+    }
     return most;
 }
 
@@ -63,11 +82,13 @@ int alloc_acts(vh_model *m, int rows, bool up_to, A &&alloc, MixActs *a) {
         return *p != nullptr;
     };
     a->rows = rows;
-    const int cols = pad_to(m->cfg.hidden, 16);
     const bool ok = get(&a->x, R * m->cfg.hidden * 4) && get(&a->h, R * w.width_pad * es) && get(&a->proj, R * w.in * es) &&
                     get(&a->cat, R * w.out * es) && get(&a->xc, R * w.xc * es) && get(&a->dtr, R * w.dtr * es) &&
                     get(&a->bc, R * w.bc * 4) && get(&a->dt, R * w.dt * 4) && get(&a->act, R * w.act * es) &&
-                    get(&a->y, slice_rows(m, rows, up_to) * cols * 4) && (!loop || get(&a->emb, R * m->cfg.hidden * 4));
+                    get(&a->y, slice_floats(m, rows, up_to) * 4) && (!loop || get(&a->emb, R * m->cfg.hidden * 4)) &&
+                    get(&a->qc, R * w.qc * es) && get(&a->qa, R * w.qa * es) && get(&a->lo, R * w.qa * es) && get(&a->z, R * w.z * es) &&
+                    get(&a->rot, R * w.rot * 4) &&
+                    (!m->mix->post_norm || get(&a->hist, R * m->cfg.hidden * (m->mix->runs.size() + 1) * 4));
     return ok ? (int)VH_OK : fail("activations of %d rows: %s", rows, vx_last_error());
 }
 
@@ -95,6 +116,13 @@ int mix_finish(vh_model *m) {
             if (!r.kv) return fail("KV pool: %s", vx_last_error());
             m->kv.back() = r.kv;
         }
+        if (l.has_latent && l.latent.kv_from < 0) {
+            r.kv = zeroed((size_t)c.block_size * c.pool_blocks * l.latent.row * es);
+            if (!r.kv) return fail("latent pool: %s", vx_last_error());
+            m->kv.back() = r.kv;
+        }
+        if (l.has_latent && l.latent.kv_from >= 0)  // (every layer runs once in a model that shares pools)
+            r.kv = x.runs[l.latent.kv_from].kv;
         if (l.has_scan) {
             r.state = (float *)zeroed((size_t)c.max_seqs * l.scan.channels * l.scan.pad * 4);
             if (!r.state) return fail("scan state: %s", vx_last_error());
@@ -103,6 +131,13 @@ int mix_finish(vh_model *m) {
             if (!r.conv) return fail("convolution state: %s", vx_last_error());
             m->adopted.push_back(r.conv);
         }
+    }
+    for (Rotation &r : x.rotations) {
+        void *p = vx_alloc_permanent(m->be, (r.freqs.size() * 8 + 15) / 16 * 16);
+        if (!p) return fail("device memory: %s", vx_last_error());
+        m->adopted.push_back(p);
+        VXC(vx_to_device(m->be, p, r.freqs.data(), r.freqs.size() * 8));
+        r.d_freqs = (const double *)p;
     }
     VHC(init_common(m));
     VHC(alloc_acts(m, c.max_batch, true, [&](size_t n) {
@@ -187,11 +222,104 @@ int run_mixers(vh_model *m, const LayerRun &r, const vx_ragged &b, const MixActs
     return VH_OK;
 }
 
+// a rotation's angles of the step's rows
+const float *rot_table(const MixModel &x, const MixActs &a, int rows, int rotation) {
+    if (rotation < 0) return nullptr;
+    size_t before = 0;
+    for (int i = 0; i < rotation; i++) before += x.rotations[i].freqs.size();
+    return a.rot + before * 2 * rows;
+}
+
+// latent attention of one layer run: a.h -> the sublayer's output as `slices` partial sums in a.y
+int run_latent(vh_model *m, const LayerRun &r, const vx_ragged &b, const MixActs &a, const MixExpand *ex, int *slices) {
+    const MixModel &x = *m->mix;
+    const MixLayer &l = x.layers[r.layer];
+    const LatentMixer &t = l.latent;
+    const size_t es = esize(x);
+    const int rows = b.rows, width_pad = pad_to(m->cfg.hidden, 64), q_cols = t.heads * t.head_cols, ldc = l.out.k;
+    const float *tab = rot_table(x, a, rows, t.rotation);
+    const auto heads_out = [&]() {  // the queries' projection: heads, their last part turned
+        vx_linear_out o = plain(a.proj, 0, q_cols, q_cols, 1);
+        if (tab) {
+            o.kind = VX_LIN_ROTARY;
+            o.split = q_cols, o.rot_stride = t.head_cols, o.rot_first = t.dim_pad, o.rot_pairs = t.rot_dim / 2, o.rot_tab = tab;
+        }
+        return o;
+    };
+    vx_latent_store_args st;
+    memset(&st, 0, sizeof st);
+    st.y = a.y, st.y_slices = 1, st.eps = x.eps, st.rot_tab = tab;
+    if (t.kv_from < 0) st.rank = t.rank, st.rot_dim = t.rot_dim, st.w_c = t.norm_c, st.pool = r.kv;
+    if (t.q_rank > 0) {  // query latent and key latent in one float32 projection
+        *slices = vx_linear_slices(m->be, l.in.n, l.in.k, rows);
+        vx_linear_out o = plain(a.y, 1, l.in.n, l.in.n, *slices);
+        VXC(vx_linear(m->be, x.act, a.h, width_pad, l.in.w, l.in.n, l.in.k, rows, &o));
+        st.y_slices = *slices, st.ldy = l.in.n, st.y_stride = (int64_t)rows * l.in.n;
+        st.c_col = t.c_col, st.kr_col = t.kr_col, st.q_rank = t.q_rank, st.w_q = t.norm_q, st.q_out = a.qc, st.ldq = t.q_up.k;
+        VXC(vx_latent_store(m->be, x.act, &b, &st));
+        o = heads_out();
+        VXC(vx_linear(m->be, x.act, a.qc, t.q_up.k, t.q_up.w, t.q_up.n, t.q_up.k, rows, &o));
+    } else {
+        vx_linear_out o = heads_out();
+        if (t.kv_cols > 0) {
+            if (!tab) o.kind = VX_LIN_SPLIT, o.split = q_cols;
+            o.out2 = a.y, o.ldo2 = t.kv_cols;
+        }
+        VXC(vx_linear(m->be, x.act, a.h, width_pad, l.in.w, l.in.n, l.in.k, rows, &o));
+        st.ldy = t.kv_cols, st.c_col = t.c_col, st.kr_col = t.kr_col;
+        if (st.rank > 0) VXC(vx_latent_store(m->be, x.act, &b, &st));
+    }
+    if (t.heads * t.v_pad < ldc) VXC(vx_fill_zero(m->be, a.cat, (size_t)rows * ldc * es));
+    // sequences with many rows: keys and values of all their tokens spelled out, once for all rows and heads
+    const int many = ex && ex->rows > 0 ? t.expand_rows : 0;
+    bool few = many == 0;
+    if (many > 0)
+        for (int s = 0; s < b.n_seqs; s++) few = few || b.q_lens[s] < many;
+    if (few) {
+        vx_linear_out o = plain(a.qa, 0, t.heads * t.rank_pad, t.rank_pad, 1);
+        o.groups = t.heads, o.a_group = t.head_cols, o.out_group = t.rank_pad;
+        VXC(vx_linear(m->be, x.act, a.proj, q_cols, t.absorb.w, t.rank_pad, t.dim_pad, rows, &o));
+        vx_latent_attn_args at_;
+        memset(&at_, 0, sizeof at_);
+        at_.heads = t.heads, at_.rank = t.rank, at_.rot_dim = t.rot_dim, at_.scale = t.scale, at_.sink = t.sink;
+        at_.q = a.qa, at_.ldq = t.heads * t.rank_pad;
+        at_.qr = at(a.proj, t.dim_pad, es), at_.ldqr = q_cols, at_.qr_stride = t.head_cols;
+        at_.pool = r.kv, at_.out = a.lo, at_.ldo = t.heads * t.rank_pad, at_.max_rows = many > 0 ? many - 1 : 0;
+        VXC(vx_attn_latent(m->be, x.act, &b, &at_));
+        o = plain(a.cat, 0, ldc, t.v_pad, 1);
+        o.groups = t.heads, o.a_group = t.rank_pad, o.out_group = t.v_pad;
+        VXC(vx_linear(m->be, x.act, a.lo, t.heads * t.rank_pad, at(t.expand.w, (size_t)q_cols * t.rank_pad, 2), t.v_pad, t.rank_pad, rows, &o));
+    }
+    if (many > 0) {
+        vx_linear_out o = plain(a.proj, 0, t.expand.n, t.expand.n, 1);  // (every column leaves for the pool)
+        o.kind = VX_LIN_KV;
+        o.k_col = 0, o.v_col = q_cols, o.kv_heads = t.heads, o.k_dim = t.head_cols, o.v_dim = t.v_pad;
+        o.block_size = b.block_size, o.pool = ex->kv, o.a_rows = ex->slots;
+        VXC(vx_linear(m->be, x.act, r.kv, t.row, t.expand.w, t.expand.n, t.rank_pad, ex->rows, &o));
+        VXC(vx_latent_spread(m->be, x.act, r.kv, t.rank, t.rot_dim, ex->slots, ex->rows, ex->kv, t.heads, t.head_cols, t.v_pad, b.block_size,
+                             t.dim_pad));
+        vx_ragged eb = b;
+        eb.table_rows = ex->table_rows, eb.block_tables = ex->tables, eb.max_blocks = ex->max_blocks;
+        eb.max_kv_len = std::min(b.max_kv_len, ex->max_blocks * b.block_size);
+        vx_attn_args at_;
+        memset(&at_, 0, sizeof at_);
+        at_.heads = at_.kv_heads = t.heads, at_.k_dim = t.head_cols, at_.v_dim = t.v_pad, at_.scale = t.scale, at_.sink = t.sink;
+        at_.q = a.proj, at_.ldq = q_cols, at_.pool = ex->kv, at_.out_scale = 1.f, at_.out = a.cat, at_.ldo = ldc, at_.min_rows = many;
+        VXC(vx_attn_ragged(m->be, x.act, &eb, &at_));
+    }
+    *slices = vx_linear_slices(m->be, l.out.n, l.out.k, rows);
+    vx_linear_out o = plain(a.y, 1, l.out.n, l.out.n, *slices);
+    VXC(vx_linear(m->be, x.act, a.cat, ldc, l.out.w, l.out.n, l.out.k, rows, &o));
+    return VH_OK;
+}
+
 int run_mlp(vh_model *m, const MixLayer &l, int rows, const MixActs &a, int *slices) {
     const MixModel &x = *m->mix;
-    vx_linear_out o = plain(a.act, 0, l.ff_pad, l.ff_pad, 1);
-    o.kind = VX_LIN_SWIGLU;
-    VXC(vx_linear(m->be, x.act, a.h, pad_to(m->cfg.hidden, 64), l.gate_up.w, l.gate_up.n, l.gate_up.k, rows, &o));
+    const int width_pad = pad_to(m->cfg.hidden, 64);
+    vx_linear_out o = plain(l.poly ? a.z : a.act, 0, l.ff_pad, l.ff_pad, 1);
+    if (!l.poly) o.kind = VX_LIN_SWIGLU;
+    VXC(vx_linear(m->be, x.act, a.h, width_pad, l.gate_up.w, l.gate_up.n, l.gate_up.k, rows, &o));
+    if (l.poly) VXC(vx_poly_norm(m->be, x.act, a.z, l.ff_pad, rows, l.ff, l.poly, x.eps, a.act, l.ff_pad));
     *slices = vx_linear_slices(m->be, l.down.n, l.down.k, rows);
     o = plain(a.y, 1, l.down.n, l.down.n, *slices);
     VXC(vx_linear(m->be, x.act, a.act, l.ff_pad, l.down.w, l.down.n, l.down.k, rows, &o));
@@ -200,15 +328,23 @@ int run_mlp(vh_model *m, const MixLayer &l, int rows, const MixActs &a, int *sli
 
 }  // namespace
 
-int mix_forward(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, const MixActs &a, const int32_t *want, int n_want,
-                float *logits) {
+namespace {
+
+int head_logits(vh_model *m, const MixActs &a, int n, float *logits) {
+    const MixModel &x = *m->mix;
+    vx_linear_out o = plain(logits, 1, m->cfg.vocab, m->cfg.vocab, 1);
+    o.softcap = x.softcap;
+    VXC(vx_linear(m->be, x.act, a.h, pad_to(m->cfg.hidden, 64), x.head.w, x.head.n, x.head.k, n, &o));
+    return VH_OK;
+}
+
+// Layers whose norms precede the sublayers: the seams add what the last one left, normed, and norm what the next one reads.
+int forward_pre_norm(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, const MixActs &a, const int32_t *want, int n_want) {
     const MixModel &x = *m->mix;
     const vh_config &c = m->cfg;
     const int rows = b.rows, width_pad = pad_to(c.hidden, 64);
-    if (rows > a.rows) return fail("internal: %d rows, activations for %d", rows, a.rows);
     float *emb = a.emb ? a.emb : a.x;
     VXC(vx_embedding(m->be, d_tokens, rows, m->embedding, emb, c.vocab, c.hidden));
-    // the seams between sublayers: what the last one left is normed and added, what the next one reads is normed
     vx_residual_norm_args s;
     memset(&s, 0, sizeof s);
     s.rows = rows, s.cols = c.hidden, s.x_in = emb, s.x_out = a.x, s.mult = x.mult, s.eps = x.eps, s.out = a.h, s.ldo = width_pad;
@@ -239,10 +375,99 @@ int mix_forward(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, const 
     s.y = post ? a.y : nullptr, s.w_post = post, s.y_slices = slices, s.ldy = pad_to(c.hidden, 16);
     s.add = nullptr, s.w_pre = m->final_norm;
     VXC(vx_residual_norm(m->be, x.act, &s));
-    vx_linear_out o = plain(logits, 1, c.vocab, c.vocab, 1);
-    VXC(vx_linear(m->be, x.act, a.h, width_pad, x.head.w, x.head.n, x.head.k, n_want, &o));
     return VH_OK;
 }
+
+// Layers whose norms follow the residual sums; the sublayers read the stream itself, and every layer's result is kept for the
+// averages of those behind it.
+int forward_post_norm(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, const MixActs &a, const MixExpand *ex, const int32_t *want,
+                      int n_want) {
+    const MixModel &x = *m->mix;
+    const vh_config &c = m->cfg;
+    const int rows = b.rows, n_runs = (int)x.runs.size();
+    VXC(vx_embedding(m->be, d_tokens, rows, m->embedding, a.hist, c.vocab, c.hidden));
+    for (size_t i = 0; i < x.rotations.size(); i++)
+        VXC(vx_rotary_table(m->be, b.token_pos, rows, (int)x.rotations[i].freqs.size(), x.rotations[i].d_freqs, x.rotations[i].factor,
+                            (float *)rot_table(x, a, rows, (int)i)));
+    vx_post_norm_args s;
+    memset(&s, 0, sizeof s);
+    s.rows = rows, s.cols = c.hidden, s.x_in = a.hist, s.eps = x.eps, s.alpha = x.alpha, s.out = a.h, s.ldo = pad_to(c.hidden, 64);
+    s.hist = a.hist, s.hist_stride = (int64_t)rows * c.hidden, s.keep = 1;
+    VXC(vx_post_norm(m->be, x.act, &s));
+    s.x_out = a.x, s.y = a.y, s.ldy = pad_to(c.hidden, 16), s.y_stride = (int64_t)rows * s.ldy;
+    for (int i = 0; i < n_runs; i++) {
+        const MixLayer &l = x.layers[x.runs[i].layer];
+        VHC(run_latent(m, x.runs[i], b, a, ex, &s.y_slices));
+        s.w = l.norm1;
+        if (l.has_mlp) {
+            VXC(vx_post_norm(m->be, x.act, &s));
+            s.x_in = a.x;
+            VHC(run_mlp(m, l, rows, a, &s.y_slices));
+            s.w = l.norm2;
+        }
+        s.avg = l.depth_avg, s.n_avg = l.depth_avg ? i + 2 : 0;
+        if (i + 1 == n_runs) {  // the rows whose logits are asked for alone, with the final norm
+            if (n_want == 0) return VH_OK;
+            s.rows = n_want, s.row_idx = want, s.keep = 0, s.x_out = nullptr, s.w_pre = m->final_norm;
+        }
+        VXC(vx_post_norm(m->be, x.act, &s));
+        s.x_in = a.x, s.n_avg = 0;
+    }
+    return VH_OK;
+}
+
+}  // namespace
+
+int mix_forward(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, const MixActs &a, const MixExpand *ex, const int32_t *want,
+                int n_want, float *logits) {
+    if (b.rows > a.rows) return fail("internal: %d rows, activations for %d", b.rows, a.rows);
+    VHC(m->mix->post_norm ? forward_post_norm(m, b, d_tokens, a, ex, want, n_want) : forward_pre_norm(m, b, d_tokens, a, want, n_want));
+    return n_want > 0 ? head_logits(m, a, n_want, logits) : (int)VH_OK;
+}
+
+namespace {
+
+// The part of a step that spells keys and values out: lens / tables of the sequences after it. Nothing when no sequence brings
+// enough rows, or when the spelled-out keys would take too much memory.
+int plan_expand(vh_model *m, int n_seqs, const int32_t *q_lens, const std::vector<int> &lens, const std::vector<std::vector<int32_t>> &tables,
+                MixExpand *ex) {
+    const MixModel &x = *m->mix;
+    const int bs = m->cfg.block_size;
+    if (x.expand_rows <= 0) return VH_OK;
+    int64_t blocks = 0, most = 0;
+    for (int i = 0; i < n_seqs; i++)
+        if (q_lens[i] >= x.expand_rows) {
+            const int64_t n = (lens[i] + bs - 1) / bs;
+            blocks += n, most = std::max(most, n);
+        }
+    size_t per_block = 0;
+    for (const MixLayer &l : x.layers)
+        if (l.has_latent && l.latent.expand_rows > 0)
+            per_block = std::max(per_block, vx_kv_block_elems(bs, l.latent.heads, l.latent.head_cols, l.latent.v_pad) * esize(x));
+    if (blocks == 0 || blocks * bs > (1 << 22) || blocks * per_block > ((size_t)8 << 30)) return VH_OK;
+    ex->rows = (int)blocks * bs, ex->max_blocks = (int)most;
+    std::vector<int32_t> up((size_t)ex->rows + (size_t)n_seqs * most + n_seqs);
+    int32_t *slots = up.data(), *tab = slots + ex->rows, *ids = tab + (size_t)n_seqs * most;
+    int64_t at = 0;
+    for (int i = 0; i < n_seqs; i++) {
+        ids[i] = i;
+        for (int64_t k = 0; k < most; k++) tab[i * most + k] = 0;
+        if (q_lens[i] < x.expand_rows) continue;
+        const int n = (lens[i] + bs - 1) / bs;
+        for (int k = 0; k < n; k++, at++) {
+            tab[i * most + k] = (int32_t)at;
+            for (int t = 0; t < bs; t++) slots[at * bs + t] = tables[i][k] * bs + t;  // (behind the last token: finite, not seen)
+        }
+    }
+    ex->kv = vx_alloc(m->be, blocks * per_block);
+    int32_t *d = (int32_t *)vx_alloc(m->be, up.size() * 4);
+    if (!ex->kv || !d) return fail("spelled-out keys: %s", vx_last_error());
+    VXC(vx_to_device(m->be, d, up.data(), up.size() * 4));
+    ex->slots = d, ex->tables = d + ex->rows, ex->table_rows = ex->tables + (size_t)n_seqs * most;
+    return VH_OK;
+}
+
+}  // namespace
 
 int mix_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_lens, const int32_t *tokens, int n_want,
              const int32_t *want_rows, float *logits_out, int32_t *argmax_out) {
@@ -267,6 +492,8 @@ int mix_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_l
     for (int w = 0; w < n_want; w++)
         if (want_rows[w] < 0 || want_rows[w] >= T) return fail("wanted row %d of %d", want_rows[w], T);
     std::vector<int32_t> slots(n_seqs), pos(n_seqs);
+    std::vector<int> lens(n_seqs);
+    std::vector<std::vector<int32_t>> seq_tables(n_seqs);  // of the sequences that may be spelled out
     int max_kv = 1;
     {
         std::lock_guard<std::mutex> g(m->pool.mu);
@@ -290,7 +517,9 @@ int mix_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_l
             SeqState *s = find_seq(m, seq_ids[i]);
             slots[i] = s->slot, pos[i] = s->seq_len;
             VHC(m->pool.ensure_blocks(*s, s->seq_len + q_lens[i]));
-            max_kv = std::max(max_kv, s->seq_len + q_lens[i]);
+            lens[i] = s->seq_len + q_lens[i];
+            max_kv = std::max(max_kv, lens[i]);
+            if (m->mix->expand_rows > 0 && q_lens[i] >= m->mix->expand_rows) seq_tables[i] = s->table;
         }
         VHC(sync_pool_to_device(m));
     }
@@ -316,11 +545,13 @@ int mix_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_l
         logits = (float *)vx_alloc(be, (size_t)n_want * c.vocab * 4);
         if (!logits) return fail("logits of %d rows: %s", n_want, vx_last_error());
     }
+    MixExpand ex;
+    if (!one_each) VHC(plan_expand(m, n_seqs, q_lens, lens, seq_tables, &ex));
     VXC(vx_pack_batch(be, d_slots, d_pos, one_each ? nullptr : d_q, n_seqs, T, m->d_tables, c.max_blocks_per_seq, m->d_num_blocks,
                       m->d_free, m->d_free_count, c.block_size, d_cu, d_tp, d_sm, d_kvl, m->d_status));
     const vx_ragged b{T, n_seqs, one_each ? nullptr : q_lens, max_kv, d_cu, d_tp, d_sm, d_slots, d_kvl, m->d_tables, c.max_blocks_per_seq,
                       c.block_size};
-    VHC(mix_forward(m, b, d_tok, acts, n_want ? d_want : nullptr, n_want, logits));
+    VHC(mix_forward(m, b, d_tok, acts, ex.rows > 0 ? &ex : nullptr, n_want ? d_want : nullptr, n_want, logits));
     if (n_want > 0 && argmax_out) {
         int32_t *d_am = n_want <= c.max_batch ? m->d_next : (int32_t *)vx_alloc(be, (size_t)n_want * 4);
         if (!d_am) return fail("arg-max rows: %s", vx_last_error());

@@ -114,22 +114,50 @@ struct ScanMixer {    // vx_conv_silu, the projections of its result, vx_selecti
     const float *dt_bias = nullptr, *a2 = nullptr, *d = nullptr;
 };
 
+struct Rotation {      // pairs (2i, 2i + 1) turn by position * freqs[i]; cosine and sine times factor
+    std::vector<double> freqs;
+    float factor = 1.f;
+    const double *d_freqs = nullptr;
+};
+
+// Latent attention (vx_latent_store, vx_attn_latent). Prompts' queries meet either the latents themselves (queries carried into
+// their space by `absorb`, results out of it by `value`) or, from expand_rows rows of a sequence on, keys and values
+// spelled out for the step (`expand`, vx_attn_ragged). Heads of the query projection: dim_pad columns, then the rotated part.
+struct LatentMixer {
+    int heads = 0, rank = 0, rot_dim = 0, q_rank = 0;
+    int dim_pad = 0, head_cols = 0, v_pad = 0, rank_pad = 0, row = 0;
+    float scale = 1.f;
+    int rotation = -1;                                 // index in MixModel::rotations, -1: nothing is rotated
+    int kv_from = -1;                                  // the layer whose pool is read, -1: its own
+    int c_col = 0, kr_col = 0, kv_cols = 0;            // in the float32 part of the input projection (q_rank > 0: all of it, the
+                                                       // query latent first; else kv_cols columns behind the heads)
+    const float *norm_c = nullptr, *norm_q = nullptr, *sink = nullptr;
+    Linear q_up;                                       // query latent -> heads (q_rank > 0)
+    Linear absorb;                                     // per head: dim_pad -> rank_pad, one behind the other
+    Linear expand;                                     // rank_pad -> heads' keys [heads * head_cols] | values [heads * v_pad]
+    int expand_rows = 0;                               // 0: never
+};
+
 // x += mult * rms(mixers(rms(x) * norm1)) * norm1b, then the same around the MLP. The mixers of a layer read one input
-// projection and write one row, which one output projection takes.
+// projection and write one row, which one output projection takes. In a model with post_norm instead: x = rms(alpha * x +
+// mixer(x)) * norm1, x = rms(alpha * x + MLP(x)) * norm2, then the average over the depth.
 struct MixLayer {
     const float *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr;
-    bool has_attn = false, has_scan = false, has_mlp = false;
+    bool has_attn = false, has_scan = false, has_latent = false, has_mlp = false;
     AttnMixer attn;
+    LatentMixer latent;
     ScanMixer scan;
     Linear in, out;
     Linear gate_up, down;
-    int ff_pad = 0;
+    int ff = 0, ff_pad = 0;
+    const float *poly = nullptr;   // set: the MLP is down(poly_norm(up)), gate_up holds up alone (vx_poly_norm)
+    const float *depth_avg = nullptr;  // weights of the embedding output and of every result up to this layer's
 };
 
 struct LayerRun {     // one pass through a layer; every pass has its own cache and state
     int layer = 0;
     bool add_embedding = false;    // the embedding output is added to the stream first
-    void *kv = nullptr;            // paged pool (owned by vh_model::kv)
+    void *kv = nullptr;            // paged pool (owned by vh_model::kv, by the run that writes it)
     void *conv = nullptr;          // [max_seqs][taps - 1][channels]
     float *state = nullptr;        // [max_seqs][channels][pad]
 };
@@ -138,11 +166,27 @@ struct MixActs {      // a step's activations for up to `rows` rows
     int rows = 0;
     float *x = nullptr, *emb = nullptr, *bc = nullptr, *dt = nullptr, *y = nullptr;
     void *h = nullptr, *proj = nullptr, *cat = nullptr, *xc = nullptr, *dtr = nullptr, *act = nullptr;
+    void *qc = nullptr, *qa = nullptr, *lo = nullptr, *z = nullptr;  // query latent; queries and results in the latents' space; up's output
+    float *hist = nullptr, *rot = nullptr;                           // results of all layers; angle tables, one after the other
+};
+
+// The sequences of a step whose keys and values are spelled out: their tokens, block after block, from row 0 on.
+struct MixExpand {
+    int rows = 0, max_blocks = 0;
+    const int32_t *slots = nullptr;    // [rows] pool slot of every token
+    const int32_t *tables = nullptr;   // [n_seqs][max_blocks] blocks of the spelled-out rows
+    const int32_t *table_rows = nullptr;  // [n_seqs] 0, 1, ..
+    void *kv = nullptr;
 };
 
 struct MixModel {
     int act = VX_ACT_BF16;
     float eps = 1e-5f, mult = 1.f;
+    bool post_norm = false;
+    float alpha = 1.f, softcap = 0.f;
+    bool recurrent = false;        // a sequence is more than its blocks
+    int expand_rows = 0;           // the smallest of the layers'
+    std::vector<Rotation> rotations;
     std::vector<MixLayer> layers;
     std::vector<LayerRun> runs;
     Linear head;
@@ -159,8 +203,8 @@ int sync_pool_to_device(vh_model *m);
 int mix_finish(vh_model *m);
 // Embedding of b.rows tokens -> layer runs -> final norm and head of n_want rows (want: device row numbers, NULL = the
 // first n_want) -> logits [n_want, vocab].
-int mix_forward(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, const MixActs &a, const int32_t *want, int n_want,
-                float *logits);
+int mix_forward(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, const MixActs &a, const MixExpand *ex, const int32_t *want,
+                int n_want, float *logits);
 // One mixed step (vh_step) of such a model.
 int mix_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_lens, const int32_t *tokens, int n_want,
              const int32_t *want_rows, float *logits_out, int32_t *argmax_out);

@@ -345,7 +345,7 @@ int forward_decode(vh_model *m, int rows, int max_kv_len) {
     if (m->mix) {
         const vx_ragged b{rows, rows, nullptr, max_kv_len, m->d_cu, m->d_token_pos, m->d_slot_map, m->d_slots, m->d_kv_lens, m->d_tables,
                           c.max_blocks_per_seq, c.block_size};
-        VHC(mix_forward(m, b, m->d_tokens, m->mix->perm, nullptr, rows, m->logits));
+        VHC(mix_forward(m, b, m->d_tokens, m->mix->perm, nullptr, nullptr, rows, m->logits));
         VXC(vx_argmax_rows(m->be, m->logits, rows, c.vocab, m->d_next));
         return VH_OK;
     }
@@ -647,7 +647,7 @@ int vh_pool_truncate_sequence(vh_model *m, int64_t seq_id, int new_len) {  // gp
     std::lock_guard<std::mutex> g(m->pool.mu);
     SeqState *s = find_seq(m, seq_id);
     if (!s || new_len >= s->seq_len) return VH_OK;
-    if (m->mix && new_len > 0) return fail("sequence %lld: its recurrent state cannot go back to length %d", (long long)seq_id, new_len);
+    if (m->mix && m->mix->recurrent && new_len > 0) return fail("sequence %lld: its recurrent state cannot go back to length %d", (long long)seq_id, new_len);
     int keep = 0;
     if (new_len > 0) keep = (new_len - 1) / m->pool.block_size + 1;
     for (int i = keep; i < (int)s->table.size(); i++) m->pool.release_block(s->table[i]);
@@ -665,7 +665,7 @@ int vh_pool_has_sequence(vh_model *m, int64_t seq_id) {
 }
 
 int vh_pool_share_blocks(vh_model *m, int64_t src_id, int64_t dst_id, int num_tokens) {  // gpu_block_pool.go:572-607
-    if (m->mix) return fail("vh_pool_share_blocks: a sequence of this model is more than its blocks (recurrent state)");
+    if (m->mix && m->mix->recurrent) return fail("vh_pool_share_blocks: a sequence of this model is more than its blocks (recurrent state)");
     std::lock_guard<std::mutex> g(m->pool.mu);
     SeqState *src = find_seq(m, src_id);
     if (!src) return fail("source sequence %lld not found", (long long)src_id);
@@ -690,7 +690,9 @@ static void release_fragment(vh_model *m, const Fragment &f) {  // fragment.go:8
 
 int vh_fragment_cache(vh_model *m, const char *name, int64_t seq_id) {  // paged_cache.go:324-343, fragment.go:36-60
     if (!m || !name) return fail("bad arguments");
-    if (m->mix) return fail("vh_fragment_cache: a sequence of this model is more than its blocks (recurrent state)");
+    if (m->mix)
+        return fail(m->mix->recurrent ? "vh_fragment_cache: a sequence of this model is more than its blocks (recurrent state)"
+                                      : "vh_fragment_cache: fragments are moved as LLaMA's K and V rows are, not this model's");
     std::lock_guard<std::mutex> g(m->pool.mu);
     SeqState *s = find_seq(m, seq_id);
     if (!s) return VH_OK;  // paged_cache.go:331-333: an unknown sequence caches nothing
@@ -737,7 +739,9 @@ int vh_fragment_delete(vh_model *m, const char *name) {  // fragment.go:71-79
 int vh_fragment_insert(vh_model *m, int64_t seq_id, const char *name, int insert_pos, int *num_tokens) {
     if (num_tokens) *num_tokens = 0;
     if (!m || !name || insert_pos < 0) return fail("bad arguments");
-    if (m->mix) return fail("vh_fragment_insert: a sequence of this model is more than its blocks (recurrent state)");
+    if (m->mix)
+        return fail(m->mix->recurrent ? "vh_fragment_insert: a sequence of this model is more than its blocks (recurrent state)"
+                                      : "vh_fragment_insert: fragments are moved as LLaMA's K and V rows are, not this model's");
     const vh_config &c = m->cfg;
     if (m->arch.rope_neox || (m->arch.rope_dim != 0 && m->arch.rope_dim != c.head_dim))
         return fail("fragments are rotated as RoPEShift rotates (whole head, pairs 2j and 2j+1): not this model's RoPE");
@@ -828,7 +832,7 @@ int vh_pool_block_table(vh_model *m, int64_t seq_id, int32_t *out, int cap) {
 }
 
 int vh_pool_adopt_blocks(vh_model *m, int64_t seq_id, const int32_t *blocks, int num_blocks, int seq_len) {
-    if (m->mix) return fail("vh_pool_adopt_blocks: a sequence of this model is more than its blocks (recurrent state)");
+    if (m->mix && m->mix->recurrent) return fail("vh_pool_adopt_blocks: a sequence of this model is more than its blocks (recurrent state)");
     std::lock_guard<std::mutex> g(m->pool.mu);
     SeqState *s = find_seq(m, seq_id);
     if (!s) return fail("sequence %lld not found", (long long)seq_id);
@@ -1198,7 +1202,9 @@ int vh_verify_tree(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_
     if (!m || n_seqs < 0 || !seq_ids || !input_tokens || !start_pos || !n_nodes || !num_accepted || !final_tokens)
         return fail("bad arguments");
     if (n_seqs == 0) return VH_OK;
-    if (m->mix) return fail("vh_verify_tree: the recurrent state of a mixer program cannot follow several branches");
+    if (m->mix)
+        return fail(m->mix->recurrent ? "vh_verify_tree: the recurrent state of a mixer program cannot follow several branches"
+                                      : "vh_verify_tree: not for mixer programs");
     VHC(check_ready(m));
     const vh_config &c = m->cfg;
     struct SeqRows { int row0, rows, node0, start, slot, pad; };
