@@ -779,6 +779,93 @@ LOZEDRA_SHAPES = {
     "4096": dict(width=4096, heads=32, kv_heads=8, dim=128, inner=8192, dt_rank=256, ff=14336, layers=4),
 }
 LOZEDRA_VOCAB = 32000
+# The runs of the layer reports: sequences at the end of a real prompt of MIX_CTX tokens each; portions (tokens, position).
+MIX_SEQS, MIX_CTX = 32, 1000
+MIX_PORTIONS = ((512, 0), (512, 3584), (2048, 0))
+MIX_SIZES = dict(pool_blocks=(MIX_SEQS * (MIX_CTX + 200) + 8192) // BLOCK, max_seqs=MIX_SEQS + 1, max_blocks_per_seq=8192 // BLOCK,
+                 max_batch=64)
+
+
+def fill_contexts(mr, vocab, rng):
+    for lo in range(0, MIX_SEQS, 4):
+        mr.step([(s, rng.integers(0, vocab, MIX_CTX).tolist()) for s in range(lo, lo + 4)], [])
+
+
+def write_folder(folder, cfg, shapes, fill):
+    """config.json + model.safetensors; fill(name, shape): the values, or (mean, deviation) of random ones (one random
+    megaword repeated)."""
+    noise = np.random.default_rng(11).standard_normal(1 << 20).astype(np.float32)
+
+    def bf16(a):
+        return ((np.ascontiguousarray(a, dtype=np.float32).view(np.uint32) + 0x8000) >> 16).astype("<u2")
+
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    head, at = {}, 0
+    for name, shape in shapes.items():
+        size = 2 * int(np.prod(shape))
+        head[name] = {"dtype": "BF16", "shape": list(shape), "data_offsets": [at, at + size]}
+        at += size
+    js = json.dumps(head).encode()
+    js += b" " * (-len(js) % 8)
+    words = {}
+    with open(os.path.join(folder, "model.safetensors"), "wb") as f:
+        f.write(len(js).to_bytes(8, "little") + js)
+        for name, shape in shapes.items():
+            v = fill(name, shape)
+            if not isinstance(v, tuple):
+                f.write(bf16(v).tobytes())
+                continue
+            if v not in words:
+                words[v] = bf16(v[0] + v[1] * noise)
+            src, left = words[v], int(np.prod(shape))
+            while left > 0:
+                f.write(src[:min(left, src.size)].tobytes())
+                left -= src.size
+
+
+def load_written(be, write, **kw):
+    """The model that write(folder) puts into a folder, which is gone afterwards."""
+    import shutil
+    import tempfile
+    from vexel_amd.runtime import ModelRuntime
+    folder = tempfile.mkdtemp()
+    try:
+        write(folder)
+        return ModelRuntime.load(be, folder, **kw)
+    finally:
+        shutil.rmtree(folder)
+
+
+def layer_rates(be, label, r, ids, layers, vocab, ctx, steps, portions, use_graph, rng):
+    """Prints a model's decode rate (greedy, ids at context ctx, replayed from a hipGraph) and the rates of single portions."""
+    tok = lambda n: rng.integers(0, vocab, n).tolist()
+    n = len(ids)
+    r.decode_graph(np.array(tok(n), dtype=np.int32), ids, [ctx] * n, 4, use_graph=use_graph)
+    be.sync()
+    t0 = time.perf_counter()
+    r.decode_graph(None, None, None, steps, use_graph=use_graph, batch=n)
+    be.sync()
+    dt = (time.perf_counter() - t0) / steps
+    print("  %-13s decode  %d x ctx %d: %8.0f tok/s  %7.3f ms/step  %6.1f us/layer" %
+          (label, n, ctx, n / dt, dt * 1e3, dt * 1e6 / layers), flush=True)
+    for n, start in portions:
+        best = 1e9
+        for rep in range(4):
+            sid, at = 5000, 0
+            while at < start:
+                m = min(512, start - at)
+                r.step([(sid, tok(m))], [])
+                at += m
+            body = tok(n)
+            be.sync()
+            t0 = time.perf_counter()
+            r.step([(sid, body)], [n - 1])
+            best = min(best, time.perf_counter() - t0) if rep else best   # (the first sizes the workspaces)
+            r.delete_sequence(sid)
+        print("  %-13s prefill %4d tokens at %4d: %8.0f tok/s  %7.3f ms      %6.1f us/layer" %
+              (label, n, start, n / best, best * 1e3, best * 1e6 / layers), flush=True)
 
 
 def write_lozedra(folder, width, heads, kv_heads, dim, inner, dt_rank, ff, layers, state=16, conv=4, bias_rows=32,
@@ -801,94 +888,96 @@ def write_lozedra(folder, width, heads, kv_heads, dim, inner, dt_rank, ff, layer
                        right + "x": (dt_rank + 2 * state, inner), right + "dt": (inner, dt_rank), right + "dt.b": (inner,),
                        right + "A_log": (inner, state), right + "D": (inner,), right + "o": (width, inner),
                        l + "mlp.gate": (ff, width), l + "mlp.up": (ff, width), l + "mlp.down": (width, ff)})
-    rng = np.random.default_rng(11)
-    noise = rng.standard_normal(1 << 20).astype(np.float32)
+    def fill(name, shape):
+        if name.endswith("A_log"):
+            return np.tile(np.log(np.arange(1, state + 1)), shape[0])
+        return (1.0, 0.05) if "norm" in name or name.endswith(".D") else (0.0, 0.02)
 
-    def bf16(a):
-        return ((np.ascontiguousarray(a, dtype=np.float32).view(np.uint32) + 0x8000) >> 16).astype("<u2")
-
-    os.makedirs(folder, exist_ok=True)
-    with open(os.path.join(folder, "config.json"), "w") as f:
-        json.dump(cfg, f)
-    head, at = {}, 0
-    for name, shape in shapes.items():
-        size = 2 * int(np.prod(shape))
-        head[name] = {"dtype": "BF16", "shape": list(shape), "data_offsets": [at, at + size]}
-        at += size
-    js = json.dumps(head).encode()
-    js += b" " * (-len(js) % 8)
-    small, ones = bf16(0.02 * noise), bf16(1.0 + 0.05 * noise)
-    with open(os.path.join(folder, "model.safetensors"), "wb") as f:
-        f.write(len(js).to_bytes(8, "little") + js)
-        for name, shape in shapes.items():
-            n = int(np.prod(shape))
-            if name.endswith("A_log"):
-                f.write(bf16(np.tile(np.log(np.arange(1, state + 1)), shape[0])).tobytes())
-                continue
-            src = ones if "norm" in name or name.endswith(".D") else small
-            left = n
-            while left > 0:
-                f.write(src[:min(left, src.size)].tobytes())
-                left -= src.size
+    write_folder(folder, cfg, shapes, fill)
 
 
 def lozedra_report(be, only=None, use_graph=True):
     """Decode and prefill rates of Lozedra layers at real sizes (random weights) beside the closest model the engine had
     before, a LLaMA layer graph with Q8_0 weights of the same width, heads and feed-forward. Decode: 32 sequences at the
     end of a real 1000-token prompt each, greedy, replayed from a hipGraph. Prefill: one portion of a prompt."""
-    import shutil
-    import tempfile
     from vexel_amd import lib
-    from vexel_amd.runtime import ModelRuntime
-    nseq, ctx, steps = 32, 1000, 32
-    portions = ((512, 0), (512, 3584), (2048, 0))
     rng = np.random.default_rng(2)
     for name, c in LOZEDRA_SHAPES.items():
         if only not in (None, name):
             continue
-        folder = tempfile.mkdtemp()
-        try:
-            write_lozedra(folder, **c)
-            mr = ModelRuntime.load(be, folder, pool_blocks=(nseq * (ctx + 200) + 8192) // BLOCK, max_seqs=nseq + 1,
-                                   max_blocks_per_seq=8192 // BLOCK, max_batch=64)
-        finally:
-            shutil.rmtree(folder)
+        mr = load_written(be, lambda f: write_lozedra(f, **c), **MIX_SIZES)
         llama = dict(num_layers=c["layers"], hidden=c["width"], num_heads=c["heads"], num_kv_heads=c["kv_heads"],
                      head_dim=c["dim"], ffn=c["ff"], vocab=LOZEDRA_VOCAB)
-        lr, lids = build_model(be, [ctx] * nseq, 200, c["layers"], llama, {"*": lib.VX_Q8_0}, spare_tokens=8192)
-        tok = lambda n: rng.integers(0, LOZEDRA_VOCAB, n).tolist()
-        for lo in range(0, nseq, 4):
-            mr.step([(s, tok(ctx)) for s in range(lo, lo + 4)], [])
-        first = np.array(tok(nseq), dtype=np.int32)
+        lr, lids = build_model(be, [MIX_CTX] * MIX_SEQS, 200, c["layers"], llama, {"*": lib.VX_Q8_0}, spare_tokens=8192)
+        fill_contexts(mr, LOZEDRA_VOCAB, rng)
         print("layers of width %s, %d of each model" % (name, c["layers"]))
-        for label, r, ids in (("Lozedra bf16", mr, list(range(nseq))), ("LLaMA Q8_0", lr, lids)):
-            r.decode_graph(first, ids, [ctx] * nseq, 4, use_graph=use_graph)
-            be.sync()
-            t0 = time.perf_counter()
-            r.decode_graph(None, None, None, steps, use_graph=use_graph, batch=nseq)
-            be.sync()
-            dt = (time.perf_counter() - t0) / steps
-            print("  %-13s decode  %d x ctx %d: %8.0f tok/s  %7.3f ms/step  %6.1f us/layer" %
-                  (label, nseq, ctx, nseq / dt, dt * 1e3, dt * 1e6 / c["layers"]), flush=True)
-            for n, start in portions:
-                best = 1e9
-                for rep in range(4):
-                    sid = 5000
-                    at = 0
-                    while at < start:
-                        m = min(512, start - at)
-                        r.step([(sid, tok(m))], [])
-                        at += m
-                    body = tok(n)
-                    be.sync()
-                    t0 = time.perf_counter()
-                    r.step([(sid, body)], [n - 1])
-                    best = min(best, time.perf_counter() - t0) if rep else best   # (the first sizes the workspaces)
-                    r.delete_sequence(sid)
-                print("  %-13s prefill %4d tokens at %4d: %8.0f tok/s  %7.3f ms      %6.1f us/layer" %
-                      (label, n, start, n / best, best * 1e3, best * 1e6 / c["layers"]), flush=True)
+        for label, r, ids in (("Lozedra bf16", mr, list(range(MIX_SEQS))), ("LLaMA Q8_0", lr, lids)):
+            layer_rates(be, label, r, ids, c["layers"], LOZEDRA_VOCAB, MIX_CTX, 32, MIX_PORTIONS, use_graph, rng)
         mr.close()
         lr.close()
+
+
+# Shapes of --tulipel-report, of the widths above; a Lozedra model of the same width, heads and feed-forward stands beside each.
+TULIPEL_SHAPES = {
+    "2048": dict(width=2048, heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=768, ff=5632, layers=6),
+    "4096": dict(width=4096, heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=1536, ff=14336, layers=4),
+}
+
+
+def write_tulipel(folder, width, heads, dim, rot_dim, vdim, kv_rank, q_rank, ff, layers, vocab=LOZEDRA_VOCAB):
+    """A Tulipel model of that shape with random weights: both kinds of layers in turn, every third of the second kind on
+    another layer's latents."""
+    common = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "scale": (dim + rot_dim) ** -0.5}
+    scaling = {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}
+    shapes = {"embed": (vocab, width), "final.norm": (width,), "head": (vocab, width)}
+    entries = []
+    for i in range(layers):
+        l, m = "l%d." % i, "l%d.mix." % i
+        mixer = dict(common)
+        qd = heads * (dim + rot_dim)
+        if i % 2 == 0:
+            mixer.update(q_rank=q_rank, rot={"base": 10000.0, "dims": rot_dim})
+            shapes.update({m + "dq": (q_rank, width), m + "dq.norm": (q_rank,), m + "uq": (qd, q_rank)})
+        else:
+            mixer.update(rot={"base": 10000.0, "dims": rot_dim, "scaling": scaling})
+            shapes[m + "q"] = (qd, width)
+            if i % 6 == 3:
+                mixer["kv_from"] = i - 2
+        if "kv_from" not in mixer:
+            shapes.update({m + "dkv": (kv_rank + rot_dim, width), m + "dkv.norm": (kv_rank,)})
+        shapes.update({m + "uk": (heads * dim, kv_rank), m + "uv": (heads * vdim, kv_rank), m + "sink": (heads,), m + "o": (width, heads * vdim),
+                       l + "norm1": (width,), l + "norm2": (width,), l + "mlp.up": (ff, width), l + "mlp.down": (width, ff),
+                       l + "mlp.act": (4,), l + "dwa": (i + 2,)})
+        entries.append({"type": "latent_attention_2" if i % 2 else "latent_attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": ff}})
+    cfg = {"architecture": "Tulipel", "layers": entries, "norm": {"eps": 1e-5}, "postln_alpha": 2.0, "logit_softcap": 30.0, "vocab": vocab,
+           "width": width}
+
+    def fill(name, shape):
+        if name.endswith(("dq.norm", "dkv.norm")):
+            return (1.0, 0.05)
+        if name.endswith("dwa"):
+            return np.array([0.2] * (shape[0] - 1) + [0.8])
+        if name.endswith("mlp.act"):
+            return np.array([0.6, 0.3, 0.1, 0.05])
+        return (0.0, 0.05) if "norm" in name else (0.0, 0.02)
+
+    write_folder(folder, cfg, shapes, fill)
+
+
+def tulipel_report(be, only=None, use_graph=True):
+    """Decode and prefill rates of Tulipel layers at real sizes (random weights) beside Lozedra layers of the same width, heads
+    and feed-forward, the closest model: the same linear maps, the same kind of step. Runs as for --lozedra-report."""
+    rng = np.random.default_rng(2)
+    for name, c in TULIPEL_SHAPES.items():
+        if only not in (None, name):
+            continue
+        print("layers of width %s, %d of each model" % (name, c["layers"]))
+        loz = dict(LOZEDRA_SHAPES[name], layers=c["layers"])
+        for label, write in (("Tulipel bf16", lambda f: write_tulipel(f, **c)), ("Lozedra bf16", lambda f: write_lozedra(f, **loz))):
+            mr = load_written(be, write, **MIX_SIZES)
+            fill_contexts(mr, LOZEDRA_VOCAB, rng)
+            layer_rates(be, label, mr, list(range(MIX_SEQS)), c["layers"], LOZEDRA_VOCAB, MIX_CTX, 32, MIX_PORTIONS, use_graph, rng)
+            mr.close()
 
 
 def main():
@@ -920,6 +1009,9 @@ def main():
     ap.add_argument("--lozedra-report", nargs="?", const="all", choices=["all"] + list(LOZEDRA_SHAPES),
                     help="decode and prefill rates of Lozedra layers at real sizes beside LLaMA Q8_0 layers of the same "
                          "sizes, then exit")
+    ap.add_argument("--tulipel-report", nargs="?", const="all", choices=["all"] + list(TULIPEL_SHAPES),
+                    help="decode and prefill rates of Tulipel layers at real sizes beside Lozedra layers of the same sizes, "
+                         "then exit")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU: this build has no multi-GPU path (run with --gpus 1)", file=sys.stderr)
@@ -943,6 +1035,9 @@ def main():
         return
     if args.lozedra_report:
         lozedra_report(be, None if args.lozedra_report == "all" else args.lozedra_report, use_graph=not args.no_graph)
+        return
+    if args.tulipel_report:
+        tulipel_report(be, None if args.tulipel_report == "all" else args.tulipel_report, use_graph=not args.no_graph)
         return
     ctx = ragged_contexts(n=args.seqs) if args.seqs != BATCH else ragged_contexts()
     nseq = len(ctx)

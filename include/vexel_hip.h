@@ -500,12 +500,13 @@ enum {
                           float32 partial sums over slices of the inputs, out[s][r * ldo + c], slice after slice */
     VX_LIN_SWIGLU = 1, /* row tiles alternate gate, up: out = silu(gate) * up, 16 columns per pair of tiles */
     VX_LIN_KV = 2,     /* PLAIN in the activation type, but columns [k_col, k_col + kv_heads * k_dim) and [v_col, ..) go
-                          to the paged pool at slot_mapping[r] (layout: vx_kv_block_elems) */
+                          to the paged pool at slot_mapping[r] (layout: vx_kv_block_elems); v_col = n: no V */
     VX_LIN_SPLIT = 3,  /* columns < split to out (activation type), the others to out2[r * ldo2 + c - split] (float32) */
     VX_LIN_SOFTPLUS = 4, /* float32 out = log(1 + exp(y + bias[c])) */
-    VX_LIN_ROTARY = 5  /* columns < split to out (activation type) in heads of rot_stride columns, whose columns rot_first ..
+    VX_LIN_ROTARY = 5, /* columns < split to out (activation type) in heads of rot_stride columns, whose columns rot_first ..
                           rot_first + 2 * rot_pairs - 1 are turned in neighbouring pairs by rot_tab (vx_rotary_table); the
                           others (split = n: none) to out2 as with SPLIT */
+    VX_LIN_V = 6       /* every column is V of the pool (v_col 0), stored as with KV, four neighbouring slots at a time */
 };
 typedef struct vx_linear_out {
     int kind, out_f32, ldo, cols, slices;
@@ -522,6 +523,7 @@ typedef struct vx_linear_out {
                                     the activations from column g * a_group on and writes from column g * out_group on */
     int rot_stride, rot_first, rot_pairs;
     const float *rot_tab;
+    int k_used;                  /* > 0: a K head's k_used first elements are what the map makes (kv_heads * k_used columns) */
 } vx_linear_out;
 /* out = a [rows, k] * W^T for a packed matrix [n, k] (padded sizes); a has lda >= k columns of the activation type, zero
  * where k was padded, rows 16-byte aligned. vx_linear_slices: into how many slices a PLAIN float32 result is best cut
@@ -618,7 +620,7 @@ typedef struct vx_latent_attn_args {
 int vx_attn_latent(vx_backend *be, int act, const vx_ragged *b, const vx_latent_attn_args *p);
 /* 1 when the matrix-core kernel takes the geometry, 0 when vx_attn_latent uses the plain one. */
 int vx_attn_latent_fast(int act, int block_size, int rank, int rot_dim);
-/* The rotated key part of row a_rows[r] of a latent pool into columns first .. of every head of row r of a K pool (layout:
+/* The rotated key part (rot_dim columns, or more with the zeros behind them) of row a_rows[r] of a latent pool into columns first .. of every head of row r of a K pool (layout:
  * vx_kv_block_elems; the slot of row r is r). */
 int vx_latent_spread(vx_backend *be, int act, const void *latent_pool, int rank, int rot_dim, const int32_t *a_rows, int rows, void *pool,
                      int kv_heads, int k_dim, int v_dim, int block_size, int first);
@@ -648,9 +650,11 @@ typedef struct vx_post_norm_args {
 int vx_post_norm(vx_backend *be, int act, const vx_post_norm_args *p);
 
 /* Polynomial activation normed over the row, in float32: out = coef[0] * N(z) + coef[1] * N(z^2) + coef[2] * N(z^3) + coef[3] with
- * N(u) = u / sqrt(mean over the row's cols columns of u^2 + eps), powers element by element. z, out: activation type;
- * columns cols .. ldo - 1 of out become zero. coef: device float32[4]. */
-int vx_poly_norm(vx_backend *be, int act, const void *z, int ldz, int rows, int cols, const float *coef, float eps, void *out, int ldo);
+ * N(u) = u / sqrt(mean over the row's cols columns of u^2 + eps), powers element by element. out: activation type; its columns
+ * cols .. ldo - 1 become zero. z: activation type (z_slices 0), or float32 in so many slices, z_stride floats from one to the
+ * next, that are added up. coef: device float32[4]. */
+int vx_poly_norm(vx_backend *be, int act, const void *z, int ldz, int z_slices, int64_t z_stride, int rows, int cols, const float *coef, float eps,
+                 void *out, int ldo);
 
 /* Causal depthwise convolution with SiLU over a mixed batch: out[r][c] = silu(b[c] + sum_t w[t][c] * x[position - (taps
  * - 1 - t)][c]), positions before the sequence's start count as zero, positions before this step's rows come from

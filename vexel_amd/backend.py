@@ -37,7 +37,7 @@ class VxRagged(C.Structure):
 class VxLinearOut(C.Structure):
     _fields_ = _fields("int kind out_f32 ldo cols slices; ptr out out2; int split ldo2; ptr bias; int k_col v_col kv_heads "
                        "k_dim v_dim block_size; ptr pool slot_mapping a_rows; float softcap; int groups a_group out_group "
-                       "rot_stride rot_first rot_pairs; ptr rot_tab")
+                       "rot_stride rot_first rot_pairs; ptr rot_tab; int k_used")
 
 
 class VxResidualNormArgs(C.Structure):
@@ -478,8 +478,8 @@ class HipBackend:
     def post_norm(self, act, args):
         self.call("vx_post_norm", act, C.byref(args))
 
-    def poly_norm(self, act, z, ldz, rows, cols, coef, eps, out, ldo):
-        self.call("vx_poly_norm", act, z, ldz, rows, cols, coef, eps, out, ldo)
+    def poly_norm(self, act, z, ldz, rows, cols, coef, eps, out, ldo, z_slices=0, z_stride=0):
+        self.call("vx_poly_norm", act, z, ldz, z_slices, z_stride, rows, cols, coef, eps, out, ldo)
 
     def conv_silu(self, act, batch, args):
         self.call("vx_conv_silu", act, C.byref(batch), C.byref(args))

@@ -292,6 +292,10 @@ __global__ void embedding_kernel(const int32_t *ids, const float *table, float *
     if (id < 0 || id >= vocab) return;  // row left untouched
     const float *src = table + (size_t)id * dim;
     float *dst = out + (size_t)t * dim;
+    if (dim % 4 == 0 && ((uintptr_t)table | (uintptr_t)out) % 16 == 0) {
+        for (int j = threadIdx.x; j < dim / 4; j += blockDim.x) ((float4 *)dst)[j] = ((const float4 *)src)[j];
+        return;
+    }
     for (int j = threadIdx.x; j < dim; j += blockDim.x) dst[j] = src[j];
 }
 

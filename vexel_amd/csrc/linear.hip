@@ -26,16 +26,20 @@ struct LinArgs {
     vx_linear_out o;
 };
 
-__device__ __forceinline__ size_t kv_elem_k(const vx_linear_out &o, int slot, int g, int d) {
-    const int kp = (o.k_dim + 7) & ~7;
-    const size_t blk = (size_t)o.kv_heads * o.block_size * (kp + o.v_dim);
-    return (size_t)(slot / o.block_size) * blk + ((size_t)g * o.block_size + slot % o.block_size) * kp + d;
+// Where K and V elements lie in the pool: a part that depends on the slot and one that depends on the column.
+struct KvSlot {
+    size_t k, v;
+};
+__device__ __forceinline__ KvSlot kv_slot(const vx_linear_out &o, int row) {
+    const int slot = o.slot_mapping ? o.slot_mapping[row] : row, kp = (o.k_dim + 7) & ~7;
+    const int blk = slot / o.block_size, in = slot - blk * o.block_size;
+    const size_t base = (size_t)blk * o.kv_heads * o.block_size * (kp + o.v_dim);
+    return {base + (size_t)in * kp, base + (size_t)o.kv_heads * o.block_size * kp + in};
 }
-__device__ __forceinline__ size_t kv_elem_v(const vx_linear_out &o, int slot, int g, int d) {
-    const int kp = (o.k_dim + 7) & ~7;
-    const size_t blk = (size_t)o.kv_heads * o.block_size * (kp + o.v_dim);
-    return (size_t)(slot / o.block_size) * blk + (size_t)o.kv_heads * o.block_size * kp +
-           ((size_t)g * o.v_dim + d) * o.block_size + slot % o.block_size;
+__device__ __forceinline__ int k_used(const vx_linear_out &o) { return o.k_used > 0 ? o.k_used : o.k_dim; }
+__device__ __forceinline__ int kv_col_k(const vx_linear_out &o, int ck) {
+    const int kp = (o.k_dim + 7) & ~7, g = ck / k_used(o);
+    return g * o.block_size * kp + ck - g * k_used(o);
 }
 
 // Where row r of the activations lies.
@@ -77,6 +81,29 @@ __device__ __forceinline__ void take_group(LinArgs &p) {
     p.o.out = p.o.out_f32 ? (void *)((float *)p.o.out + g * p.o.out_group) : (void *)((T *)p.o.out + g * p.o.out_group);
 }
 
+// Columns c .. c + 3 of a map with K and V; at: the row's slot, col_k: kv_col_k of the first column where that is K.
+template <typename T, int KIND>
+__device__ __forceinline__ void emit_kv(const LinArgs &p, KvSlot at, int row, int c, int col_k, f32x4 v) {
+    const vx_linear_out &o = p.o;
+    const int kw = o.kv_heads * k_used(o), vw = o.kv_heads * o.v_dim, ck = c - o.k_col, cv = c - o.v_col;
+    T *pool = (T *)o.pool;
+    if (KIND == VX_LIN_KV && ck >= 0 && ck < kw) {
+        if ((k_used(o) & 3) == 0 && (o.k_dim & 3) == 0) {
+            store4(pool + at.k + col_k, v);
+        } else {
+#pragma unroll
+            for (int r = 0; r < 4; r++)
+                if (ck + r < kw) pool[at.k + kv_col_k(o, ck + r)] = (T)v[r];
+        }
+    } else if (cv >= 0 && cv < vw) {
+#pragma unroll
+        for (int r = 0; r < 4; r++)
+            if (cv + r < vw) pool[at.v + (size_t)(cv + r) * o.block_size] = (T)v[r];
+    } else if (KIND == VX_LIN_KV) {
+        put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
+    }
+}
+
 // Columns c .. c + 3 of activation row `row`.
 template <typename T, int KIND>
 __device__ __forceinline__ void emit(const LinArgs &p, int slice, int row, int c, f32x4 v) {
@@ -110,29 +137,24 @@ __device__ __forceinline__ void emit(const LinArgs &p, int slice, int row, int c
             u[r] = softplus_f(v[r] + (c + r < o.cols ? o.bias[c + r] : 0.f));
         }
         put4((float *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, u);
-    } else {  // VX_LIN_KV: K and V columns leave for the pool (segments start at multiples of 16 columns)
-        const auto slot_of = [&](int r) { return o.slot_mapping ? o.slot_mapping[r] : r; };
-        const int kw = o.kv_heads * o.k_dim, vw = o.kv_heads * o.v_dim;
-        const int ck = c - o.k_col, cv = c - o.v_col;
-        if (ck >= 0 && ck < kw) {
-            const int slot = slot_of(row);
-            T *pool = (T *)o.pool;
-            if ((o.k_dim & 3) == 0) {
-                store4(pool + kv_elem_k(o, slot, ck / o.k_dim, ck % o.k_dim), v);
-            } else {
+    } else {  // VX_LIN_KV, VX_LIN_V: K and V columns leave for the pool (segments start at multiples of 16 columns)
+        emit_kv<T, KIND>(p, kv_slot(o, row), row, c, KIND == VX_LIN_KV && c >= o.k_col ? kv_col_k(o, c - o.k_col) : 0, v);
+    }
+}
+
+// VX_LIN_V, from a tile whose operands were exchanged: rows `row` .. row + 3, column c. Neighbouring slots of a block are
+// neighbours in V as it lies in the pool.
+template <typename T>
+__device__ __forceinline__ void emit_v(const LinArgs &p, const KvSlot *at, bool together, int row, int c, f32x4 v) {
+    const vx_linear_out &o = p.o;
+    if (row >= p.rows || c >= o.kv_heads * o.v_dim) return;
+    T *pool = (T *)o.pool + (size_t)c * o.block_size;
+    if (together) {
+        store4(pool + at[0].v, v);
+    } else {
 #pragma unroll
-                for (int r = 0; r < 4; r++)
-                    if (ck + r < kw) pool[kv_elem_k(o, slot, (ck + r) / o.k_dim, (ck + r) % o.k_dim)] = (T)v[r];
-            }
-        } else if (cv >= 0 && cv < vw) {
-            const int slot = slot_of(row);
-            T *pool = (T *)o.pool;
-#pragma unroll
-            for (int r = 0; r < 4; r++)
-                if (cv + r < vw) pool[kv_elem_v(o, slot, (cv + r) / o.v_dim, (cv + r) % o.v_dim)] = (T)v[r];
-        } else {
-            put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
-        }
+        for (int r = 0; r < 4; r++)
+            if (row + r < p.rows) pool[at[r].v] = (T)v[r];
     }
 }
 
@@ -255,6 +277,8 @@ __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_til
 #pragma unroll
             for (int t = 0; t < NI; t++) wf[h][t] = *(const bf16x8 *)(w[t] + (size_t)(kt * 2 + h) * 512);
     };
+    // V columns alone: the operands are exchanged, so that a lane ends with four rows of one column
+    constexpr bool EXCHANGED = KIND == VX_LIN_V;
     f32x4 acc[NI][MI];
 #pragma unroll
     for (int t = 0; t < NI; t++)
@@ -293,10 +317,42 @@ __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_til
 #pragma unroll
             for (int t = 0; t < NI; t++)
 #pragma unroll
-                for (int m = 0; m < MI; m++) acc[t][m] = mma(cur[h][t], af[m], acc[t][m]);
+                for (int m = 0; m < MI; m++) acc[t][m] = EXCHANGED ? mma_act(af[m], cur[h][t], acc[t][m]) : mma(cur[h][t], af[m], acc[t][m]);
         }
     }
     const int q4 = (lane >> 4) * 4;
+    if constexpr (EXCHANGED) {
+#pragma unroll
+        for (int m = 0; m < MI; m++) {
+            const int row = m0 + wm + m * 16 + q4;
+            KvSlot at[4];
+#pragma unroll
+            for (int r = 0; r < 4; r++) at[r] = kv_slot(p.o, min(row + r, p.rows - 1));
+            const bool together = row + 4 <= p.rows && (p.o.block_size & 3) == 0 && (at[0].v & 3) == 0 && at[1].v == at[0].v + 1 && at[2].v == at[0].v + 2 &&
+                                  at[3].v == at[0].v + 3;
+#pragma unroll
+            for (int t = 0; t < NI; t++)
+                if (tile0 + wn + t < n_tiles) emit_v<T>(p, at, together, row, (tile0 + wn + t) * 16 + (lane & 15), acc[t][m]);
+        }
+        return;
+    } else if constexpr (KIND == VX_LIN_KV) {
+        int col_k[NI];
+#pragma unroll
+        for (int t = 0; t < NI; t++) {
+            const int ck = (tile0 + wn + t) * 16 + q4 - p.o.k_col;
+            col_k[t] = ck >= 0 ? kv_col_k(p.o, ck) : 0;
+        }
+#pragma unroll
+        for (int m = 0; m < MI; m++) {
+            const int row = m0 + wm + m * 16 + (lane & 15);
+            if (row >= p.rows) continue;
+            const KvSlot at = kv_slot(p.o, row);
+#pragma unroll
+            for (int t = 0; t < NI; t++)
+                if (tile0 + wn + t < n_tiles) emit_kv<T, KIND>(p, at, row, (tile0 + wn + t) * 16 + q4, col_k[t], acc[t][m]);
+        }
+        return;
+    }
 #pragma unroll
     for (int m = 0; m < MI; m++) {
         const int row = m0 + wm + m * 16 + (lane & 15);
@@ -388,7 +444,7 @@ int pick_slices(int n, int k, int rows) {
     int64_t wgs;
     int want, least;
     if (rows <= 64) {
-        wgs = n / 16, want = wgs >= 192 ? 512 : 192, least = 16;  // (a wave's four steps of 32 inputs, eight waves)
+        wgs = n / 16, want = 1024, least = 4;  // (as many workgroups as the chip holds; a wave's step of 32 inputs)
         if (wgs >= want) return 1;
     } else {
         wgs = (int64_t)ceil_div(rows, 128) * ceil_div(n, 128), want = 512, least = 12;
@@ -434,6 +490,7 @@ int dispatch(vx_backend *be, const LinArgs &p, int slices) {
         case VX_LIN_KV: return launch<T, VX_LIN_KV>(be, p, slices);
         case VX_LIN_SPLIT: return launch<T, VX_LIN_SPLIT>(be, p, slices);
         case VX_LIN_ROTARY: return launch<T, VX_LIN_ROTARY>(be, p, slices);
+        case VX_LIN_V: return launch<T, VX_LIN_V>(be, p, slices);
         default: return launch<T, VX_LIN_SOFTPLUS>(be, p, slices);
     }
 }
@@ -507,7 +564,7 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
     VX_REQUIRE(n >= 16 && n % 16 == 0 && k >= 64 && k % 64 == 0 && lda >= k && lda % 8 == 0 && (uintptr_t)a % 16 == 0 &&
                    (uintptr_t)w % 16 == 0 && (uintptr_t)o->out % 16 == 0,
                "vx_linear: sizes or alignment (n %d, k %d, lda %d)", n, k, lda);
-    VX_REQUIRE(o->kind >= VX_LIN_PLAIN && o->kind <= VX_LIN_ROTARY, "vx_linear: unknown kind %d", o->kind);
+    VX_REQUIRE(o->kind >= VX_LIN_PLAIN && o->kind <= VX_LIN_V, "vx_linear: unknown kind %d", o->kind);
     VX_REQUIRE(o->cols >= 1 && o->ldo >= o->cols, "vx_linear: %d columns in rows of %d", o->cols, o->ldo);
     const int slices = o->slices > 1 ? o->slices : 1;
     VX_REQUIRE(slices == 1 || (o->kind == VX_LIN_PLAIN && o->out_f32 && slices <= 64), "vx_linear: slices need a plain float32 result");
@@ -528,11 +585,13 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
         VX_REQUIRE(o->cols <= n, "vx_linear: %d columns of %d", o->cols, n);
     }
     if (o->kind == VX_LIN_SOFTPLUS) VX_REQUIRE(o->bias != nullptr, "vx_linear: null bias");
-    if (o->kind == VX_LIN_KV)
+    if (o->kind == VX_LIN_KV || o->kind == VX_LIN_V)
         VX_REQUIRE(o->pool && o->kv_heads >= 1 && o->k_dim >= 1 && o->v_dim >= 1 && o->block_size >= 1 &&
                        o->k_col % 16 == 0 && o->v_col % 16 == 0 && o->k_col >= 0 && o->v_col >= 0 &&
-                       o->k_col + o->kv_heads * o->k_dim <= n && o->v_col + o->kv_heads * o->v_dim <= n,
+                       (o->kind == VX_LIN_V || (o->k_used >= 0 && o->k_used <= o->k_dim && o->k_col + o->kv_heads * (o->k_used > 0 ? o->k_used : o->k_dim) <= n)) &&
+                       ((o->kind == VX_LIN_KV && o->v_col == n) || o->v_col + o->kv_heads * o->v_dim <= n),
                    "vx_linear: bad K/V columns");
+    if (o->kind == VX_LIN_V) VX_REQUIRE(o->v_col == 0 && o->kv_heads * o->v_dim + 15 >= n, "vx_linear: columns beside V");
     VX_REQUIRE(o->softcap == 0.f || (o->softcap > 0.f && o->kind == VX_LIN_PLAIN && slices == 1), "vx_linear: a cap needs a plain whole result");
     LinArgs p{a, w, lda, n, k, rows, *o};
     if (o->groups > 1) {
@@ -545,7 +604,7 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
     }
     if (o->kind != VX_LIN_ROTARY) p.o.rot_tab = nullptr;
     if (o->kind == VX_LIN_SPLIT || o->kind == VX_LIN_ROTARY) {  // (narrow and deep as a rule) in slices, added up by a kernel of their own
-        const int cut = pick_slices(n, k, rows);
+        const int cut = k >= 2048 ? pick_slices(n, k, rows) : 1;  // (a short map is over before the second launch pays)
         if (cut > 1) {
             const size_t bytes = (size_t)cut * rows * n * 4;
             rc = ensure_ws(be, &be->part_ws, &be->part_ws_bytes, bytes, "partial sums");

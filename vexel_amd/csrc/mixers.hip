@@ -248,12 +248,15 @@ __global__ void __launch_bounds__(1024) post_norm_kernel(vx_post_norm_args p) {
 }
 
 // A row per workgroup; NV > 0: cols is a multiple of 8 and at most 8 * NV * blockDim.x, rows aligned: they live in registers.
-template <typename T, int NV>
-__global__ void __launch_bounds__(1024) poly_norm_kernel(const T *z, int ldz, int cols, const float *coef, float eps, T *out, int ldo) {
+// Z: bfloat16 or float32, the latter in `slices` parts that are added up.
+template <typename T, typename Z, int NV>
+__global__ void __launch_bounds__(1024) poly_norm_kernel(const Z *z, int ldz, int slices, int64_t stride, int cols, const float *coef, float eps, T *out,
+                                                         int ldo) {
     typedef typename Vec8<T>::type V8;
+    typedef typename Vec8<Z>::type Z8;
     __shared__ float sm[3][16];
     const int tid = threadIdx.x, nt = blockDim.x, waves = nt >> 6;
-    const T *zr = z + (size_t)blockIdx.x * ldz;
+    const Z *zr = z + (size_t)blockIdx.x * ldz;
     T *o = out + (size_t)blockIdx.x * ldo;
     float s[3] = {0.f, 0.f, 0.f};
     const auto add = [&](float t) {
@@ -262,12 +265,21 @@ __global__ void __launch_bounds__(1024) poly_norm_kernel(const T *z, int ldz, in
         s[1] = fmaf(q, q, s[1]);
         s[2] = fmaf(q * q, q, s[2]);
     };
-    V8 v[NV > 0 ? NV : 1];
+    const auto at = [&](int c) {
+        float t = (float)zr[c];
+        if constexpr (sizeof(Z) == 4)
+            for (int k = 1; k < slices; k++) t += zr[(size_t)k * stride + c];
+        return t;
+    };
+    Z8 v[NV > 0 ? NV : 1];
     if constexpr (NV > 0) {
 #pragma unroll
         for (int i = 0; i < NV; i++) {
             const int c = (tid + i * nt) * 8;
-            if (c < cols) v[i] = *(const V8 *)(zr + c);
+            if (c < cols) v[i] = *(const Z8 *)(zr + c);
+            if constexpr (sizeof(Z) == 4)
+                for (int k = 1; k < slices; k++)
+                    if (c < cols) v[i] += *(const Z8 *)(zr + (size_t)k * stride + c);
         }
 #pragma unroll
         for (int i = 0; i < NV; i++)
@@ -275,7 +287,7 @@ __global__ void __launch_bounds__(1024) poly_norm_kernel(const T *z, int ldz, in
 #pragma unroll
                 for (int e = 0; e < 8; e++) add((float)v[i][e]);
     } else {
-        for (int c = tid; c < cols; c += nt) add((float)zr[c]);
+        for (int c = tid; c < cols; c += nt) add(at(c));
     }
     float f[3];
 #pragma unroll
@@ -305,7 +317,7 @@ __global__ void __launch_bounds__(1024) poly_norm_kernel(const T *z, int ldz, in
             }
         }
     } else {
-        for (int c = tid; c < cols; c += nt) o[c] = (T)value((float)zr[c]);
+        for (int c = tid; c < cols; c += nt) o[c] = (T)value(at(c));
     }
     for (int c = cols + tid; c < ldo; c += nt) o[c] = (T)0.f;
 }
@@ -590,22 +602,22 @@ void launch_post_norm(vx_backend *be, const vx_post_norm_args &p) {
         post_norm_kernel<T, 8><<<p.rows, threads, 0, be->stream>>>(p);
 }
 
-template <typename T>
-void launch_poly_norm(vx_backend *be, const T *z, int ldz, int rows, int cols, const float *coef, float eps, T *out, int ldo) {
-    const bool vec = cols % 8 == 0 && ldz % 8 == 0 && ldo % 8 == 0 && (uintptr_t)z % 16 == 0 && (uintptr_t)out % 16 == 0;
+template <typename T, typename Z>
+void launch_poly_norm(vx_backend *be, const Z *z, int ldz, int slices, int64_t stride, int rows, int cols, const float *coef, float eps, T *out, int ldo) {
+    const bool vec = cols % 8 == 0 && ldz % 8 == 0 && ldo % 8 == 0 && (slices == 1 || stride % 8 == 0) && (uintptr_t)z % 16 == 0 && (uintptr_t)out % 16 == 0;
     const int n8 = cols / 8;
     int threads = rows <= 256 ? 1024 : 256;
     while (threads > 64 && threads / 2 >= n8) threads /= 2;
     while (threads < 1024 && n8 > 4 * threads) threads *= 2;
     const int nv = ceil_div(n8, threads);
     if (!vec || nv > 4)
-        poly_norm_kernel<T, 0><<<rows, 1024, 0, be->stream>>>(z, ldz, cols, coef, eps, out, ldo);
+        poly_norm_kernel<T, Z, 0><<<rows, 1024, 0, be->stream>>>(z, ldz, slices, stride, cols, coef, eps, out, ldo);
     else if (nv <= 1)
-        poly_norm_kernel<T, 1><<<rows, threads, 0, be->stream>>>(z, ldz, cols, coef, eps, out, ldo);
+        poly_norm_kernel<T, Z, 1><<<rows, threads, 0, be->stream>>>(z, ldz, slices, stride, cols, coef, eps, out, ldo);
     else if (nv <= 2)
-        poly_norm_kernel<T, 2><<<rows, threads, 0, be->stream>>>(z, ldz, cols, coef, eps, out, ldo);
+        poly_norm_kernel<T, Z, 2><<<rows, threads, 0, be->stream>>>(z, ldz, slices, stride, cols, coef, eps, out, ldo);
     else
-        poly_norm_kernel<T, 4><<<rows, threads, 0, be->stream>>>(z, ldz, cols, coef, eps, out, ldo);
+        poly_norm_kernel<T, Z, 4><<<rows, threads, 0, be->stream>>>(z, ldz, slices, stride, cols, coef, eps, out, ldo);
 }
 
 }  // namespace
@@ -629,15 +641,18 @@ int vx_post_norm(vx_backend *be, int act, const vx_post_norm_args *a) {
     return VX_OK;
 }
 
-int vx_poly_norm(vx_backend *be, int act, const void *z, int ldz, int rows, int cols, const float *coef, float eps, void *out, int ldo) {
+int vx_poly_norm(vx_backend *be, int act, const void *z, int ldz, int z_slices, int64_t z_stride, int rows, int cols, const float *coef, float eps,
+                 void *out, int ldo) {
     int rc = enter(be);
     if (rc) return rc;
     VX_REQUIRE(act == VX_ACT_F32 || act == VX_ACT_BF16, "vx_poly_norm: unknown activation type %d", act);
-    VX_REQUIRE(z && coef && out && z != out && rows >= 1 && cols >= 1 && ldz >= cols && ldo >= cols, "vx_poly_norm: bad arguments");
-    if (act == VX_ACT_BF16)
-        launch_poly_norm<bf16>(be, (const bf16 *)z, ldz, rows, cols, coef, eps, (bf16 *)out, ldo);
+    VX_REQUIRE(z && coef && out && z != out && rows >= 1 && cols >= 1 && ldz >= cols && ldo >= cols && z_slices >= 0, "vx_poly_norm: bad arguments");
+    if (act == VX_ACT_F32)
+        launch_poly_norm<float, float>(be, (const float *)z, ldz, z_slices > 1 ? z_slices : 1, z_stride, rows, cols, coef, eps, (float *)out, ldo);
+    else if (z_slices > 0)
+        launch_poly_norm<bf16, float>(be, (const float *)z, ldz, z_slices, z_stride, rows, cols, coef, eps, (bf16 *)out, ldo);
     else
-        launch_poly_norm<float>(be, (const float *)z, ldz, rows, cols, coef, eps, (float *)out, ldo);
+        launch_poly_norm<bf16, bf16>(be, (const bf16 *)z, ldz, 1, 0, rows, cols, coef, eps, (bf16 *)out, ldo);
     VX_CHECK_LAUNCH();
     return VX_OK;
 }

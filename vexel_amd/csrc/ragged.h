@@ -29,6 +29,13 @@ __device__ __forceinline__ f32x4 mma(bf16x8 a, f32x8 b, f32x4 acc) {  // bfloat1
     for (int j = 0; j < 8; j++) acc = __builtin_amdgcn_mfma_f32_16x16x4f32((float)a[j], b[j], acc, 0, 0, 0);
     return acc;
 }
+// The same product with the activations as A and the weights as B.
+__device__ __forceinline__ f32x4 mma_act(bf16x8 a, bf16x8 b, f32x4 acc) { return mma(a, b, acc); }
+__device__ __forceinline__ f32x4 mma_act(f32x8 a, bf16x8 b, f32x4 acc) {
+#pragma unroll
+    for (int j = 0; j < 8; j++) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], (float)b[j], acc, 0, 0, 0);
+    return acc;
+}
 
 // The hardware's exponential and reciprocal are good to a unit in the last place; the exponent's own rounding adds |z| times
 // that.

@@ -718,12 +718,13 @@ int build_tulipel(Builder &b, const Json &config, MixModel *x, vh_config *cfg) {
         }
         VHC(b.vec(mix + "sink", s.heads, &t.sink));
         // out of the latents: keys of all heads, then values; into them: per head, the keys' matrix transposed
-        VHC(b.packed(&t.expand, q_cols + s.heads * t.v_pad, t.rank_pad));
-        VHC(b.pack_rows(mix + "uk", s.heads * s.dim, s.rank, q_cols, t.expand, 0, [&](int r) {
-            const int h = r / t.head_cols, d = r % t.head_cols;
+        const int k_cols = s.heads * t.dim_pad;
+        VHC(b.packed(&t.expand, k_cols + s.heads * t.v_pad, t.rank_pad));
+        VHC(b.pack_rows(mix + "uk", s.heads * s.dim, s.rank, k_cols, t.expand, 0, [&](int r) {
+            const int h = r / t.dim_pad, d = r % t.dim_pad;
             return d < s.dim ? h * s.dim + d : -1;
         }));
-        VHC(b.pack_rows(mix + "uv", s.heads * s.vdim, s.rank, s.heads * t.v_pad, t.expand, q_cols, [&](int r) {
+        VHC(b.pack_rows(mix + "uv", s.heads * s.vdim, s.rank, s.heads * t.v_pad, t.expand, k_cols, [&](int r) {
             const int h = r / t.v_pad, d = r % t.v_pad;
             return d < s.vdim ? h * s.vdim + d : -1;
         }));

@@ -25,7 +25,7 @@ size_t esize(const MixModel &x) { return x.act == VX_ACT_F32 ? 4 : 2; }
 
 struct Widths {
     int width_pad = 0, in = 0, out = 0, xc = 0, dtr = 0, bc = 0, dt = 0, act = 0;
-    int qc = 0, qa = 0, z = 0, rot = 0;
+    int qc = 0, qa = 0, rot = 0;
 };
 
 Widths widths(const vh_model *m) {
@@ -45,10 +45,22 @@ Widths widths(const vh_model *m) {
             w.qc = std::max(w.qc, l.latent.q_up.k);
             w.qa = std::max(w.qa, l.latent.heads * l.latent.rank_pad);
         }
-        if (l.poly) w.z = std::max(w.z, l.ff_pad);
     }
     for (const Rotation &r : m->mix->rotations) w.rot += 2 * (int)r.freqs.size();
     return w;
+}
+
+// bytes of the up projection's output in front of vx_poly_norm, which may come as float32 slices
+size_t up_bytes(const vh_model *m, int rows, bool up_to) {
+    size_t most = 1;
+    for (const MixLayer &l : m->mix->layers) {
+        if (!l.poly) continue;
+        for (int r = up_to ? 1 : rows; r <= rows; r++) {
+            const size_t cut = vx_linear_slices(m->be, l.gate_up.n, l.gate_up.k, r);
+            most = std::max(most, (size_t)r * l.ff_pad * (cut > 1 ? cut * 4 : esize(*m->mix)));
+        }
+    }
+    return most;
 }
 
 // floats of sliced sublayer outputs, and of latent projections, that a step of up to `rows` rows may need
@@ -86,7 +98,7 @@ int alloc_acts(vh_model *m, int rows, bool up_to, A &&alloc, MixActs *a) {
                     get(&a->cat, R * w.out * es) && get(&a->xc, R * w.xc * es) && get(&a->dtr, R * w.dtr * es) &&
                     get(&a->bc, R * w.bc * 4) && get(&a->dt, R * w.dt * 4) && get(&a->act, R * w.act * es) &&
                     get(&a->y, slice_floats(m, rows, up_to) * 4) && (!loop || get(&a->emb, R * m->cfg.hidden * 4)) &&
-                    get(&a->qc, R * w.qc * es) && get(&a->qa, R * w.qa * es) && get(&a->lo, R * w.qa * es) && get(&a->z, R * w.z * es) &&
+                    get(&a->qc, R * w.qc * es) && get(&a->qa, R * w.qa * es) && get(&a->lo, R * w.qa * es) && get(&a->z, up_bytes(m, rows, up_to)) &&
                     get(&a->rot, R * w.rot * 4) &&
                     (!m->mix->post_norm || get(&a->hist, R * m->cfg.hidden * (m->mix->runs.size() + 1) * 4));
     return ok ? (int)VH_OK : fail("activations of %d rows: %s", rows, vx_last_error());
@@ -271,6 +283,8 @@ int run_latent(vh_model *m, const LayerRun &r, const vx_ragged &b, const MixActs
     }
     if (t.heads * t.v_pad < ldc) VXC(vx_fill_zero(m->be, a.cat, (size_t)rows * ldc * es));
     // sequences with many rows: keys and values of all their tokens spelled out, once for all rows and heads
+    const int k_cols = t.heads * t.dim_pad;
+    const void *values = at(t.expand.w, (size_t)k_cols * t.rank_pad, 2);
     const int many = ex && ex->rows > 0 ? t.expand_rows : 0;
     bool few = many == 0;
     if (many > 0)
@@ -288,15 +302,17 @@ int run_latent(vh_model *m, const LayerRun &r, const vx_ragged &b, const MixActs
         VXC(vx_attn_latent(m->be, x.act, &b, &at_));
         o = plain(a.cat, 0, ldc, t.v_pad, 1);
         o.groups = t.heads, o.a_group = t.rank_pad, o.out_group = t.v_pad;
-        VXC(vx_linear(m->be, x.act, a.lo, t.heads * t.rank_pad, at(t.expand.w, (size_t)q_cols * t.rank_pad, 2), t.v_pad, t.rank_pad, rows, &o));
+        VXC(vx_linear(m->be, x.act, a.lo, t.heads * t.rank_pad, values, t.v_pad, t.rank_pad, rows, &o));
     }
     if (many > 0) {
-        vx_linear_out o = plain(a.proj, 0, t.expand.n, t.expand.n, 1);  // (every column leaves for the pool)
+        vx_linear_out o = plain(a.proj, 0, k_cols, k_cols, 1);  // (every column leaves for the pool)
         o.kind = VX_LIN_KV;
-        o.k_col = 0, o.v_col = q_cols, o.kv_heads = t.heads, o.k_dim = t.head_cols, o.v_dim = t.v_pad;
+        o.kv_heads = t.heads, o.k_dim = t.head_cols, o.k_used = t.dim_pad, o.v_dim = t.v_pad, o.v_col = k_cols;
         o.block_size = b.block_size, o.pool = ex->kv, o.a_rows = ex->slots;
-        VXC(vx_linear(m->be, x.act, r.kv, t.row, t.expand.w, t.expand.n, t.rank_pad, ex->rows, &o));
-        VXC(vx_latent_spread(m->be, x.act, r.kv, t.rank, t.rot_dim, ex->slots, ex->rows, ex->kv, t.heads, t.head_cols, t.v_pad, b.block_size,
+        VXC(vx_linear(m->be, x.act, r.kv, t.row, t.expand.w, k_cols, t.rank_pad, ex->rows, &o));
+        o.kind = VX_LIN_V, o.v_col = 0, o.cols = o.ldo = t.heads * t.v_pad;
+        VXC(vx_linear(m->be, x.act, r.kv, t.row, values, t.heads * t.v_pad, t.rank_pad, ex->rows, &o));
+        VXC(vx_latent_spread(m->be, x.act, r.kv, t.rank, t.head_cols - t.dim_pad, ex->slots, ex->rows, ex->kv, t.heads, t.head_cols, t.v_pad, b.block_size,
                              t.dim_pad));
         vx_ragged eb = b;
         eb.table_rows = ex->table_rows, eb.block_tables = ex->tables, eb.max_blocks = ex->max_blocks;
@@ -316,10 +332,12 @@ int run_latent(vh_model *m, const LayerRun &r, const vx_ragged &b, const MixActs
 int run_mlp(vh_model *m, const MixLayer &l, int rows, const MixActs &a, int *slices) {
     const MixModel &x = *m->mix;
     const int width_pad = pad_to(m->cfg.hidden, 64);
-    vx_linear_out o = plain(l.poly ? a.z : a.act, 0, l.ff_pad, l.ff_pad, 1);
+    const int cut = l.poly ? vx_linear_slices(m->be, l.gate_up.n, l.gate_up.k, rows) : 1;
+    vx_linear_out o = plain(l.poly ? a.z : a.act, cut > 1, l.ff_pad, l.ff_pad, cut);
     if (!l.poly) o.kind = VX_LIN_SWIGLU;
     VXC(vx_linear(m->be, x.act, a.h, width_pad, l.gate_up.w, l.gate_up.n, l.gate_up.k, rows, &o));
-    if (l.poly) VXC(vx_poly_norm(m->be, x.act, a.z, l.ff_pad, rows, l.ff, l.poly, x.eps, a.act, l.ff_pad));
+    if (l.poly)
+        VXC(vx_poly_norm(m->be, x.act, a.z, l.ff_pad, cut > 1 ? cut : 0, (int64_t)rows * l.ff_pad, rows, l.ff, l.poly, x.eps, a.act, l.ff_pad));
     *slices = vx_linear_slices(m->be, l.down.n, l.down.k, rows);
     o = plain(a.y, 1, l.down.n, l.down.n, *slices);
     VXC(vx_linear(m->be, x.act, a.act, l.ff_pad, l.down.w, l.down.n, l.down.k, rows, &o));

@@ -134,7 +134,7 @@ struct LatentMixer {
     const float *norm_c = nullptr, *norm_q = nullptr, *sink = nullptr;
     Linear q_up;                                       // query latent -> heads (q_rank > 0)
     Linear absorb;                                     // per head: dim_pad -> rank_pad, one behind the other
-    Linear expand;                                     // rank_pad -> heads' keys [heads * head_cols] | values [heads * v_pad]
+    Linear expand;                                     // rank_pad -> heads' keys [heads * dim_pad] | values [heads * v_pad]
     int expand_rows = 0;                               // 0: never
 };
 

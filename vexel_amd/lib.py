@@ -10,7 +10,7 @@ LIB_PATH = os.path.join(HERE, "libvexel_hip.so")
 VX_OK, VX_ERR_INVALID, VX_ERR_OOM, VX_ERR_HIP, VX_ERR_UNSUPPORTED = 0, 1, 2, 3, 4
 VX_Q4_0, VX_Q8_0, VX_Q4_K, VX_Q6_K = 1, 2, 3, 4
 VX_ACT_F32, VX_ACT_BF16 = 0, 1
-VX_LIN_PLAIN, VX_LIN_SWIGLU, VX_LIN_KV, VX_LIN_SPLIT, VX_LIN_SOFTPLUS, VX_LIN_ROTARY = 0, 1, 2, 3, 4, 5
+VX_LIN_PLAIN, VX_LIN_SWIGLU, VX_LIN_KV, VX_LIN_SPLIT, VX_LIN_SOFTPLUS, VX_LIN_ROTARY, VX_LIN_V = 0, 1, 2, 3, 4, 5, 6
 
 _vp, _i, _f, _sz, _i64 = C.c_void_p, C.c_int, C.c_float, C.c_size_t, C.c_int64
 
@@ -130,7 +130,7 @@ SIGNATURES = {
     "vx_attn_latent_fast": (_i, [_i, _i, _i, _i]),
     "vx_latent_spread": (_i, [_vp, _i, _vp, _i, _i, _vp, _i, _vp, _i, _i, _i, _i, _i]),
     "vx_post_norm": (_i, [_vp, _i, _vp]),
-    "vx_poly_norm": (_i, [_vp, _i, _vp, _i, _i, _i, _vp, _f, _vp, _i]),
+    "vx_poly_norm": (_i, [_vp, _i, _vp, _i, _i, _i64, _i, _i, _vp, _f, _vp, _i]),
     "vx_conv_silu": (_i, [_vp, _i, _vp, _vp]),
     "vx_scan_state_pad": (_i, [_i]),
     "vx_selective_scan": (_i, [_vp, _i, _vp, _vp]),
