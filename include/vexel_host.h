@@ -245,6 +245,12 @@ int vh_check_config(const char *json_text);
 /* Bucket of a key `distance` >= 0 back in a distance-bias table of `rows` rows: distances under rows/2 have a bucket each,
  * larger ones share them logarithmically up to bias_max, from which on it is the last. -1: rows or bias_max out of range. */
 int vh_distance_bucket(int distance, int rows, int bias_max);
+/* Radians per position of the dims / 2 rotated pairs, base^(-2i / dims), and the factor of cosine and sine (1). With factor > 0 YaRN's
+ * blend of them with their quotient by factor, by how many turns (fast .. slow) a pair makes over `original` positions, and
+ * 0.1 ln(factor) + 1. */
+int vh_rotary_frequencies(int dims, double base, double factor, double original, double fast, double slow, double *freqs, double *both);
+/* From how many new rows of a sequence on latent attention of these sizes spells keys and values out (bfloat16); 0: never. */
+int vh_spell_out_rows(int rank, int dim, int vdim);
 /* Hands a vx_alloc_permanent buffer to the model, which frees it in vh_model_destroy. */
 void vh_model_adopt_buffer(vh_model *m, void *device_ptr);
 

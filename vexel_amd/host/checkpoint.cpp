@@ -649,10 +649,10 @@ void rotary_frequencies(int dims, double base, bool yarn, double factor, double 
 // From how many rows of a sequence on it pays to spell its keys and values out: per (row, key, head) that takes 2 rank - dim - vdim
 // products less, and rank (dim + vdim) per (key, head) once. Half as many rows again, since the keys before the sequence's
 // new rows count in full and the spelled-out ones have to be written and read.
-int spell_out_rows(const LatentMixer &t, int dim, int vdim) {
-    const int64_t less = 2 * (int64_t)t.rank - dim - vdim;
+int spell_out_rows(int rank, int dim, int vdim) {
+    const int64_t less = 2 * (int64_t)rank - dim - vdim;
     if (less <= 0) return 0;
-    const int64_t rows = (3 * (int64_t)t.rank * (dim + vdim) / 2 + less - 1) / less;
+    const int64_t rows = (3 * (int64_t)rank * (dim + vdim) / 2 + less - 1) / less;
     return rows < (1 << 20) ? (int)(rows < 2 ? 2 : rows) : 0;
 }
 
@@ -740,7 +740,7 @@ int build_tulipel(Builder &b, const Json &config, MixModel *x, vh_config *cfg) {
         }));
         if (x->act == VX_ACT_BF16 && vx_attn_latent_fast(x->act, b.block_size, s.rank, s.rot_dim) &&
             vx_attn_ragged_fast(x->act, b.block_size, s.heads, s.heads, t.head_cols, t.v_pad)) {
-            t.expand_rows = spell_out_rows(t, s.dim + b.pad(s.rot_dim, 16) - s.rot_dim, s.vdim);
+            t.expand_rows = spell_out_rows(s.rank, s.dim, s.vdim);
             if (t.expand_rows > 0 && (x->expand_rows == 0 || t.expand_rows < x->expand_rows)) x->expand_rows = t.expand_rows;
         }
         if (s.ff > 0) {
@@ -809,6 +809,16 @@ const char *vh_architecture_name(int i) {
 }
 
 int vh_distance_bucket(int distance, int rows, int bias_max) { return distance_bucket(distance, rows, bias_max); }
+
+int vh_rotary_frequencies(int dims, double base, double factor, double original, double fast, double slow, double *freqs, double *both) {
+    if (dims < 2 || dims % 2 || !(base > 1.0) || !freqs || !both) return fail("vh_rotary_frequencies: bad arguments");
+    std::vector<double> f;
+    rotary_frequencies(dims, base, factor > 0, factor, original, fast, slow, &f, both);
+    memcpy(freqs, f.data(), f.size() * sizeof(double));
+    return VH_OK;
+}
+
+int vh_spell_out_rows(int rank, int dim, int vdim) { return rank > 0 && dim > 0 && vdim > 0 ? spell_out_rows(rank, dim, vdim) : 0; }
 
 int vh_check_config(const char *json_text) {
     Json config;

@@ -81,6 +81,8 @@ def load_host():
         h.vh_architecture_name.restype = C.c_char_p
         h.vh_check_config.argtypes = [C.c_char_p]
         h.vh_distance_bucket.argtypes = [C.c_int, C.c_int, C.c_int]
+        h.vh_rotary_frequencies.argtypes = [C.c_int] + [C.c_double] * 5 + [C.POINTER(C.c_double)] * 2
+        h.vh_spell_out_rows.argtypes = [C.c_int, C.c_int, C.c_int]
         h.vh_step.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p]
         h.vh_model_mixed_batches.argtypes = [C.c_void_p]
         h.vh_model_set_fused.argtypes = [C.c_void_p, C.c_int]
