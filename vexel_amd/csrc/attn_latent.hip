@@ -28,7 +28,7 @@ struct Args {
     int decode;               // items are the sequences that bring one row; otherwise tiles of the others
     int min_rows, max_rows, tiles;
     int pieces, goal, cap, n_rows;  // pieces: room for so many of a sequence; goal, cap: see piece_of
-    float *partial;           // [row][piece][head][pad], then the same of (maximum, sum)
+    float *partial;           // [row, or sequence][piece][head][pad], then the same of (maximum, sum)
 };
 
 // Keys of one piece of a sequence of `len` tokens: `goal` pieces of whole tiles, more where they would be longer than cap.
@@ -268,7 +268,7 @@ __global__ void __launch_bounds__(512, 2) latent_kernel(Args a) {
 #pragma unroll
             for (int v = 0; v < TD; v++) store4(out + (wave * TD + v) * 16, o[t][v] * inv);
         } else {
-            const size_t at = ((size_t)(row0 + tok) * a.pieces + piece) * H + head;
+            const size_t at = ((size_t)(a.decode ? seq : row0 + tok) * a.pieces + piece) * H + head;
             float *dst = a.partial + at * (RT * 64) + lq * 4;
 #pragma unroll
             for (int v = 0; v < TD; v++) *(f32x4 *)(dst + (wave * TD + v) * 16) = o[t][v];
@@ -283,12 +283,12 @@ __global__ void __launch_bounds__(512, 2) latent_kernel(Args a) {
 // One (row, head): its pieces become one.
 __global__ void __launch_bounds__(128) latent_merge_kernel(Args a, int pad) {
     __shared__ float s_w[MAX_PIECES];
-    const int h = blockIdx.x, row = blockIdx.y, lane = threadIdx.x & 63;
-    const int seq = a.one_token ? row : seq_of_row(a.cu, a.n_seqs, row);
+    const int h = blockIdx.x, own = blockIdx.y, lane = threadIdx.x & 63;  // own: the partial results' row
+    const int row = a.decode && !a.one_token ? a.cu[own] : own, seq = a.decode ? own : seq_of_row(a.cu, a.n_seqs, row);
     const int brings = a.one_token ? 1 : a.cu[seq + 1] - a.cu[seq];
     if (a.decode ? brings != 1 : (brings < a.min_rows || (a.max_rows > 0 && brings > a.max_rows))) return;
     const int n = a.pos[row] / piece_of(a, a.kv_lens[seq]) + 1, H = a.p.heads;
-    const size_t at = (size_t)row * a.pieces * H + h;
+    const size_t at = (size_t)own * a.pieces * H + h;
     const float *src = a.partial + at * pad, *ml = a.partial + (size_t)a.n_rows * H * a.pieces * pad + at * 2;
     float m = -INFINITY, l = 0.f;
     for (int i = lane; i < n; i += 64) m = fmaxf(m, ml[(size_t)2 * i * H]);
@@ -325,17 +325,17 @@ int run_latent(vx_backend *be, Args a, const vx_ragged *b) {
             one += b->q_lens[s] == 1;
             if (b->q_lens[s] > 1 && (a.max_rows <= 0 || b->q_lens[s] <= a.max_rows) && b->q_lens[s] > longest) longest = b->q_lens[s];
         }
-    a.n_rows = b->rows;
     // Pieces, so that the launch fills the chip. The lengths may be known as a bound only (max_kv_len), so that a sequence's own
     // length decides about its pieces on the device.
     const auto split = [&](int64_t wgs, int cap) -> int {
-        const int64_t room = most / ((int64_t)b->rows * H * (pad + 2) * 4), tiles = ceil_div(b->max_kv_len, 128);
+        a.n_rows = a.decode ? b->n_seqs : b->rows;  // (single tokens: one row a sequence)
+        const int64_t room = most / ((int64_t)a.n_rows * H * (pad + 2) * 4), tiles = ceil_div(b->max_kv_len, 128);
         const auto bounded = [&](int64_t n) { return (int)std::max<int64_t>(1, std::min({n, tiles, room, (int64_t)MAX_PIECES})); };
         a.goal = bounded(ceil_div64(256, wgs));
         a.pieces = bounded(std::max<int64_t>(a.goal, ceil_div(b->max_kv_len, cap)));
         a.cap = std::max(cap, ceil_div(ceil_div(b->max_kv_len, a.pieces), 128) * 128);
         if (a.pieces == 1) return VX_OK;
-        const size_t bytes = (size_t)b->rows * H * a.pieces * (pad + 2) * 4;
+        const size_t bytes = (size_t)a.n_rows * H * a.pieces * (pad + 2) * 4;
         const int rc = ensure_ws(be, &be->attn_ws, &be->attn_ws_bytes, bytes, "attention");
         a.partial = (float *)be->attn_ws;
         be->split.batch = 0;  // (whatever an earlier call left there is gone)
@@ -343,7 +343,7 @@ int run_latent(vx_backend *be, Args a, const vx_ragged *b) {
     };
     const auto merge = [&]() {
         if (a.pieces > 1)
-            latent_merge_kernel<<<dim3(H, b->rows), pad / 4 < 64 ? 64 : 128, 0, be->stream>>>(a, pad);
+            latent_merge_kernel<<<dim3(H, a.n_rows), pad / 4 < 64 ? 64 : 128, 0, be->stream>>>(a, pad);
     };
     if (longest > 0) {
         const int mt = query_tiles(longest * H);
