@@ -506,7 +506,8 @@ enum {
     VX_LIN_ROTARY = 5, /* columns < split to out (activation type) in heads of rot_stride columns, whose columns rot_first ..
                           rot_first + 2 * rot_pairs - 1 are turned in neighbouring pairs by rot_tab (vx_rotary_table); the
                           others (split = n: none) to out2 as with SPLIT */
-    VX_LIN_V = 6       /* every column is V of the pool (v_col 0), stored as with KV, four neighbouring slots at a time */
+    VX_LIN_V = 6,      /* every column is V of the pool (v_col 0), stored as with KV, four neighbouring slots at a time */
+    VX_LIN_SILU = 7    /* columns < split: silu(y) to out (activation type); the others, as they are, to out2 as with SPLIT */
 };
 typedef struct vx_linear_out {
     int kind, out_f32, ldo, cols, slices;
@@ -524,6 +525,8 @@ typedef struct vx_linear_out {
     int rot_stride, rot_first, rot_pairs;
     const float *rot_tab;
     int k_used;                  /* > 0: a K head's k_used first elements are what the map makes (kv_heads * k_used columns) */
+    float glu_limit, glu_alpha, glu_add; /* glu_limit > 0 (SWIGLU): g = min(gate, limit), u = up cut to -limit .. limit, and
+                                    out = g * sigmoid(glu_alpha * g) * (u + glu_add) */
 } vx_linear_out;
 /* out = a [rows, k] * W^T for a packed matrix [n, k] (padded sizes); a has lda >= k columns of the activation type, zero
  * where k was padded, rows 16-byte aligned. vx_linear_slices: into how many slices a PLAIN float32 result is best cut
@@ -531,9 +534,49 @@ typedef struct vx_linear_out {
 int vx_linear_slices(vx_backend *be, int n, int k, int rows);
 int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, int n, int k, int rows, const vx_linear_out *o);
 
+/* Mixtures of experts. vx_route chooses each row's experts and sorts the (row, choice) pairs by expert:
+ *   s = sigmoid(z[r]), choice scores c = s + correction; with groups > 1 only experts of the `keep` groups (of neighbours) whose two
+ *   largest choice scores have the largest sums; the `top` experts with the largest choice scores; weights[r][j] = s of the j-th.
+ * z: float32 in slices that are added up. A pair's place in the sorted order is places[r][j], and order[place] = r. With shared != 0
+ * every row has one more place, rows * top + r, with an expert of its own, number `experts`. tiles (device int32[4 + 4 *
+ * vx_route_max_tiles]): their count, then from tiles[4] on (expert, first place, places, 0) each; a tile holds at most tile_rows
+ * places of one expert. */
+typedef struct vx_route_args {
+    int rows, experts, top, groups, keep, shared, tile_rows;
+    const float *z;
+    int z_slices, ldz;
+    int64_t z_stride;
+    const float *correction;     /* [experts]; NULL: 0 */
+    float *weights;              /* [rows][top] */
+    int32_t *places;             /* [rows][top] */
+    int32_t *order;              /* [rows * (top + (shared != 0))] */
+    int32_t *tiles;
+} vx_route_args;
+int vx_route(vx_backend *be, const vx_route_args *p);
+/* places of a tile as vx_linear_experts wants them for that many rows of a step; the most tiles vx_route may make of them */
+int vx_route_tile_rows(int act, int rows, int experts, int top);
+int vx_route_max_tiles(int rows, int experts, int top, int shared, int tile_rows);
+/* The experts' maps over the places that vx_route made: activation row of a place: a_rows[place], or the place itself (NULL); result
+ * rows are places. Expert e < experts: the packed matrix [n, k] at w + e * n * k elements; expert `experts`: w_shared [n_shared,
+ * k_shared], which may have another size (out rows then hold the larger of the two). SWIGLU (glu_* and, for the shared expert,
+ * shared_limit; 0: its gate and up are not cut) or PLAIN in the activation type. n % 32 == 0. */
+typedef struct vx_experts_args {
+    int kind, rows, experts, shared, n, k, n_shared, k_shared, tile_rows, max_tiles;
+    const void *a, *w, *w_shared;
+    int lda;
+    const int32_t *tiles, *a_rows;
+    float glu_limit, shared_limit, glu_alpha, glu_add;
+    void *out;
+    int ldo, cols, cols_shared;
+} vx_experts_args;
+int vx_linear_experts(vx_backend *be, int act, const vx_experts_args *p);
+
 /* The seam between two sublayers, one row at a time, in float32:
- *   x = x_in[r];  if y: x += mult * rmsnorm(sum over slices of y[s][r]) * w_post;  if add: x += add[r];  x_out[r] = x;
+ *   x = x_in[r];  if y: x += mult * rmsnorm(sum over slices of y[s][r]) * w_post   (w_post NULL: x += mult * (the sum + y_bias));
+ *   if e_rows: x += sum over j < e_top of e_weights[r][j] * e_rows[e_places[r][j]], + e_rows[e_shared + r] (e_shared >= 0);
+ *   if add: x += add[r];  x_out[r] = x;
  *   if w_pre: out[i] = rmsnorm(x) * w_pre in the activation type, columns cols .. ldo - 1 zero.
+ * e_rows: activation type.
  * r = row_idx ? row_idx[i] : i for i < rows. x_out may be x_in or NULL. rmsnorm(v) = v / sqrt(mean(v^2) + eps). */
 typedef struct vx_residual_norm_args {
     int rows, cols;
@@ -547,6 +590,11 @@ typedef struct vx_residual_norm_args {
     const float *w_pre;
     void *out;
     int ldo;
+    const float *y_bias;         /* [cols] or NULL; with w_post NULL only */
+    const void *e_rows;
+    int lde, e_top, e_shared;
+    const int32_t *e_places;
+    const float *e_weights;
 } vx_residual_norm_args;
 int vx_residual_norm(vx_backend *be, int act, const vx_residual_norm_args *p);
 
@@ -570,10 +618,19 @@ typedef struct vx_attn_args {
     float out_scale;
     void *out;
     int ldo;
-    const float *sink;           /* [heads]: the softmax's denominator also holds exp(sink[h]); NULL: none */
+    const float *sink;           /* [heads * maps]: the softmax's denominator also holds exp(sink[h]); NULL: none */
     int min_rows;                /* > 1: only the rows of sequences that bring at least so many */
+    int window, chunk;           /* > 0: a row sees only keys with i - j < window, or with floor(i / chunk) = floor(j / chunk) */
+    float softcap;               /* > 0: scores become softcap * tanh(score / softcap) (before the bias) */
+    int maps;                    /* 2: differential attention, see below; 0 or 1: one map */
+    float diff_lambda, diff_scale, diff_eps;
 } vx_attn_args;
+/* maps = 2: every head has two queries, and every K/V head two keys, side by side (head h, map m at (h * 2 + m) * k_dim); both maps
+ * attend on their own to the K/V head's values, and with their results a1 and a2
+ *   o = a1 - diff_lambda * a2,  out = diff_scale * o / sqrt(mean over v_dim of o^2 + diff_eps)      (no gate)
+ * K of such a pool is [kv_heads * 2][block_size][k_pad]: vx_kv_block_elems2 counts the heads of K and of V apart. */
 size_t vx_kv_block_elems(int block_size, int kv_heads, int k_dim, int v_dim);
+size_t vx_kv_block_elems2(int block_size, int k_heads, int k_dim, int v_heads, int v_dim);
 int vx_attn_ragged(vx_backend *be, int act, const vx_ragged *b, const vx_attn_args *p);
 /* 1 when the matrix-core kernels take the geometry, 0 when vx_attn_ragged uses the plain one. */
 int vx_attn_ragged_fast(int act, int block_size, int heads, int kv_heads, int k_dim, int v_dim);
@@ -670,6 +727,62 @@ typedef struct vx_conv_args {
     int ldo;
 } vx_conv_args;
 int vx_conv_silu(vx_backend *be, int act, const vx_ragged *b, const vx_conv_args *p);
+
+/* Token embeddings with pairs: out[r] = embed[token] + pairs[row], row = (previous token * mul_prev + token * mul_cur) mod buckets, and
+ * `buckets` for a sequence's first token (pairs has buckets + 1 rows). token_pool [slots of the paged pool] keeps the
+ * sequences' tokens by slot: this step's are written, the one before a sequence's first new row is read. */
+typedef struct vx_pair_embedding_args {
+    int cols, vocab, buckets;
+    int64_t mul_prev, mul_cur;
+    const int32_t *tokens;       /* [rows] */
+    const float *embed, *pairs;
+    int32_t *token_pool;
+    float *out;                  /* [rows][cols] */
+} vx_pair_embedding_args;
+int vx_pair_embedding(vx_backend *be, const vx_ragged *b, const vx_pair_embedding_args *p);
+
+/* Query, key and value heads from a float32 projection (slices added up, bias added) to where vx_attn_ragged reads them:
+ *   queries and keys: dimensions i and i + rot_pairs (i < rot_pairs) turned by rot_tab (vx_rotary_table; rot_pairs 0: not), then, with norm,
+ *   v / sqrt(mean(v^2) + eps) over the head, times w_q or w_k [dim] (NULL: 1)
+ * Heads lie side by side from their column on: q_heads and k_heads of dim, v_heads of v_dim. Queries go to q (activation type, head h at h *
+ * dim), keys and values to the pool (layout: vx_kv_block_elems2) at slot_mapping[r]. v_col < 0: a value is its key head as
+ * projected, before rotation and norm (v_heads = k_heads, v_dim = dim). */
+typedef struct vx_heads_args {
+    int q_heads, k_heads, v_heads, dim, v_dim;
+    const float *y;
+    int y_slices, ldy;
+    int64_t y_stride;
+    const float *bias;           /* [ldy] or NULL */
+    int q_col, k_col, v_col;
+    int rot_pairs;
+    const float *rot_tab;
+    int norm;
+    float eps;
+    const float *w_q, *w_k;
+    void *q, *pool;
+    int ldq;
+} vx_heads_args;
+int vx_heads_store(vx_backend *be, int act, const vx_ragged *b, const vx_heads_args *p);
+
+/* Linear attention with a constant decay per head over a mixed batch (states and sums in float32):
+ *   S = decay * S + k v^T,  out = S^T q,  S [dim][vdim] per head
+ * dim a multiple of 32 up to 512, vdim one of 16 up to 512 (columns that pad a head are zero in q, k and v, and in out). q, k, v: activation
+ * type, head h at columns h * dim and h * vdim, rows 16-byte aligned; out float32 [rows][ldo], head h at h * vdim. decay
+ * [heads][2] float32: decay - 1 and log2(decay), the latter finite. state [slots][heads][dim][vdim] float32. A sequence at position 0 starts from zero. */
+typedef struct vx_decay_args {
+    int heads, dim, vdim;
+    const float *decay;
+    const void *q, *k, *v;
+    int ldq, ldk, ldv;
+    float *state;
+    float *out;
+    int ldo;
+} vx_decay_args;
+int vx_decay_attn(vx_backend *be, int act, const vx_ragged *b, const vx_decay_args *p);
+/* out[r] = x[r] / sqrt(sum(x[r]^2) / count + eps) * w * sigmoid(gate[r]): x and gate float32, out activation type, columns cols .. ldo - 1
+ * zero. count: how many of the columns are not padding. */
+int vx_gated_norm(vx_backend *be, int act, const float *x, int ldx, const float *gate, int ldg, const float *w, float eps, int rows, int cols,
+                  int count, void *out, int ldo);
 
 /* Selective scan over a mixed batch, all in float32:
  *   S[c][n] = exp(dt[c] * A[c][n]) * S[c][n] + dt[c] * x[c] * B[n];  y[c] = sum_n S[c][n] * C[n] + D[c] * x[c]

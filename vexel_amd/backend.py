@@ -37,17 +37,41 @@ class VxRagged(C.Structure):
 class VxLinearOut(C.Structure):
     _fields_ = _fields("int kind out_f32 ldo cols slices; ptr out out2; int split ldo2; ptr bias; int k_col v_col kv_heads "
                        "k_dim v_dim block_size; ptr pool slot_mapping a_rows; float softcap; int groups a_group out_group "
-                       "rot_stride rot_first rot_pairs; ptr rot_tab; int k_used")
+                       "rot_stride rot_first rot_pairs; ptr rot_tab; int k_used; float glu_limit glu_alpha glu_add")
 
 
 class VxResidualNormArgs(C.Structure):
     _fields_ = _fields("int rows cols; ptr row_idx x_in add x_out y w_post; int y_slices ldy; i64 y_stride; float mult eps; "
-                       "ptr w_pre out; int ldo")
+                       "ptr w_pre out; int ldo; ptr y_bias e_rows; int lde e_top e_shared; ptr e_places e_weights")
+
+
+class VxRouteArgs(C.Structure):
+    _fields_ = _fields("int rows experts top groups keep shared tile_rows; ptr z; int z_slices ldz; i64 z_stride; "
+                       "ptr correction weights places order tiles")
+
+
+class VxExpertsArgs(C.Structure):
+    _fields_ = _fields("int kind rows experts shared n k n_shared k_shared tile_rows max_tiles; ptr a w w_shared; int lda; "
+                       "ptr tiles a_rows; float glu_limit shared_limit glu_alpha glu_add; ptr out; int ldo cols cols_shared")
+
+
+class VxPairEmbeddingArgs(C.Structure):
+    _fields_ = _fields("int cols vocab buckets; i64 mul_prev mul_cur; ptr tokens embed pairs token_pool out")
+
+
+class VxHeadsArgs(C.Structure):
+    _fields_ = _fields("int q_heads k_heads v_heads dim v_dim; ptr y; int y_slices ldy; i64 y_stride; ptr bias; "
+                       "int q_col k_col v_col rot_pairs; ptr rot_tab; int norm; float eps; ptr w_q w_k q pool; int ldq")
+
+
+class VxDecayArgs(C.Structure):
+    _fields_ = _fields("int heads dim vdim; ptr decay q k v; int ldq ldk ldv; ptr state out; int ldo")
 
 
 class VxAttnArgs(C.Structure):
     _fields_ = _fields("int heads kv_heads k_dim v_dim; float scale temp_coef; int temp_every; ptr bias; int bias_len; "
-                       "ptr q gate; int ldq ldg; ptr pool; float out_scale; ptr out; int ldo; ptr sink; int min_rows")
+                       "ptr q gate; int ldq ldg; ptr pool; float out_scale; ptr out; int ldo; ptr sink; int min_rows window chunk; "
+                       "float softcap; int maps; float diff_lambda diff_scale diff_eps")
 
 
 class VxLatentStoreArgs(C.Structure):
@@ -456,6 +480,24 @@ class HipBackend:
 
     def linear(self, act, a, lda, w, n, k, rows, out):
         self.call("vx_linear", act, a, lda, w, n, k, rows, C.byref(out))
+
+    def route(self, args):
+        self.call("vx_route", C.byref(args))
+
+    def linear_experts(self, act, args):
+        self.call("vx_linear_experts", act, C.byref(args))
+
+    def pair_embedding(self, batch, args):
+        self.call("vx_pair_embedding", C.byref(batch), C.byref(args))
+
+    def heads_store(self, act, batch, args):
+        self.call("vx_heads_store", act, C.byref(batch), C.byref(args))
+
+    def decay_attn(self, act, batch, args):
+        self.call("vx_decay_attn", act, C.byref(batch), C.byref(args))
+
+    def gated_norm(self, act, x, ldx, gate, ldg, w, eps, rows, cols, count, out, ldo):
+        self.call("vx_gated_norm", act, x, ldx, gate, ldg, w, eps, rows, cols, count, out, ldo)
 
     def residual_norm(self, act, args):
         self.call("vx_residual_norm", act, C.byref(args))

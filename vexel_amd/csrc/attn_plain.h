@@ -15,6 +15,13 @@ __device__ __forceinline__ float query_temperature(float coef, int every, int po
     return 1.0f + coef * logf((float)((pos + 1) / every) + 1.0f);
 }
 
+// The first key a row sees: all are (0), those of a window of so many tokens, those of its chunk.
+__device__ __forceinline__ int first_visible(int window, int chunk, int pos) {
+    int f = window > 0 && pos >= window ? pos - window + 1 : 0;
+    if (chunk > 0) f = max(f, pos - pos % chunk);
+    return f;
+}
+
 struct PlainPart {      // one part of a head's query: head h's elements lie at h * stride, and are multiplied with the key row's
     const void *p;      // elements from `first` on; they fill `room` places there, zero beyond n
     int ld, n, first, room, stride;
@@ -34,6 +41,9 @@ struct PlainAttn {
     float out_scale;
     void *out;
     int ldo, out_head, out_cols;              // head h at columns h * out_head; columns v_dim .. out_cols - 1 become zero
+    int maps, out_f32;                        // maps (0: 1) queries share a head's values; out is float32 whatever T is
+    int window, chunk;
+    float softcap;
     int min_rows, max_rows;                   // rows of sequences with so many rows only (0: no limit)
     const int32_t *cu, *pos, *rows, *tables;
     int n_seqs, max_blocks, block_size, one_token;
@@ -43,13 +53,13 @@ template <typename T>
 __global__ void __launch_bounds__(256) attn_plain_kernel(PlainAttn p) {
     extern __shared__ float s_q[];  // [row]
     __shared__ float s_s[PL_CHUNK], s_red[4];
-    const int h = blockIdx.x, row = blockIdx.y, g = h / p.group, tid = threadIdx.x;
+    const int h = blockIdx.x, row = blockIdx.y, maps = max(p.maps, 1), g = h / maps / p.group, tid = threadIdx.x;
     const int seq = p.one_token ? row : seq_of_row(p.cu, p.n_seqs, row);
     const int brings = p.one_token ? 1 : p.cu[seq + 1] - p.cu[seq];
     if ((p.min_rows > 0 && brings < p.min_rows) || (p.max_rows > 0 && brings > p.max_rows)) return;
-    const int pos = p.pos[row], len = pos + 1;
+    const int pos = p.pos[row], len = pos + 1, first = first_visible(p.window, p.chunk, pos);
     const int32_t *bt = p.tables + (size_t)p.rows[seq] * p.max_blocks;
-    const T *kpool = (const T *)p.pool + g * p.k_head, *vpool = (const T *)p.pool + p.v_first + g * p.v_head;
+    const T *kpool = (const T *)p.pool + (g * maps + h % maps) * p.k_head, *vpool = (const T *)p.pool + p.v_first + g * p.v_head;
     const float qf = p.scale * query_temperature(p.temp_coef, p.temp_every, pos);
 #pragma unroll
     for (int i = 0; i < 2; i++)
@@ -62,7 +72,7 @@ __global__ void __launch_bounds__(256) attn_plain_kernel(PlainAttn p) {
 #pragma unroll
     for (int i = 0; i < MAXV; i++) acc[i] = 0.f;
     float m = -INFINITY, l = 0.f;
-    for (int c0 = 0; c0 < len; c0 += PL_CHUNK) {
+    for (int c0 = first; c0 < len; c0 += PL_CHUNK) {
         const int cn = min(PL_CHUNK, len - c0);
         __syncthreads();
         float mx = -INFINITY;
@@ -72,6 +82,7 @@ __global__ void __launch_bounds__(256) attn_plain_kernel(PlainAttn p) {
             float dot = 0.f;
             for (int d = 0; d < p.row; d++) dot = fmaf(s_q[d], (float)k[d], dot);
             float s = dot * qf;
+            if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
             if (p.bias) s += p.bias[(size_t)h * p.bias_len + min(pos - key, p.bias_len - 1)];
             s_s[i] = s;
             mx = fmaxf(mx, s);
@@ -109,7 +120,9 @@ __global__ void __launch_bounds__(256) attn_plain_kernel(PlainAttn p) {
     }
     if (p.sink) l += expf(p.sink[h] - m);
     __syncthreads();
-    T *out = (T *)p.out + (size_t)row * p.ldo + h * p.out_head;
+    const size_t at = (size_t)row * p.ldo + h * p.out_head;
+    T *out = (T *)p.out + at;
+    float *fout = p.out_f32 ? (float *)p.out + at : nullptr;
     float *s_acc = s_s;  // [kg][width]
     for (int v = 0; v < MAXV; v++) {
         const int d = md + v * 256;
@@ -121,7 +134,10 @@ __global__ void __launch_bounds__(256) attn_plain_kernel(PlainAttn p) {
             for (int i = 0; i < kg; i++) t += s_acc[i * width + md];
             t = t / l * p.out_scale;
             if (p.gate) t *= sigmoid_f((float)((const T *)p.gate)[(size_t)row * p.ldg + h * p.v_dim + d]);
-            out[d] = (T)t;
+            if (fout)
+                fout[d] = t;
+            else
+                out[d] = (T)t;
         }
         __syncthreads();
     }

@@ -1,0 +1,171 @@
+// What stands at either end of mixed-batch attention: token embeddings with a table of pairs (vx_pair_embedding), and query, key
+// and value heads on their way from a float32 projection to the queries' rows and the paged pool (vx_heads_store).
+#include "ragged.h"
+
+using namespace vx;
+
+namespace {
+
+struct PairArgs {
+    vx_pair_embedding_args p;
+    const int32_t *cu, *pos, *slot_map, *table_rows, *tables;
+    int n_seqs, max_blocks, block_size, one_token;
+};
+
+// A row per workgroup. The token before a sequence's first new row was written by an earlier step.
+template <bool VEC>
+__global__ void __launch_bounds__(256) pair_embedding_kernel(PairArgs a) {
+    const vx_pair_embedding_args &p = a.p;
+    const int row = blockIdx.x, pos = a.pos[row], tok = p.tokens[row];
+    const int seq = a.one_token ? row : seq_of_row(a.cu, a.n_seqs, row);
+    int pair = p.buckets;
+    if (pos > 0) {
+        int prev;
+        if (!a.one_token && row > a.cu[seq]) {
+            prev = p.tokens[row - 1];
+        } else {
+            const int at = pos - 1, blk = a.tables[(size_t)a.table_rows[seq] * a.max_blocks + at / a.block_size];
+            prev = p.token_pool[(size_t)blk * a.block_size + at % a.block_size];
+        }
+        pair = (int)(((int64_t)prev * p.mul_prev + (int64_t)tok * p.mul_cur) % p.buckets);
+    }
+    if (threadIdx.x == 0) p.token_pool[a.slot_map[row]] = tok;
+    const float *e = p.embed + (size_t)tok * p.cols, *b = p.pairs + (size_t)pair * p.cols;
+    float *out = p.out + (size_t)row * p.cols;
+    if constexpr (VEC) {
+        for (int c = threadIdx.x * 4; c < p.cols; c += 1024) *(f32x4 *)(out + c) = *(const f32x4 *)(e + c) + *(const f32x4 *)(b + c);
+    } else {
+        for (int c = threadIdx.x; c < p.cols; c += 256) out[c] = e[c] + b[c];
+    }
+}
+
+struct HeadArgs {
+    vx_heads_args p;
+    const int32_t *slot_map;
+    int rows, block_size, units;
+};
+
+// A wave takes one head of one row; 64 * NV >= its dimensions. The element a rotation pairs with is read a second time.
+template <typename T, int NV>
+__global__ void __launch_bounds__(256) heads_kernel(HeadArgs a) {
+    const vx_heads_args &p = a.p;
+    const int groups = (a.units + 3) / 4, lane = threadIdx.x & 63;
+    const int row = blockIdx.x / groups, unit = blockIdx.x % groups * 4 + (threadIdx.x >> 6);
+    if (unit >= a.units) return;  // (nothing is shared between waves)
+    const bool is_q = unit < p.q_heads, is_k = !is_q && unit < p.q_heads + p.k_heads;
+    const int h = is_q ? unit : is_k ? unit - p.q_heads : unit - p.q_heads - p.k_heads;
+    const int dim = is_q || is_k ? p.dim : p.v_dim, col = (is_q ? p.q_col : is_k ? p.k_col : p.v_col) + h * dim;
+    const float *y = p.y + (size_t)row * p.ldy + col, *bias = p.bias ? p.bias + col : nullptr;
+    const auto raw = [&](int d) {
+        float t = y[d];
+        for (int s = 1; s < p.y_slices; s++) t += y[(size_t)s * p.y_stride + d];
+        return bias ? t + bias[d] : t;
+    };
+    const int kp = (p.dim + 7) & ~7;
+    const int slot = is_q ? 0 : a.slot_map[row], blk = is_q ? 0 : slot / a.block_size, in = slot - blk * a.block_size;
+    T *pool = (T *)p.pool + (size_t)blk * a.block_size * ((size_t)p.k_heads * kp + (size_t)p.v_heads * p.v_dim);
+    T *vpool = pool + (size_t)p.k_heads * a.block_size * kp + (size_t)h * p.v_dim * a.block_size + in;
+    float v[NV];
+#pragma unroll
+    for (int i = 0; i < NV; i++) v[i] = lane + i * 64 < dim ? raw(lane + i * 64) : 0.f;
+    if ((is_k && p.v_col < 0) || (!is_q && !is_k)) {
+#pragma unroll
+        for (int i = 0; i < NV; i++)
+            if (lane + i * 64 < dim) vpool[(size_t)(lane + i * 64) * a.block_size] = (T)v[i];
+        if (!is_k) return;
+    }
+    if (p.rot_pairs > 0) {
+        const float *tab = p.rot_tab + (size_t)row * p.rot_pairs * 2;
+#pragma unroll
+        for (int i = 0; i < NV; i++) {
+            const int d = lane + i * 64;
+            if (d < 2 * p.rot_pairs) {
+                const bool low = d < p.rot_pairs;
+                const int pair = low ? d : d - p.rot_pairs;
+                const float o = raw(low ? d + p.rot_pairs : d - p.rot_pairs), c = tab[2 * pair], s = tab[2 * pair + 1];
+                v[i] = low ? v[i] * c - o * s : v[i] * c + o * s;
+            }
+        }
+    }
+    if (p.norm) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < NV; i++) ss = fmaf(v[i], v[i], ss);
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+        const float inv = 1.0f / sqrtf(ss / (float)dim + p.eps);
+        const float *w = is_q ? p.w_q : p.w_k;
+#pragma unroll
+        for (int i = 0; i < NV; i++) v[i] *= w && lane + i * 64 < dim ? inv * w[lane + i * 64] : inv;
+    }
+    T *out = is_q ? (T *)p.q + (size_t)row * p.ldq + h * dim : pool + ((size_t)h * a.block_size + in) * kp;
+#pragma unroll
+    for (int i = 0; i < NV; i++)
+        if (lane + i * 64 < dim) out[lane + i * 64] = (T)v[i];
+}
+
+template <typename T>
+void launch_heads(vx_backend *be, const HeadArgs &a) {
+    const int wide = a.p.dim > a.p.v_dim ? a.p.dim : a.p.v_dim;
+    const unsigned grid = (unsigned)a.rows * (unsigned)ceil_div(a.units, 4);
+    if (wide <= 64)
+        heads_kernel<T, 1><<<grid, 256, 0, be->stream>>>(a);
+    else if (wide <= 128)
+        heads_kernel<T, 2><<<grid, 256, 0, be->stream>>>(a);
+    else if (wide <= 256)
+        heads_kernel<T, 4><<<grid, 256, 0, be->stream>>>(a);
+    else
+        heads_kernel<T, 32><<<grid, 256, 0, be->stream>>>(a);
+}
+
+}  // namespace
+
+extern "C" {
+
+int vx_pair_embedding(vx_backend *be, const vx_ragged *b, const vx_pair_embedding_args *p) {
+    int rc = enter(be);
+    if (rc) return rc;
+    rc = check_ragged(b, "vx_pair_embedding");
+    if (rc) return rc;
+    VX_REQUIRE(p && p->cols >= 1 && p->vocab >= 1 && p->buckets >= 1 && p->mul_prev >= 0 && p->mul_cur >= 0 && p->tokens && p->embed && p->pairs &&
+                   p->token_pool && p->out,
+               "vx_pair_embedding: bad arguments");
+    VX_REQUIRE(p->mul_prev < ((int64_t)1 << 31) && p->mul_cur < ((int64_t)1 << 31), "vx_pair_embedding: factors of 2^31 or more");
+    const PairArgs a{*p, b->cu_seqlens, b->token_pos, b->slot_mapping, b->table_rows, b->block_tables, b->n_seqs, b->max_blocks, b->block_size,
+                     b->q_lens ? 0 : 1};
+    const auto al = [](const void *q) { return (uintptr_t)q % 16 == 0; };
+    if (p->cols % 4 == 0 && al(p->embed) && al(p->pairs) && al(p->out))
+        pair_embedding_kernel<true><<<b->rows, 256, 0, be->stream>>>(a);
+    else
+        pair_embedding_kernel<false><<<b->rows, 256, 0, be->stream>>>(a);
+    VX_CHECK_LAUNCH();
+    return VX_OK;
+}
+
+int vx_heads_store(vx_backend *be, int act, const vx_ragged *b, const vx_heads_args *p) {
+    int rc = enter(be);
+    if (rc) return rc;
+    rc = check_ragged(b, "vx_heads_store");
+    if (rc) return rc;
+    VX_REQUIRE(act == VX_ACT_F32 || act == VX_ACT_BF16, "vx_heads_store: unknown activation type %d", act);
+    VX_REQUIRE(p && p->q_heads >= 1 && p->k_heads >= 1 && p->v_heads >= 1 && p->dim >= 1 && p->v_dim >= 1 && p->dim <= 2048 && p->v_dim <= 2048 && p->y &&
+                   p->y_slices >= 1 && p->q && p->pool && p->q_col >= 0 && p->k_col >= 0,
+               "vx_heads_store: bad arguments");
+    VX_REQUIRE(p->v_col >= 0 || (p->v_heads == p->k_heads && p->v_dim == p->dim), "vx_heads_store: values are keys of another size");
+    const int64_t q_end = p->q_col + (int64_t)p->q_heads * p->dim, k_end = p->k_col + (int64_t)p->k_heads * p->dim;
+    VX_REQUIRE(q_end <= p->ldy && k_end <= p->ldy && (p->v_col < 0 || p->v_col + (int64_t)p->v_heads * p->v_dim <= p->ldy) &&
+                   p->ldq >= (int64_t)p->q_heads * p->dim,
+               "vx_heads_store: heads beyond their row");
+    VX_REQUIRE(p->rot_pairs >= 0 && 2 * p->rot_pairs <= p->dim && (p->rot_pairs == 0 || p->rot_tab), "vx_heads_store: %d pairs in heads of %d", p->rot_pairs,
+               p->dim);
+    HeadArgs a{*p, b->slot_mapping, b->rows, b->block_size, p->q_heads + p->k_heads + (p->v_col < 0 ? 0 : p->v_heads)};
+    VX_REQUIRE((int64_t)b->rows * ceil_div(a.units, 4) < ((int64_t)1 << 31), "vx_heads_store: %d rows of %d heads", b->rows, a.units);
+    if (act == VX_ACT_BF16)
+        launch_heads<bf16>(be, a);
+    else
+        launch_heads<float>(be, a);
+    VX_CHECK_LAUNCH();
+    return VX_OK;
+}
+
+}  // extern "C"

@@ -1,4 +1,5 @@
-// Linear maps with bfloat16 weights for mixed batches (vx_linear_pack, vx_linear).
+// Linear maps with bfloat16 weights for mixed batches (vx_linear_pack, vx_linear), and those of experts over the rows that
+// were sorted by expert (vx_linear_experts).
 //
 // The weights lie in tiles of 16 outputs x 32 inputs, each stored in the order in which the 64 lanes of a wave hold a
 // matrix-core operand: a wave reads a tile as one contiguous kilobyte. Both kernels compute W * a^T, so that a lane ends
@@ -11,6 +12,9 @@
 //
 // Activations are bfloat16 or float32 (template parameter T); with float32 the weights are widened and the float32
 // matrix instruction multiplies them, so that nothing is rounded to fewer bits.
+#include <string.h>
+
+#include <algorithm>
 #include <type_traits>
 
 #include "ragged.h"
@@ -24,7 +28,37 @@ struct LinArgs {
     const void *w;
     int lda, n, k, rows;
     vx_linear_out o;
+    // experts (EX): row0 .. rows - 1 are the places of the workgroup's tile
+    int row0;
+    const int32_t *tiles;
+    int experts, n_shared, k_shared, cols_shared;
+    const void *w_shared;
+    float shared_limit;
 };
+
+// The expert and the places of tile `t`; false beyond the last.
+__device__ __forceinline__ bool take_tile(LinArgs &p, int t) {
+    if (t >= p.tiles[0]) return false;
+    const int32_t *r = p.tiles + 4 + 4 * t;
+    const int e = r[0];
+    p.row0 = r[1], p.rows = r[1] + r[2];
+    if (e < p.experts) {
+        p.w = (const bf16 *)p.w + (size_t)e * p.n * p.k;
+    } else {
+        p.w = p.w_shared, p.n = p.n_shared, p.k = p.k_shared, p.o.cols = p.cols_shared, p.o.glu_limit = p.shared_limit;
+    }
+    return true;
+}
+
+// A gate column times its up column.
+__device__ __forceinline__ float glu(const vx_linear_out &o, float g, float u) {
+    if (o.glu_limit <= 0.f && o.glu_alpha == 0.f) return silu_f(g) * u;
+    if (o.glu_limit > 0.f) {
+        g = fminf(g, o.glu_limit);
+        u = fminf(fmaxf(u, -o.glu_limit), o.glu_limit);
+    }
+    return g * sigmoid_f(o.glu_alpha * g) * (u + o.glu_add);
+}
 
 // Where K and V elements lie in the pool: a part that depends on the slot and one that depends on the column.
 struct KvSlot {
@@ -120,6 +154,14 @@ __device__ __forceinline__ void emit(const LinArgs &p, int slice, int row, int c
             put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
     } else if constexpr (KIND == VX_LIN_SWIGLU) {
         put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
+    } else if constexpr (KIND == VX_LIN_SILU) {
+        if (c < o.split) {
+#pragma unroll
+            for (int r = 0; r < 4; r++) v[r] = silu_f(v[r]);
+            put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
+        } else {
+            put4(o.out2 + (size_t)row * o.ldo2, c - o.split, o.ldo2, o.ldo2, v);
+        }
     } else if constexpr (KIND == VX_LIN_SPLIT) {
         if (c < o.split)
             put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
@@ -159,11 +201,19 @@ __device__ __forceinline__ void emit_v(const LinArgs &p, const KvSlot *at, bool 
 }
 
 // ---------------------------------------------------------------- up to 64 rows
-template <typename T, int MT, int NT, int WAVES, int KIND>
+// EX: a workgroup takes one row tile of one expert's map, for all of the expert's rows (grid.z: the experts that have any).
+template <typename T, int MT, int NT, int WAVES, int KIND, bool EX>
 __global__ void __launch_bounds__(64 * WAVES) linear_few_kernel(LinArgs p) {
     typedef typename Vec8<T>::type A8;
     __shared__ f32x4 red[WAVES][NT * MT][64];
-    if constexpr (KIND == VX_LIN_PLAIN) take_group<T>(p);
+    int mt = MT;  // 16-row tiles that have rows
+    if constexpr (EX) {  // (n is a multiple of 32: both of a workgroup's row tiles exist)
+        if (!take_tile(p, blockIdx.z) || (int)blockIdx.x * NT >= p.n >> 4) return;
+        mt = (p.rows - p.row0 + 15) >> 4;
+    } else if constexpr (KIND == VX_LIN_PLAIN) {
+        take_group<T>(p);
+    }
+    const int row0 = EX ? p.row0 : 0;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int steps = p.k >> 5, slices = gridDim.y, slice = blockIdx.y;
     const int s0 = (int)((int64_t)steps * slice / slices), s1 = (int)((int64_t)steps * (slice + 1) / slices);
@@ -171,7 +221,7 @@ __global__ void __launch_bounds__(64 * WAVES) linear_few_kernel(LinArgs p) {
     const bf16 *w = (const bf16 *)p.w + ((size_t)tile * steps) * 512 + lane * 8;
     const T *a[MT];
 #pragma unroll
-    for (int m = 0; m < MT; m++) a[m] = (const T *)p.a + a_row(p, min(m * 16 + (lane & 15), p.rows - 1)) * p.lda + (lane >> 4) * 8;
+    for (int m = 0; m < MT; m++) a[m] = (const T *)p.a + a_row(p, min(row0 + m * 16 + (lane & 15), p.rows - 1)) * p.lda + (lane >> 4) * 8;
     f32x4 acc[NT][MT];
 #pragma unroll
     for (int t = 0; t < NT; t++)
@@ -188,14 +238,16 @@ __global__ void __launch_bounds__(64 * WAVES) linear_few_kernel(LinArgs p) {
             for (int t = 0; t < NT; t++)
                 wf[u][t] = __builtin_nontemporal_load((const bf16x8 *)(w + ((size_t)t * steps + s + u * WAVES) * 512));
 #pragma unroll
-            for (int m = 0; m < MT; m++) af[u][m] = *(const A8 *)(a[m] + (size_t)(s + u * WAVES) * 32);
+            for (int m = 0; m < MT; m++)
+                if (!EX || m < mt) af[u][m] = *(const A8 *)(a[m] + (size_t)(s + u * WAVES) * 32);
         }
 #pragma unroll
         for (int u = 0; u < U; u++)
 #pragma unroll
             for (int t = 0; t < NT; t++)
 #pragma unroll
-                for (int m = 0; m < MT; m++) acc[t][m] = mma(wf[u][t], af[u][m], acc[t][m]);
+                for (int m = 0; m < MT; m++)
+                    if (!EX || m < mt) acc[t][m] = mma(wf[u][t], af[u][m], acc[t][m]);
     }
     for (; s < s1; s += WAVES) {
         bf16x8 wf[NT];
@@ -203,6 +255,7 @@ __global__ void __launch_bounds__(64 * WAVES) linear_few_kernel(LinArgs p) {
         for (int t = 0; t < NT; t++) wf[t] = __builtin_nontemporal_load((const bf16x8 *)(w + ((size_t)t * steps + s) * 512));
 #pragma unroll
         for (int m = 0; m < MT; m++) {
+            if (EX && m >= mt) break;
             const A8 af = *(const A8 *)(a[m] + (size_t)s * 32);
 #pragma unroll
             for (int t = 0; t < NT; t++) acc[t][m] = mma(wf[t], af, acc[t][m]);
@@ -216,16 +269,17 @@ __global__ void __launch_bounds__(64 * WAVES) linear_few_kernel(LinArgs p) {
     constexpr int ITEMS = (KIND == VX_LIN_SWIGLU ? 1 : NT) * MT * 64;
     for (int i = threadIdx.x; i < ITEMS; i += 64 * WAVES) {
         const int l = i & 63, tm = i >> 6, t = tm / MT, m = tm % MT;
+        if (EX && m >= mt) continue;
         f32x4 v = red[0][tm][l];
 #pragma unroll
         for (int x = 1; x < WAVES; x++) v += red[x][tm][l];
-        const int row = m * 16 + (l & 15);
+        const int row = row0 + m * 16 + (l & 15);
         if constexpr (KIND == VX_LIN_SWIGLU) {
             f32x4 u = red[0][MT + m][l];
 #pragma unroll
             for (int x = 1; x < WAVES; x++) u += red[x][MT + m][l];
 #pragma unroll
-            for (int r = 0; r < 4; r++) v[r] = silu_f(v[r]) * u[r];
+            for (int r = 0; r < 4; r++) v[r] = glu(p.o, v[r], u[r]);
             emit<T, KIND>(p, slice, row, (tile / 2) * 16 + (l >> 4) * 4, v);
         } else {
             emit<T, KIND>(p, slice, row, (tile + t) * 16 + (l >> 4) * 4, v);
@@ -234,7 +288,8 @@ __global__ void __launch_bounds__(64 * WAVES) linear_few_kernel(LinArgs p) {
 }
 
 // ---------------------------------------------------------------- more rows
-template <typename T, int BM, int BN, int KIND>
+// EX: a row tile is a tile of one expert's places.
+template <typename T, int BM, int BN, int KIND, bool EX>
 __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_tiles) {
     typedef typename Vec8<T>::type A8;
     constexpr int EPC = 16 / (int)sizeof(T);           // elements of a 16-byte piece
@@ -243,11 +298,12 @@ __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_til
     constexpr int MI = BM / 32, NI = BN / 32;          // 16-wide tiles per wave in each direction
     typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
     extern __shared__ u32x4 lds[];                     // [2][BM][CPR], pieces of a row permuted by the row's low bits
-    if constexpr (KIND == VX_LIN_PLAIN) take_group<T>(p);
+    if constexpr (KIND == VX_LIN_PLAIN && !EX) take_group<T>(p);
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int wm = (wave & 1) * (BM / 2), wn = (wave >> 1) * NI;
     const int rt = blockIdx.x % row_tiles, nt = blockIdx.x / row_tiles;  // the row tiles of one weight tile run together
-    const int m0 = rt * BM, tile0 = nt * (BN / 16);
+    if (EX && (!take_tile(p, rt) || nt * BN >= p.n)) return;
+    const int m0 = EX ? p.row0 : rt * BM, tile0 = nt * (BN / 16);
     const int n_tiles = p.n >> 4;
     const int ktiles = p.k >> 6, slices = gridDim.y, slice = blockIdx.y;
     const int k0 = (int)((int64_t)ktiles * slice / slices), k1 = (int)((int64_t)ktiles * (slice + 1) / slices);
@@ -362,7 +418,7 @@ __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_til
                 if (tile0 + wn + t >= n_tiles) continue;
                 f32x4 v;
 #pragma unroll
-                for (int r = 0; r < 4; r++) v[r] = silu_f(acc[t][m][r]) * acc[t + 1][m][r];
+                for (int r = 0; r < 4; r++) v[r] = glu(p.o, acc[t][m][r], acc[t + 1][m][r]);
                 emit<T, KIND>(p, slice, row, (tile0 + wn + t) / 2 * 16 + q4, v);
             }
         } else {
@@ -373,7 +429,7 @@ __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_til
     }
 }
 
-// Adds up the slices of a VX_LIN_SPLIT or VX_LIN_ROTARY map and deals the columns to its two results.
+// Adds up the slices of a VX_LIN_SPLIT, VX_LIN_ROTARY or VX_LIN_SILU map and deals the columns to its two results.
 template <typename T>
 __global__ void __launch_bounds__(256) split_sum_kernel(const float *part, int slices, int rows, int n, vx_linear_out o) {
     const int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x;
@@ -382,6 +438,9 @@ __global__ void __launch_bounds__(256) split_sum_kernel(const float *part, int s
     const float *src = part + (size_t)row * n + c;
     f32x4 v = *(const f32x4 *)src;
     for (int s = 1; s < slices; s++) v += *(const f32x4 *)(src + (size_t)s * rows * n);
+    if (c < o.split && o.kind == VX_LIN_SILU)
+#pragma unroll
+        for (int r = 0; r < 4; r++) v[r] = silu_f(v[r]);
     if (c < o.split)
         put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, o.rot_tab ? turned(o, row, c, v) : v);
     else
@@ -404,7 +463,7 @@ __global__ void fill_zero_kernel(uint32_t *p, size_t n) {
 // ---------------------------------------------------------------- launches
 template <typename T, int MT, int NT, int WAVES, int KIND>
 void launch_few_as(vx_backend *be, const LinArgs &p, int slices) {
-    linear_few_kernel<T, MT, NT, WAVES, KIND><<<dim3((p.n >> 4) / NT, slices, p.o.groups), 64 * WAVES, 0, be->stream>>>(p);
+    linear_few_kernel<T, MT, NT, WAVES, KIND, false><<<dim3((p.n >> 4) / NT, slices, p.o.groups), 64 * WAVES, 0, be->stream>>>(p);
 }
 template <typename T, int MT, int KIND>
 void launch_few(vx_backend *be, const LinArgs &p, int slices) {
@@ -425,7 +484,7 @@ void launch_few(vx_backend *be, const LinArgs &p, int slices) {
 template <typename T, int BM, int BN, int KIND>
 void launch_many(vx_backend *be, const LinArgs &p, int slices) {
     const int rt = ceil_div(p.rows, BM), nt = ceil_div(p.n, BN);
-    linear_many_kernel<T, BM, BN, KIND><<<dim3(rt * nt, slices, p.o.groups), 256, 2 * BM * 64 * sizeof(T), be->stream>>>(p, rt);
+    linear_many_kernel<T, BM, BN, KIND, false><<<dim3(rt * nt, slices, p.o.groups), 256, 2 * BM * 64 * sizeof(T), be->stream>>>(p, rt);
 }
 
 // The widest tiles that still give every compute unit a workgroup.
@@ -490,9 +549,35 @@ int dispatch(vx_backend *be, const LinArgs &p, int slices) {
         case VX_LIN_KV: return launch<T, VX_LIN_KV>(be, p, slices);
         case VX_LIN_SPLIT: return launch<T, VX_LIN_SPLIT>(be, p, slices);
         case VX_LIN_ROTARY: return launch<T, VX_LIN_ROTARY>(be, p, slices);
+        case VX_LIN_SILU: return launch<T, VX_LIN_SILU>(be, p, slices);
         case VX_LIN_V: return launch<T, VX_LIN_V>(be, p, slices);
         default: return launch<T, VX_LIN_SOFTPLUS>(be, p, slices);
     }
+}
+
+// Experts' maps. Up to 64 rows in the step: an expert's rows are one tile, and every active expert's weights are read once.
+template <typename T, int KIND>
+int launch_experts(vx_backend *be, const LinArgs &p, int step_rows, int max_tiles, int tile_rows) {
+    const int n = std::max(p.n, p.n_shared);
+    if (step_rows <= 64) {
+        constexpr int NT = 2;
+        const dim3 grid(ceil_div(n >> 4, NT), 1, max_tiles);
+        if (step_rows <= 16)
+            linear_few_kernel<T, 1, NT, 8, KIND, true><<<grid, 512, 0, be->stream>>>(p);
+        else if (step_rows <= 32)
+            linear_few_kernel<T, 2, NT, 8, KIND, true><<<grid, 512, 0, be->stream>>>(p);
+        else
+            linear_few_kernel<T, 4, NT, 4, KIND, true><<<grid, 256, 0, be->stream>>>(p);
+    } else if (sizeof(T) == 2 && tile_rows == 128) {
+        if constexpr (sizeof(T) == 2)
+            linear_many_kernel<T, 128, 128, KIND, true><<<max_tiles * ceil_div(n, 128), 256, 2 * 128 * 64 * sizeof(T), be->stream>>>(p, max_tiles);
+    } else if constexpr (sizeof(T) == 2) {
+        linear_many_kernel<T, 64, 128, KIND, true><<<max_tiles * ceil_div(n, 128), 256, 2 * 64 * 64 * sizeof(T), be->stream>>>(p, max_tiles);
+    } else {
+        linear_many_kernel<T, 64, 64, KIND, true><<<max_tiles * ceil_div(n, 64), 256, 2 * 64 * 64 * sizeof(T), be->stream>>>(p, max_tiles);
+    }
+    VX_CHECK_LAUNCH();
+    return VX_OK;
 }
 
 }  // namespace
@@ -564,13 +649,14 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
     VX_REQUIRE(n >= 16 && n % 16 == 0 && k >= 64 && k % 64 == 0 && lda >= k && lda % 8 == 0 && (uintptr_t)a % 16 == 0 &&
                    (uintptr_t)w % 16 == 0 && (uintptr_t)o->out % 16 == 0,
                "vx_linear: sizes or alignment (n %d, k %d, lda %d)", n, k, lda);
-    VX_REQUIRE(o->kind >= VX_LIN_PLAIN && o->kind <= VX_LIN_V, "vx_linear: unknown kind %d", o->kind);
+    VX_REQUIRE(o->kind >= VX_LIN_PLAIN && o->kind <= VX_LIN_SILU, "vx_linear: unknown kind %d", o->kind);
     VX_REQUIRE(o->cols >= 1 && o->ldo >= o->cols, "vx_linear: %d columns in rows of %d", o->cols, o->ldo);
     const int slices = o->slices > 1 ? o->slices : 1;
     VX_REQUIRE(slices == 1 || (o->kind == VX_LIN_PLAIN && o->out_f32 && slices <= 64), "vx_linear: slices need a plain float32 result");
     if (o->kind == VX_LIN_SWIGLU) {
         VX_REQUIRE(n % 32 == 0 && o->cols <= n / 2, "vx_linear: gate|up pairs of %d rows for %d columns", n, o->cols);
-    } else if (o->kind == VX_LIN_SPLIT) {
+        VX_REQUIRE(o->glu_limit >= 0.f, "vx_linear: negative limit");
+    } else if (o->kind == VX_LIN_SPLIT || o->kind == VX_LIN_SILU) {
         VX_REQUIRE(o->out2 && o->split % 16 == 0 && o->split > 0 && o->split < n && o->cols == o->split && o->ldo2 >= n - o->split &&
                        (uintptr_t)o->out2 % 16 == 0,
                    "vx_linear: bad split");
@@ -593,7 +679,9 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
                    "vx_linear: bad K/V columns");
     if (o->kind == VX_LIN_V) VX_REQUIRE(o->v_col == 0 && o->kv_heads * o->v_dim + 15 >= n, "vx_linear: columns beside V");
     VX_REQUIRE(o->softcap == 0.f || (o->softcap > 0.f && o->kind == VX_LIN_PLAIN && slices == 1), "vx_linear: a cap needs a plain whole result");
-    LinArgs p{a, w, lda, n, k, rows, *o};
+    LinArgs p;
+    memset(&p, 0, sizeof p);
+    p.a = a, p.w = w, p.lda = lda, p.n = n, p.k = k, p.rows = rows, p.o = *o;
     if (o->groups > 1) {
         VX_REQUIRE(o->kind == VX_LIN_PLAIN && slices == 1 && o->groups <= 65535 && o->a_group >= 0 && o->out_group >= o->cols &&
                        o->a_group % 8 == 0 && o->out_group % 4 == 0 && lda >= (o->groups - 1) * (int64_t)o->a_group + k &&
@@ -603,7 +691,7 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
         p.o.groups = 1;
     }
     if (o->kind != VX_LIN_ROTARY) p.o.rot_tab = nullptr;
-    if (o->kind == VX_LIN_SPLIT || o->kind == VX_LIN_ROTARY) {  // (narrow and deep as a rule) in slices, added up by a kernel of their own
+    if (o->kind == VX_LIN_SPLIT || o->kind == VX_LIN_ROTARY || o->kind == VX_LIN_SILU) {  // (narrow and deep as a rule) in slices, added up by a kernel of their own
         const int cut = k >= 2048 ? pick_slices(n, k, rows) : 1;  // (a short map is over before the second launch pays)
         if (cut > 1) {
             const size_t bytes = (size_t)cut * rows * n * 4;
@@ -622,6 +710,43 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
         }
     }
     return act == VX_ACT_BF16 ? dispatch<bf16>(be, p, slices) : dispatch<float>(be, p, slices);
+}
+
+int vx_route_tile_rows(int act, int rows, int experts, int top) {
+    if (rows <= 64 || act != VX_ACT_BF16) return 64;
+    return (int64_t)rows * top >= (int64_t)experts * 96 ? 128 : 64;
+}
+
+int vx_linear_experts(vx_backend *be, int act, const vx_experts_args *e) {
+    int rc = enter(be);
+    if (rc) return rc;
+    VX_REQUIRE(act == VX_ACT_F32 || act == VX_ACT_BF16, "vx_linear_experts: unknown activation type %d", act);
+    VX_REQUIRE(e && e->a && e->w && e->tiles && e->out && e->rows >= 1 && e->experts >= 1 && e->max_tiles >= 1, "vx_linear_experts: bad arguments");
+    VX_REQUIRE(e->kind == VX_LIN_PLAIN || e->kind == VX_LIN_SWIGLU, "vx_linear_experts: kind %d", e->kind);
+    VX_REQUIRE((e->rows <= 64 && e->tile_rows == 64) || (e->rows > 64 && (e->tile_rows == 64 || (e->tile_rows == 128 && act == VX_ACT_BF16))),
+               "vx_linear_experts: tiles of %d of %d rows", e->tile_rows, e->rows);
+    const int per = e->kind == VX_LIN_SWIGLU ? 2 : 1;  // outputs of a result column
+    const auto fits = [&](const void *w, int n, int k, int cols) {
+        return w && (uintptr_t)w % 16 == 0 && n >= 32 && n % 32 == 0 && k >= 64 && k % 64 == 0 && e->lda >= k && cols >= 1 && cols * per <= n &&
+               cols <= e->ldo;
+    };
+    VX_REQUIRE(fits(e->w, e->n, e->k, e->cols) && (!e->shared || fits(e->w_shared, e->n_shared, e->k_shared, e->cols_shared)) && e->lda % 8 == 0 &&
+                   (uintptr_t)e->a % 16 == 0 && (uintptr_t)e->out % 16 == 0,
+               "vx_linear_experts: sizes or alignment (n %d, k %d, lda %d)", e->n, e->k, e->lda);
+    VX_REQUIRE(e->glu_limit >= 0.f && e->shared_limit >= 0.f && e->max_tiles <= 65535 * 16, "vx_linear_experts: bad limit or tile count");
+    VX_REQUIRE(e->rows > 64 || e->max_tiles <= 65535, "vx_linear_experts: %d tiles", e->max_tiles);
+    LinArgs p;
+    memset(&p, 0, sizeof p);
+    p.a = e->a, p.w = e->w, p.lda = e->lda, p.n = e->n, p.k = e->k;
+    p.o.kind = e->kind, p.o.out = e->out, p.o.ldo = e->ldo, p.o.cols = e->cols, p.o.a_rows = e->a_rows, p.o.groups = 1;
+    p.o.glu_limit = e->glu_limit, p.o.glu_alpha = e->glu_alpha, p.o.glu_add = e->glu_add;
+    p.tiles = e->tiles, p.experts = e->experts;
+    if (e->shared) p.w_shared = e->w_shared, p.n_shared = e->n_shared, p.k_shared = e->k_shared, p.cols_shared = e->cols_shared, p.shared_limit = e->shared_limit;
+    if (e->kind == VX_LIN_SWIGLU)
+        return act == VX_ACT_BF16 ? launch_experts<bf16, VX_LIN_SWIGLU>(be, p, e->rows, e->max_tiles, e->tile_rows)
+                                  : launch_experts<float, VX_LIN_SWIGLU>(be, p, e->rows, e->max_tiles, e->tile_rows);
+    return act == VX_ACT_BF16 ? launch_experts<bf16, VX_LIN_PLAIN>(be, p, e->rows, e->max_tiles, e->tile_rows)
+                              : launch_experts<float, VX_LIN_PLAIN>(be, p, e->rows, e->max_tiles, e->tile_rows);
 }
 
 }  // extern "C"

@@ -22,6 +22,21 @@ __device__ __forceinline__ float block_sum(float v, float *sm) {
     return t;
 }
 
+// What row r's experts add to columns c ..: W is a vector of float32 columns.
+template <typename T, typename W>
+__device__ __forceinline__ void add_experts(const vx_residual_norm_args &p, int r, int c, W *x) {
+    const T *rows = (const T *)p.e_rows + c;
+    const auto read = [&](size_t place) {
+        if constexpr (sizeof(W) == 4) {
+            return (W)rows[place * p.lde];
+        } else {
+            return __builtin_convertvector(*(const typename Vec4<T>::type *)(rows + place * p.lde), f32x4);
+        }
+    };
+    for (int j = 0; j < p.e_top; j++) *x += p.e_weights[(size_t)r * p.e_top + j] * read(p.e_places[(size_t)r * p.e_top + j]);
+    if (p.e_shared >= 0) *x += read((size_t)p.e_shared + r);
+}
+
 // NV > 0: cols is a multiple of 4 and at most 4 * NV * blockDim.x, everything aligned: a row lives in registers.
 template <typename T, int NV>
 __global__ void __launch_bounds__(1024) residual_norm_kernel(vx_residual_norm_args p) {
@@ -53,17 +68,31 @@ __global__ void __launch_bounds__(1024) residual_norm_kernel(vx_residual_norm_ar
 #pragma unroll
                 for (int e = 0; e < 4; e++) ss = fmaf(y[v][e], y[v][e], ss);
             }
-            const float inv = 1.0f / sqrtf(block_sum(ss, sm) / (float)p.cols + p.eps);
+            if (p.w_post) {
+                const float inv = 1.0f / sqrtf(block_sum(ss, sm) / (float)p.cols + p.eps);
 #pragma unroll
-            for (int v = 0; v < NV; v++) {
-                const int c = tid + v * nt;
-                if (c < n4) {
-                    const f32x4 w = ((const f32x4 *)p.w_post)[c];
+                for (int v = 0; v < NV; v++) {
+                    const int c = tid + v * nt;
+                    if (c < n4) {
+                        const f32x4 w = ((const f32x4 *)p.w_post)[c];
 #pragma unroll
-                    for (int e = 0; e < 4; e++) x[v][e] = fmaf(p.mult, y[v][e] * inv * w[e], x[v][e]);
+                        for (int e = 0; e < 4; e++) x[v][e] = fmaf(p.mult, y[v][e] * inv * w[e], x[v][e]);
+                    }
+                }
+            } else {
+#pragma unroll
+                for (int v = 0; v < NV; v++) {
+                    const int c = tid + v * nt;
+                    if (c < n4 && p.y_bias) y[v] += ((const f32x4 *)p.y_bias)[c];
+#pragma unroll
+                    for (int e = 0; e < 4; e++) x[v][e] = fmaf(p.mult, y[v][e], x[v][e]);
                 }
             }
         }
+        if (p.e_rows)
+#pragma unroll
+            for (int v = 0; v < NV; v++)
+                if (tid + v * nt < n4) add_experts<T>(p, r, (tid + v * nt) * 4, &x[v]);
         float ss = 0.f;
 #pragma unroll
         for (int v = 0; v < NV; v++) {
@@ -96,7 +125,7 @@ __global__ void __launch_bounds__(1024) residual_norm_kernel(vx_residual_norm_ar
             return t;
         };
         float inv_y = 0.f;
-        if (p.y) {
+        if (p.y && p.w_post) {
             float ss = 0.f;
             for (int c = tid; c < p.cols; c += nt) {
                 const float t = yat(c);
@@ -106,7 +135,8 @@ __global__ void __launch_bounds__(1024) residual_norm_kernel(vx_residual_norm_ar
         }
         auto xat = [&](int c) {
             float t = xr[c];
-            if (p.y) t = fmaf(p.mult, yat(c) * inv_y * p.w_post[c], t);
+            if (p.y) t = fmaf(p.mult, p.w_post ? yat(c) * inv_y * p.w_post[c] : p.y_bias ? yat(c) + p.y_bias[c] : yat(c), t);
+            if (p.e_rows) add_experts<T>(p, r, c, &t);
             return ar ? t + ar[c] : t;
         };
         float ss = 0.f;
@@ -563,7 +593,7 @@ template <typename T>
 void launch_norm(vx_backend *be, const vx_residual_norm_args &p) {
     const auto al = [](const void *q) { return (uintptr_t)q % 16 == 0; };
     const bool vec = p.cols % 4 == 0 && al(p.x_in) && al(p.add) && al(p.x_out) && al(p.y) && al(p.w_post) && al(p.w_pre) &&
-                     al(p.out) && (!p.y || (p.ldy % 4 == 0 && p.y_stride % 4 == 0)) && (!p.w_pre || p.ldo % 4 == 0);
+                     al(p.out) && al(p.y_bias) && al(p.e_rows) && (!p.e_rows || p.lde % 4 == 0) && (!p.y || (p.ldy % 4 == 0 && p.y_stride % 4 == 0)) && (!p.w_pre || p.ldo % 4 == 0);
     const int n4 = p.cols / 4;
     // few rows: many threads each, so that a decode step's rows are short
     int threads = p.rows <= 256 ? 1024 : 256;
@@ -662,7 +692,8 @@ int vx_residual_norm(vx_backend *be, int act, const vx_residual_norm_args *a) {
     if (rc) return rc;
     VX_REQUIRE(a && a->rows >= 1 && a->cols >= 1 && a->x_in, "vx_residual_norm: bad arguments");
     VX_REQUIRE(act == VX_ACT_F32 || act == VX_ACT_BF16, "vx_residual_norm: unknown activation type %d", act);
-    VX_REQUIRE(!a->y || (a->w_post && a->y_slices >= 1 && a->ldy >= a->cols), "vx_residual_norm: incomplete sublayer output");
+    VX_REQUIRE(!a->y || (a->y_slices >= 1 && a->ldy >= a->cols && !(a->w_post && a->y_bias)), "vx_residual_norm: incomplete sublayer output");
+    VX_REQUIRE(!a->e_rows || (a->lde >= a->cols && a->e_top >= 0 && (a->e_top == 0 || (a->e_places && a->e_weights))), "vx_residual_norm: incomplete experts");
     VX_REQUIRE(!a->w_pre || (a->out && a->ldo >= a->cols), "vx_residual_norm: incomplete output");
     VX_REQUIRE(a->w_pre || a->x_out, "vx_residual_norm: nothing to write");
     if (act == VX_ACT_BF16)

@@ -14,6 +14,7 @@
 #include <sys/stat.h>
 #include <unistd.h>
 
+#include <functional>
 #include <utility>
 
 #include "model.h"
@@ -772,6 +773,290 @@ int check_tulipel(const Json &config) {
     return parse_tulipel(config, &c);
 }
 
+// ---------------------------------------------------------------- Kitodra
+struct KitodraLayer {
+    enum Kind { DIFFERENTIAL, KEY_VALUE, LIGHTNING } kind = LIGHTNING;
+    int weights_of = -1;          // >= 0: a layer whose tensors this one uses; the rest of its entry says the same
+    int heads = 1, kv_heads = 1, dim = 1, vdim = 1, mask = 0, rot_dims = 0;
+    double rot_base = 1.0;
+    float scale = 1.f, softcap = 0.f, diff = 0.f;
+    std::vector<double> decay;
+    bool experts = false, shared = false;
+    int n_experts = 1, top = 1, groups = 1, keep = 1, ff = 1, shared_ff = 1;
+    float limit = 0.f, shared_limit = 0.f;
+};
+struct KitodraConfig {
+    std::vector<KitodraLayer> layers;
+    std::vector<int> own;         // the layer whose tensors layer i uses
+    float eps = 1e-5f;
+    int vocab = 1, width = 1, buckets = 0;
+    int64_t mul_prev = 0, mul_cur = 0;
+};
+
+int parse_kitodra(const Json &j, KitodraConfig *c) {
+    int rc = VH_OK;
+    const Fields root("config", &j, &rc);
+    c->vocab = root.count("vocab");
+    c->width = root.count("width", 1, 1 << 20);
+    c->eps = (float)root.sub("norm").num("eps");
+    if (root.has("embedding") && root.sub("embedding").has("bigram")) {
+        const Fields p = root.sub("embedding").sub("bigram");
+        c->buckets = p.count("buckets", 1, 1 << 30);
+        c->mul_prev = p.count("mul_prev", 0, 0x7fffffff), c->mul_cur = p.count("mul_cur", 0, 0x7fffffff);
+    }
+    const Json *layers = root.need("layers", Json::ARR);
+    if (rc != VH_OK) return rc;
+    if (layers->arr.empty()) return fail("config.json: no layers");
+    for (size_t i = 0; i < layers->arr.size(); i++) {
+        const Fields l("layers[" + std::to_string(i) + "]", &layers->arr[i], &rc);
+        const Json *type = l.need("type", Json::STR);
+        if (rc != VH_OK) return rc;
+        KitodraLayer o;
+        if (type->str == "attention")
+            o.kind = KitodraLayer::DIFFERENTIAL;
+        else if (type->str == "attention_2")
+            o.kind = KitodraLayer::KEY_VALUE;
+        else if (type->str != "lightning")
+            return fail("config.json: layer %zu has the unknown mixer type '%s'", i, type->str.c_str());
+        if (l.has("weights_of")) o.weights_of = l.count("weights_of", 0, (int)layers->arr.size() - 1);
+        const Fields mx = l.sub("mixer");
+        const bool light = o.kind == KitodraLayer::LIGHTNING;
+        o.heads = mx.count("heads", 1, 4096);
+        o.dim = mx.count("dim", 1, light ? 512 : 2048), o.vdim = mx.count("vdim", 1, light ? 512 : 2048);
+        if (light) {
+            const Json *decay = mx.need("decay", Json::ARR);
+            if (rc != VH_OK) return rc;
+            for (const Json &d : decay->arr) {
+                if (d.type != Json::NUM || !(d.num >= 0.0 && d.num <= 1.0)) return fail("config.json: layer %zu: mixer.decay is not between 0 and 1", i);
+                o.decay.push_back(d.num);
+            }
+            if ((int)o.decay.size() != o.heads) return fail("config.json: layer %zu: mixer.decay holds %zu numbers for %d heads", i, o.decay.size(), o.heads);
+        } else {
+            o.kv_heads = mx.count("kv_heads", 1, 4096);
+            o.scale = (float)mx.num("scale");
+            if (mx.has("mask")) o.mask = mx.sub("mask").count("size", 1, 1 << 30);
+            if (mx.has("softcap")) {
+                o.softcap = (float)mx.num("softcap");
+                if (rc == VH_OK && !(o.softcap > 0.f)) return fail("config.json: layer %zu: mixer.softcap is not above 0", i);
+            }
+            if (o.kind == KitodraLayer::DIFFERENTIAL) o.diff = (float)mx.num("diff");
+            if (o.kind == KitodraLayer::KEY_VALUE && mx.has("rot")) {
+                const Fields rot = mx.sub("rot");
+                o.rot_dims = rot.count("dims", 0, 2048), o.rot_base = rot.num("base");
+            }
+        }
+        if (l.has("mlp")) {
+            const Fields mlp = l.sub("mlp"), router = mlp.sub("router"), expert = mlp.sub("expert");
+            const Json *kind = mlp.need("kind", Json::STR);
+            if (rc == VH_OK && kind->str != "moe") return fail("config.json: layer %zu has the unknown feed-forward '%s'", i, kind->str.c_str());
+            o.experts = true;
+            o.n_experts = router.count("experts", 1, 1024), o.top = router.count("top", 1, 1024);
+            if (router.has("groups")) {
+                const Fields g = router.sub("groups");
+                o.groups = g.count("count", 1, 1024), o.keep = g.count("keep", 1, 1024);
+            }
+            const auto cut = [&](const Fields &f) {
+                const float v = f.has("limit") ? (float)f.num("limit") : 0.f;
+                if (rc == VH_OK && f.has("limit") && !(v > 0.f)) rc = fail("config.json: %s.limit is not above 0", f.where.c_str());
+                return v;
+            };
+            o.ff = expert.count("ff", 1, 1 << 20), o.limit = cut(expert);
+            if (mlp.has("shared")) {
+                o.shared = true;
+                o.shared_ff = mlp.sub("shared").count("ff", 1, 1 << 20), o.shared_limit = cut(mlp.sub("shared"));
+            }
+        }
+        if (rc != VH_OK) return rc;
+        if (o.heads % o.kv_heads) return fail("config.json: layer %zu: %d heads are no multiple of %d", i, o.heads, o.kv_heads);
+        if (o.kind == KitodraLayer::KEY_VALUE && o.vdim != o.dim) return fail("config.json: layer %zu: keys of %d are values of %d", i, o.dim, o.vdim);
+        if (o.rot_dims % 2 || o.rot_dims > o.dim) return fail("config.json: layer %zu turns %d of %d dimensions", i, o.rot_dims, o.dim);
+        if (o.rot_dims > 0 && !(o.rot_base > 0.0)) return fail("config.json: layer %zu: rot.base is not above 0", i);
+        if (o.n_experts % o.groups || o.keep > o.groups) return fail("config.json: layer %zu: %d of %d groups of %d experts", i, o.keep, o.groups, o.n_experts);
+        if (o.top > (o.groups > 1 ? o.keep * (o.n_experts / o.groups) : o.n_experts))
+            return fail("config.json: layer %zu: %d of %d experts in %d groups", i, o.top, o.n_experts, o.keep);
+        c->layers.push_back(o);
+    }
+    for (size_t i = 0; i < c->layers.size(); i++) {
+        int at = (int)i;
+        for (size_t n = 0; c->layers[at].weights_of >= 0; n++) {
+            if (n == c->layers.size()) return fail("config.json: layer %zu: weights_of leads in a circle", i);
+            at = c->layers[at].weights_of;
+        }
+        const KitodraLayer &a = c->layers[i], &b = c->layers[at];
+        if (a.kind != b.kind || a.heads != b.heads || a.kv_heads != b.kv_heads || a.dim != b.dim || a.vdim != b.vdim || a.experts != b.experts)
+            return fail("config.json: layer %zu is of another kind than layer %d, whose weights it uses", i, at);
+        c->own.push_back(at);
+    }
+    return rc;
+}
+
+// A float32 logarithm of a decay that a kernel may multiply with any count of tokens: 0 becomes a decay that nothing outlives.
+float decay_log2(double d) { return d > 0.0 ? (float)fmax(log2(d), -1e4) : -1e4f; }
+
+int build_kitodra_attention(Builder &b, const KitodraLayer &s, const std::string &l, int W, int router_cols, MixModel *x, MixLayer *o, int *router_col) {
+    const std::string mix = l + "mix.";
+    const bool diff = s.kind == KitodraLayer::DIFFERENTIAL;
+    AttnMixer &a = o->attn;
+    o->has_attn = true;
+    a.by_heads = a.norm = true;
+    a.heads = s.heads, a.kv_heads = s.kv_heads, a.k_dim = s.dim, a.v_dim = s.vdim, a.scale = s.scale, a.softcap = s.softcap, a.maps = diff ? 2 : 1;
+    const int qd = s.heads * a.maps * s.dim, kd = s.kv_heads * a.maps * s.dim, vd = s.kv_heads * s.vdim, od = s.heads * s.vdim;
+    a.k_col = b.pad(qd, 16), a.v_col = diff ? a.k_col + b.pad(kd, 16) : -1;
+    *router_col = diff ? a.v_col + b.pad(vd, 16) : a.k_col + b.pad(kd, 16);
+    VHC(b.packed(&o->in, *router_col + router_cols, W));
+    std::vector<float> bias(o->in.n, 0.f), v;
+    const auto part = [&](const char *name, int n, int col) -> int {
+        VHC(b.pack(mix + name, n, W, 0, n, o->in, col, 1, 0));
+        VHC(b.floats(mix + name + ".b", {n}, &v));
+        std::copy(v.begin(), v.end(), bias.begin() + col);
+        return VH_OK;
+    };
+    VHC(part("q", qd, a.q_col));
+    VHC(part("k", kd, a.k_col));
+    if (diff) VHC(part("v", vd, a.v_col));
+    VHC(b.upload(bias, &a.in_bias));
+    VHC(b.packed(&o->out, W, od));
+    VHC(b.pack(mix + "o", W, od, 0, W, o->out, 0, 1, 0));
+    VHC(b.vec(mix + "o.b", W, &o->out_bias));
+    if (diff) {
+        a.chunk = s.mask;
+        VHC(b.vec(mix + "q.norm", s.dim, &a.norm_q));
+        VHC(b.vec(mix + "k.norm", s.dim, &a.norm_k));
+        double sum[2] = {0, 0};
+        for (int n = 0; n < 2; n++) {
+            std::vector<float> q, k;
+            VHC(b.floats(mix + (n ? "lq2" : "lq1"), {s.dim}, &q));
+            VHC(b.floats(mix + (n ? "lk2" : "lk1"), {s.dim}, &k));
+            for (int d = 0; d < s.dim; d++) sum[n] += (double)q[d] * k[d];
+        }
+        a.diff_lambda = (float)(exp(sum[0]) - exp(sum[1]) + s.diff), a.diff_scale = 1.f - s.diff;
+    } else {
+        a.window = s.mask;
+        VHC(b.upload(std::vector<float>(s.heads, 0.f), &a.sink));
+        if (s.rot_dims > 0) {
+            Rotation r;
+            double both;
+            rotary_frequencies(s.rot_dims, s.rot_base, false, 0, 0, 0, 0, &r.freqs, &both);
+            for (size_t k = 0; k < x->rotations.size(); k++)
+                if (x->rotations[k].freqs == r.freqs) a.rotation = (int)k;
+            if (a.rotation < 0) {
+                a.rotation = (int)x->rotations.size();
+                x->rotations.push_back(r);
+            }
+        }
+    }
+    return VH_OK;
+}
+
+int build_kitodra_lightning(Builder &b, const KitodraLayer &s, const std::string &l, int W, int router_cols, MixLayer *o, int *router_col) {
+    const std::string mix = l + "mix.";
+    DecayMixer &t = o->decay;
+    o->has_decay = true;
+    t.heads = s.heads, t.vdim = s.vdim, t.dim_pad = b.pad(s.dim, 32), t.v_pad = b.pad(s.vdim, 16);
+    const int qs = s.heads * t.dim_pad, vs = s.heads * t.v_pad, vd = s.heads * s.vdim;
+    t.split = 2 * qs + vs, t.g_col = 0;
+    *router_col = vs;
+    VHC(b.packed(&o->in, t.split + vs + router_cols, W));
+    // heads of `dim` rows spread to heads of `to`
+    const auto spread = [&](const char *name, int dim, int to, int row0) {
+        return b.pack_rows(mix + name, s.heads * dim, W, s.heads * to, o->in, row0, [&](int r) { return r % to < dim ? r / to * dim + r % to : -1; });
+    };
+    VHC(spread("q", s.dim, t.dim_pad, 0));
+    VHC(spread("k", s.dim, t.dim_pad, qs));
+    VHC(spread("v", s.vdim, t.v_pad, 2 * qs));
+    VHC(spread("g", s.vdim, t.v_pad, t.split));
+    std::vector<float> w, wp(vs, 0.f), decay;
+    VHC(b.floats(mix + "norm", {vd}, &w));
+    for (int i = 0; i < vd; i++) wp[i / s.vdim * t.v_pad + i % s.vdim] = w[i];
+    VHC(b.upload(wp, &t.norm));
+    for (double d : s.decay) {
+        decay.push_back((float)(d - 1.0));
+        decay.push_back(decay_log2(d));
+    }
+    VHC(b.upload(decay, &t.decay));
+    VHC(b.packed(&o->out, W, vs));
+    return b.pack_placed(mix + "o", W, vd, W, vs, o->out, 0, [&](int r, int k) -> int64_t {
+        return k % t.v_pad < s.vdim ? (int64_t)r * vd + k / t.v_pad * s.vdim + k % t.v_pad : -1;
+    });
+}
+
+int build_kitodra_experts(Builder &b, const KitodraLayer &s, const std::string &mlp, int W, MixLayer *o) {
+    ExpertMlp &e = o->moe;
+    o->has_experts = true;
+    e.experts = s.n_experts, e.top = s.top, e.groups = s.groups, e.keep = s.keep, e.shared = s.shared;
+    e.limit = s.limit, e.shared_limit = s.shared_limit, e.alpha = 1.702f, e.add = 1.f;
+    VHC(b.vec(mlp + "correction", s.n_experts, &e.correction));
+    // n maps of that feed-forward size, one behind the other
+    const auto maps = [&](int n, int ff, const std::function<std::string(int)> &name, Linear *gate_up, Linear *down, int *ff_pad) -> int {
+        const int fp = *ff_pad = b.pad(ff, 64), wp = b.pad(W, 32);
+        VHC(b.packed(gate_up, n * 2 * fp, W));
+        VHC(b.packed(down, n * wp, ff));
+        for (int i = 0; i < n; i++) {
+            const std::string p = mlp + name(i);
+            VHC(b.pack(p + ".gate", ff, W, 0, ff, *gate_up, i * 2 * fp, 2, 0));
+            VHC(b.pack(p + ".up", ff, W, 0, ff, *gate_up, i * 2 * fp + 16, 2, 0));
+            VHC(b.pack(p + ".down", W, ff, 0, W, *down, i * wp, 1, 0));
+        }
+        gate_up->n /= n, down->n /= n;
+        return VH_OK;
+    };
+    VHC(maps(s.n_experts, s.ff, [](int i) { return "e" + std::to_string(i); }, &e.gate_up, &e.down, &e.ff_pad));
+    if (s.shared) VHC(maps(1, s.shared_ff, [](int) { return std::string("shared"); }, &e.shared_gate_up, &e.shared_down, &e.shared_pad));
+    return VH_OK;
+}
+
+int build_kitodra(Builder &b, const Json &config, MixModel *x, vh_config *cfg) {
+    KitodraConfig c;
+    VHC(parse_kitodra(config, &c));
+    cfg->hidden = c.width, cfg->vocab = c.vocab, cfg->eps = c.eps;
+    x->eps = c.eps;
+    const int W = c.width;
+    std::vector<int> place(c.layers.size(), -1);  // of a layer with tensors of its own, in the program
+    for (size_t i = 0; i < c.layers.size(); i++) {
+        if (c.own[i] != (int)i) continue;
+        const KitodraLayer &s = c.layers[i];
+        const std::string l = "l" + std::to_string(i) + ".";
+        MixLayer o;
+        VHC(b.vec(l + "norm1", W, &o.norm1));
+        int router_col = 0;
+        const int router_cols = s.experts ? s.n_experts : 0;
+        if (s.kind == KitodraLayer::LIGHTNING) {
+            VHC(build_kitodra_lightning(b, s, l, W, router_cols, &o, &router_col));
+            x->recurrent = true;
+        } else {
+            VHC(build_kitodra_attention(b, s, l, W, router_cols, x, &o, &router_col));
+        }
+        if (s.experts) {
+            VHC(b.pack(l + "mlp.router", s.n_experts, W, 0, s.n_experts, o.in, (o.has_decay ? o.decay.split : 0) + router_col, 1, 0));
+            VHC(build_kitodra_experts(b, s, l + "mlp.", W, &o));
+            o.moe.router_col = router_col;
+        }
+        place[i] = (int)x->layers.size();
+        x->layers.push_back(o);
+    }
+    for (size_t i = 0; i < c.layers.size(); i++) {
+        LayerRun r;
+        r.layer = place[c.own[i]];
+        x->runs.push_back(r);
+    }
+    std::vector<float> emb;
+    VHC(b.floats("embed", {c.vocab, W}, &emb));
+    VHC(b.upload(emb, &b.m->embedding));
+    if (c.buckets > 0) {
+        VHC(b.floats("bigram", {c.buckets + 1, W}, &emb));
+        VHC(b.upload(emb, &x->pairs));
+        x->buckets = c.buckets, x->mul_prev = c.mul_prev, x->mul_cur = c.mul_cur;
+    }
+    VHC(b.vec("final.norm", W, &b.m->final_norm));
+    VHC(b.packed(&x->head, c.vocab, W));
+    return b.pack("embed", c.vocab, W, 0, c.vocab, x->head, 0, 1, 0);
+}
+
+int check_kitodra(const Json &config) {
+    KitodraConfig c;
+    return parse_kitodra(config, &c);
+}
+
 // ---------------------------------------------------------------- registry
 struct Architecture {
     const char *name;                                                    // config.json "architecture"
@@ -781,6 +1066,7 @@ struct Architecture {
 const Architecture kArchitectures[] = {
     {"Lozedra", check_lozedra, build_lozedra},
     {"Tulipel", check_tulipel, build_tulipel},
+    {"Kitodra", check_kitodra, build_kitodra},
 };
 
 const Architecture *find_architecture(const Json &config) {

@@ -3,6 +3,9 @@
 // A step is a set of sequences with any number of new tokens each. Its rows run through every layer together:
 //   norm | input projection (K and V leave for the paged pool on the way) | attention and / or convolution + scan | output
 //   projection | norm, residual, norm | gate|up with SiLU | down | norm, residual, and the next layer's norm
+// or, with a mixer and experts that read the same normed input,
+//   norm | input projection with the router | routing | heads to their places, attention, or decaying states with their norm and
+//   gate | output projection | experts' gate|up | down | residual with all of them, and the next layer's norm
 // or, with the norm behind the residual sum and latent attention,
 //   input projection (queries turned on the way) | norms, latents to the paged pool | queries into the latents' space |
 //   attention | results out of it | output projection | residual, norm | up | activation | down | residual, norm, average
@@ -23,16 +26,22 @@ namespace {
 int pad_to(int n, int m) { return (n + m - 1) / m * m; }
 size_t esize(const MixModel &x) { return x.act == VX_ACT_F32 ? 4 : 2; }
 
+int by_heads_ldq(const AttnMixer &t) { return pad_to(t.heads * t.maps * t.k_dim, 8); }
+
 struct Widths {
     int width_pad = 0, in = 0, out = 0, xc = 0, dtr = 0, bc = 0, dt = 0, act = 0;
     int qc = 0, qa = 0, rot = 0;
+    int o = 0, e_act = 0, e_out = 0, top = 0, places = 0, experts = 0;  // top, places: of a row
 };
 
 Widths widths(const vh_model *m) {
     Widths w;
     w.width_pad = pad_to(m->cfg.hidden, 64);
     for (const MixLayer &l : m->mix->layers) {
-        w.in = std::max(w.in, l.has_latent ? l.latent.heads * l.latent.head_cols : l.in.n);
+        w.in = std::max(w.in, l.has_latent                    ? l.latent.heads * l.latent.head_cols
+                              : l.has_decay                     ? l.decay.split
+                              : l.has_attn && l.attn.by_heads ? by_heads_ldq(l.attn)
+                                                                : l.in.n);
         w.out = std::max(w.out, l.out.k);
         w.act = std::max(w.act, l.ff_pad);
         if (l.has_scan) {
@@ -44,6 +53,16 @@ Widths widths(const vh_model *m) {
         if (l.has_latent) {
             w.qc = std::max(w.qc, l.latent.q_up.k);
             w.qa = std::max(w.qa, l.latent.heads * l.latent.rank_pad);
+        }
+    }
+    for (const MixLayer &l : m->mix->layers) {
+        if (l.has_decay) w.o = std::max(w.o, l.decay.heads * l.decay.v_pad);
+        if (l.has_experts) {
+            const ExpertMlp &e = l.moe;
+            w.e_act = std::max({w.e_act, e.ff_pad, e.shared_pad});
+            w.e_out = std::max(w.e_out, e.down.n);
+            w.top = std::max(w.top, e.top), w.places = std::max(w.places, e.top + (e.shared ? 1 : 0));
+            w.experts = std::max(w.experts, e.experts);
         }
     }
     for (const Rotation &r : m->mix->rotations) w.rot += 2 * (int)r.freqs.size();
@@ -74,6 +93,8 @@ size_t slice_floats(const vh_model *m, int rows, bool up_to) {
     for (const MixLayer &l : m->mix->layers) {
         sliced(l.out, cols);
         sliced(l.down, cols);
+        if (l.has_attn && l.attn.by_heads) sliced(l.in, l.in.n);
+        if (l.has_decay) most = std::max(most, (size_t)rows * (l.in.n - l.decay.split));
         if (!l.has_latent) continue;
         if (l.latent.q_rank > 0)
             sliced(l.in, l.in.n);
@@ -99,7 +120,10 @@ int alloc_acts(vh_model *m, int rows, bool up_to, A &&alloc, MixActs *a) {
                     get(&a->bc, R * w.bc * 4) && get(&a->dt, R * w.dt * 4) && get(&a->act, R * w.act * es) &&
                     get(&a->y, slice_floats(m, rows, up_to) * 4) && (!loop || get(&a->emb, R * m->cfg.hidden * 4)) &&
                     get(&a->qc, R * w.qc * es) && get(&a->qa, R * w.qa * es) && get(&a->lo, R * w.qa * es) && get(&a->z, up_bytes(m, rows, up_to)) &&
-                    get(&a->rot, R * w.rot * 4) &&
+                    get(&a->rot, R * w.rot * 4) && get(&a->o, R * w.o * 4) && get(&a->e_act, R * w.places * w.e_act * es) &&
+                    get(&a->e_out, R * w.places * w.e_out * es) && get(&a->e_weights, R * w.top * 4) && get(&a->e_places, R * w.top * 4) &&
+                    get(&a->e_order, R * w.places * 4) &&
+                    get(&a->e_tiles, w.top > 0 ? (4 + 4 * (size_t)vx_route_max_tiles(rows, w.experts, w.top, 1, 64)) * 4 : 0) &&
                     (!m->mix->post_norm || get(&a->hist, R * m->cfg.hidden * (m->mix->runs.size() + 1) * 4));
     return ok ? (int)VH_OK : fail("activations of %d rows: %s", rows, vx_last_error());
 }
@@ -124,7 +148,7 @@ int mix_finish(vh_model *m) {
         m->kv.push_back(nullptr);
         if (l.has_attn) {
             // (what a kernel may read beyond a sequence's tokens is a finite number from the start)
-            r.kv = zeroed(vx_kv_block_elems(c.block_size, l.attn.kv_heads, l.attn.k_dim, l.attn.v_dim) * c.pool_blocks * es);
+            r.kv = zeroed(vx_kv_block_elems2(c.block_size, l.attn.kv_heads * l.attn.maps, l.attn.k_dim, l.attn.kv_heads, l.attn.v_dim) * c.pool_blocks * es);
             if (!r.kv) return fail("KV pool: %s", vx_last_error());
             m->kv.back() = r.kv;
         }
@@ -143,6 +167,18 @@ int mix_finish(vh_model *m) {
             if (!r.conv) return fail("convolution state: %s", vx_last_error());
             m->adopted.push_back(r.conv);
         }
+    }
+    for (LayerRun &r : x.runs) {
+        const MixLayer &l = x.layers[r.layer];
+        if (!l.has_decay) continue;
+        r.state = (float *)zeroed((size_t)c.max_seqs * l.decay.heads * l.decay.dim_pad * l.decay.v_pad * 4);
+        if (!r.state) return fail("decaying state: %s", vx_last_error());
+        m->adopted.push_back(r.state);
+    }
+    if (x.pairs) {
+        x.token_pool = (int32_t *)zeroed((size_t)c.block_size * c.pool_blocks * 4);
+        if (!x.token_pool) return fail("token pool: %s", vx_last_error());
+        m->adopted.push_back(x.token_pool);
     }
     for (Rotation &r : x.rotations) {
         void *p = vx_alloc_permanent(m->be, (r.freqs.size() * 8 + 15) / 16 * 16);
@@ -172,6 +208,127 @@ vx_linear_out plain(void *out, int out_f32, int ldo, int cols, int slices) {
 }
 
 void *at(void *p, size_t elems, size_t es) { return (char *)p + elems * es; }
+
+// a rotation's angles of the step's rows
+const float *rot_table(const MixModel &x, const MixActs &a, int rows, int rotation) {
+    if (rotation < 0) return nullptr;
+    size_t before = 0;
+    for (int i = 0; i < rotation; i++) before += x.rotations[i].freqs.size();
+    return a.rot + before * 2 * rows;
+}
+
+int rot_tables(vh_model *m, const vx_ragged &b, const MixActs &a) {
+    const MixModel &x = *m->mix;
+    for (size_t i = 0; i < x.rotations.size(); i++)
+        VXC(vx_rotary_table(m->be, b.token_pos, b.rows, (int)x.rotations[i].freqs.size(), x.rotations[i].d_freqs, x.rotations[i].factor,
+                            (float *)rot_table(x, a, b.rows, (int)i)));
+    return VH_OK;
+}
+
+int embed(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, float *out) {
+    const MixModel &x = *m->mix;
+    if (!x.pairs) {
+        VXC(vx_embedding(m->be, d_tokens, b.rows, m->embedding, out, m->cfg.vocab, m->cfg.hidden));
+        return VH_OK;
+    }
+    vx_pair_embedding_args e;
+    memset(&e, 0, sizeof e);
+    e.cols = m->cfg.hidden, e.vocab = m->cfg.vocab, e.buckets = x.buckets, e.mul_prev = x.mul_prev, e.mul_cur = x.mul_cur;
+    e.tokens = d_tokens, e.embed = m->embedding, e.pairs = x.pairs, e.token_pool = x.token_pool, e.out = out;
+    VXC(vx_pair_embedding(m->be, &b, &e));
+    return VH_OK;
+}
+
+// the experts of every row, from the router's logits z (float32, in slices)
+int run_router(vh_model *m, const MixLayer &l, int rows, const MixActs &a, const float *z, int slices, int ldz) {
+    const ExpertMlp &e = l.moe;
+    vx_route_args r;
+    memset(&r, 0, sizeof r);
+    r.rows = rows, r.experts = e.experts, r.top = e.top, r.groups = e.groups, r.keep = e.keep, r.shared = e.shared;
+    r.tile_rows = vx_route_tile_rows(m->mix->act, rows, e.experts, e.top);
+    r.z = z + e.router_col, r.z_slices = slices, r.ldz = ldz, r.z_stride = (int64_t)rows * ldz;
+    r.correction = e.correction, r.weights = a.e_weights, r.places = a.e_places, r.order = a.e_order, r.tiles = a.e_tiles;
+    VXC(vx_route(m->be, &r));
+    return VH_OK;
+}
+
+// a.h -> the chosen experts' results in a.e_out, by place
+int run_experts(vh_model *m, const MixLayer &l, int rows, const MixActs &a) {
+    const MixModel &x = *m->mix;
+    const ExpertMlp &e = l.moe;
+    vx_experts_args g;
+    memset(&g, 0, sizeof g);
+    g.rows = rows, g.experts = e.experts, g.shared = e.shared;
+    g.tile_rows = vx_route_tile_rows(m->mix->act, rows, e.experts, e.top);
+    g.max_tiles = vx_route_max_tiles(rows, e.experts, e.top, e.shared, g.tile_rows);
+    g.tiles = a.e_tiles;
+    g.kind = VX_LIN_SWIGLU, g.a = a.h, g.lda = pad_to(m->cfg.hidden, 64), g.a_rows = a.e_order;
+    g.w = e.gate_up.w, g.n = e.gate_up.n, g.k = e.gate_up.k, g.w_shared = e.shared_gate_up.w, g.n_shared = e.shared_gate_up.n, g.k_shared = e.shared_gate_up.k;
+    g.glu_limit = e.limit, g.shared_limit = e.shared_limit, g.glu_alpha = e.alpha, g.glu_add = e.add;
+    g.out = a.e_act, g.ldo = std::max(e.ff_pad, e.shared_pad), g.cols = e.ff_pad, g.cols_shared = e.shared_pad;
+    VXC(vx_linear_experts(m->be, x.act, &g));
+    g.kind = VX_LIN_PLAIN, g.a = a.e_act, g.lda = g.ldo, g.a_rows = nullptr;
+    g.w = e.down.w, g.n = e.down.n, g.k = e.down.k, g.w_shared = e.shared_down.w, g.n_shared = e.shared_down.n, g.k_shared = e.shared_down.k;
+    g.out = a.e_out, g.ldo = g.cols = g.cols_shared = e.down.n;
+    VXC(vx_linear_experts(m->be, x.act, &g));
+    return VH_OK;
+}
+
+int run_out(vh_model *m, const MixLayer &l, int rows, const MixActs &a, int *slices) {
+    *slices = vx_linear_slices(m->be, l.out.n, l.out.k, rows);
+    vx_linear_out o = plain(a.y, 1, l.out.n, l.out.n, *slices);
+    VXC(vx_linear(m->be, m->mix->act, a.cat, l.out.k, l.out.w, l.out.n, l.out.k, rows, &o));
+    return VH_OK;
+}
+
+// A layer of one mixer beside experts: a.h -> the mixer's output as `slices` partial sums in a.y, and the choice of experts.
+int run_beside_experts(vh_model *m, const LayerRun &r, const vx_ragged &b, const MixActs &a, int *slices) {
+    const MixModel &x = *m->mix;
+    const MixLayer &l = x.layers[r.layer];
+    const size_t es = esize(x);
+    const int rows = b.rows, width_pad = pad_to(m->cfg.hidden, 64), ldc = l.out.k;
+    if (l.has_decay) {
+        const DecayMixer &t = l.decay;
+        const int side = l.in.n - t.split, vs = t.heads * t.v_pad;
+        vx_linear_out o = plain(a.proj, 0, t.split, t.split, 1);
+        o.kind = VX_LIN_SILU;
+        o.split = t.split, o.out2 = a.y, o.ldo2 = side;
+        VXC(vx_linear(m->be, x.act, a.h, width_pad, l.in.w, l.in.n, l.in.k, rows, &o));
+        if (l.has_experts) VHC(run_router(m, l, rows, a, a.y, 1, side));
+        vx_decay_args d;
+        memset(&d, 0, sizeof d);
+        d.heads = t.heads, d.dim = t.dim_pad, d.vdim = t.v_pad, d.decay = t.decay;
+        d.q = a.proj, d.k = at(a.proj, (size_t)t.heads * t.dim_pad, es), d.v = at(a.proj, (size_t)2 * t.heads * t.dim_pad, es);
+        d.ldq = d.ldk = d.ldv = t.split;
+        d.state = r.state, d.out = a.o, d.ldo = vs;
+        VXC(vx_decay_attn(m->be, x.act, &b, &d));
+        VXC(vx_gated_norm(m->be, x.act, a.o, vs, a.y + t.g_col, side, t.norm, x.eps, rows, vs, t.heads * t.vdim, a.cat, ldc));
+        return run_out(m, l, rows, a, slices);
+    }
+    const AttnMixer &t = l.attn;
+    *slices = vx_linear_slices(m->be, l.in.n, l.in.k, rows);
+    vx_linear_out o = plain(a.y, 1, l.in.n, l.in.n, *slices);
+    VXC(vx_linear(m->be, x.act, a.h, width_pad, l.in.w, l.in.n, l.in.k, rows, &o));
+    if (l.has_experts) VHC(run_router(m, l, rows, a, a.y, *slices, l.in.n));
+    vx_heads_args h;
+    memset(&h, 0, sizeof h);
+    h.q_heads = t.heads * t.maps, h.k_heads = t.kv_heads * t.maps, h.v_heads = t.kv_heads, h.dim = t.k_dim, h.v_dim = t.v_dim;
+    h.y = a.y, h.y_slices = *slices, h.ldy = l.in.n, h.y_stride = (int64_t)rows * l.in.n, h.bias = t.in_bias;
+    h.q_col = t.q_col, h.k_col = t.k_col, h.v_col = t.v_col;
+    if (t.rotation >= 0) h.rot_pairs = (int)x.rotations[t.rotation].freqs.size(), h.rot_tab = rot_table(x, a, rows, t.rotation);
+    h.norm = t.norm, h.eps = x.eps, h.w_q = t.norm_q, h.w_k = t.norm_k;
+    h.q = a.proj, h.ldq = by_heads_ldq(t), h.pool = r.kv;
+    VXC(vx_heads_store(m->be, x.act, &b, &h));
+    if (t.heads * t.v_dim < ldc) VXC(vx_fill_zero(m->be, a.cat, (size_t)rows * ldc * es));
+    vx_attn_args at_;
+    memset(&at_, 0, sizeof at_);
+    at_.heads = t.heads, at_.kv_heads = t.kv_heads, at_.k_dim = t.k_dim, at_.v_dim = t.v_dim, at_.scale = t.scale, at_.sink = t.sink;
+    at_.window = t.window, at_.chunk = t.chunk, at_.softcap = t.softcap;
+    at_.maps = t.maps, at_.diff_lambda = t.diff_lambda, at_.diff_scale = t.diff_scale, at_.diff_eps = x.eps;
+    at_.q = a.proj, at_.ldq = h.ldq, at_.pool = r.kv, at_.out_scale = 1.f, at_.out = a.cat, at_.ldo = ldc;
+    VXC(vx_attn_ragged(m->be, x.act, &b, &at_));
+    return run_out(m, l, rows, a, slices);
+}
 
 // mixers of one layer run: a.h -> the sublayer's output as `slices` partial sums in a.y
 int run_mixers(vh_model *m, const LayerRun &r, const vx_ragged &b, const MixActs &a, int *slices) {
@@ -228,18 +385,7 @@ int run_mixers(vh_model *m, const LayerRun &r, const vx_ragged &b, const MixActs
         at_.pool = r.kv, at_.out_scale = t.out_scale, at_.out = a.cat, at_.ldo = ldc;
         VXC(vx_attn_ragged(m->be, x.act, &b, &at_));
     }
-    *slices = vx_linear_slices(m->be, l.out.n, l.out.k, rows);
-    o = plain(a.y, 1, l.out.n, l.out.n, *slices);
-    VXC(vx_linear(m->be, x.act, a.cat, ldc, l.out.w, l.out.n, l.out.k, rows, &o));
-    return VH_OK;
-}
-
-// a rotation's angles of the step's rows
-const float *rot_table(const MixModel &x, const MixActs &a, int rows, int rotation) {
-    if (rotation < 0) return nullptr;
-    size_t before = 0;
-    for (int i = 0; i < rotation; i++) before += x.rotations[i].freqs.size();
-    return a.rot + before * 2 * rows;
+    return run_out(m, l, rows, a, slices);
 }
 
 // latent attention of one layer run: a.h -> the sublayer's output as `slices` partial sums in a.y
@@ -323,10 +469,7 @@ int run_latent(vh_model *m, const LayerRun &r, const vx_ragged &b, const MixActs
         at_.q = a.proj, at_.ldq = q_cols, at_.pool = ex->kv, at_.out_scale = 1.f, at_.out = a.cat, at_.ldo = ldc, at_.min_rows = many;
         VXC(vx_attn_ragged(m->be, x.act, &eb, &at_));
     }
-    *slices = vx_linear_slices(m->be, l.out.n, l.out.k, rows);
-    vx_linear_out o = plain(a.y, 1, l.out.n, l.out.n, *slices);
-    VXC(vx_linear(m->be, x.act, a.cat, ldc, l.out.w, l.out.n, l.out.k, rows, &o));
-    return VH_OK;
+    return run_out(m, l, rows, a, slices);
 }
 
 int run_mlp(vh_model *m, const MixLayer &l, int rows, const MixActs &a, int *slices) {
@@ -362,15 +505,28 @@ int forward_pre_norm(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, c
     const vh_config &c = m->cfg;
     const int rows = b.rows, width_pad = pad_to(c.hidden, 64);
     float *emb = a.emb ? a.emb : a.x;
-    VXC(vx_embedding(m->be, d_tokens, rows, m->embedding, emb, c.vocab, c.hidden));
+    VHC(embed(m, b, d_tokens, emb));
+    VHC(rot_tables(m, b, a));
     vx_residual_norm_args s;
     memset(&s, 0, sizeof s);
     s.rows = rows, s.cols = c.hidden, s.x_in = emb, s.x_out = a.x, s.mult = x.mult, s.eps = x.eps, s.out = a.h, s.ldo = width_pad;
-    const float *post = nullptr;  // the norm that waits for the sublayer output in a.y
+    bool pending = false;         // a sublayer's output waits in a.y, for the norm `post` (or none)
+    const float *post = nullptr;
+    const MixLayer *beside = nullptr;  // whose experts' results wait in a.e_out
     int slices = 1;
-    auto seam = [&](const float *next, const float *add) {
-        s.y = post ? a.y : nullptr;
+    auto take = [&]() {
+        s.y = pending ? a.y : nullptr;
         s.w_post = post, s.y_slices = slices, s.ldy = pad_to(c.hidden, 16), s.y_stride = (int64_t)rows * s.ldy;
+        s.e_rows = nullptr, s.y_bias = nullptr;
+        if (!beside) return;
+        s.y_bias = beside->out_bias;
+        if (!beside->has_experts) return;
+        const ExpertMlp &e = beside->moe;
+        s.e_rows = a.e_out, s.lde = e.down.n, s.e_top = e.top, s.e_shared = e.shared ? rows * e.top : -1;
+        s.e_places = a.e_places, s.e_weights = a.e_weights;
+    };
+    auto seam = [&](const float *next, const float *add) {
+        take();
         s.add = add, s.w_pre = next;
         const int rc = vx_residual_norm(m->be, x.act, &s);
         s.x_in = a.x;
@@ -379,6 +535,14 @@ int forward_pre_norm(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, c
     for (const LayerRun &r : x.runs) {
         const MixLayer &l = x.layers[r.layer];
         VXC(seam(l.norm1, r.add_embedding ? emb : nullptr));
+        pending = true;
+        if (!l.norm1b) {
+            VHC(run_beside_experts(m, r, b, a, &slices));
+            if (l.has_experts) VHC(run_experts(m, l, rows, a));
+            post = nullptr, beside = &l;
+            continue;
+        }
+        beside = nullptr;
         VHC(run_mixers(m, r, b, a, &slices));
         post = l.norm1b;
         if (l.has_mlp) {
@@ -388,9 +552,8 @@ int forward_pre_norm(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, c
         }
     }
     if (n_want == 0) return VH_OK;
+    take();
     s.rows = n_want, s.row_idx = want, s.x_out = nullptr;
-    s.y_stride = (int64_t)rows * pad_to(c.hidden, 16);
-    s.y = post ? a.y : nullptr, s.w_post = post, s.y_slices = slices, s.ldy = pad_to(c.hidden, 16);
     s.add = nullptr, s.w_pre = m->final_norm;
     VXC(vx_residual_norm(m->be, x.act, &s));
     return VH_OK;
@@ -403,10 +566,8 @@ int forward_post_norm(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, 
     const MixModel &x = *m->mix;
     const vh_config &c = m->cfg;
     const int rows = b.rows, n_runs = (int)x.runs.size();
-    VXC(vx_embedding(m->be, d_tokens, rows, m->embedding, a.hist, c.vocab, c.hidden));
-    for (size_t i = 0; i < x.rotations.size(); i++)
-        VXC(vx_rotary_table(m->be, b.token_pos, rows, (int)x.rotations[i].freqs.size(), x.rotations[i].d_freqs, x.rotations[i].factor,
-                            (float *)rot_table(x, a, rows, (int)i)));
+    VHC(embed(m, b, d_tokens, a.hist));
+    VHC(rot_tables(m, b, a));
     vx_post_norm_args s;
     memset(&s, 0, sizeof s);
     s.rows = rows, s.cols = c.hidden, s.x_in = a.hist, s.eps = x.eps, s.alpha = x.alpha, s.out = a.h, s.ldo = pad_to(c.hidden, 64);

@@ -94,7 +94,9 @@ struct Linear {       // packed bfloat16 weights (vx_linear_pack), padded sizes
     int n = 0, k = 0;
 };
 
-struct AttnMixer {    // vx_attn_ragged; columns are places in the layer's input projection
+// vx_attn_ragged; columns are places in the layer's input projection. Keys and values leave for the pool in the projection's
+// epilogue, or (by_heads) queries, keys and values pass through vx_heads_store, from a float32 projection.
+struct AttnMixer {
     int heads = 0, kv_heads = 0, k_dim = 0, v_dim = 0;
     float scale = 1.f, temp_coef = 0.f;
     int temp_every = 0;
@@ -102,7 +104,33 @@ struct AttnMixer {    // vx_attn_ragged; columns are places in the layer's input
     int bias_len = 0;
     bool gate = false;
     float out_scale = 1.f;
-    int q_col = 0, k_col = 0, v_col = 0, g_col = 0;
+    int q_col = 0, k_col = 0, v_col = 0, g_col = 0;    // v_col < 0: values are keys as projected
+    bool by_heads = false, norm = false;
+    const float *in_bias = nullptr, *norm_q = nullptr, *norm_k = nullptr;
+    int rotation = -1;                                 // index in MixModel::rotations, halves of a head's first dimensions
+    int window = 0, chunk = 0;
+    float softcap = 0.f;
+    const float *sink = nullptr;
+    int maps = 1;                                      // 2: differential heads
+    float diff_lambda = 0.f, diff_scale = 1.f;
+};
+
+// vx_decay_attn and vx_gated_norm. Projection: q | k | v with SiLU, heads padded to dim_pad and v_pad columns; behind them, in float32, the
+// gate.
+struct DecayMixer {
+    int heads = 0, vdim = 0, dim_pad = 0, v_pad = 0;
+    int split = 0, g_col = 0;                          // columns of q | k | v; the gate's among the others
+    const float *decay = nullptr, *norm = nullptr;     // [heads][2]; [heads * v_pad]
+};
+
+// vx_route and vx_linear_experts over the layer's normed input; the router's logits are columns of the input projection's float32 part.
+struct ExpertMlp {
+    int experts = 0, top = 0, groups = 1, keep = 1;
+    bool shared = false;
+    int router_col = 0, ff_pad = 0, shared_pad = 0;
+    float limit = 0.f, shared_limit = 0.f, alpha = 0.f, add = 0.f;
+    const float *correction = nullptr;
+    Linear gate_up, down, shared_gate_up, shared_down; // the experts' one behind the other: n counts one expert's
 };
 
 struct ScanMixer {    // vx_conv_silu, the projections of its result, vx_selective_scan
@@ -114,7 +142,7 @@ struct ScanMixer {    // vx_conv_silu, the projections of its result, vx_selecti
     const float *dt_bias = nullptr, *a2 = nullptr, *d = nullptr;
 };
 
-struct Rotation {      // pairs (2i, 2i + 1) turn by position * freqs[i]; cosine and sine times factor
+struct Rotation {      // pair i turns by position * freqs[i]; cosine and sine times factor
     std::vector<double> freqs;
     float factor = 1.f;
     const double *d_freqs = nullptr;
@@ -140,11 +168,15 @@ struct LatentMixer {
 
 // x += mult * rms(mixers(rms(x) * norm1)) * norm1b, then the same around the MLP. The mixers of a layer read one input
 // projection and write one row, which one output projection takes. In a model with post_norm instead: x = rms(alpha * x +
-// mixer(x)) * norm1, x = rms(alpha * x + MLP(x)) * norm2, then the average over the depth.
+// mixer(x)) * norm1, x = rms(alpha * x + MLP(x)) * norm2, then the average over the depth. A layer with experts instead: x +=
+// mixer(h) + experts(h), h = rms(x) * norm1.
 struct MixLayer {
     const float *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr;
-    bool has_attn = false, has_scan = false, has_latent = false, has_mlp = false;
+    bool has_attn = false, has_scan = false, has_latent = false, has_decay = false, has_mlp = false, has_experts = false;
     AttnMixer attn;
+    DecayMixer decay;
+    ExpertMlp moe;
+    const float *out_bias = nullptr;   // of the output projection, in layers without norm1b
     LatentMixer latent;
     ScanMixer scan;
     Linear in, out;
@@ -159,7 +191,7 @@ struct LayerRun {     // one pass through a layer; every pass has its own cache 
     bool add_embedding = false;    // the embedding output is added to the stream first
     void *kv = nullptr;            // paged pool (owned by vh_model::kv, by the run that writes it)
     void *conv = nullptr;          // [max_seqs][taps - 1][channels]
-    float *state = nullptr;        // [max_seqs][channels][pad]
+    float *state = nullptr;        // [max_seqs][channels][pad], or [max_seqs][heads][dim_pad][v_pad]
 };
 
 struct MixActs {      // a step's activations for up to `rows` rows
@@ -168,6 +200,10 @@ struct MixActs {      // a step's activations for up to `rows` rows
     void *h = nullptr, *proj = nullptr, *cat = nullptr, *xc = nullptr, *dtr = nullptr, *act = nullptr;
     void *qc = nullptr, *qa = nullptr, *lo = nullptr, *z = nullptr;  // query latent; queries and results in the latents' space; up's output
     float *hist = nullptr, *rot = nullptr;                           // results of all layers; angle tables, one after the other
+    float *o = nullptr;                                              // what the decaying states gave
+    void *e_act = nullptr, *e_out = nullptr;                         // by place in the experts' order
+    float *e_weights = nullptr;
+    int32_t *e_places = nullptr, *e_order = nullptr, *e_tiles = nullptr;
 };
 
 // The sequences of a step whose keys and values are spelled out: their tokens, block after block, from row 0 on.
@@ -186,6 +222,10 @@ struct MixModel {
     float alpha = 1.f, softcap = 0.f;
     bool recurrent = false;        // a sequence is more than its blocks
     int expand_rows = 0;           // the smallest of the layers'
+    const float *pairs = nullptr;  // set: the embedding has a table of token pairs (vx_pair_embedding)
+    int buckets = 0;
+    int64_t mul_prev = 0, mul_cur = 0;
+    int32_t *token_pool = nullptr;
     std::vector<Rotation> rotations;
     std::vector<MixLayer> layers;
     std::vector<LayerRun> runs;

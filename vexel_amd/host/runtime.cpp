@@ -833,6 +833,7 @@ int vh_pool_block_table(vh_model *m, int64_t seq_id, int32_t *out, int cap) {
 
 int vh_pool_adopt_blocks(vh_model *m, int64_t seq_id, const int32_t *blocks, int num_blocks, int seq_len) {
     if (m->mix && m->mix->recurrent) return fail("vh_pool_adopt_blocks: a sequence of this model is more than its blocks (recurrent state)");
+    if (m->mix && m->mix->pairs) return fail("vh_pool_adopt_blocks: the model needs the tokens that the blocks hold");
     std::lock_guard<std::mutex> g(m->pool.mu);
     SeqState *s = find_seq(m, seq_id);
     if (!s) return fail("sequence %lld not found", (long long)seq_id);

@@ -120,6 +120,15 @@ SIGNATURES = {
     "vx_linear": (_i, [_vp, _i, _vp, _i, _vp, _i, _i, _i, _vp]),
     "vx_residual_norm": (_i, [_vp, _i, _vp]),
     "vx_kv_block_elems": (_sz, [_i, _i, _i, _i]),
+    "vx_kv_block_elems2": (_sz, [_i, _i, _i, _i, _i]),
+    "vx_route": (_i, [_vp, _vp]),
+    "vx_route_tile_rows": (_i, [_i, _i, _i, _i]),
+    "vx_route_max_tiles": (_i, [_i, _i, _i, _i, _i]),
+    "vx_linear_experts": (_i, [_vp, _i, _vp]),
+    "vx_pair_embedding": (_i, [_vp, _vp, _vp]),
+    "vx_heads_store": (_i, [_vp, _i, _vp, _vp]),
+    "vx_decay_attn": (_i, [_vp, _i, _vp, _vp]),
+    "vx_gated_norm": (_i, [_vp, _i, _vp, _i, _vp, _i, _vp, _f, _i, _i, _i, _vp, _i]),
     "vx_attn_ragged": (_i, [_vp, _i, _vp, _vp]),
     "vx_attn_ragged_fast": (_i, [_i, _i, _i, _i, _i, _i]),
     "vx_latent_pad": (_i, [_i]),
