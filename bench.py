@@ -980,6 +980,65 @@ def tulipel_report(be, only=None, use_graph=True):
             mr.close()
 
 
+# Shapes of --kitodra-report, of the widths above: a layer of each mixer. A row's experts with the shared one have the feed-forward
+# size of the Lozedra layers that stand beside them.
+KITODRA_SHAPES = {
+    "2048": dict(width=2048, heads=16, kv_heads=4, dim=128, experts=64, top=6, ff=704, shared=1408),
+    "4096": dict(width=4096, heads=32, kv_heads=8, dim=128, experts=32, top=6, ff=1792, shared=3584),
+}
+KITODRA_MIXERS = ("lightning", "attention_2", "attention")
+
+
+def write_kitodra(folder, width, heads, kv_heads, dim, experts, top, ff, shared, window=1024, chunk=8192, mixers=KITODRA_MIXERS, vocab=LOZEDRA_VOCAB):
+    """A Kitodra model of that shape with random weights, a layer per mixer (differential heads: two maps of dim / 2)."""
+    shapes = {"embed": (vocab, width), "bigram": (vocab + 1, width), "final.norm": (width,)}
+    mlp = {"kind": "moe", "expert": {"ff": ff, "limit": 7.0}, "shared": {"ff": shared, "limit": 7.0},
+           "router": {"experts": experts, "top": top, "groups": {"count": 8, "keep": 4}}}
+    entries = []
+    for i, kind in enumerate(mixers):
+        l, m = "l%d." % i, "l%d.mix." % i
+        maps, d = (2, dim // 2) if kind == "attention" else (1, dim)
+        mixer = {"heads": heads, "dim": d, "vdim": dim}
+        qd, kd, vd, od = heads * maps * d, kv_heads * maps * d, kv_heads * dim, heads * dim
+        if kind == "lightning":
+            mixer["decay"] = [math.exp(-2.0 ** (-8.0 * h / heads)) for h in range(1, heads + 1)]
+            shapes.update({m + "q": (od, width), m + "k": (od, width), m + "v": (od, width), m + "g": (od, width), m + "norm": (od,)})
+        else:
+            mixer.update(kv_heads=kv_heads, scale=d ** -0.5, mask={"size": chunk if kind == "attention" else window})
+            shapes.update({m + "q": (qd, width), m + "q.b": (qd,), m + "k": (kd, width), m + "k.b": (kd,), m + "o.b": (width,)})
+        if kind == "attention":
+            mixer.update(softcap=30.0, diff=0.5)
+            shapes.update({m + "v": (vd, width), m + "v.b": (vd,), m + "q.norm": (d,), m + "k.norm": (d,), m + "lq1": (d,), m + "lk1": (d,),
+                           m + "lq2": (d,), m + "lk2": (d,)})
+        elif kind == "attention_2":
+            mixer["rot"] = {"base": 10000.0, "dims": dim // 2}
+        shapes.update({m + "o": (width, od), l + "norm1": (width,), l + "mlp.router": (experts, width), l + "mlp.correction": (experts,)})
+        for name, n in [("e%d" % e, ff) for e in range(experts)] + [("shared", shared)]:
+            p = l + "mlp." + name
+            shapes.update({p + ".gate": (n, width), p + ".up": (n, width), p + ".down": (width, n)})
+        entries.append({"type": kind, "mixer": mixer, "mlp": mlp})
+    cfg = {"architecture": "Kitodra", "embedding": {"bigram": {"buckets": vocab, "mul_prev": 31, "mul_cur": 17}}, "layers": entries,
+           "norm": {"eps": 1e-5}, "vocab": vocab, "width": width}
+    write_folder(folder, cfg, shapes, lambda name, shape: (1.0, 0.05) if "norm" in name else (0.0, 0.02))
+
+
+def kitodra_report(be, only=None, use_graph=True):
+    """Decode and prefill rates of Kitodra layers at real sizes (random weights) beside Lozedra layers of the same width, heads
+    and feed-forward per row, the closest model. Runs as for --lozedra-report."""
+    rng = np.random.default_rng(2)
+    for name, c in KITODRA_SHAPES.items():
+        if only not in (None, name):
+            continue
+        n = len(KITODRA_MIXERS)
+        print("layers of width %s, %d of each model" % (name, n), flush=True)
+        loz = dict(LOZEDRA_SHAPES[name], layers=n)
+        for label, write in (("Kitodra bf16", lambda f: write_kitodra(f, **c)), ("Lozedra bf16", lambda f: write_lozedra(f, **loz))):
+            mr = load_written(be, write, **MIX_SIZES)
+            fill_contexts(mr, LOZEDRA_VOCAB, rng)
+            layer_rates(be, label, mr, list(range(MIX_SEQS)), n, LOZEDRA_VOCAB, MIX_CTX, 32, MIX_PORTIONS, use_graph, rng)
+            mr.close()
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -1012,6 +1071,9 @@ def main():
     ap.add_argument("--tulipel-report", nargs="?", const="all", choices=["all"] + list(TULIPEL_SHAPES),
                     help="decode and prefill rates of Tulipel layers at real sizes beside Lozedra layers of the same sizes, "
                          "then exit")
+    ap.add_argument("--kitodra-report", nargs="?", const="all", choices=["all"] + list(KITODRA_SHAPES),
+                    help="decode and prefill rates of Kitodra layers (one of each mixer) at real sizes beside Lozedra layers of the "
+                         "same sizes, then exit")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU: this build has no multi-GPU path (run with --gpus 1)", file=sys.stderr)
@@ -1038,6 +1100,9 @@ def main():
         return
     if args.tulipel_report:
         tulipel_report(be, None if args.tulipel_report == "all" else args.tulipel_report, use_graph=not args.no_graph)
+        return
+    if args.kitodra_report:
+        kitodra_report(be, None if args.kitodra_report == "all" else args.kitodra_report, use_graph=not args.no_graph)
         return
     ctx = ragged_contexts(n=args.seqs) if args.seqs != BATCH else ragged_contexts()
     nseq = len(ctx)

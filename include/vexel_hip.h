@@ -536,7 +536,7 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
 
 /* Mixtures of experts. vx_route chooses each row's experts and sorts the (row, choice) pairs by expert:
  *   s = sigmoid(z[r]), choice scores c = s + correction; with groups > 1 only experts of the `keep` groups (of neighbours) whose two
- *   largest choice scores have the largest sums; the `top` experts with the largest choice scores; weights[r][j] = s of the j-th.
+ *   largest choice scores have the largest sums; the `top` experts with the largest choice scores; weights[r][j] = s of the j-th, in the experts' order.
  * z: float32 in slices that are added up. A pair's place in the sorted order is places[r][j], and order[place] = r. With shared != 0
  * every row has one more place, rows * top + r, with an expert of its own, number `experts`. tiles (device int32[4 + 4 *
  * vx_route_max_tiles]): their count, then from tiles[4] on (expert, first place, places, 0) each; a tile holds at most tile_rows

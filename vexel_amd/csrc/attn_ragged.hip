@@ -44,6 +44,7 @@ struct Args {
     // decode
     const int32_t *items;
     int piece, pieces;
+    int from_start;    // pieces count from the sequence's start (else from the group of 32 that holds the first key seen)
     float *partial;
 };
 
@@ -409,7 +410,7 @@ __global__ void __launch_bounds__(256) prefill_kernel(Args a) {
 }
 
 template <int KD, int VD, int MAPS>
-__global__ void __launch_bounds__(256) decode_kernel(Args a) {
+__global__ void __launch_bounds__(256, VD <= 8 && MAPS * KD <= 6 ? 2 : 1) decode_kernel(Args a) {
     constexpr int QT = MAPS;
     extern __shared__ float s_dyn[];
     __shared__ float s_m[4][QT * 16], s_l[4][QT * 16];
@@ -426,8 +427,8 @@ __global__ void __launch_bounds__(256) decode_kernel(Args a) {
     const int row = a.one_token ? seq : a.cu[seq];
     if (!a.one_token && a.cu[seq + 1] - row != 1) return;
     const int len = a.kv_lens[seq], pos = len - 1, first = first_key(a.p, pos);
-    const int k_lo = first / 32 * 32 + piece * a.piece, k_hi = min(len, k_lo + a.piece);
-    if (k_lo >= len) return;
+    const int start = first / 32 * 32, p_lo = (a.from_start ? 0 : start) + piece * a.piece, k_lo = max(p_lo, start), k_hi = min(len, p_lo + a.piece);
+    if (k_lo >= k_hi) return;
     load_lut(a, g, s_lut);
     const int last_blk = pos / BS;
     const int32_t *bt = a.tables + (size_t)a.rows[seq] * a.max_blocks;
@@ -507,12 +508,13 @@ __global__ void __launch_bounds__(64) merge_kernel(Args a) {
     const int h = blockIdx.x, seq = blockIdx.y, vd = a.p.v_dim;
     const int row = a.one_token ? seq : a.cu[seq];
     if (!a.one_token && a.cu[seq + 1] - row != 1) return;
-    const int len = a.kv_lens[seq], n = (len - first_key(a.p, len - 1) / 32 * 32 + a.piece - 1) / a.piece;
+    const int len = a.kv_lens[seq], start = first_key(a.p, len - 1) / 32 * 32, skip = a.from_start ? start / a.piece : 0;  // pieces nobody sees
+    const int n = (len - (a.from_start ? skip * a.piece : start) + a.piece - 1) / a.piece;
     const float *src[MAPS];
     float m[MAPS], inv[MAPS];
 #pragma unroll
     for (int x = 0; x < MAPS; x++) {
-        src[x] = a.partial + (((size_t)seq * a.p.heads + h) * MAPS + x) * a.pieces * (vd + 2);
+        src[x] = a.partial + ((((size_t)seq * a.p.heads + h) * MAPS + x) * a.pieces + skip) * (vd + 2);
         m[x] = -INFINITY;
         for (int i = threadIdx.x; i < n; i += 64) m[x] = fmaxf(m[x], src[x][(size_t)i * (vd + 2)]);
 #pragma unroll
@@ -645,7 +647,8 @@ int run_fast(vx_backend *be, Args a, const vx_ragged *b) {
         be->split.batch = 0;  // (whatever an earlier call left there is gone)
         dim3 grid(a.p.kv_heads, a.pieces, b->n_seqs);
         // vx_pack_batch's list of pieces of 256 tokens, when it was made for this batch
-        if (a.piece == ATTN_TPW / 2 && a.p.window <= 0 && a.p.chunk <= 0 && be->items.valid && be->items.kv_lens == b->kv_lens && be->items.table_rows == b->table_rows &&
+        a.from_start = span == b->max_kv_len;  // (also when windows or chunks start somewhere: they are not much shorter)
+        if (a.piece == ATTN_TPW / 2 && a.from_start && be->items.valid && be->items.kv_lens == b->kv_lens && be->items.table_rows == b->table_rows &&
             be->items.batch == b->n_seqs && b->n_seqs * (int64_t)a.pieces <= 65535 &&
             2 * be->items.cap >= (size_t)b->n_seqs * a.pieces) {
             a.items = be->items.buf + (be->items.cap + 1) * 4;

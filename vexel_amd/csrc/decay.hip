@@ -30,7 +30,10 @@ struct DecayArgs {
     int n_seqs, one_token;
     int max_rows;     // step_kernel: sequences with more rows are left out
     int subs;         // sub-chunks of a chunk
-    float *h;         // [chunks][heads][dim][vdim]
+    // [chunks][heads][dim / 32][vdim / 16][64 lanes][8]: what a chunk adds to the state, in the order in which a wave's lanes hold it as
+    // an operand (lane: column lane % 16, rows 8 (lane / 16) ..); then, in its place, the state before the chunk as eight high and
+    // eight low bfloat16 parts per lane
+    float *h;
 };
 
 __device__ __forceinline__ void split(float v, bf16 *hi, bf16 *lo) {
@@ -162,50 +165,67 @@ __global__ void __launch_bounds__(256) chunk_kernel(DecayArgs a) {
             for (int v = 0; v < VB / 16; v++) {
                 if (v >= tiles) break;
                 const bf16x8 vt = column8(s_v, LDV, ks * 32, v * 16, lane);
-                acc[v] = mma(vt, hi, acc[v]);
-                acc[v] = mma(vt, lo, acc[v]);
+                acc[v] = mma(hi, vt, acc[v]);
+                acc[v] = mma(lo, vt, acc[v]);
             }
         }
     }
-    const int d = d0 + wave * 16 + (lane & 15);
+    // rows d0 + 16 wave + 4 (lane / 16) .. of columns lane % 16: four of the eight elements of a lane of the operand
+    const int d = d0 + wave * 16 + (lane >> 4) * 4;
     if (d >= p.dim) return;
-    float *out = a.h + (((size_t)blockIdx.x * p.heads + h) * p.dim + d) * p.vdim + v0 + (lane >> 4) * 4;
+    float *out = a.h + (size_t)(blockIdx.x * p.heads + h) * p.dim * p.vdim + ((size_t)(d >> 5) * (p.vdim >> 4) + (v0 >> 4)) * 512 +
+                 (((d & 31) >> 3) * 16 + (lane & 15)) * 8 + (d & 7);
 #pragma unroll
     for (int v = 0; v < VB / 16; v++)
-        if (v < tiles) *(f32x4 *)(out + v * 16) = acc[v];
+        if (v < tiles) *(f32x4 *)(out + v * 512) = acc[v];
 }
 
-// Four columns of a state row per thread.
+// Eight rows of one state column per thread: a lane's part of an operand.
 __global__ void __launch_bounds__(256) carry_kernel(DecayArgs a) {
     const vx_decay_args &p = a.p;
-    const int seq = blockIdx.x, h = blockIdx.y, per = p.dim * p.vdim, e = (blockIdx.z * 256 + threadIdx.x) * 4;
+    const int seq = blockIdx.x, h = blockIdx.y, per = p.dim * p.vdim, e = blockIdx.z * 256 + threadIdx.x;
     const int size = a.subs * SUB, rows = a.cu[seq + 1] - a.cu[seq], chunks = (rows + size - 1) / size;
-    if (rows <= FEW || e >= per) return;
+    if (rows <= FEW || e >= per / 8) return;
     int first = 0;
     for (int s = 0; s < seq; s++) {
         const int n = a.cu[s + 1] - a.cu[s];
         if (n > FEW) first += (n + size - 1) / size;
     }
-    float *state = p.state + ((size_t)a.slots[seq] * p.heads + h) * per + e;
-    float *hp = a.h + ((size_t)first * p.heads + h) * per + e;
+    const int lane = e & 63, tile = e >> 6, vt = p.vdim >> 4, d = tile / vt * 32 + (lane >> 4) * 8, v = tile % vt * 16 + (lane & 15);
+    float *state = p.state + ((size_t)a.slots[seq] * p.heads + h) * per + (size_t)d * p.vdim + v;
+    float *hp = a.h + (size_t)(first * p.heads + h) * per + (size_t)e * 8;
     const size_t step = (size_t)p.heads * per;
-    f32x4 S = a.pos[a.cu[seq]] > 0 ? *(const f32x4 *)state : f32x4{0.f, 0.f, 0.f, 0.f};
+    const bool old = a.pos[a.cu[seq]] > 0;
+    float S[8];
+#pragma unroll
+    for (int j = 0; j < 8; j++) S[j] = old ? state[(size_t)j * p.vdim] : 0.f;
     const float lg = p.decay[2 * h + 1], whole = __builtin_amdgcn_exp2f((float)size * lg);
     constexpr int U = 4;
     for (int k = 0; k < chunks; k += U) {
-        f32x4 own[U];
+        f32x4 own[U][2];
 #pragma unroll
-        for (int u = 0; u < U; u++) own[u] = *(const f32x4 *)(hp + (size_t)min(k + u, chunks - 1) * step);
+        for (int u = 0; u < U; u++)
+#pragma unroll
+            for (int x = 0; x < 2; x++) own[u][x] = *(const f32x4 *)(hp + (size_t)min(k + u, chunks - 1) * step + x * 4);
 #pragma unroll
         for (int u = 0; u < U; u++) {
             if (k + u >= chunks) break;
-            *(f32x4 *)(hp + (size_t)(k + u) * step) = S;
+            bf16x8 hi, lo;
+#pragma unroll
+            for (int j = 0; j < 8; j++) {
+                bf16 x, y;
+                split(S[j], &x, &y);
+                hi[j] = x, lo[j] = y;
+            }
+            bf16x8 *at = (bf16x8 *)(hp + (size_t)(k + u) * step);
+            at[0] = hi, at[1] = lo;
             const float f = k + u + 1 < chunks ? whole : __builtin_amdgcn_exp2f((float)(rows - (chunks - 1) * size) * lg);
 #pragma unroll
-            for (int r = 0; r < 4; r++) S[r] = fmaf(f, S[r], own[u][r]);
+            for (int j = 0; j < 8; j++) S[j] = fmaf(f, S[j], own[u][j >> 2][j & 3]);
         }
     }
-    *(f32x4 *)state = S;
+#pragma unroll
+    for (int j = 0; j < 8; j++) state[(size_t)j * p.vdim] = S[j];
 }
 
 __global__ void __launch_bounds__(256) out_kernel(DecayArgs a) {
@@ -234,31 +254,35 @@ __global__ void __launch_bounds__(256) out_kernel(DecayArgs a) {
 #pragma unroll
         for (int it = 0; it < 4; it++) acc[x][it] = f32x4{0.f, 0.f, 0.f, 0.f};
     if ((chunk > 0 || a.pos[row0] > 0) && wave * 2 < tiles) {  // (a chunk behind the first starts at a position above 0 as well)
-        const float *S = a.h + (((size_t)(first + chunk) * p.heads + h) * p.dim + q8) * p.vdim + v0 + l16;
+        const bf16x8 *S = (const bf16x8 *)(a.h + (size_t)((first + chunk) * p.heads + h) * p.dim * p.vdim) + lane * 2;
+        int tile[2];
+#pragma unroll
+        for (int x = 0; x < 2; x++) tile[x] = (v0 >> 4) + min(wave * 2 + x, tiles - 1);
+        bf16x8 hi[2], lo[2], qf[4];
+        const auto fetch = [&](int ds) {
+#pragma unroll
+            for (int x = 0; x < 2; x++) {
+                const bf16x8 *at = S + ((size_t)(ds >> 5) * (p.vdim >> 4) + tile[x]) * 128;
+                hi[x] = at[0], lo[x] = at[1];
+            }
+#pragma unroll
+            for (int it = 0; it < 4; it++) qf[it] = *(const bf16x8 *)(q + (size_t)min(i0 + it * 16 + l16, len - 1) * p.ldq + ds);
+        };
+        fetch(0);
         for (int ds = 0; ds < p.dim; ds += 32) {
-            float raw[2][8];
+            bf16x8 ch[2], cl[2], cq[4];
+#pragma unroll
+            for (int x = 0; x < 2; x++) ch[x] = hi[x], cl[x] = lo[x];
+#pragma unroll
+            for (int it = 0; it < 4; it++) cq[it] = qf[it];
+            if (ds + 32 < p.dim) fetch(ds + 32);
 #pragma unroll
             for (int x = 0; x < 2; x++)
 #pragma unroll
-                for (int j = 0; j < 8; j++) raw[x][j] = S[(size_t)(ds + j) * p.vdim + min(wave * 2 + x, tiles - 1) * 16];
-            bf16x8 qf[4];
-#pragma unroll
-            for (int it = 0; it < 4; it++) qf[it] = *(const bf16x8 *)(q + (size_t)min(i0 + it * 16 + l16, len - 1) * p.ldq + ds);
-#pragma unroll
-            for (int x = 0; x < 2; x++) {
-                bf16x8 hi, lo;
-#pragma unroll
-                for (int j = 0; j < 8; j++) {
-                    bf16 y, z;
-                    split(raw[x][j], &y, &z);
-                    hi[j] = y, lo[j] = z;
-                }
-#pragma unroll
                 for (int it = 0; it < 4; it++) {
-                    acc[x][it] = mma(hi, qf[it], acc[x][it]);
-                    acc[x][it] = mma(lo, qf[it], acc[x][it]);
+                    acc[x][it] = mma(ch[x], cq[it], acc[x][it]);
+                    acc[x][it] = mma(cl[x], cq[it], acc[x][it]);
                 }
-            }
         }
 #pragma unroll
         for (int it = 0; it < 4; it++) {
@@ -449,7 +473,7 @@ int vx_decay_attn(vx_backend *be, int act, const vx_ragged *b, const vx_decay_ar
         a.h = (float *)be->scan_ws;
         chunk_kernel<<<dim3(chunks, p->heads, ceil_div(p->vdim, VB) * ceil_div(p->dim, DB)), 256, 0, be->stream>>>(a);
         VX_CHECK_LAUNCH();
-        carry_kernel<<<dim3(b->n_seqs, p->heads, ceil_div(p->dim * p->vdim, 1024)), 256, 0, be->stream>>>(a);
+        carry_kernel<<<dim3(b->n_seqs, p->heads, ceil_div(p->dim * p->vdim, 2048)), 256, 0, be->stream>>>(a);
         VX_CHECK_LAUNCH();
         out_kernel<<<dim3(subs, p->heads, ceil_div(p->vdim, VB)), 256, 0, be->stream>>>(a);
         VX_CHECK_LAUNCH();

@@ -4,7 +4,9 @@
 //  * choose: a wave per row. Every lane ranks its experts among all by counting, so that nothing waits for a chain of maxima.
 //  * place: one workgroup counts, adds up and deals out places; its atomics are in LDS. The order of an expert's rows among
 //    themselves does not matter to anyone's result.
-// Few rows (a decode step): one workgroup does both.
+// Few rows (a decode step): one workgroup does both, and the choices stay in LDS between them.
+#include <type_traits>
+
 #include "ragged.h"
 
 using namespace vx;
@@ -13,49 +15,70 @@ namespace {
 
 constexpr int MAX_EXPERTS = 1024;
 constexpr int FEW = 64;            // rows that one workgroup chooses for
+constexpr int FEW_LDS = 48 * 1024; // bytes it may keep them in
 constexpr int THREADS = 1024;
 
-// c: [experts] choice scores of the row in LDS, s: its scores; both this wave's own.
-__device__ __forceinline__ void choose_row(const vx_route_args &p, int row, int lane, float *c, float *s, float *g, int32_t *chosen) {
-    const float *z = p.z + (size_t)row * p.ldz;
-    for (int e = lane; e < p.experts; e += 64) {
-        float t = z[e];
-        for (int k = 1; k < p.z_slices; k++) t += z[(size_t)k * p.z_stride + e];
-        t = 1.0f / (1.0f + expf(-t));
-        s[e] = t;
-        c[e] = p.correction ? t + p.correction[e] : t;
+__device__ __forceinline__ float score(const vx_route_args &p, int row, int e) {
+    const float *z = p.z + (size_t)row * p.ldz + e;
+    float t = z[0];
+#pragma unroll 4
+    for (int k = 1; k < p.z_slices; k++) t += z[(size_t)k * p.z_stride];
+    return 1.0f / (1.0f + expf(-t));
+}
+
+// How many of a[0 .. n - 1] come before element i, which is v: the larger ones, and with TIES equal ones of a lower index. Reads up to
+// three elements beyond n - 1, which have to be -infinity.
+template <bool TIES>
+__device__ __forceinline__ int rank_of(const float *a, int n, float v, int i) {
+    int rank = 0;
+#pragma unroll 4
+    for (int k = 0; k < n; k += 4) {
+        const f32x4 x = *(const f32x4 *)(a + k);
+#pragma unroll
+        for (int e = 0; e < 4; e++) rank += x[e] > v || (TIES && x[e] == v && k + e < i);
     }
-    __builtin_amdgcn_wave_barrier();
+    return rank;
+}
+
+__host__ __device__ __forceinline__ int up4(int n) { return (n + 3) & ~3; }
+
+// c: [up4(experts)] choice scores of the row in LDS, s: its scores, g: [up4(groups)]; this wave's own. chosen, weights: [top].
+__device__ __forceinline__ void choose_row(const vx_route_args &p, int lane, float *c, const float *s, float *g, int32_t *chosen, float *weights) {
     if (p.groups > 1) {
         const int size = p.experts / p.groups;
-        for (int i = lane; i < p.groups; i += 64) {
+        for (int i = lane; i < up4(p.groups); i += 64) {
             float a = -INFINITY, b = -INFINITY;
-            for (int k = 0; k < size; k++) {
-                const float v = c[i * size + k];
-                b = fmaxf(b, fminf(a, v));
-                a = fmaxf(a, v);
-            }
+            if (i < p.groups)
+#pragma unroll 4
+                for (int k = 0; k < size; k++) {
+                    const float v = c[i * size + k];
+                    b = fmaxf(b, fminf(a, v));
+                    a = fmaxf(a, v);
+                }
             g[i] = size > 1 ? a + b : a;
         }
         __builtin_amdgcn_wave_barrier();
         for (int e = lane; e < p.experts; e += 64) {
             const int own = e / size;
-            const float v = g[own];
-            int rank = 0;
-            for (int i = 0; i < p.groups; i++) rank += g[i] > v || (g[i] == v && i < own);
-            if (rank >= p.keep) c[e] = -INFINITY;
+            if (rank_of<true>(g, p.groups, g[own], own) >= p.keep) c[e] = -INFINITY;
         }
         __builtin_amdgcn_wave_barrier();
     }
-    for (int e = lane; e < p.experts; e += 64) {
-        const float v = c[e];
-        int rank = 0;
-        for (int i = 0; i < p.experts; i++) rank += c[i] > v || (c[i] == v && i < e);
-        if (rank < p.top) {
-            chosen[(size_t)row * p.top + rank] = e;
-            p.weights[(size_t)row * p.top + rank] = s[e];
+    // The experts that fewer than `top` others surpass, in the order of their numbers; more than `top` when the last of them has an
+    // equal: then equals rank by number.
+    const auto deal = [&](auto ties) {
+        int n = 0;
+        for (int e0 = 0; e0 < p.experts; e0 += 64) {
+            const int e = e0 + lane;
+            const bool takes = e < p.experts && rank_of<decltype(ties)::value>(c, p.experts, c[min(e, p.experts - 1)], e) < p.top;
+            const uint64_t mask = __ballot(takes);
+            const int slot = n + __popcll(mask & (((uint64_t)1 << lane) - 1));
+            if (takes && slot < p.top) chosen[slot] = e, weights[slot] = s[e];
+            n += __popcll(mask);
         }
-    }
+        return n;
+    };
+    if (deal(std::false_type()) != p.top) deal(std::true_type());
     __builtin_amdgcn_wave_barrier();
 }
 
@@ -106,12 +129,19 @@ __device__ __forceinline__ void place_rows(const vx_route_args &p, const int32_t
         for (int i = tid; i < p.rows; i += THREADS) p.order[pairs + i] = i;
 }
 
-// dynamic LDS: per wave [experts] choice scores | [experts] scores | [groups] sums
+// dynamic LDS: per wave choice scores | scores | groups' sums
 __global__ void __launch_bounds__(256) route_choose_kernel(vx_route_args p) {
     extern __shared__ float s_dyn[];
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, row = blockIdx.x * 4 + wave;
-    float *c = s_dyn + (size_t)wave * (2 * p.experts + p.groups);
-    if (row < p.rows) choose_row(p, row, lane, c, c + p.experts, c + 2 * p.experts, p.places);  // (nothing is shared between waves)
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, row = blockIdx.x * 4 + wave, ne = up4(p.experts);
+    float *c = s_dyn + (size_t)wave * (2 * ne + up4(p.groups)), *s = c + ne;
+    if (row >= p.rows) return;  // (nothing is shared between waves)
+    for (int e = lane; e < ne; e += 64) {
+        const float t = e < p.experts ? score(p, row, e) : 0.f;
+        s[e] = t;
+        c[e] = e < p.experts ? (p.correction ? t + p.correction[e] : t) : -INFINITY;
+    }
+    __builtin_amdgcn_wave_barrier();
+    choose_row(p, lane, c, s, s + ne, p.places + (size_t)row * p.top, p.weights + (size_t)row * p.top);
 }
 
 __global__ void __launch_bounds__(THREADS) route_place_kernel(vx_route_args p) {
@@ -119,14 +149,24 @@ __global__ void __launch_bounds__(THREADS) route_place_kernel(vx_route_args p) {
     place_rows(p, p.places, count, first, scan);
 }
 
+// dynamic LDS: [rows] choice scores | [rows] scores | per wave groups' sums | [rows][top] choices
 __global__ void __launch_bounds__(THREADS) route_few_kernel(vx_route_args p) {
     extern __shared__ float s_dyn[];
     __shared__ int count[MAX_EXPERTS], first[MAX_EXPERTS], scan[32];
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    float *c = s_dyn + (size_t)wave * (2 * p.experts + p.groups);
-    for (int row = wave; row < p.rows; row += THREADS / 64) choose_row(p, row, lane, c, c + p.experts, c + 2 * p.experts, p.places);
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, ne = up4(p.experts);
+    float *c = s_dyn, *s = c + p.rows * ne, *g = s + p.rows * ne;
+    int32_t *chosen = (int32_t *)(g + THREADS / 64 * up4(p.groups));
+    for (int i = threadIdx.x; i < p.rows * ne; i += THREADS) {
+        const int row = i / ne, e = i - row * ne;
+        const float t = e < p.experts ? score(p, row, e) : 0.f;
+        s[i] = t;
+        c[i] = e < p.experts ? (p.correction ? t + p.correction[e] : t) : -INFINITY;
+    }
     __syncthreads();
-    place_rows(p, p.places, count, first, scan);
+    for (int row = wave; row < p.rows; row += THREADS / 64)
+        choose_row(p, lane, c + row * ne, s + row * ne, g + wave * up4(p.groups), chosen + row * p.top, p.weights + (size_t)row * p.top);
+    __syncthreads();
+    place_rows(p, chosen, count, first, scan);
 }
 
 }  // namespace
@@ -151,11 +191,11 @@ int vx_route(vx_backend *be, const vx_route_args *p) {
                a.experts);
     VX_REQUIRE(a.top >= 1 && a.top <= (a.groups == 1 ? a.experts : a.keep * (a.experts / a.groups)), "vx_route: %d of %d experts", a.top, a.experts);
     VX_REQUIRE((int64_t)a.rows * (a.top + 1) < ((int64_t)1 << 30), "vx_route: %d rows", a.rows);
-    const size_t per = (size_t)(2 * a.experts + a.groups) * 4;
-    if (a.rows <= FEW && THREADS / 64 * per <= 48 * 1024) {
-        route_few_kernel<<<1, THREADS, THREADS / 64 * per, be->stream>>>(a);
+    const size_t few = ((size_t)a.rows * (2 * up4(a.experts) + a.top) + THREADS / 64 * up4(a.groups)) * 4;
+    if (a.rows <= FEW && few <= FEW_LDS) {
+        route_few_kernel<<<1, THREADS, few, be->stream>>>(a);
     } else {
-        route_choose_kernel<<<ceil_div(a.rows, 4), 256, 4 * per, be->stream>>>(a);
+        route_choose_kernel<<<ceil_div(a.rows, 4), 256, 4 * (size_t)(2 * up4(a.experts) + up4(a.groups)) * 4, be->stream>>>(a);
         VX_CHECK_LAUNCH();
         route_place_kernel<<<1, THREADS, 0, be->stream>>>(a);
     }

@@ -104,9 +104,83 @@ __global__ void __launch_bounds__(256) heads_kernel(HeadArgs a) {
         if (lane + i * 64 < dim) out[lane + i * 64] = (T)v[i];
 }
 
+// The same where everything is a multiple of four: LANES lanes take a head, four neighbouring elements each; 4 * LANES >= its
+// dimensions. A rotation's partner is LANES' lane rot_pairs / 4 further on.
+template <typename T, int LANES>
+__global__ void __launch_bounds__(256) heads4_kernel(HeadArgs a) {
+    const vx_heads_args &p = a.p;
+    const int64_t id = ((int64_t)blockIdx.x * 256 + threadIdx.x) / LANES;
+    const int row_ = (int)(id / a.units), unit = (int)(id - (int64_t)row_ * a.units), d = threadIdx.x % LANES * 4;
+    const bool live = row_ < a.rows;  // (all lanes stay for the shuffles)
+    const int row = live ? row_ : a.rows - 1;
+    const bool is_q = unit < p.q_heads, is_k = !is_q && unit < p.q_heads + p.k_heads;
+    const int h = is_q ? unit : is_k ? unit - p.q_heads : unit - p.q_heads - p.k_heads;
+    const int dim = is_q || is_k ? p.dim : p.v_dim, col = (is_q ? p.q_col : is_k ? p.k_col : p.v_col) + h * dim;
+    const bool in_head = d < dim;
+    f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (in_head) {
+        const float *y = p.y + (size_t)row * p.ldy + col + d;
+        v = *(const f32x4 *)y;
+#pragma unroll 4
+        for (int s = 1; s < p.y_slices; s++) v += *(const f32x4 *)(y + (size_t)s * p.y_stride);
+        if (p.bias) v += *(const f32x4 *)(p.bias + col + d);
+    }
+    const int kp = (p.dim + 7) & ~7;
+    const int slot = is_q ? 0 : a.slot_map[row], blk = is_q ? 0 : slot / a.block_size, in = slot - blk * a.block_size;
+    T *pool = (T *)p.pool + (size_t)blk * a.block_size * ((size_t)p.k_heads * kp + (size_t)p.v_heads * p.v_dim);
+    if (live && in_head && !is_q && (!is_k || p.v_col < 0)) {
+        T *vp = pool + (size_t)p.k_heads * a.block_size * kp + ((size_t)h * p.v_dim + d) * a.block_size + in;
+#pragma unroll
+        for (int e = 0; e < 4; e++) vp[(size_t)e * a.block_size] = (T)v[e];
+    }
+    if (p.rot_pairs > 0) {
+        const bool low = d < p.rot_pairs, turns = (is_q || is_k) && d < 2 * p.rot_pairs;
+        const int other = (threadIdx.x & 63) + (turns ? (low ? p.rot_pairs : -p.rot_pairs) / 4 : 0);
+        f32x4 o;
+#pragma unroll
+        for (int e = 0; e < 4; e++) o[e] = __shfl(v[e], other, 64);
+        if (turns) {
+            const float *tab = p.rot_tab + ((size_t)row * p.rot_pairs + (low ? d : d - p.rot_pairs)) * 2;
+            const f32x4 t0 = *(const f32x4 *)tab, t1 = *(const f32x4 *)(tab + 4);
+            const f32x4 c = f32x4{t0[0], t0[2], t1[0], t1[2]}, s = f32x4{t0[1], t0[3], t1[1], t1[3]};
+            v = low ? v * c - o * s : v * c + o * s;
+        }
+    }
+    if (p.norm) {
+        float ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < 4; e++) ss = fmaf(v[e], v[e], ss);
+#pragma unroll
+        for (int off = LANES / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+        const float inv = 1.0f / sqrtf(ss / (float)dim + p.eps);
+        const float *w = is_q ? p.w_q : p.w_k;
+        v *= inv;
+        if (w && in_head && (is_q || is_k)) v *= *(const f32x4 *)(w + d);
+    }
+    if (live && in_head && (is_q || is_k)) store4((is_q ? (T *)p.q + (size_t)row * p.ldq + h * dim : pool + ((size_t)h * a.block_size + in) * kp) + d, v);
+}
+
+template <typename T, int LANES>
+void launch_heads4(vx_backend *be, const HeadArgs &a) {
+    heads4_kernel<T, LANES><<<(unsigned)ceil_div64((int64_t)a.rows * a.units * LANES, 256), 256, 0, be->stream>>>(a);
+}
+
 template <typename T>
 void launch_heads(vx_backend *be, const HeadArgs &a) {
+    const vx_heads_args &p = a.p;
     const int wide = a.p.dim > a.p.v_dim ? a.p.dim : a.p.v_dim;
+    const auto al = [](const void *q) { return (uintptr_t)q % 16 == 0; };
+    if (p.dim % 4 == 0 && p.v_dim % 4 == 0 && p.ldy % 4 == 0 && p.q_col % 4 == 0 && p.k_col % 4 == 0 && (p.v_col < 0 || p.v_col % 4 == 0) &&
+        p.rot_pairs % 4 == 0 && p.ldq % 4 == 0 && (p.y_slices == 1 || p.y_stride % 4 == 0) && al(p.y) && al(p.bias) && al(p.rot_tab) && al(p.w_q) &&
+        al(p.w_k) && al(p.q) && al(p.pool) && wide <= 256) {
+        if (wide <= 64)
+            launch_heads4<T, 16>(be, a);
+        else if (wide <= 128)
+            launch_heads4<T, 32>(be, a);
+        else
+            launch_heads4<T, 64>(be, a);
+        return;
+    }
     const unsigned grid = (unsigned)a.rows * (unsigned)ceil_div(a.units, 4);
     if (wide <= 64)
         heads_kernel<T, 1><<<grid, 256, 0, be->stream>>>(a);
@@ -159,7 +233,7 @@ int vx_heads_store(vx_backend *be, int act, const vx_ragged *b, const vx_heads_a
     VX_REQUIRE(p->rot_pairs >= 0 && 2 * p->rot_pairs <= p->dim && (p->rot_pairs == 0 || p->rot_tab), "vx_heads_store: %d pairs in heads of %d", p->rot_pairs,
                p->dim);
     HeadArgs a{*p, b->slot_mapping, b->rows, b->block_size, p->q_heads + p->k_heads + (p->v_col < 0 ? 0 : p->v_heads)};
-    VX_REQUIRE((int64_t)b->rows * ceil_div(a.units, 4) < ((int64_t)1 << 31), "vx_heads_store: %d rows of %d heads", b->rows, a.units);
+    VX_REQUIRE((int64_t)b->rows * a.units < ((int64_t)1 << 31), "vx_heads_store: %d rows of %d heads", b->rows, a.units);
     if (act == VX_ACT_BF16)
         launch_heads<bf16>(be, a);
     else
