@@ -34,6 +34,7 @@ struct LinArgs {
     int experts, n_shared, k_shared, cols_shared;
     const void *w_shared;
     float shared_limit;
+    int common, shared_tiles;  // linear_many_kernel: workgroups for the columns that every tile has, and the shared expert's tiles
 };
 
 // The expert and the places of tile `t`; false beyond the last.
@@ -301,7 +302,14 @@ __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_til
     if constexpr (KIND == VX_LIN_PLAIN && !EX) take_group<T>(p);
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int wm = (wave & 1) * (BM / 2), wn = (wave >> 1) * NI;
-    const int rt = blockIdx.x % row_tiles, nt = blockIdx.x / row_tiles;  // the row tiles of one weight tile run together
+    // the row tiles of one weight tile run together, with experts on one die (workgroup ids are dealt to the eight dies in turn)
+    const int id = EX ? (int)(blockIdx.x & 7) * (int)(gridDim.x >> 3) + (int)(blockIdx.x >> 3) : (int)blockIdx.x;
+    int rt = id % row_tiles, nt = id / row_tiles;
+    if (EX && id >= p.common) {  // more columns of the shared expert, whose tiles are the last
+        if (p.shared_tiles == 0) return;
+        const int k = id - p.common;
+        rt = p.tiles[0] - p.shared_tiles + k % p.shared_tiles, nt = p.common / row_tiles + k / p.shared_tiles;
+    }
     if (EX && (!take_tile(p, rt) || nt * BN >= p.n)) return;
     const int m0 = EX ? p.row0 : rt * BM, tile0 = nt * (BN / 16);
     const int n_tiles = p.n >> 4;
@@ -555,6 +563,14 @@ int dispatch(vx_backend *be, const LinArgs &p, int slices) {
     }
 }
 
+template <typename T, int BM, int BN, int KIND>
+void launch_many_experts(vx_backend *be, LinArgs p, int step_rows, int max_tiles) {
+    const int nts = ceil_div(p.n, BN), more = p.n_shared > p.n ? ceil_div(p.n_shared, BN) - nts : 0;
+    p.common = max_tiles * nts, p.shared_tiles = more > 0 ? ceil_div(step_rows, BM) : 0;
+    const int grid = ceil_div(p.common + p.shared_tiles * more, 8) * 8;
+    linear_many_kernel<T, BM, BN, KIND, true><<<grid, 256, 2 * BM * 64 * sizeof(T), be->stream>>>(p, max_tiles);
+}
+
 // Experts' maps. Up to 64 rows in the step: an expert's rows are one tile, and every active expert's weights are read once.
 template <typename T, int KIND>
 int launch_experts(vx_backend *be, const LinArgs &p, int step_rows, int max_tiles, int tile_rows) {
@@ -570,11 +586,11 @@ int launch_experts(vx_backend *be, const LinArgs &p, int step_rows, int max_tile
             linear_few_kernel<T, 4, NT, 4, KIND, true><<<grid, 256, 0, be->stream>>>(p);
     } else if (sizeof(T) == 2 && tile_rows == 128) {
         if constexpr (sizeof(T) == 2)
-            linear_many_kernel<T, 128, 128, KIND, true><<<max_tiles * ceil_div(n, 128), 256, 2 * 128 * 64 * sizeof(T), be->stream>>>(p, max_tiles);
+            launch_many_experts<T, 128, 128, KIND>(be, p, step_rows, max_tiles);
     } else if constexpr (sizeof(T) == 2) {
-        linear_many_kernel<T, 64, 128, KIND, true><<<max_tiles * ceil_div(n, 128), 256, 2 * 64 * 64 * sizeof(T), be->stream>>>(p, max_tiles);
+        launch_many_experts<T, 64, 128, KIND>(be, p, step_rows, max_tiles);
     } else {
-        linear_many_kernel<T, 64, 64, KIND, true><<<max_tiles * ceil_div(n, 64), 256, 2 * 64 * 64 * sizeof(T), be->stream>>>(p, max_tiles);
+        launch_many_experts<T, 64, 64, KIND>(be, p, step_rows, max_tiles);
     }
     VX_CHECK_LAUNCH();
     return VX_OK;
