@@ -243,8 +243,8 @@ __device__ __forceinline__ float score_factor(const vx_attn_args &p, int pos) {
     return p.softcap > 0.f ? f * (2.0f / p.softcap) : f;
 }
 
-// Columns v * 16 + 4 (lane / 16) .. of the difference of two maps' results, normed over the head: o1, o2(v) are the lane's columns
-// of tile v, each to be multiplied by its inv; the head's columns lie in the four lanes lane % 16 + 16 i.
+// What the difference of two maps' results is multiplied with. diff(v): columns v * 16 + 4 (lane / 16) .. of it; the head's columns lie
+// in the four lanes lane % 16 + 16 i.
 template <int VD, class O>
 __device__ __forceinline__ float diff_factor(const Args &a, int lane, O &&diff) {
     float ss = 0.f;

@@ -1,5 +1,5 @@
-// The pieces of mixed-batch layers beside linear maps and attention: the norm | residual | norm seam, the residual | norm |
-// average over the depth seam, the normed polynomial activation, the causal depthwise convolution and the selective scan. All of them in float32 on activations that are bfloat16 or float32 (T).
+// The pieces of mixed-batch layers beside linear maps and attention: the norm | residual | norm seam (which also adds experts'
+// rows), the residual | norm | average over the depth seam, the normed polynomial activation, the causal depthwise convolution and the selective scan. All of them in float32 on activations that are bfloat16 or float32 (T).
 //
 // Scan: a lane keeps 8 states of one channel in registers, LP = padded / 8 neighbouring lanes make up the channel. A
 // sequence's rows are cut into chunks of CHUNK; where a sequence has several, a first pass finds what every chunk adds to
