@@ -507,7 +507,10 @@ enum {
                           rot_first + 2 * rot_pairs - 1 are turned in neighbouring pairs by rot_tab (vx_rotary_table); the
                           others (split = n: none) to out2 as with SPLIT */
     VX_LIN_V = 6,      /* every column is V of the pool (v_col 0), stored as with KV, four neighbouring slots at a time */
-    VX_LIN_SILU = 7    /* columns < split: silu(y) to out (activation type); the others, as they are, to out2 as with SPLIT */
+    VX_LIN_SILU = 7,   /* columns < split: silu(y) to out (activation type); the others, as they are, to out2 as with SPLIT */
+    VX_LIN_FORGET = 8, /* columns < silu_cols: silu(y) to out, < split: y to out (activation type); the others, c = column - split,
+                          to out2 as keep[c] * sigmoid(-(y + bias[c])): one minus a forget gate whose lower bound is 1 - keep */
+    VX_LIN_RELU2 = 9   /* out = max(y + bias[c], 0)^2 in the activation type (bias NULL: 0) */
 };
 typedef struct vx_linear_out {
     int kind, out_f32, ldo, cols, slices;
@@ -527,6 +530,9 @@ typedef struct vx_linear_out {
     int k_used;                  /* > 0: a K head's k_used first elements are what the map makes (kv_heads * k_used columns) */
     float glu_limit, glu_alpha, glu_add; /* glu_limit > 0 (SWIGLU): g = min(gate, limit), u = up cut to -limit .. limit, and
                                     out = g * sigmoid(glu_alpha * g) * (u + glu_add) */
+    int silu_cols;
+    const float *keep;
+    float mult;                  /* not 0 (PLAIN, one slice): y *= mult (ahead of the cap) */
 } vx_linear_out;
 /* out = a [rows, k] * W^T for a packed matrix [n, k] (padded sizes); a has lda >= k columns of the activation type, zero
  * where k was padded, rows 16-byte aligned. vx_linear_slices: into how many slices a PLAIN float32 result is best cut
@@ -537,6 +543,7 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
 /* Mixtures of experts. vx_route chooses each row's experts and sorts the (row, choice) pairs by expert:
  *   s = sigmoid(z[r]), choice scores c = s + correction; with groups > 1 only experts of the `keep` groups (of neighbours) whose two
  *   largest choice scores have the largest sums; the `top` experts with the largest choice scores; weights[r][j] = s of the j-th, in the experts' order.
+ *   softmax != 0: s = z[r] + bias instead (correction and groups as above), and the weights are the softmax over the chosen s.
  * z: float32 in slices that are added up. A pair's place in the sorted order is places[r][j], and order[place] = r. With shared != 0
  * every row has one more place, rows * top + r, with an expert of its own, number `experts`. tiles (device int32[4 + 4 *
  * vx_route_max_tiles]): their count, then from tiles[4] on (expert, first place, places, 0) each; a tile holds at most tile_rows
@@ -551,6 +558,8 @@ typedef struct vx_route_args {
     int32_t *places;             /* [rows][top] */
     int32_t *order;              /* [rows * (top + (shared != 0))] */
     int32_t *tiles;
+    const float *bias;           /* [experts], added to z; NULL: 0 */
+    int softmax;
 } vx_route_args;
 int vx_route(vx_backend *be, const vx_route_args *p);
 /* places of a tile as vx_linear_experts wants them for that many rows of a step; the most tiles vx_route may make of them */
@@ -559,7 +568,7 @@ int vx_route_max_tiles(int rows, int experts, int top, int shared, int tile_rows
 /* The experts' maps over the places that vx_route made: activation row of a place: a_rows[place], or the place itself (NULL); result
  * rows are places. Expert e < experts: the packed matrix [n, k] at w + e * n * k elements; expert `experts`: w_shared [n_shared,
  * k_shared], which may have another size (out rows then hold the larger of the two). SWIGLU (glu_* and, for the shared expert,
- * shared_limit; 0: its gate and up are not cut) or PLAIN in the activation type. n % 32 == 0. */
+ * shared_limit; 0: its gate and up are not cut), PLAIN or RELU2 (no bias) in the activation type. n % 32 == 0. */
 typedef struct vx_experts_args {
     int kind, rows, experts, shared, n, k, n_shared, k_shared, tile_rows, max_tiles;
     const void *a, *w, *w_shared;
@@ -624,7 +633,12 @@ typedef struct vx_attn_args {
     float softcap;               /* > 0: scores become softcap * tanh(score / softcap) (before the bias) */
     int maps;                    /* 2: differential attention, see below; 0 or 1: one map */
     float diff_lambda, diff_scale, diff_eps;
+    const float *slopes;         /* [heads]: slopes[h] * (i - j) is taken off a score (no bias table beside it); NULL: not */
+    const void *talk;            /* bfloat16 [heads][heads] on the device: scores mixed across heads, see below; NULL: not */
 } vx_attn_args;
+/* talk: score_h(i, j) = sum over g of talk[h][g] * (temp(i) * scale * q_i[g] . k_j[g's K/V head]), then bias, slopes, mask and softmax.
+ * (A slope per head that is taken off ahead of the mixing is the slope sum over g of talk[h][g] * slope[g] behind it.) One map, no
+ * cap; the products' scores enter the mixing as two bfloat16 parts, or in float32 with the plain kernel. */
 /* maps = 2: every head has two queries, and every K/V head two keys, side by side (head h, map m at (h * 2 + m) * k_dim); both maps
  * attend on their own to the K/V head's values, and with their results a1 and a2
  *   o = a1 - diff_lambda * a2,  out = diff_scale * o / sqrt(mean over v_dim of o^2 + diff_eps)      (no gate)
@@ -633,6 +647,7 @@ size_t vx_kv_block_elems(int block_size, int kv_heads, int k_dim, int v_dim);
 size_t vx_kv_block_elems2(int block_size, int k_heads, int k_dim, int v_heads, int v_dim);
 int vx_attn_ragged(vx_backend *be, int act, const vx_ragged *b, const vx_attn_args *p);
 /* 1 when the matrix-core kernels take the geometry, 0 when vx_attn_ragged uses the plain one. */
+int vx_attn_talk_fast(int act, int block_size, int heads, int kv_heads, int k_dim, int v_dim);   /* with talk */
 int vx_attn_ragged_fast(int act, int block_size, int heads, int kv_heads, int k_dim, int v_dim);
 
 /* ---- latent attention: a token is kept as one normed vector c [rank] and one rotated key part kr [rot_dim] for all heads.
@@ -706,6 +721,33 @@ typedef struct vx_post_norm_args {
 } vx_post_norm_args;
 int vx_post_norm(vx_backend *be, int act, const vx_post_norm_args *p);
 
+/* The seam behind a sublayer whose output is layer-normed before it joins the stream, one row at a time, in float32:
+ *   v = (y: sum over slices of y[s][r] + y_bias) (e_rows: + sum over j < e_top of e_weights[r][j] * e_rows[e_places[r][j]])
+ *   x = x_in[r] + ln(v; w, b)   (w NULL: x = x_in[r]);   x_out[r] = x (NULL: not)
+ *   out[i] = x, or ln(x; w_pre, b_pre), in the activation type, columns cols .. ldo - 1 zero
+ * ln(v; w, b) = (v - mean) / sqrt(mean((v - mean)^2) + eps) * w + b. r = row_idx ? row_idx[i] : i for i < rows. x_out may be x_in.
+ * tokens (w NULL, no row_idx): x = ln(x_in[tokens[r]] + positions[token_pos[r]]; w_pre, b_pre) goes to x_out and out alike. */
+typedef struct vx_branch_norm_args {
+    int rows, cols;
+    const int32_t *row_idx;
+    const float *x_in, *y, *y_bias;
+    int y_slices, ldy;
+    int64_t y_stride;
+    float eps;
+    const float *w, *b;
+    const void *e_rows;          /* activation type */
+    int lde, e_top;
+    const int32_t *e_places;
+    const float *e_weights;
+    float *x_out;
+    const float *w_pre, *b_pre;
+    void *out;
+    int ldo;
+    const int32_t *tokens, *token_pos;
+    const float *positions;
+} vx_branch_norm_args;
+int vx_branch_norm(vx_backend *be, int act, const vx_branch_norm_args *p);
+
 /* Polynomial activation normed over the row, in float32: out = coef[0] * N(z) + coef[1] * N(z^2) + coef[2] * N(z^3) + coef[3] with
  * N(u) = u / sqrt(mean over the row's cols columns of u^2 + eps), powers element by element. out: activation type; its columns
  * cols .. ldo - 1 become zero. z: activation type (z_slices 0), or float32 in so many slices, z_stride floats from one to the
@@ -744,7 +786,8 @@ int vx_pair_embedding(vx_backend *be, const vx_ragged *b, const vx_pair_embeddin
 /* Query, key and value heads from a float32 projection (slices added up, bias added) to where vx_attn_ragged reads them:
  *   queries and keys: dimensions i and i + rot_pairs (i < rot_pairs) turned by rot_tab (vx_rotary_table; rot_pairs 0: not), then, with norm,
  *   v / sqrt(mean(v^2) + eps) over the head, times w_q or w_k [dim] (NULL: 1)
- * Heads lie side by side from their column on: q_heads and k_heads of dim, v_heads of v_dim. Queries go to q (activation type, head h at h *
+ * (norm 2: over all the row's query heads at once, and over all its key heads; w_q [q_heads * dim], w_k [k_heads * dim])
+ * Heads lie side by side from their column on: q_heads and k_heads of dim, v_heads of v_dim (k_heads = v_heads = 0: queries alone). Queries go to q (activation type, head h at h *
  * dim), keys and values to the pool (layout: vx_kv_block_elems2) at slot_mapping[r]. v_col < 0: a value is its key head as
  * projected, before rotation and norm (v_heads = k_heads, v_dim = dim). */
 typedef struct vx_heads_args {
@@ -783,6 +826,29 @@ int vx_decay_attn(vx_backend *be, int act, const vx_ragged *b, const vx_decay_ar
  * zero. count: how many of the columns are not padding. */
 int vx_gated_norm(vx_backend *be, int act, const float *x, int ldx, const float *gate, int ldg, const float *w, float eps, int rows, int cols,
                   int count, void *out, int ldo);
+
+/* Linear attention with a forget gate per channel whose complement is what is written, over a mixed batch (states, gates and sums in
+ * float32):
+ *   S[d] = (1 - g[d]) * S[d] + g[d] * v,  out = S^T q,  S [dim][vdim] per head
+ * dim a multiple of 32 up to 512, vdim one of 16 up to 512 (in columns that pad a head q, g and v are zero). q, v: activation type, head h at
+ * columns h * dim and h * vdim, rows 16-byte aligned; g float32 [rows][ldg], 0 .. 1, head h at h * dim; out float32 [rows][ldo], head h at
+ * h * vdim. state [slots][heads][dim][vdim] float32. A sequence at position 0 starts from zero. */
+typedef struct vx_forget_args {
+    int heads, dim, vdim;
+    const void *q, *v;
+    const float *g;
+    int ldq, ldv, ldg;
+    float *state;
+    float *out;
+    int ldo;
+} vx_forget_args;
+int vx_forget_attn(vx_backend *be, int act, const vx_ragged *b, const vx_forget_args *p);
+/* 1 when prompts of that geometry take the matrix-core kernels, 0 when their rows are walked. */
+int vx_forget_attn_fast(int act, int dim, int vdim);
+/* out[r] = x[r], every head of vdim columns divided by its root mean square (sum of squares / count + eps) and multiplied by w [vdim]; x
+ * float32, out activation type, columns heads * vdim .. ldo - 1 zero. count: how many of a head's columns are not padding. */
+int vx_head_norm(vx_backend *be, int act, const float *x, int ldx, const float *w, float eps, int rows, int heads, int vdim, int count, void *out,
+                 int ldo);
 
 /* Selective scan over a mixed batch, all in float32:
  *   S[c][n] = exp(dt[c] * A[c][n]) * S[c][n] + dt[c] * x[c] * B[n];  y[c] = sum_n S[c][n] * C[n] + D[c] * x[c]

@@ -146,6 +146,9 @@ int vh_sample_last_logits(vh_model *m, int rows, const float *temperature, const
 int vh_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_lens, const int32_t *tokens, int n_want,
             const int32_t *want_rows, float *logits_out, int32_t *argmax_out);
 int vh_model_mixed_batches(const vh_model *m);
+/* How many tokens a sequence may hold because the model has no more positions; 0: no such limit. Steps beyond are refused; the
+ * scheduler refuses longer prompts and ends a sequence that gets there. */
+int vh_model_max_positions(const vh_model *m);
 /* Speculative verification of a whole candidate tree for each of n_seqs sequences in one forward pass, greedy
  * acceptance and rollback. The reference's runTreeMedusaDecodeStep (scheduler/medusa_scheduler.go:733-861)
  * handles one sequence and verifies only the most confident path with VerifySpeculativeWithPagedKV

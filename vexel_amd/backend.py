@@ -37,7 +37,8 @@ class VxRagged(C.Structure):
 class VxLinearOut(C.Structure):
     _fields_ = _fields("int kind out_f32 ldo cols slices; ptr out out2; int split ldo2; ptr bias; int k_col v_col kv_heads "
                        "k_dim v_dim block_size; ptr pool slot_mapping a_rows; float softcap; int groups a_group out_group "
-                       "rot_stride rot_first rot_pairs; ptr rot_tab; int k_used; float glu_limit glu_alpha glu_add")
+                       "rot_stride rot_first rot_pairs; ptr rot_tab; int k_used; float glu_limit glu_alpha glu_add; "
+                       "int silu_cols; ptr keep; float mult")
 
 
 class VxResidualNormArgs(C.Structure):
@@ -47,7 +48,7 @@ class VxResidualNormArgs(C.Structure):
 
 class VxRouteArgs(C.Structure):
     _fields_ = _fields("int rows experts top groups keep shared tile_rows; ptr z; int z_slices ldz; i64 z_stride; "
-                       "ptr correction weights places order tiles")
+                       "ptr correction weights places order tiles bias; int softmax")
 
 
 class VxExpertsArgs(C.Structure):
@@ -71,7 +72,7 @@ class VxDecayArgs(C.Structure):
 class VxAttnArgs(C.Structure):
     _fields_ = _fields("int heads kv_heads k_dim v_dim; float scale temp_coef; int temp_every; ptr bias; int bias_len; "
                        "ptr q gate; int ldq ldg; ptr pool; float out_scale; ptr out; int ldo; ptr sink; int min_rows window chunk; "
-                       "float softcap; int maps; float diff_lambda diff_scale diff_eps")
+                       "float softcap; int maps; float diff_lambda diff_scale diff_eps; ptr slopes talk")
 
 
 class VxLatentStoreArgs(C.Structure):
@@ -86,6 +87,15 @@ class VxLatentAttnArgs(C.Structure):
 class VxPostNormArgs(C.Structure):
     _fields_ = _fields("int rows cols; ptr row_idx x_in y; int y_slices ldy; i64 y_stride; float alpha eps; ptr w hist; "
                        "i64 hist_stride; ptr avg; int n_avg keep; ptr x_out w_pre out; int ldo")
+
+
+class VxBranchNormArgs(C.Structure):
+    _fields_ = _fields("int rows cols; ptr row_idx x_in y y_bias; int y_slices ldy; i64 y_stride; float eps; ptr w b e_rows; "
+                       "int lde e_top; ptr e_places e_weights x_out w_pre b_pre out; int ldo; ptr tokens token_pos positions")
+
+
+class VxForgetArgs(C.Structure):
+    _fields_ = _fields("int heads dim vdim; ptr q v g; int ldq ldv ldg; ptr state out; int ldo")
 
 
 class VxConvArgs(C.Structure):
@@ -522,6 +532,15 @@ class HipBackend:
 
     def poly_norm(self, act, z, ldz, rows, cols, coef, eps, out, ldo, z_slices=0, z_stride=0):
         self.call("vx_poly_norm", act, z, ldz, z_slices, z_stride, rows, cols, coef, eps, out, ldo)
+
+    def branch_norm(self, act, args):
+        self.call("vx_branch_norm", act, C.byref(args))
+
+    def forget_attn(self, act, batch, args):
+        self.call("vx_forget_attn", act, C.byref(batch), C.byref(args))
+
+    def head_norm(self, act, x, ldx, w, eps, rows, heads, vdim, count, out, ldo):
+        self.call("vx_head_norm", act, x, ldx, w, eps, rows, heads, vdim, count, out, ldo)
 
     def conv_silu(self, act, batch, args):
         self.call("vx_conv_silu", act, C.byref(batch), C.byref(args))

@@ -14,7 +14,7 @@ OBJ_DIR = os.path.join(HERE, "build")
 
 SOURCES = ["backend.hip", "elementwise.hip", "attention.hip", "qgemm.hip", "qstream.hip", "qmatvec.hip", "pack.hip", "sampler.hip", "medusa.hip",
            "linear.hip", "mixers.hip", "attn_ragged.hip", "attn_latent.hip", "heads.hip",
-           "decay.hip", "experts.hip"]
+           "decay.hip", "experts.hip", "forget.hip", "attn_talk.hip"]
 HOST_SOURCES = ["runtime.cpp", "gguf.cpp", "scheduler.cpp", "layers.cpp", "checkpoint.cpp"]
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")

@@ -34,7 +34,8 @@ struct PlainAttn {
     int64_t block, k_head, k_tok, v_first, v_head, v_tok, v_elem;  // strides in elements
     float scale, temp_coef;
     int temp_every;
-    const float *bias, *sink;
+    const float *bias, *sink, *slopes;
+    const bf16 *talk;                         // [heads][heads]: scores are mixed across heads (one map, q[0] alone)
     int bias_len;
     const void *gate;
     int ldg;
@@ -51,7 +52,7 @@ struct PlainAttn {
 
 template <typename T>
 __global__ void __launch_bounds__(256) attn_plain_kernel(PlainAttn p) {
-    extern __shared__ float s_q[];  // [row]
+    extern __shared__ float s_q[];  // [row], or with mixed heads [K/V heads][row]
     __shared__ float s_s[PL_CHUNK], s_red[4];
     const int h = blockIdx.x, row = blockIdx.y, maps = max(p.maps, 1), g = h / maps / p.group, tid = threadIdx.x;
     const int seq = p.one_token ? row : seq_of_row(p.cu, p.n_seqs, row);
@@ -59,11 +60,25 @@ __global__ void __launch_bounds__(256) attn_plain_kernel(PlainAttn p) {
     if ((p.min_rows > 0 && brings < p.min_rows) || (p.max_rows > 0 && brings > p.max_rows)) return;
     const int pos = p.pos[row], len = pos + 1, first = first_visible(p.window, p.chunk, pos);
     const int32_t *bt = p.tables + (size_t)p.rows[seq] * p.max_blocks;
-    const T *kpool = (const T *)p.pool + (g * maps + h % maps) * p.k_head, *vpool = (const T *)p.pool + p.v_first + g * p.v_head;
+    const T *kpool = (const T *)p.pool + (g * maps + h % maps) * p.k_head;
+    const T *vpool = (const T *)p.pool + p.v_first + g * p.v_head;
     const float qf = p.scale * query_temperature(p.temp_coef, p.temp_every, pos);
+    // mixed heads: a sum of products with weights is the product with a weighted sum, one for every K/V head
+    const int parts = p.talk ? p.heads / p.group : 1;
+    if (p.talk) {
+        kpool = (const T *)p.pool;
+        const bf16 *w = p.talk + (size_t)h * p.heads;
+        for (int d = tid; d < parts * p.row; d += 256) {
+            const int c = d / p.row, e = d - c * p.row;
+            float t = 0.f;
+            for (int i = c * p.group; i < (c + 1) * p.group; i++)
+                t = fmaf((float)w[i], (float)((const T *)p.q[0].p)[(size_t)row * p.q[0].ld + i * p.q[0].stride + e], t);
+            s_q[d] = t;
+        }
+    }
 #pragma unroll
     for (int i = 0; i < 2; i++)
-        for (int d = tid; d < p.q[i].room; d += 256)
+        for (int d = tid; d < p.q[i].room && !p.talk; d += 256)
             s_q[p.q[i].first + d] = d < p.q[i].n ? (float)((const T *)p.q[i].p)[(size_t)row * p.q[i].ld + h * p.q[i].stride + d] : 0.f;
     // thread t accumulates dimension t % width over the keys t / width, t / width + groups, ..; wider heads: several each
     const int width = p.v_dim < 256 ? p.v_dim : 256, kg = 256 / width, md = tid % width, mg = tid / width;
@@ -80,10 +95,12 @@ __global__ void __launch_bounds__(256) attn_plain_kernel(PlainAttn p) {
             const int key = c0 + i;
             const T *k = kpool + (size_t)bt[key / p.block_size] * p.block + key % p.block_size * p.k_tok;
             float dot = 0.f;
-            for (int d = 0; d < p.row; d++) dot = fmaf(s_q[d], (float)k[d], dot);
+            for (int c = 0; c < parts; c++)
+                for (int d = 0; d < p.row; d++) dot = fmaf(s_q[c * p.row + d], (float)k[c * p.k_head + d], dot);
             float s = dot * qf;
             if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
             if (p.bias) s += p.bias[(size_t)h * p.bias_len + min(pos - key, p.bias_len - 1)];
+            if (p.slopes) s -= p.slopes[h] * (float)(pos - key);
             s_s[i] = s;
             mx = fmaxf(mx, s);
         }
@@ -149,7 +166,7 @@ inline void launch_plain(vx_backend *be, int act, const vx_ragged *b, PlainAttn 
     t.cu = b->cu_seqlens, t.pos = b->token_pos, t.rows = b->table_rows, t.tables = b->block_tables;
     t.n_seqs = b->n_seqs, t.max_blocks = b->max_blocks, t.block_size = b->block_size, t.one_token = b->q_lens ? 0 : 1;
     const dim3 grid(t.heads, b->rows);
-    const size_t lds = (size_t)t.row * 4;
+    const size_t lds = (size_t)t.row * 4 * (t.talk ? t.heads / t.group : 1);
     if (act == VX_ACT_BF16)
         attn_plain_kernel<bf16><<<grid, 256, lds, be->stream>>>(t);
     else

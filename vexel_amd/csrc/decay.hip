@@ -9,14 +9,11 @@
 //      out_kernel     a sub-chunk's rows: Q S with the state before the chunk, and (Q K^T, decayed) V inside the chunk
 //    Float32 operands (decayed keys, scores, states) enter the products as two bfloat16 parts (16 bits of the 24). Products whose
 //    inner dimension is the token read their operands transposed from LDS (ds_read_tr).
-#include "ragged.h"
+#include "state_tiles.h"
 
 using namespace vx;
 
 namespace {
-
-typedef short s16x4 __attribute__((ext_vector_type(4)));
-typedef short s16x8 __attribute__((ext_vector_type(8)));
 
 constexpr int FEW = 16;        // rows of a sequence up to which it is walked
 constexpr int SUB = 64;
@@ -35,24 +32,6 @@ struct DecayArgs {
     // eight low bfloat16 parts per lane
     float *h;
 };
-
-__device__ __forceinline__ void split(float v, bf16 *hi, bf16 *lo) {
-    *hi = (bf16)v;
-    *lo = (bf16)(v - (float)*hi);
-}
-
-// Four rows x 16 columns of 16-bit elements, transposed on the way: of a group of 16 lanes, lane i points at columns 4 (i & 3) ..
-// of row i >> 2 and gets column i of the four rows.
-__device__ __forceinline__ s16x4 read_transposed(const void *p) {
-    return __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4 *)p);
-}
-// Rows r0 + 8 (lane / 16) .. + 7 of column c0 + lane % 16.
-__device__ __forceinline__ bf16x8 column8(const bf16 *tile, int ld, int r0, int c0, int lane) {
-    const int i = lane & 15;
-    const bf16 *p = tile + (r0 + (lane >> 4) * 8 + (i >> 2)) * ld + c0 + (i & 3) * 4;
-    const s16x4 a = read_transposed(p), b = read_transposed(p + 4 * ld);
-    return __builtin_bit_cast(bf16x8, __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7));
-}
 
 // ---------------------------------------------------------------- few rows
 // Thread: columns 4 (tid % 8) .. of the workgroup's 32, state rows tid / 8 + 32 i.

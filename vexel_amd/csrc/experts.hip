@@ -23,7 +23,8 @@ __device__ __forceinline__ float score(const vx_route_args &p, int row, int e) {
     float t = z[0];
 #pragma unroll 4
     for (int k = 1; k < p.z_slices; k++) t += z[(size_t)k * p.z_stride];
-    return 1.0f / (1.0f + expf(-t));
+    if (p.bias) t += p.bias[e];
+    return p.softmax ? t : 1.0f / (1.0f + expf(-t));
 }
 
 // How many of a[0 .. n - 1] come before element i, which is v: the larger ones, and with TIES equal ones of a lower index. Reads up to
@@ -66,19 +67,42 @@ __device__ __forceinline__ void choose_row(const vx_route_args &p, int lane, flo
     }
     // The experts that fewer than `top` others surpass, in the order of their numbers; more than `top` when the last of them has an
     // equal: then equals rank by number.
+    // Softmax: relative to the largest s of all (with no correction that is the first choice), and divided by their sum in a second round.
+    float top_s = -INFINITY, inv = 1.0f;
+    if (p.softmax) {
+        for (int e = lane; e < p.experts; e += 64) top_s = fmaxf(top_s, s[e]);
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) top_s = fmaxf(top_s, __shfl_xor(top_s, off, 64));
+    }
+    const auto weight = [&](int e) { return p.softmax ? expf(s[e] - top_s) : s[e]; };
+    float sum = 0.f;  // of this lane's
     const auto deal = [&](auto ties) {
         int n = 0;
+        sum = 0.f;
         for (int e0 = 0; e0 < p.experts; e0 += 64) {
             const int e = e0 + lane;
             const bool takes = e < p.experts && rank_of<decltype(ties)::value>(c, p.experts, c[min(e, p.experts - 1)], e) < p.top;
             const uint64_t mask = __ballot(takes);
             const int slot = n + __popcll(mask & (((uint64_t)1 << lane) - 1));
-            if (takes && slot < p.top) chosen[slot] = e, weights[slot] = s[e];
+            if (takes && slot < p.top) {
+                const float w = weight(e);
+                chosen[slot] = e, weights[slot] = w * inv, sum += w;
+            }
             n += __popcll(mask);
         }
         return n;
     };
-    if (deal(std::false_type()) != p.top) deal(std::true_type());
+    const bool ties = deal(std::false_type()) != p.top;
+    if (ties) deal(std::true_type());
+    if (p.softmax) {
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) sum += __shfl_xor(sum, off, 64);
+        inv = 1.0f / sum;
+        if (ties)
+            deal(std::true_type());
+        else
+            deal(std::false_type());
+    }
     __builtin_amdgcn_wave_barrier();
 }
 

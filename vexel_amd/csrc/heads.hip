@@ -160,6 +160,85 @@ __global__ void __launch_bounds__(256) heads4_kernel(HeadArgs a) {
     if (live && in_head && (is_q || is_k)) store4((is_q ? (T *)p.q + (size_t)row * p.ldq + h * dim : pool + ((size_t)h * a.block_size + in) * kp) + d, v);
 }
 
+// Norms over all heads of a row: a workgroup takes a row's queries, its keys or its values (blockIdx.y), in pieces of VEC columns; up to
+// NV pieces of a thread stay in registers, wider rows are read again.
+template <typename T, int VEC, int NV>
+__global__ void __launch_bounds__(1024) rows_kernel(HeadArgs a) {
+    typedef float F __attribute__((ext_vector_type(VEC)));
+    __shared__ float sm[16];
+    const vx_heads_args &p = a.p;
+    const int row = blockIdx.x, part = blockIdx.y, tid = threadIdx.x, nt = blockDim.x;  // 0: queries, 1: keys, 2: values
+    const int dim = part < 2 ? p.dim : p.v_dim, cols = (part == 0 ? p.q_heads : part == 1 ? p.k_heads : p.v_heads) * dim;
+    const int col = part == 0 ? p.q_col : part == 1 ? p.k_col : p.v_col;
+    const float *y = p.y + (size_t)row * p.ldy + col, *bias = p.bias ? p.bias + col : nullptr, *w = part == 0 ? p.w_q : part == 1 ? p.w_k : nullptr;
+    const auto raw = [&](int c) {
+        F t = *(const F *)(y + c);
+#pragma unroll 4
+        for (int s = 1; s < p.y_slices; s++) t += *(const F *)(y + (size_t)s * p.y_stride + c);
+        return bias ? t + *(const F *)(bias + c) : t;
+    };
+    F v[NV];
+    float inv = 1.0f, ss = 0.f;
+    const auto square = [&](F t) {
+#pragma unroll
+        for (int e = 0; e < VEC; e++) ss = fmaf(t[e], t[e], ss);
+    };
+#pragma unroll
+    for (int i = 0; i < NV; i++)
+        if (const int c = (tid + i * nt) * VEC; c < cols) {
+            v[i] = raw(c);
+            square(v[i]);
+        }
+    if (part < 2) {
+        for (int c = (tid + NV * nt) * VEC; c < cols; c += nt * VEC) square(raw(c));
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+        if ((tid & 63) == 0) sm[tid >> 6] = ss;
+        __syncthreads();
+        ss = 0.f;
+        for (int i = 0; i < (nt >> 6); i++) ss += sm[i];
+        inv = 1.0f / sqrtf(ss / (float)cols + p.eps);
+    }
+    const int kp = (p.dim + 7) & ~7;
+    const int slot = part == 0 ? 0 : a.slot_map[row], blk = part == 0 ? 0 : slot / a.block_size, in = slot - blk * a.block_size;
+    T *pool = (T *)p.pool + (size_t)blk * a.block_size * ((size_t)p.k_heads * kp + (size_t)p.v_heads * p.v_dim);
+    T *vpool = pool + (size_t)p.k_heads * a.block_size * kp + in;
+    const auto put = [&](int c, F t) {
+        if (part == 2) {
+#pragma unroll
+            for (int e = 0; e < VEC; e++) vpool[(size_t)(c + e) * a.block_size] = (T)t[e];
+            return;
+        }
+        t *= inv;
+        if (w) t *= *(const F *)(w + c);
+        T *out = part == 0 ? (T *)p.q + (size_t)row * p.ldq + c : pool + ((size_t)(c / dim) * a.block_size + in) * kp + c % dim;
+        if constexpr (VEC == 4) {
+            store4(out, t);
+        } else {
+            out[0] = (T)t[0];
+        }
+    };
+#pragma unroll
+    for (int i = 0; i < NV; i++)
+        if (const int c = (tid + i * nt) * VEC; c < cols) put(c, v[i]);
+    for (int c = (tid + NV * nt) * VEC; c < cols; c += nt * VEC) put(c, raw(c));
+}
+
+template <typename T>
+void launch_rows(vx_backend *be, const HeadArgs &a) {
+    const vx_heads_args &p = a.p;
+    const auto al = [](const void *q) { return (uintptr_t)q % 16 == 0; };
+    const bool vec = p.dim % 4 == 0 && p.v_dim % 4 == 0 && p.ldy % 4 == 0 && p.q_col % 4 == 0 && p.k_col % 4 == 0 && p.v_col % 4 == 0 && p.ldq % 4 == 0 &&
+                     (p.y_slices == 1 || p.y_stride % 4 == 0) && al(p.y) && al(p.bias) && al(p.w_q) && al(p.w_k) && al(p.q) && al(p.pool);
+    const dim3 grid(a.rows, p.k_heads > 0 ? 3 : 1);
+    int threads = a.rows <= 256 ? 1024 : 256;
+    while (threads > 64 && threads * 2 >= p.q_heads * p.dim) threads /= 2;
+    if (vec)
+        rows_kernel<T, 4, 4><<<grid, threads, 0, be->stream>>>(a);
+    else
+        rows_kernel<T, 1, 4><<<grid, threads, 0, be->stream>>>(a);
+}
+
 template <typename T, int LANES>
 void launch_heads4(vx_backend *be, const HeadArgs &a) {
     heads4_kernel<T, LANES><<<(unsigned)ceil_div64((int64_t)a.rows * a.units * LANES, 256), 256, 0, be->stream>>>(a);
@@ -168,6 +247,7 @@ void launch_heads4(vx_backend *be, const HeadArgs &a) {
 template <typename T>
 void launch_heads(vx_backend *be, const HeadArgs &a) {
     const vx_heads_args &p = a.p;
+    if (p.norm == 2) return launch_rows<T>(be, a);
     const int wide = a.p.dim > a.p.v_dim ? a.p.dim : a.p.v_dim;
     const auto al = [](const void *q) { return (uintptr_t)q % 16 == 0; };
     if (p.dim % 4 == 0 && p.v_dim % 4 == 0 && p.ldy % 4 == 0 && p.q_col % 4 == 0 && p.k_col % 4 == 0 && (p.v_col < 0 || p.v_col % 4 == 0) &&
@@ -222,14 +302,15 @@ int vx_heads_store(vx_backend *be, int act, const vx_ragged *b, const vx_heads_a
     rc = check_ragged(b, "vx_heads_store");
     if (rc) return rc;
     VX_REQUIRE(act == VX_ACT_F32 || act == VX_ACT_BF16, "vx_heads_store: unknown activation type %d", act);
-    VX_REQUIRE(p && p->q_heads >= 1 && p->k_heads >= 1 && p->v_heads >= 1 && p->dim >= 1 && p->v_dim >= 1 && p->dim <= 2048 && p->v_dim <= 2048 && p->y &&
-                   p->y_slices >= 1 && p->q && p->pool && p->q_col >= 0 && p->k_col >= 0,
+    VX_REQUIRE(p && p->q_heads >= 1 && p->k_heads >= 0 && p->v_heads >= 0 && (p->k_heads > 0) == (p->v_heads > 0) && p->dim >= 1 && p->v_dim >= 1 && p->dim <= 2048 && p->v_dim <= 2048 && p->y &&
+                   p->y_slices >= 1 && p->q && (p->pool || p->k_heads == 0) && p->q_col >= 0 && p->k_col >= 0,
                "vx_heads_store: bad arguments");
     VX_REQUIRE(p->v_col >= 0 || (p->v_heads == p->k_heads && p->v_dim == p->dim), "vx_heads_store: values are keys of another size");
     const int64_t q_end = p->q_col + (int64_t)p->q_heads * p->dim, k_end = p->k_col + (int64_t)p->k_heads * p->dim;
     VX_REQUIRE(q_end <= p->ldy && k_end <= p->ldy && (p->v_col < 0 || p->v_col + (int64_t)p->v_heads * p->v_dim <= p->ldy) &&
                    p->ldq >= (int64_t)p->q_heads * p->dim,
                "vx_heads_store: heads beyond their row");
+    VX_REQUIRE(p->norm >= 0 && p->norm <= 2 && (p->norm < 2 || (p->rot_pairs == 0 && p->v_col >= 0)), "vx_heads_store: norm %d", p->norm);
     VX_REQUIRE(p->rot_pairs >= 0 && 2 * p->rot_pairs <= p->dim && (p->rot_pairs == 0 || p->rot_tab), "vx_heads_store: %d pairs in heads of %d", p->rot_pairs,
                p->dim);
     HeadArgs a{*p, b->slot_mapping, b->rows, b->block_size, p->q_heads + p->k_heads + (p->v_col < 0 ? 0 : p->v_heads)};

@@ -61,6 +61,12 @@ __device__ __forceinline__ float glu(const vx_linear_out &o, float g, float u) {
     return g * sigmoid_f(o.glu_alpha * g) * (u + o.glu_add);
 }
 
+// One element of a VX_LIN_FORGET map: column c of the activations, or c >= split of the gates.
+__device__ __forceinline__ float forget(const vx_linear_out &o, int c, float y) {
+    if (c >= o.split) return o.keep[c - o.split] * sigmoid_f(-(y + o.bias[c - o.split]));
+    return c < o.silu_cols ? silu_f(y) : y;
+}
+
 // Where K and V elements lie in the pool: a part that depends on the slot and one that depends on the column.
 struct KvSlot {
     size_t k, v;
@@ -145,6 +151,7 @@ __device__ __forceinline__ void emit(const LinArgs &p, int slice, int row, int c
     const vx_linear_out &o = p.o;
     if (row >= p.rows) return;
     if constexpr (KIND == VX_LIN_PLAIN) {
+        if (o.mult != 0.f) v *= o.mult;
         if (o.softcap > 0.f) {
 #pragma unroll
             for (int r = 0; r < 4; r++) v[r] = o.softcap * tanhf(v[r] / o.softcap);
@@ -163,6 +170,20 @@ __device__ __forceinline__ void emit(const LinArgs &p, int slice, int row, int c
         } else {
             put4(o.out2 + (size_t)row * o.ldo2, c - o.split, o.ldo2, o.ldo2, v);
         }
+    } else if constexpr (KIND == VX_LIN_FORGET) {
+#pragma unroll
+        for (int r = 0; r < 4; r++) v[r] = forget(o, c + r, v[r]);
+        if (c < o.split)
+            put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
+        else
+            put4(o.out2 + (size_t)row * o.ldo2, c - o.split, o.ldo2, o.ldo2, v);
+    } else if constexpr (KIND == VX_LIN_RELU2) {
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            const float t = fmaxf(o.bias && c + r < o.cols ? v[r] + o.bias[c + r] : v[r], 0.f);
+            v[r] = t * t;
+        }
+        put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
     } else if constexpr (KIND == VX_LIN_SPLIT) {
         if (c < o.split)
             put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, v);
@@ -437,7 +458,7 @@ __global__ void __launch_bounds__(256) linear_many_kernel(LinArgs p, int row_til
     }
 }
 
-// Adds up the slices of a VX_LIN_SPLIT, VX_LIN_ROTARY or VX_LIN_SILU map and deals the columns to its two results.
+// Adds up the slices of a VX_LIN_SPLIT, VX_LIN_ROTARY, VX_LIN_SILU or VX_LIN_FORGET map and deals the columns to its two results.
 template <typename T>
 __global__ void __launch_bounds__(256) split_sum_kernel(const float *part, int slices, int rows, int n, vx_linear_out o) {
     const int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x;
@@ -449,6 +470,9 @@ __global__ void __launch_bounds__(256) split_sum_kernel(const float *part, int s
     if (c < o.split && o.kind == VX_LIN_SILU)
 #pragma unroll
         for (int r = 0; r < 4; r++) v[r] = silu_f(v[r]);
+    if (o.kind == VX_LIN_FORGET)
+#pragma unroll
+        for (int r = 0; r < 4; r++) v[r] = forget(o, c + r, v[r]);
     if (c < o.split)
         put4((T *)o.out + (size_t)row * o.ldo, c, o.cols, o.ldo, o.rot_tab ? turned(o, row, c, v) : v);
     else
@@ -559,6 +583,8 @@ int dispatch(vx_backend *be, const LinArgs &p, int slices) {
         case VX_LIN_ROTARY: return launch<T, VX_LIN_ROTARY>(be, p, slices);
         case VX_LIN_SILU: return launch<T, VX_LIN_SILU>(be, p, slices);
         case VX_LIN_V: return launch<T, VX_LIN_V>(be, p, slices);
+        case VX_LIN_FORGET: return launch<T, VX_LIN_FORGET>(be, p, slices);
+        case VX_LIN_RELU2: return launch<T, VX_LIN_RELU2>(be, p, slices);
         default: return launch<T, VX_LIN_SOFTPLUS>(be, p, slices);
     }
 }
@@ -665,14 +691,14 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
     VX_REQUIRE(n >= 16 && n % 16 == 0 && k >= 64 && k % 64 == 0 && lda >= k && lda % 8 == 0 && (uintptr_t)a % 16 == 0 &&
                    (uintptr_t)w % 16 == 0 && (uintptr_t)o->out % 16 == 0,
                "vx_linear: sizes or alignment (n %d, k %d, lda %d)", n, k, lda);
-    VX_REQUIRE(o->kind >= VX_LIN_PLAIN && o->kind <= VX_LIN_SILU, "vx_linear: unknown kind %d", o->kind);
+    VX_REQUIRE(o->kind >= VX_LIN_PLAIN && o->kind <= VX_LIN_RELU2, "vx_linear: unknown kind %d", o->kind);
     VX_REQUIRE(o->cols >= 1 && o->ldo >= o->cols, "vx_linear: %d columns in rows of %d", o->cols, o->ldo);
     const int slices = o->slices > 1 ? o->slices : 1;
     VX_REQUIRE(slices == 1 || (o->kind == VX_LIN_PLAIN && o->out_f32 && slices <= 64), "vx_linear: slices need a plain float32 result");
     if (o->kind == VX_LIN_SWIGLU) {
         VX_REQUIRE(n % 32 == 0 && o->cols <= n / 2, "vx_linear: gate|up pairs of %d rows for %d columns", n, o->cols);
         VX_REQUIRE(o->glu_limit >= 0.f, "vx_linear: negative limit");
-    } else if (o->kind == VX_LIN_SPLIT || o->kind == VX_LIN_SILU) {
+    } else if (o->kind == VX_LIN_SPLIT || o->kind == VX_LIN_SILU || o->kind == VX_LIN_FORGET) {
         VX_REQUIRE(o->out2 && o->split % 16 == 0 && o->split > 0 && o->split < n && o->cols == o->split && o->ldo2 >= n - o->split &&
                        (uintptr_t)o->out2 % 16 == 0,
                    "vx_linear: bad split");
@@ -686,7 +712,9 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
     } else {
         VX_REQUIRE(o->cols <= n, "vx_linear: %d columns of %d", o->cols, n);
     }
-    if (o->kind == VX_LIN_SOFTPLUS) VX_REQUIRE(o->bias != nullptr, "vx_linear: null bias");
+    if (o->kind == VX_LIN_SOFTPLUS || o->kind == VX_LIN_FORGET) VX_REQUIRE(o->bias != nullptr, "vx_linear: null bias");
+    if (o->kind == VX_LIN_FORGET) VX_REQUIRE(o->keep && o->silu_cols >= 0 && o->silu_cols <= o->split, "vx_linear: incomplete gates");
+    VX_REQUIRE(o->mult == 0.f || (o->kind == VX_LIN_PLAIN && slices == 1), "vx_linear: a factor needs a plain whole result");
     if (o->kind == VX_LIN_KV || o->kind == VX_LIN_V)
         VX_REQUIRE(o->pool && o->kv_heads >= 1 && o->k_dim >= 1 && o->v_dim >= 1 && o->block_size >= 1 &&
                        o->k_col % 16 == 0 && o->v_col % 16 == 0 && o->k_col >= 0 && o->v_col >= 0 &&
@@ -707,7 +735,7 @@ int vx_linear(vx_backend *be, int act, const void *a, int lda, const void *w, in
         p.o.groups = 1;
     }
     if (o->kind != VX_LIN_ROTARY) p.o.rot_tab = nullptr;
-    if (o->kind == VX_LIN_SPLIT || o->kind == VX_LIN_ROTARY || o->kind == VX_LIN_SILU) {  // (narrow and deep as a rule) in slices, added up by a kernel of their own
+    if (o->kind == VX_LIN_SPLIT || o->kind == VX_LIN_ROTARY || o->kind == VX_LIN_SILU || o->kind == VX_LIN_FORGET) {  // (narrow and deep as a rule) in slices, added up by a kernel of their own
         const int cut = k >= 2048 ? pick_slices(n, k, rows) : 1;  // (a short map is over before the second launch pays)
         if (cut > 1) {
             const size_t bytes = (size_t)cut * rows * n * 4;
@@ -738,7 +766,7 @@ int vx_linear_experts(vx_backend *be, int act, const vx_experts_args *e) {
     if (rc) return rc;
     VX_REQUIRE(act == VX_ACT_F32 || act == VX_ACT_BF16, "vx_linear_experts: unknown activation type %d", act);
     VX_REQUIRE(e && e->a && e->w && e->tiles && e->out && e->rows >= 1 && e->experts >= 1 && e->max_tiles >= 1, "vx_linear_experts: bad arguments");
-    VX_REQUIRE(e->kind == VX_LIN_PLAIN || e->kind == VX_LIN_SWIGLU, "vx_linear_experts: kind %d", e->kind);
+    VX_REQUIRE(e->kind == VX_LIN_PLAIN || e->kind == VX_LIN_SWIGLU || e->kind == VX_LIN_RELU2, "vx_linear_experts: kind %d", e->kind);
     VX_REQUIRE((e->rows <= 64 && e->tile_rows == 64) || (e->rows > 64 && (e->tile_rows == 64 || (e->tile_rows == 128 && act == VX_ACT_BF16))),
                "vx_linear_experts: tiles of %d of %d rows", e->tile_rows, e->rows);
     const int per = e->kind == VX_LIN_SWIGLU ? 2 : 1;  // outputs of a result column
@@ -761,6 +789,9 @@ int vx_linear_experts(vx_backend *be, int act, const vx_experts_args *e) {
     if (e->kind == VX_LIN_SWIGLU)
         return act == VX_ACT_BF16 ? launch_experts<bf16, VX_LIN_SWIGLU>(be, p, e->rows, e->max_tiles, e->tile_rows)
                                   : launch_experts<float, VX_LIN_SWIGLU>(be, p, e->rows, e->max_tiles, e->tile_rows);
+    if (e->kind == VX_LIN_RELU2)
+        return act == VX_ACT_BF16 ? launch_experts<bf16, VX_LIN_RELU2>(be, p, e->rows, e->max_tiles, e->tile_rows)
+                                  : launch_experts<float, VX_LIN_RELU2>(be, p, e->rows, e->max_tiles, e->tile_rows);
     return act == VX_ACT_BF16 ? launch_experts<bf16, VX_LIN_PLAIN>(be, p, e->rows, e->max_tiles, e->tile_rows)
                               : launch_experts<float, VX_LIN_PLAIN>(be, p, e->rows, e->max_tiles, e->tile_rows);
 }

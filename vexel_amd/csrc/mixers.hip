@@ -277,6 +277,128 @@ __global__ void __launch_bounds__(1024) post_norm_kernel(vx_post_norm_args p) {
         for (int c = p.cols + tid; c < p.ldo; c += nt) out[c] = (T)0.f;
 }
 
+// A row's mean and 1 / standard deviation from its columns in registers (zero beyond cols; n4: how many pieces of four there are).
+template <int NV>
+__device__ __forceinline__ float mean_and_scale(const f32x4 (&v)[NV], int n4, int cols, float eps, float *sm, float *mean) {
+    const int tid = threadIdx.x, nt = blockDim.x;
+    float t = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; i++) t += (v[i][0] + v[i][1]) + (v[i][2] + v[i][3]);
+    *mean = block_sum(t, sm) / (float)cols;
+    t = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; i++)
+        if (tid + i * nt < n4)
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const float d = v[i][e] - *mean;
+                t = fmaf(d, d, t);
+            }
+    return 1.0f / sqrtf(block_sum(t, sm) / (float)cols + eps);
+}
+
+// NV > 0: as for residual_norm_kernel. NV 0: the sublayer's row passes through LDS (cols floats).
+template <typename T, int NV>
+__global__ void __launch_bounds__(1024) branch_norm_kernel(vx_branch_norm_args p) {
+    extern __shared__ float s_row[];
+    __shared__ float sm[16];
+    const int i = blockIdx.x, r = p.row_idx ? p.row_idx[i] : i, tid = threadIdx.x, nt = blockDim.x;
+    const float *xr = p.x_in + (size_t)(p.tokens ? p.tokens[r] : r) * p.cols;
+    const float *pr = p.tokens ? p.positions + (size_t)p.token_pos[r] * p.cols : nullptr;
+    float *xo = p.x_out ? p.x_out + (size_t)r * p.cols : nullptr;
+    T *out = p.out ? (T *)p.out + (size_t)i * p.ldo : nullptr;
+    vx_residual_norm_args ex;  // (what add_experts reads)
+    ex.e_rows = p.e_rows, ex.lde = p.lde, ex.e_top = p.e_top, ex.e_shared = -1, ex.e_places = p.e_places, ex.e_weights = p.e_weights;
+    float mean, inv;
+    if constexpr (NV > 0) {
+        f32x4 x[NV];
+        const int n4 = p.cols >> 2;
+        if (p.w) {
+            f32x4 y[NV];
+#pragma unroll
+            for (int v = 0; v < NV; v++) {
+                const int c = tid + v * nt;
+                y[v] = x[v] = f32x4{0.f, 0.f, 0.f, 0.f};
+                if (c >= n4) continue;
+                x[v] = ((const f32x4 *)xr)[c];
+                if (p.y) {
+                    const float *yr = p.y + (size_t)r * p.ldy + c * 4;
+                    y[v] = *(const f32x4 *)yr;
+                    for (int s = 1; s < p.y_slices; s++) y[v] += *(const f32x4 *)(yr + (size_t)s * p.y_stride);
+                    if (p.y_bias) y[v] += ((const f32x4 *)p.y_bias)[c];
+                }
+                if (p.e_rows) add_experts<T>(ex, r, c * 4, &y[v]);
+            }
+            inv = mean_and_scale<NV>(y, n4, p.cols, p.eps, sm, &mean);
+#pragma unroll
+            for (int v = 0; v < NV; v++)
+                if (const int c = tid + v * nt; c < n4) x[v] += (y[v] - mean) * inv * ((const f32x4 *)p.w)[c] + ((const f32x4 *)p.b)[c];
+        } else {
+#pragma unroll
+            for (int v = 0; v < NV; v++) {
+                const int c = tid + v * nt;
+                x[v] = c < n4 ? ((const f32x4 *)xr)[c] : f32x4{0.f, 0.f, 0.f, 0.f};
+                if (pr && c < n4) x[v] += ((const f32x4 *)pr)[c];
+            }
+        }
+        const auto keep = [&]() {
+#pragma unroll
+            for (int v = 0; v < NV; v++)
+                if (const int c = tid + v * nt; xo && c < n4) ((f32x4 *)xo)[c] = x[v];
+        };
+        if (!p.tokens) keep();
+        if (p.w_pre) {
+            inv = mean_and_scale<NV>(x, n4, p.cols, p.eps, sm, &mean);
+#pragma unroll
+            for (int v = 0; v < NV; v++)
+                if (const int c = tid + v * nt; c < n4) x[v] = (x[v] - mean) * inv * ((const f32x4 *)p.w_pre)[c] + ((const f32x4 *)p.b_pre)[c];
+        }
+        if (p.tokens) keep();
+        if (!out) return;
+#pragma unroll
+        for (int v = 0; v < NV; v++)
+            if (const int c = tid + v * nt; c < n4) store4(out + c * 4, x[v]);
+    } else {  // (a thread reads and writes its own columns only)
+        const auto norm = [&]() {
+            float t = 0.f;
+            for (int c = tid; c < p.cols; c += nt) t += s_row[c];
+            mean = block_sum(t, sm) / (float)p.cols;
+            t = 0.f;
+            for (int c = tid; c < p.cols; c += nt) t = fmaf(s_row[c] - mean, s_row[c] - mean, t);
+            inv = 1.0f / sqrtf(block_sum(t, sm) / (float)p.cols + p.eps);
+        };
+        for (int c = tid; c < p.cols; c += nt) {
+            float y = 0.f;
+            if (p.w) {
+                if (p.y) {
+                    y = p.y[(size_t)r * p.ldy + c];
+                    for (int s = 1; s < p.y_slices; s++) y += p.y[(size_t)s * p.y_stride + (size_t)r * p.ldy + c];
+                    if (p.y_bias) y += p.y_bias[c];
+                }
+                if (p.e_rows) add_experts<T>(ex, r, c, &y);
+            } else {
+                y = pr ? xr[c] + pr[c] : xr[c];
+            }
+            s_row[c] = y;
+        }
+        if (p.w) {
+            norm();
+            for (int c = tid; c < p.cols; c += nt) s_row[c] = xr[c] + ((s_row[c] - mean) * inv * p.w[c] + p.b[c]);
+        }
+        if (xo && !p.tokens)
+            for (int c = tid; c < p.cols; c += nt) xo[c] = s_row[c];
+        if (p.w_pre) {
+            norm();
+            for (int c = tid; c < p.cols; c += nt) s_row[c] = (s_row[c] - mean) * inv * p.w_pre[c] + p.b_pre[c];
+        }
+        if (xo && p.tokens)
+            for (int c = tid; c < p.cols; c += nt) xo[c] = s_row[c];
+        if (!out) return;
+        for (int c = tid; c < p.cols; c += nt) out[c] = (T)s_row[c];
+    }
+    for (int c = p.cols + tid; c < p.ldo; c += nt) out[c] = (T)0.f;
+}
+
 // A row per workgroup; NV > 0: cols is a multiple of 8 and at most 8 * NV * blockDim.x, rows aligned: they live in registers.
 // Z: bfloat16 or float32, the latter in `slices` parts that are added up.
 template <typename T, typename Z, int NV>
@@ -632,6 +754,29 @@ void launch_post_norm(vx_backend *be, const vx_post_norm_args &p) {
         post_norm_kernel<T, 8><<<p.rows, threads, 0, be->stream>>>(p);
 }
 
+template <typename T>
+void launch_branch_norm(vx_backend *be, const vx_branch_norm_args &p) {
+    const auto al = [](const void *q) { return (uintptr_t)q % 16 == 0; };
+    const bool vec = p.cols % 4 == 0 && al(p.x_in) && al(p.x_out) && al(p.y) && al(p.y_bias) && al(p.w) && al(p.b) && al(p.w_pre) && al(p.b_pre) && al(p.out) &&
+                     al(p.positions) && al(p.e_rows) && (!p.e_rows || p.lde % 4 == 0) && (!p.y || (p.ldy % 4 == 0 && p.y_stride % 4 == 0)) &&
+                     (!p.out || p.ldo % 4 == 0);
+    const int n4 = p.cols / 4;
+    int threads = p.rows <= 256 ? 1024 : 256;
+    while (threads > 64 && threads / 2 >= n4) threads /= 2;
+    while (threads < 1024 && n4 > 8 * threads) threads *= 2;
+    const int nv = ceil_div(n4, threads);
+    if (!vec || nv > 8)
+        branch_norm_kernel<T, 0><<<p.rows, 256, (size_t)p.cols * 4, be->stream>>>(p);
+    else if (nv <= 1)
+        branch_norm_kernel<T, 1><<<p.rows, threads, 0, be->stream>>>(p);
+    else if (nv <= 2)
+        branch_norm_kernel<T, 2><<<p.rows, threads, 0, be->stream>>>(p);
+    else if (nv <= 4)
+        branch_norm_kernel<T, 4><<<p.rows, threads, 0, be->stream>>>(p);
+    else
+        branch_norm_kernel<T, 8><<<p.rows, threads, 0, be->stream>>>(p);
+}
+
 template <typename T, typename Z>
 void launch_poly_norm(vx_backend *be, const Z *z, int ldz, int slices, int64_t stride, int rows, int cols, const float *coef, float eps, T *out, int ldo) {
     const bool vec = cols % 8 == 0 && ldz % 8 == 0 && ldo % 8 == 0 && (slices == 1 || stride % 8 == 0) && (uintptr_t)z % 16 == 0 && (uintptr_t)out % 16 == 0;
@@ -667,6 +812,28 @@ int vx_post_norm(vx_backend *be, int act, const vx_post_norm_args *a) {
         launch_post_norm<bf16>(be, *a);
     else
         launch_post_norm<float>(be, *a);
+    VX_CHECK_LAUNCH();
+    return VX_OK;
+}
+
+int vx_branch_norm(vx_backend *be, int act, const vx_branch_norm_args *a) {
+    int rc = enter(be);
+    if (rc) return rc;
+    VX_REQUIRE(a && a->rows >= 1 && a->cols >= 1 && a->x_in, "vx_branch_norm: bad arguments");
+    VX_REQUIRE(a->cols <= 15360 || a->cols % 4 == 0, "vx_branch_norm: rows of %d columns", a->cols);
+    VX_REQUIRE(a->cols <= 32768, "vx_branch_norm: rows of %d columns", a->cols);
+    VX_REQUIRE(act == VX_ACT_F32 || act == VX_ACT_BF16, "vx_branch_norm: unknown activation type %d", act);
+    VX_REQUIRE(!a->w || (a->b && (a->y || a->e_rows)), "vx_branch_norm: incomplete norm");
+    VX_REQUIRE(!a->y || (a->y_slices >= 1 && a->ldy >= a->cols), "vx_branch_norm: incomplete sublayer output");
+    VX_REQUIRE(!a->e_rows || (a->lde >= a->cols && a->e_top >= 1 && a->e_places && a->e_weights), "vx_branch_norm: incomplete experts");
+    VX_REQUIRE(!a->w_pre || a->b_pre, "vx_branch_norm: incomplete norm of the result");
+    VX_REQUIRE(!a->tokens || (!a->w && !a->row_idx && a->token_pos && a->positions && a->w_pre), "vx_branch_norm: incomplete embedding");
+    VX_REQUIRE(!a->out || a->ldo >= a->cols, "vx_branch_norm: rows of %d for %d columns", a->ldo, a->cols);
+    VX_REQUIRE(a->out || a->x_out, "vx_branch_norm: nothing to write");
+    if (act == VX_ACT_BF16)
+        launch_branch_norm<bf16>(be, *a);
+    else
+        launch_branch_norm<float>(be, *a);
     VX_CHECK_LAUNCH();
     return VX_OK;
 }

@@ -1057,6 +1057,221 @@ int check_kitodra(const Json &config) {
     return parse_kitodra(config, &c);
 }
 
+// ---------------------------------------------------------------- Fitevik
+struct FitevikLayer {
+    bool states = false;          // hgrn2, else attention
+    int heads = 1, kv_heads = 1, dim = 1, vdim = 1, window = 0, kv_from = -1;
+    float scale = 1.f;
+    enum Ff { NONE, DENSE, EXPERTS } mlp = NONE;
+    int ff = 1, experts = 1, top = 1;
+};
+struct FitevikConfig {
+    std::vector<FitevikLayer> layers;
+    float eps = 1e-5f, logit_scale = 1.f;
+    int vocab = 1, width = 1, max_positions = 1;
+};
+
+int parse_fitevik(const Json &j, FitevikConfig *c) {
+    int rc = VH_OK;
+    const Fields root("config", &j, &rc);
+    c->vocab = root.count("vocab");
+    c->width = root.count("width", 1, 15360);
+    c->max_positions = root.count("max_positions");
+    c->logit_scale = (float)root.num("logit_scale");
+    c->eps = (float)root.sub("norm").num("eps");
+    const Json *layers = root.need("layers", Json::ARR);
+    if (rc != VH_OK) return rc;
+    if (layers->arr.empty()) return fail("config.json: no layers");
+    for (size_t i = 0; i < layers->arr.size(); i++) {
+        const Fields l("layers[" + std::to_string(i) + "]", &layers->arr[i], &rc);
+        const Json *type = l.need("type", Json::STR);
+        if (rc != VH_OK) return rc;
+        FitevikLayer o;
+        o.states = type->str == "hgrn2";
+        if (!o.states && type->str != "attention") return fail("config.json: layer %zu has the unknown mixer type '%s'", i, type->str.c_str());
+        const Fields mx = l.sub("mixer");
+        o.heads = mx.count("heads", 1, 4096);
+        o.dim = mx.count("dim", 1, o.states ? 512 : 2048), o.vdim = mx.count("vdim", 1, o.states ? 512 : 2048);
+        if (!o.states) {
+            o.kv_heads = mx.count("kv_heads", 1, 4096);
+            o.scale = (float)mx.num("scale");
+            if (mx.has("mask")) o.window = mx.sub("mask").count("size", 1, 1 << 30);
+            if (mx.has("kv_from")) o.kv_from = mx.count("kv_from", 0, 1 << 16);
+        }
+        if (l.has("mlp")) {
+            const Fields mlp = l.sub("mlp");
+            const Json *kind = mlp.need("kind", Json::STR);
+            if (rc != VH_OK) return rc;
+            if (kind->str == "dense") {
+                o.mlp = FitevikLayer::DENSE;
+                o.ff = mlp.count("ff", 1, 1 << 20);
+            } else if (kind->str == "moe") {
+                o.mlp = FitevikLayer::EXPERTS;
+                o.experts = mlp.sub("router").count("experts", 1, 1024), o.top = mlp.sub("router").count("top", 1, 1024);
+                o.ff = mlp.sub("expert").count("ff", 1, 1 << 20);
+            } else {
+                return fail("config.json: layer %zu has the unknown feed-forward '%s'", i, kind->str.c_str());
+            }
+        }
+        if (rc != VH_OK) return rc;
+        if (o.heads % o.kv_heads) return fail("config.json: layer %zu: %d heads are no multiple of %d", i, o.heads, o.kv_heads);
+        if (!o.states && (int64_t)o.kv_heads * o.dim > 15360) return fail("config.json: layer %zu: %d key heads of %d", i, o.kv_heads, o.dim);
+        if (o.top > o.experts) return fail("config.json: layer %zu: %d of %d experts", i, o.top, o.experts);
+        if (o.kv_from >= 0) {
+            if (o.kv_from >= (int)i || c->layers[o.kv_from].states || c->layers[o.kv_from].kv_from >= 0)
+                return fail("config.json: layer %zu: layer %d holds no keys for it", i, o.kv_from);
+            const FitevikLayer &f = c->layers[o.kv_from];
+            if (f.kv_heads != o.kv_heads || f.dim != o.dim || f.vdim != o.vdim)
+                return fail("config.json: layer %zu: the keys of layer %d are of another kind", i, o.kv_from);
+        }
+        c->layers.push_back(o);
+    }
+    return rc;
+}
+
+int build_fitevik_attention(Builder &b, const FitevikLayer &s, const std::string &mix, int W, MixLayer *o) {
+    AttnMixer &a = o->attn;
+    o->has_attn = true;
+    a.by_heads = a.row_norm = true;
+    a.heads = s.heads, a.kv_heads = s.kv_heads, a.k_dim = s.dim, a.v_dim = s.vdim, a.scale = s.scale, a.window = s.window, a.kv_from = s.kv_from;
+    const int qd = s.heads * s.dim, kd = s.kv_heads * s.dim, vd = s.kv_heads * s.vdim, od = s.heads * s.vdim;
+    a.k_col = b.pad(qd, 16), a.v_col = a.k_col + b.pad(kd, 16);
+    VHC(b.packed(&o->in, s.kv_from < 0 ? a.v_col + vd : qd, W));
+    VHC(b.pack(mix + "q", qd, W, 0, qd, o->in, a.q_col, 1, 0));
+    VHC(b.vec(mix + "q.norm", qd, &a.norm_q));
+    if (s.kv_from < 0) {
+        VHC(b.pack(mix + "k", kd, W, 0, kd, o->in, a.k_col, 1, 0));
+        VHC(b.pack(mix + "v", vd, W, 0, vd, o->in, a.v_col, 1, 0));
+        VHC(b.vec(mix + "k.norm", kd, &a.norm_k));
+    } else {
+        a.k_col = a.v_col = 0;
+    }
+    VHC(b.packed(&o->out, W, od));
+    VHC(b.pack(mix + "o", W, od, 0, W, o->out, 0, 1, 0));
+    VHC(b.vec(mix + "sink", s.heads, &a.sink));
+    // the matrix that mixes scores, and every head's slope as the mixing leaves it
+    const TensorView *t;
+    VHC(b.view(mix + "talk", {s.heads, s.heads}, &t));
+    const size_t bytes = (size_t)s.heads * s.heads * 2;
+    void *p = vx_alloc_permanent(b.be, (bytes + 15) / 16 * 16 + 16);
+    if (!p) return fail("device memory: %s", vx_last_error());
+    b.m->adopted.push_back(p);
+    VXC(vx_to_device(b.be, p, t->data, bytes));
+    a.talk = p;
+    std::vector<float> talk, slopes;
+    VHC(b.floats(mix + "talk", {s.heads, s.heads}, &talk));
+    for (int h = 0; h < s.heads; h++) {
+        double sum = 0.0;
+        for (int g = 0; g < s.heads; g++) sum += (double)talk[(size_t)h * s.heads + g] * exp2(-8.0 * (g + 1) / s.heads);
+        slopes.push_back((float)sum);
+    }
+    return b.upload(slopes, &a.slopes);
+}
+
+int build_fitevik_states(Builder &b, const FitevikLayer &s, const std::string &mix, int W, MixLayer *o) {
+    ForgetMixer &t = o->forget;
+    o->has_forget = true;
+    t.heads = s.heads, t.vdim = s.vdim, t.dim_pad = b.pad(s.dim, 32), t.v_pad = b.pad(s.vdim, 16);
+    const int qs = s.heads * t.dim_pad, vs = s.heads * t.v_pad, vd = s.heads * s.vdim, fd = s.heads * s.dim;
+    VHC(b.packed(&o->in, 2 * qs + vs, W));
+    const auto spread = [&](const char *name, int dim, int to, int row0) {  // heads of `dim` rows to heads of `to`
+        return b.pack_rows(mix + name, s.heads * dim, W, s.heads * to, o->in, row0, [&](int r) { return r % to < dim ? r / to * dim + r % to : -1; });
+    };
+    VHC(spread("q", s.dim, t.dim_pad, 0));
+    VHC(spread("v", s.vdim, t.v_pad, qs));
+    VHC(spread("f", s.dim, t.dim_pad, qs + vs));
+    std::vector<float> fb, lower, bias(qs, 0.f), keep(qs, 0.f), w;  // (channels that pad a head write nothing)
+    VHC(b.floats(mix + "f.b", {fd}, &fb));
+    VHC(b.floats(mix + "lower", {fd}, &lower));
+    for (int i = 0; i < fd; i++) {
+        const int at = i / s.dim * t.dim_pad + i % s.dim;
+        bias[at] = fb[i], keep[at] = (float)(1.0 - (double)lower[i]);
+    }
+    VHC(b.upload(bias, &t.bias));
+    VHC(b.upload(keep, &t.keep));
+    VHC(b.floats(mix + "norm", {s.vdim}, &w));
+    w.resize(t.v_pad, 0.f);
+    VHC(b.upload(w, &t.norm));
+    VHC(b.packed(&o->out, W, vs));
+    return b.pack_placed(mix + "o", W, vd, W, vs, o->out, 0, [&](int r, int k) -> int64_t {
+        return k % t.v_pad < s.vdim ? (int64_t)r * vd + k / t.v_pad * s.vdim + k % t.v_pad : -1;
+    });
+}
+
+int build_fitevik_mlp(Builder &b, const FitevikLayer &s, const std::string &mlp, int W, MixLayer *o) {
+    if (s.mlp == FitevikLayer::DENSE) {
+        o->has_mlp = o->relu2 = true;
+        o->ff = s.ff, o->ff_pad = b.pad(s.ff, 64);
+        VHC(b.packed(&o->gate_up, o->ff_pad, W));
+        VHC(b.pack(mlp + "up", s.ff, W, 0, s.ff, o->gate_up, 0, 1, 0));
+        VHC(b.packed(&o->down, W, s.ff));
+        VHC(b.pack(mlp + "down", W, s.ff, 0, W, o->down, 0, 1, 0));
+        std::vector<float> up;
+        VHC(b.floats(mlp + "up.b", {s.ff}, &up));
+        up.resize(o->ff_pad, 0.f);
+        VHC(b.upload(up, &o->up_bias));
+        return b.vec(mlp + "down.b", W, &o->down_bias);
+    }
+    ExpertMlp &e = o->moe;
+    o->has_experts = true;
+    e.experts = s.experts, e.top = s.top, e.relu2 = e.softmax = true;
+    VHC(b.packed(&e.router, s.experts, W));
+    VHC(b.pack(mlp + "router", s.experts, W, 0, s.experts, e.router, 0, 1, 0));
+    VHC(b.vec(mlp + "router.b", s.experts, &e.router_bias));
+    const int fp = e.ff_pad = b.pad(s.ff, 64), wp = b.pad(W, 32);
+    VHC(b.packed(&e.gate_up, s.experts * fp, W));
+    VHC(b.packed(&e.down, s.experts * wp, s.ff));
+    for (int i = 0; i < s.experts; i++) {
+        const std::string p = mlp + "e" + std::to_string(i);
+        VHC(b.pack(p + ".up", s.ff, W, 0, s.ff, e.gate_up, i * fp, 1, 0));
+        VHC(b.pack(p + ".down", W, s.ff, 0, W, e.down, i * wp, 1, 0));
+    }
+    e.gate_up.n = fp, e.down.n = wp;
+    return VH_OK;
+}
+
+int build_fitevik(Builder &b, const Json &config, MixModel *x, vh_config *cfg) {
+    FitevikConfig c;
+    VHC(parse_fitevik(config, &c));
+    cfg->hidden = c.width, cfg->vocab = c.vocab, cfg->eps = c.eps;
+    x->eps = c.eps, x->branch_norm = true, x->logit_mult = c.logit_scale, x->max_positions = c.max_positions;
+    const int W = c.width;
+    for (size_t i = 0; i < c.layers.size(); i++) {
+        const FitevikLayer &s = c.layers[i];
+        const std::string l = "l" + std::to_string(i) + ".";
+        MixLayer o;
+        VHC(b.vec(l + "norm1", W, &o.norm1));
+        VHC(b.vec(l + "norm1.b", W, &o.norm1b));
+        VHC(s.states ? build_fitevik_states(b, s, l + "mix.", W, &o) : build_fitevik_attention(b, s, l + "mix.", W, &o));
+        x->recurrent = x->recurrent || s.states;
+        if (s.mlp != FitevikLayer::NONE) {
+            VHC(b.vec(l + "norm2", W, &o.norm2));
+            VHC(b.vec(l + "norm2.b", W, &o.norm2b));
+            VHC(build_fitevik_mlp(b, s, l + "mlp.", W, &o));
+        }
+        x->layers.push_back(o);
+        LayerRun r;
+        r.layer = (int)i;
+        x->runs.push_back(r);
+    }
+    std::vector<float> emb;
+    VHC(b.floats("embed", {c.vocab, W}, &emb));
+    VHC(b.upload(emb, &b.m->embedding));
+    VHC(b.floats("pos", {c.max_positions, W}, &emb));
+    VHC(b.upload(emb, &x->positions));
+    VHC(b.vec("embed.norm", W, &x->emb_norm));
+    VHC(b.vec("embed.norm.b", W, &x->emb_norm_b));
+    VHC(b.vec("final.norm", W, &b.m->final_norm));
+    VHC(b.vec("final.norm.b", W, &x->final_norm_b));
+    VHC(b.packed(&x->head, c.vocab, W));
+    return b.pack("head", c.vocab, W, 0, c.vocab, x->head, 0, 1, 0);
+}
+
+int check_fitevik(const Json &config) {
+    FitevikConfig c;
+    return parse_fitevik(config, &c);
+}
+
 // ---------------------------------------------------------------- registry
 struct Architecture {
     const char *name;                                                    // config.json "architecture"
@@ -1067,6 +1282,7 @@ const Architecture kArchitectures[] = {
     {"Lozedra", check_lozedra, build_lozedra},
     {"Tulipel", check_tulipel, build_tulipel},
     {"Kitodra", check_kitodra, build_kitodra},
+    {"Fitevik", check_fitevik, build_fitevik},
 };
 
 const Architecture *find_architecture(const Json &config) {

@@ -9,6 +9,9 @@
 // or, with the norm behind the residual sum and latent attention,
 //   input projection (queries turned on the way) | norms, latents to the paged pool | queries into the latents' space |
 //   attention | results out of it | output projection | residual, norm | up | activation | down | residual, norm, average
+// or, with a layer norm on what a sublayer adds,
+//   input projection | heads to their places, or gates | attention, or states and their norm | output projection | norm, residual |
+//   up | down, or router | routing | experts' up | down | norm, residual
 // The block tables, the pool's bookkeeping and the sequence slots are the runtime's own; recurrent state lies in one slot
 // per sequence (the row of its block table), and a sequence at position 0 starts from nothing whatever the slot holds.
 #include <math.h>
@@ -40,6 +43,7 @@ Widths widths(const vh_model *m) {
     for (const MixLayer &l : m->mix->layers) {
         w.in = std::max(w.in, l.has_latent                    ? l.latent.heads * l.latent.head_cols
                               : l.has_decay                     ? l.decay.split
+                              : l.has_forget                    ? l.forget.heads * (l.forget.dim_pad + l.forget.v_pad)
                               : l.has_attn && l.attn.by_heads ? by_heads_ldq(l.attn)
                                                                 : l.in.n);
         w.out = std::max(w.out, l.out.k);
@@ -57,6 +61,7 @@ Widths widths(const vh_model *m) {
     }
     for (const MixLayer &l : m->mix->layers) {
         if (l.has_decay) w.o = std::max(w.o, l.decay.heads * l.decay.v_pad);
+        if (l.has_forget) w.o = std::max(w.o, l.forget.heads * l.forget.v_pad);
         if (l.has_experts) {
             const ExpertMlp &e = l.moe;
             w.e_act = std::max({w.e_act, e.ff_pad, e.shared_pad});
@@ -94,6 +99,8 @@ size_t slice_floats(const vh_model *m, int rows, bool up_to) {
         sliced(l.out, cols);
         sliced(l.down, cols);
         if (l.has_attn && l.attn.by_heads) sliced(l.in, l.in.n);
+        if (l.has_experts) sliced(l.moe.router, l.moe.router.n);
+        if (l.has_forget) most = std::max(most, (size_t)rows * l.forget.heads * l.forget.dim_pad);
         if (l.has_decay) most = std::max(most, (size_t)rows * (l.in.n - l.decay.split));
         if (!l.has_latent) continue;
         if (l.latent.q_rank > 0)
@@ -146,7 +153,7 @@ int mix_finish(vh_model *m) {
     for (LayerRun &r : x.runs) {
         const MixLayer &l = x.layers[r.layer];
         m->kv.push_back(nullptr);
-        if (l.has_attn) {
+        if (l.has_attn && l.attn.kv_from < 0) {
             // (what a kernel may read beyond a sequence's tokens is a finite number from the start)
             r.kv = zeroed(vx_kv_block_elems2(c.block_size, l.attn.kv_heads * l.attn.maps, l.attn.k_dim, l.attn.kv_heads, l.attn.v_dim) * c.pool_blocks * es);
             if (!r.kv) return fail("KV pool: %s", vx_last_error());
@@ -159,6 +166,7 @@ int mix_finish(vh_model *m) {
         }
         if (l.has_latent && l.latent.kv_from >= 0)  // (every layer runs once in a model that shares pools)
             r.kv = x.runs[l.latent.kv_from].kv;
+        if (l.has_attn && l.attn.kv_from >= 0) r.kv = x.runs[l.attn.kv_from].kv;
         if (l.has_scan) {
             r.state = (float *)zeroed((size_t)c.max_seqs * l.scan.channels * l.scan.pad * 4);
             if (!r.state) return fail("scan state: %s", vx_last_error());
@@ -170,9 +178,10 @@ int mix_finish(vh_model *m) {
     }
     for (LayerRun &r : x.runs) {
         const MixLayer &l = x.layers[r.layer];
-        if (!l.has_decay) continue;
-        r.state = (float *)zeroed((size_t)c.max_seqs * l.decay.heads * l.decay.dim_pad * l.decay.v_pad * 4);
-        if (!r.state) return fail("decaying state: %s", vx_last_error());
+        if (!l.has_decay && !l.has_forget) continue;
+        const size_t per = l.has_decay ? (size_t)l.decay.heads * l.decay.dim_pad * l.decay.v_pad : (size_t)l.forget.heads * l.forget.dim_pad * l.forget.v_pad;
+        r.state = (float *)zeroed(c.max_seqs * per * 4);
+        if (!r.state) return fail("states: %s", vx_last_error());
         m->adopted.push_back(r.state);
     }
     if (x.pairs) {
@@ -247,6 +256,7 @@ int run_router(vh_model *m, const MixLayer &l, int rows, const MixActs &a, const
     r.rows = rows, r.experts = e.experts, r.top = e.top, r.groups = e.groups, r.keep = e.keep, r.shared = e.shared;
     r.tile_rows = vx_route_tile_rows(m->mix->act, rows, e.experts, e.top);
     r.z = z + e.router_col, r.z_slices = slices, r.ldz = ldz, r.z_stride = (int64_t)rows * ldz;
+    r.bias = e.router_bias, r.softmax = e.softmax;
     r.correction = e.correction, r.weights = a.e_weights, r.places = a.e_places, r.order = a.e_order, r.tiles = a.e_tiles;
     VXC(vx_route(m->be, &r));
     return VH_OK;
@@ -262,7 +272,7 @@ int run_experts(vh_model *m, const MixLayer &l, int rows, const MixActs &a) {
     g.tile_rows = vx_route_tile_rows(m->mix->act, rows, e.experts, e.top);
     g.max_tiles = vx_route_max_tiles(rows, e.experts, e.top, e.shared, g.tile_rows);
     g.tiles = a.e_tiles;
-    g.kind = VX_LIN_SWIGLU, g.a = a.h, g.lda = pad_to(m->cfg.hidden, 64), g.a_rows = a.e_order;
+    g.kind = e.relu2 ? VX_LIN_RELU2 : VX_LIN_SWIGLU, g.a = a.h, g.lda = pad_to(m->cfg.hidden, 64), g.a_rows = a.e_order;
     g.w = e.gate_up.w, g.n = e.gate_up.n, g.k = e.gate_up.k, g.w_shared = e.shared_gate_up.w, g.n_shared = e.shared_gate_up.n, g.k_shared = e.shared_gate_up.k;
     g.glu_limit = e.limit, g.shared_limit = e.shared_limit, g.glu_alpha = e.alpha, g.glu_add = e.add;
     g.out = a.e_act, g.ldo = std::max(e.ff_pad, e.shared_pad), g.cols = e.ff_pad, g.cols_shared = e.shared_pad;
@@ -281,12 +291,29 @@ int run_out(vh_model *m, const MixLayer &l, int rows, const MixActs &a, int *sli
     return VH_OK;
 }
 
-// A layer of one mixer beside experts: a.h -> the mixer's output as `slices` partial sums in a.y, and the choice of experts.
-int run_beside_experts(vh_model *m, const LayerRun &r, const vx_ragged &b, const MixActs &a, int *slices) {
+// A layer's one mixer: a.h -> its output as `slices` partial sums in a.y; where experts stand beside it, their choice as well.
+int run_mixer(vh_model *m, const LayerRun &r, const vx_ragged &b, const MixActs &a, int *slices) {
     const MixModel &x = *m->mix;
     const MixLayer &l = x.layers[r.layer];
     const size_t es = esize(x);
     const int rows = b.rows, width_pad = pad_to(m->cfg.hidden, 64), ldc = l.out.k;
+    const bool beside = l.has_experts && !l.moe.router.w;
+    if (l.has_forget) {
+        const ForgetMixer &t = l.forget;
+        const int qs = t.heads * t.dim_pad, vs = t.heads * t.v_pad;
+        vx_linear_out o = plain(a.proj, 0, qs + vs, qs + vs, 1);
+        o.kind = VX_LIN_FORGET;
+        o.split = qs + vs, o.silu_cols = qs, o.out2 = a.y, o.ldo2 = qs, o.bias = t.bias, o.keep = t.keep;
+        VXC(vx_linear(m->be, x.act, a.h, width_pad, l.in.w, l.in.n, l.in.k, rows, &o));
+        vx_forget_args d;
+        memset(&d, 0, sizeof d);
+        d.heads = t.heads, d.dim = t.dim_pad, d.vdim = t.v_pad;
+        d.q = a.proj, d.v = at(a.proj, qs, es), d.g = a.y, d.ldq = d.ldv = qs + vs, d.ldg = qs;
+        d.state = r.state, d.out = a.o, d.ldo = vs;
+        VXC(vx_forget_attn(m->be, x.act, &b, &d));
+        VXC(vx_head_norm(m->be, x.act, a.o, vs, t.norm, x.eps, rows, t.heads, t.v_pad, t.vdim, a.cat, ldc));
+        return run_out(m, l, rows, a, slices);
+    }
     if (l.has_decay) {
         const DecayMixer &t = l.decay;
         const int side = l.in.n - t.split, vs = t.heads * t.v_pad;
@@ -294,7 +321,7 @@ int run_beside_experts(vh_model *m, const LayerRun &r, const vx_ragged &b, const
         o.kind = VX_LIN_SILU;
         o.split = t.split, o.out2 = a.y, o.ldo2 = side;
         VXC(vx_linear(m->be, x.act, a.h, width_pad, l.in.w, l.in.n, l.in.k, rows, &o));
-        if (l.has_experts) VHC(run_router(m, l, rows, a, a.y, 1, side));
+        if (beside) VHC(run_router(m, l, rows, a, a.y, 1, side));
         vx_decay_args d;
         memset(&d, 0, sizeof d);
         d.heads = t.heads, d.dim = t.dim_pad, d.vdim = t.v_pad, d.decay = t.decay;
@@ -309,14 +336,15 @@ int run_beside_experts(vh_model *m, const LayerRun &r, const vx_ragged &b, const
     *slices = vx_linear_slices(m->be, l.in.n, l.in.k, rows);
     vx_linear_out o = plain(a.y, 1, l.in.n, l.in.n, *slices);
     VXC(vx_linear(m->be, x.act, a.h, width_pad, l.in.w, l.in.n, l.in.k, rows, &o));
-    if (l.has_experts) VHC(run_router(m, l, rows, a, a.y, *slices, l.in.n));
+    if (beside) VHC(run_router(m, l, rows, a, a.y, *slices, l.in.n));
     vx_heads_args h;
     memset(&h, 0, sizeof h);
-    h.q_heads = t.heads * t.maps, h.k_heads = t.kv_heads * t.maps, h.v_heads = t.kv_heads, h.dim = t.k_dim, h.v_dim = t.v_dim;
+    h.q_heads = t.heads * t.maps, h.dim = t.k_dim, h.v_dim = t.v_dim;
     h.y = a.y, h.y_slices = *slices, h.ldy = l.in.n, h.y_stride = (int64_t)rows * l.in.n, h.bias = t.in_bias;
     h.q_col = t.q_col, h.k_col = t.k_col, h.v_col = t.v_col;
     if (t.rotation >= 0) h.rot_pairs = (int)x.rotations[t.rotation].freqs.size(), h.rot_tab = rot_table(x, a, rows, t.rotation);
-    h.norm = t.norm, h.eps = x.eps, h.w_q = t.norm_q, h.w_k = t.norm_k;
+    if (t.kv_from < 0) h.k_heads = t.kv_heads * t.maps, h.v_heads = t.kv_heads;
+    h.norm = t.row_norm ? 2 : t.norm, h.eps = x.eps, h.w_q = t.norm_q, h.w_k = t.norm_k;
     h.q = a.proj, h.ldq = by_heads_ldq(t), h.pool = r.kv;
     VXC(vx_heads_store(m->be, x.act, &b, &h));
     if (t.heads * t.v_dim < ldc) VXC(vx_fill_zero(m->be, a.cat, (size_t)rows * ldc * es));
@@ -324,6 +352,7 @@ int run_beside_experts(vh_model *m, const LayerRun &r, const vx_ragged &b, const
     memset(&at_, 0, sizeof at_);
     at_.heads = t.heads, at_.kv_heads = t.kv_heads, at_.k_dim = t.k_dim, at_.v_dim = t.v_dim, at_.scale = t.scale, at_.sink = t.sink;
     at_.window = t.window, at_.chunk = t.chunk, at_.softcap = t.softcap;
+    at_.slopes = t.slopes, at_.talk = t.talk;
     at_.maps = t.maps, at_.diff_lambda = t.diff_lambda, at_.diff_scale = t.diff_scale, at_.diff_eps = x.eps;
     at_.q = a.proj, at_.ldq = h.ldq, at_.pool = r.kv, at_.out_scale = 1.f, at_.out = a.cat, at_.ldo = ldc;
     VXC(vx_attn_ragged(m->be, x.act, &b, &at_));
@@ -477,7 +506,8 @@ int run_mlp(vh_model *m, const MixLayer &l, int rows, const MixActs &a, int *sli
     const int width_pad = pad_to(m->cfg.hidden, 64);
     const int cut = l.poly ? vx_linear_slices(m->be, l.gate_up.n, l.gate_up.k, rows) : 1;
     vx_linear_out o = plain(l.poly ? a.z : a.act, cut > 1, l.ff_pad, l.ff_pad, cut);
-    if (!l.poly) o.kind = VX_LIN_SWIGLU;
+    if (!l.poly) o.kind = l.relu2 ? VX_LIN_RELU2 : VX_LIN_SWIGLU;
+    o.bias = l.up_bias;
     VXC(vx_linear(m->be, x.act, a.h, width_pad, l.gate_up.w, l.gate_up.n, l.gate_up.k, rows, &o));
     if (l.poly)
         VXC(vx_poly_norm(m->be, x.act, a.z, l.ff_pad, cut > 1 ? cut : 0, (int64_t)rows * l.ff_pad, rows, l.ff, l.poly, x.eps, a.act, l.ff_pad));
@@ -494,7 +524,7 @@ namespace {
 int head_logits(vh_model *m, const MixActs &a, int n, float *logits) {
     const MixModel &x = *m->mix;
     vx_linear_out o = plain(logits, 1, m->cfg.vocab, m->cfg.vocab, 1);
-    o.softcap = x.softcap;
+    o.softcap = x.softcap, o.mult = x.logit_mult;
     VXC(vx_linear(m->be, x.act, a.h, pad_to(m->cfg.hidden, 64), x.head.w, x.head.n, x.head.k, n, &o));
     return VH_OK;
 }
@@ -537,7 +567,7 @@ int forward_pre_norm(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, c
         VXC(seam(l.norm1, r.add_embedding ? emb : nullptr));
         pending = true;
         if (!l.norm1b) {
-            VHC(run_beside_experts(m, r, b, a, &slices));
+            VHC(run_mixer(m, r, b, a, &slices));
             if (l.has_experts) VHC(run_experts(m, l, rows, a));
             post = nullptr, beside = &l;
             continue;
@@ -595,12 +625,58 @@ int forward_post_norm(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, 
     return VH_OK;
 }
 
+// Layers whose sublayers read the stream itself and are layer-normed before they join it.
+int forward_branch_norm(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, const MixActs &a, const int32_t *want, int n_want) {
+    const MixModel &x = *m->mix;
+    const vh_config &c = m->cfg;
+    const int rows = b.rows, n_runs = (int)x.runs.size();
+    VHC(rot_tables(m, b, a));
+    vx_branch_norm_args s;
+    memset(&s, 0, sizeof s);
+    s.rows = rows, s.cols = c.hidden, s.eps = x.eps, s.x_out = a.x, s.out = a.h, s.ldo = pad_to(c.hidden, 64);
+    s.x_in = m->embedding, s.tokens = d_tokens, s.token_pos = b.token_pos, s.positions = x.positions, s.w_pre = x.emb_norm, s.b_pre = x.emb_norm_b;
+    VXC(vx_branch_norm(m->be, x.act, &s));
+    s.x_in = a.x, s.tokens = nullptr, s.w_pre = s.b_pre = nullptr;
+    s.ldy = pad_to(c.hidden, 16), s.y_stride = (int64_t)rows * s.ldy;
+    const auto join = [&](const float *w, const float *bias, bool last) {
+        s.w = w, s.b = bias;
+        if (last) s.rows = n_want, s.row_idx = want, s.x_out = nullptr, s.w_pre = m->final_norm, s.b_pre = x.final_norm_b;
+        return vx_branch_norm(m->be, x.act, &s);
+    };
+    for (int i = 0; i < n_runs; i++) {
+        const MixLayer &l = x.layers[x.runs[i].layer];
+        const bool last = i + 1 == n_runs, ff = l.has_mlp || l.has_experts;
+        VHC(run_mixer(m, x.runs[i], b, a, &s.y_slices));
+        s.y = a.y, s.y_bias = l.out_bias, s.e_rows = nullptr;
+        if (last && n_want == 0 && !ff) return VH_OK;
+        VXC(join(l.norm1, l.norm1b, last && !ff));
+        if (!ff) continue;
+        if (last && n_want == 0) return VH_OK;  // (nothing behind the last layer's mixer is kept)
+        if (l.has_mlp) {
+            VHC(run_mlp(m, l, rows, a, &s.y_slices));
+            s.y_bias = l.down_bias;
+        } else {
+            const ExpertMlp &e = l.moe;
+            const int cut = vx_linear_slices(m->be, e.router.n, e.router.k, rows);
+            vx_linear_out o = plain(a.y, 1, e.router.n, e.router.n, cut);
+            VXC(vx_linear(m->be, x.act, a.h, pad_to(c.hidden, 64), e.router.w, e.router.n, e.router.k, rows, &o));
+            VHC(run_router(m, l, rows, a, a.y, cut, e.router.n));
+            VHC(run_experts(m, l, rows, a));
+            s.y = s.y_bias = nullptr;
+            s.e_rows = a.e_out, s.lde = e.down.n, s.e_top = e.top, s.e_places = a.e_places, s.e_weights = a.e_weights;
+        }
+        VXC(join(l.norm2, l.norm2b, last));
+    }
+    return VH_OK;
+}
+
 }  // namespace
 
 int mix_forward(vh_model *m, const vx_ragged &b, const int32_t *d_tokens, const MixActs &a, const MixExpand *ex, const int32_t *want,
                 int n_want, float *logits) {
     if (b.rows > a.rows) return fail("internal: %d rows, activations for %d", b.rows, a.rows);
-    VHC(m->mix->post_norm ? forward_post_norm(m, b, d_tokens, a, ex, want, n_want) : forward_pre_norm(m, b, d_tokens, a, want, n_want));
+    VHC(m->mix->branch_norm ? forward_branch_norm(m, b, d_tokens, a, want, n_want)
+        : m->mix->post_norm ? forward_post_norm(m, b, d_tokens, a, ex, want, n_want) : forward_pre_norm(m, b, d_tokens, a, want, n_want));
     return n_want > 0 ? head_logits(m, a, n_want, logits) : (int)VH_OK;
 }
 
@@ -686,6 +762,8 @@ int mix_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_l
             if (blocks > c.max_blocks_per_seq)
                 return fail("sequence %lld: %d tokens need %d blocks, max_blocks_per_seq is %d", (long long)seq_ids[i], len, blocks,
                             c.max_blocks_per_seq);
+            if (m->mix->max_positions > 0 && len > m->mix->max_positions)
+                return fail("sequence %lld: %d tokens, the model has %d positions", (long long)seq_ids[i], len, m->mix->max_positions);
             need += std::max(0, blocks - have);
         }
         if (fresh > m->pool.free_slots.size()) return fail("more than %d live sequences", c.max_seqs);

@@ -106,6 +106,10 @@ struct AttnMixer {
     float out_scale = 1.f;
     int q_col = 0, k_col = 0, v_col = 0, g_col = 0;    // v_col < 0: values are keys as projected
     bool by_heads = false, norm = false;
+    bool row_norm = false;                             // the norms are over all heads of a row
+    int kv_from = -1;                                  // the layer whose pool is read, -1: its own
+    const float *slopes = nullptr;                     // [heads], as they are behind the mixing of heads
+    const void *talk = nullptr;                        // bfloat16 [heads][heads]
     const float *in_bias = nullptr, *norm_q = nullptr, *norm_k = nullptr;
     int rotation = -1;                                 // index in MixModel::rotations, halves of a head's first dimensions
     int window = 0, chunk = 0;
@@ -123,13 +127,25 @@ struct DecayMixer {
     const float *decay = nullptr, *norm = nullptr;     // [heads][2]; [heads * v_pad]
 };
 
-// vx_route and vx_linear_experts over the layer's normed input; the router's logits are columns of the input projection's float32 part.
+// vx_forget_attn and vx_head_norm. Projection: q with SiLU | v, heads padded to dim_pad and v_pad columns; behind them, in float32, one minus
+// the gates.
+struct ForgetMixer {
+    int heads = 0, vdim = 0, dim_pad = 0, v_pad = 0;
+    const float *bias = nullptr, *keep = nullptr;      // [heads * dim_pad]: of the gates' projection; one minus their lower bound
+    const float *norm = nullptr;                       // [v_pad]
+};
+
+// vx_route and vx_linear_experts over the layer's normed input; the router's logits are columns of the input projection's float32 part,
+// or a map of their own. Experts: gate|up pairs, or (relu2) up alone.
 struct ExpertMlp {
     int experts = 0, top = 0, groups = 1, keep = 1;
     bool shared = false;
     int router_col = 0, ff_pad = 0, shared_pad = 0;
     float limit = 0.f, shared_limit = 0.f, alpha = 0.f, add = 0.f;
     const float *correction = nullptr;
+    bool relu2 = false, softmax = false;
+    Linear router;
+    const float *router_bias = nullptr;
     Linear gate_up, down, shared_gate_up, shared_down; // the experts' one behind the other: n counts one expert's
 };
 
@@ -169,12 +185,14 @@ struct LatentMixer {
 // x += mult * rms(mixers(rms(x) * norm1)) * norm1b, then the same around the MLP. The mixers of a layer read one input
 // projection and write one row, which one output projection takes. In a model with post_norm instead: x = rms(alpha * x +
 // mixer(x)) * norm1, x = rms(alpha * x + MLP(x)) * norm2, then the average over the depth. A layer with experts instead: x +=
-// mixer(h) + experts(h), h = rms(x) * norm1.
+// mixer(h) + experts(h), h = rms(x) * norm1. In a model with branch_norm: x += ln(mixer(x); norm1, norm1b), x += ln(MLP(x); norm2,
+// norm2b), MLP dense or experts.
 struct MixLayer {
     const float *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr;
-    bool has_attn = false, has_scan = false, has_latent = false, has_decay = false, has_mlp = false, has_experts = false;
+    bool has_attn = false, has_scan = false, has_latent = false, has_decay = false, has_forget = false, has_mlp = false, has_experts = false;
     AttnMixer attn;
     DecayMixer decay;
+    ForgetMixer forget;
     ExpertMlp moe;
     const float *out_bias = nullptr;   // of the output projection, in layers without norm1b
     LatentMixer latent;
@@ -182,6 +200,8 @@ struct MixLayer {
     Linear in, out;
     Linear gate_up, down;
     int ff = 0, ff_pad = 0;
+    bool relu2 = false;            // the MLP is down(relu(up + up_bias)^2) + down_bias, gate_up holds up alone
+    const float *up_bias = nullptr, *down_bias = nullptr;
     const float *poly = nullptr;   // set: the MLP is down(poly_norm(up)), gate_up holds up alone (vx_poly_norm)
     const float *depth_avg = nullptr;  // weights of the embedding output and of every result up to this layer's
 };
@@ -200,7 +220,7 @@ struct MixActs {      // a step's activations for up to `rows` rows
     void *h = nullptr, *proj = nullptr, *cat = nullptr, *xc = nullptr, *dtr = nullptr, *act = nullptr;
     void *qc = nullptr, *qa = nullptr, *lo = nullptr, *z = nullptr;  // query latent; queries and results in the latents' space; up's output
     float *hist = nullptr, *rot = nullptr;                           // results of all layers; angle tables, one after the other
-    float *o = nullptr;                                              // what the decaying states gave
+    float *o = nullptr;                                              // what states gave
     void *e_act = nullptr, *e_out = nullptr;                         // by place in the experts' order
     float *e_weights = nullptr;
     int32_t *e_places = nullptr, *e_order = nullptr, *e_tiles = nullptr;
@@ -219,7 +239,11 @@ struct MixModel {
     int act = VX_ACT_BF16;
     float eps = 1e-5f, mult = 1.f;
     bool post_norm = false;
-    float alpha = 1.f, softcap = 0.f;
+    bool branch_norm = false;
+    float alpha = 1.f, softcap = 0.f, logit_mult = 0.f;
+    // branch_norm: the embedding is ln(token's + position's; emb_norm, emb_norm_b), the last norm has a bias
+    const float *positions = nullptr, *emb_norm = nullptr, *emb_norm_b = nullptr, *final_norm_b = nullptr;
+    int max_positions = 0;         // > 0: a sequence holds no more tokens
     bool recurrent = false;        // a sequence is more than its blocks
     int expand_rows = 0;           // the smallest of the layers'
     const float *pairs = nullptr;  // set: the embedding has a table of token pairs (vx_pair_embedding)

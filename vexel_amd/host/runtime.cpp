@@ -1141,6 +1141,8 @@ int vh_prefill(vh_model *m, const int32_t *tokens, int n, int64_t seq_id, int st
 }
 
 // ------------------------------------------------------------------ a step of portions and single tokens
+int vh_model_max_positions(const vh_model *m) { return m && m->mix ? m->mix->max_positions : 0; }
+
 int vh_model_mixed_batches(const vh_model *m) { return m && m->mix ? 1 : 0; }
 
 int vh_step(vh_model *m, int n_seqs, const int64_t *seq_ids, const int32_t *q_lens, const int32_t *tokens, int n_want,
@@ -1476,6 +1478,9 @@ static int check_room(vh_model *m, const int64_t *seq_ids, const int32_t *positi
         if (blocks > m->cfg.max_blocks_per_seq)
             return fail("sequence %lld: %d more tokens need %d blocks, max_blocks_per_seq is %d", (long long)seq_ids[i], steps,
                         blocks, m->cfg.max_blocks_per_seq);
+        if (m->mix && m->mix->max_positions > 0 && positions[i] + steps > m->mix->max_positions)
+            return fail("sequence %lld: %d more tokens at position %d, the model has %d positions", (long long)seq_ids[i], steps, positions[i],
+                        m->mix->max_positions);
         need += std::max(0, blocks - (int)s->table.size());
     }
     if (need > (long long)m->pool.free_list.size())

@@ -180,6 +180,8 @@ int vh_sched_add_sequence(vh_scheduler *s, int64_t seq_id, const int32_t *prompt
     if (s->seqs.count(seq_id)) return sfail("sequence %lld already exists", (long long)seq_id);
     for (int i = 0; i < n; i++)
         if (prompt[i] < 0 || prompt[i] >= s->mc.vocab) return sfail("prompt token %d out of range", prompt[i]);
+    const int most = vh_model_max_positions(s->m);
+    if (most > 0 && n > most) return sfail("a prompt of %d tokens, the model has %d positions", n, most);
     if (vh_pool_create_sequence(s->m, seq_id) != VH_OK) return VH_ERR;
     Seq q;
     q.prompt.assign(prompt, prompt + n);
@@ -272,6 +274,7 @@ int vh_sched_step(vh_scheduler *s, int *tokens_out) {
     };
     int produced = 0;
     if (vh_model_mixed_batches(s->m)) {
+        const int most = vh_model_max_positions(s->m);
         // one batch: the next piece of every prompt and the next token of every decoding sequence
         std::vector<int64_t> ids;
         std::vector<int32_t> tokens, lens, want;
@@ -316,7 +319,7 @@ int vh_sched_step(vh_scheduler *s, int *tokens_out) {
             const int tok = am[w++];
             q.generated.push_back(tok);
             produced++;
-            if (is_stop(tok) || q.reached_max(s->cfg.max_tokens)) q.state = VH_SEQ_FINISHED;
+            if (is_stop(tok) || q.reached_max(s->cfg.max_tokens) || (most > 0 && q.position >= most)) q.state = VH_SEQ_FINISHED;
         }
         if (tokens_out) *tokens_out = produced;
         return VH_OK;

@@ -130,6 +130,11 @@ SIGNATURES = {
     "vx_decay_attn": (_i, [_vp, _i, _vp, _vp]),
     "vx_gated_norm": (_i, [_vp, _i, _vp, _i, _vp, _i, _vp, _f, _i, _i, _i, _vp, _i]),
     "vx_attn_ragged": (_i, [_vp, _i, _vp, _vp]),
+    "vx_branch_norm": (_i, [_vp, _i, _vp]),
+    "vx_forget_attn": (_i, [_vp, _i, _vp, _vp]),
+    "vx_forget_attn_fast": (_i, [_i, _i, _i]),
+    "vx_head_norm": (_i, [_vp, _i, _vp, _i, _vp, _f, _i, _i, _i, _i, _vp, _i]),
+    "vx_attn_talk_fast": (_i, [_i, _i, _i, _i, _i, _i]),
     "vx_attn_ragged_fast": (_i, [_i, _i, _i, _i, _i, _i]),
     "vx_latent_pad": (_i, [_i]),
     "vx_latent_row": (_i, [_i, _i]),

@@ -85,6 +85,7 @@ def load_host():
         h.vh_spell_out_rows.argtypes = [C.c_int, C.c_int, C.c_int]
         h.vh_step.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p]
         h.vh_model_mixed_batches.argtypes = [C.c_void_p]
+        h.vh_model_max_positions.argtypes = [C.c_void_p]
         h.vh_model_set_fused.argtypes = [C.c_void_p, C.c_int]
         h.vh_model_set_fused.restype = None
         h.vh_model_set_layer.argtypes = [C.c_void_p, C.c_int, C.POINTER(VhLayerWeights)]
@@ -448,6 +449,11 @@ class ModelRuntime:
     def mixed_batches(self):
         """Whether a step of this model is one batch of portions and single tokens (a mixer program)."""
         return bool(self._h.vh_model_mixed_batches(self._m))
+
+    @property
+    def max_positions(self):
+        """How many tokens a sequence may hold because the model has no more positions; 0: no such limit."""
+        return self._h.vh_model_max_positions(self._m)
 
     def verify_tree(self, seq_ids, input_tokens, start_pos, trees, want_logits=True):
         """One verification pass over a candidate tree per sequence (vh_verify_tree). trees: one
