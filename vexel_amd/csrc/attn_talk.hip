@@ -40,7 +40,7 @@ template <int KD, int VD, int TPW, bool SHARE>
 __global__ void __launch_bounds__(64 * MAX_WAVES) talk_kernel(TalkArgs t) {
     extern __shared__ float s_dyn[];
     const AttnArgs &a = t.a;
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6, l16 = lane & 15, q4 = (lane >> 4) * 4, q8 = (lane >> 4) * 8;
+    const int tid = threadIdx.x, lane = tid & 63, wave = wave_id(), nw = blockDim.x >> 6, l16 = lane & 15, q4 = (lane >> 4) * 4, q8 = (lane >> 4) * 8;
     const int per_die = (t.items + 7) >> 3;
     const int id = t.many ? (int)(blockIdx.x & 7) * per_die + (int)(blockIdx.x >> 3) : (int)blockIdx.x;  // neighbours share keys: on one die
     if (id >= t.items) return;

@@ -135,7 +135,7 @@ __global__ void __launch_bounds__(512) prepare_kernel(ForgetArgs a) {
     float *s_m = s_e + NB * DIM;                         // of the blocks between a pair of blocks: (2, 0), (3, 1), (3, 0)
     bf16 *s_qh = (bf16 *)(s_m + 3 * DIM), *s_ql = s_qh + CH * LD, *s_kh = s_ql + CH * LD, *s_kl = s_kh + CH * LD;
     const vx_forget_args &p = a.p;
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.y, l16 = lane & 15, q4 = (lane >> 4) * 4, q8 = (lane >> 4) * 8;
+    const int tid = threadIdx.x, lane = tid & 63, wave = wave_id(), h = blockIdx.y, l16 = lane & 15, q4 = (lane >> 4) * 4, q8 = (lane >> 4) * 8;
     int seq, ci, chunks;
     if (!item_of_seq(a.cu, a.n_seqs, CH, FEW + 1, blockIdx.x, &seq, &ci, &chunks)) return;
     const int row0 = a.cu[seq] + ci * CH, len = min(CH, a.cu[seq + 1] - row0);
@@ -268,7 +268,7 @@ __global__ void __launch_bounds__(256) walk_kernel(ForgetArgs a) {
     constexpr int DIM = DT * 32, LD = DIM + 8, LV = VC + 8, TILES = DIM / 16, TP = (TILES + 3) / 4, NV = VC / 16;
     __shared__ bf16 s_h[2][VC * LD], s_l[2][VC * LD], s_v[2][CH * LV];
     const vx_forget_args &p = a.p;
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.y, v0 = blockIdx.z * VC;
+    const int tid = threadIdx.x, lane = tid & 63, wave = wave_id(), h = blockIdx.y, v0 = blockIdx.z * VC;
     const int l16 = lane & 15, q4 = (lane >> 4) * 4, q8 = (lane >> 4) * 8, seq = blockIdx.x;
     const int row0 = a.cu[seq], rows = a.cu[seq + 1] - row0, chunks = (rows + CH - 1) / CH;
     if (rows <= FEW) return;

@@ -37,6 +37,10 @@ __device__ __forceinline__ f32x4 mma_act(f32x8 a, bf16x8 b, f32x4 acc) {
     return acc;
 }
 
+// The wave's number as a scalar: matrix products take no account of lanes that a condition leaves out, so such conditions have to be
+// branches of the whole wave.
+__device__ __forceinline__ int wave_id() { return __builtin_amdgcn_readfirstlane(threadIdx.x >> 6); }
+
 // The hardware's exponential and reciprocal are good to a unit in the last place; the exponent's own rounding adds |z| times
 // that.
 __device__ __forceinline__ float sigmoid_f(float z) {
