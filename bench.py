@@ -1039,6 +1039,73 @@ def kitodra_report(be, only=None, use_graph=True):
             mr.close()
 
 
+# Shapes of --fitevik-report, of the widths above: both mixers twice, an attention layer on another's keys, experts and dense
+# feed-forwards in turn. A row's experts have the dense feed-forward's size, which is that of a Kitodra row beside it.
+FITEVIK_SHAPES = {
+    "2048": dict(width=2048, heads=16, kv_heads=4, dim=128, experts=64, top=8, ff=704),
+    "4096": dict(width=4096, heads=32, kv_heads=8, dim=128, experts=32, top=8, ff=1792),
+}
+FITEVIK_MIXERS = ("attention", "hgrn2", "attention", "hgrn2")
+
+
+def write_fitevik(folder, width, heads, kv_heads, dim, experts, top, ff, window=1024, vocab=LOZEDRA_VOCAB, positions=8192):
+    """A Fitevik model of that shape with random weights."""
+    shapes = {"embed": (vocab, width), "pos": (positions, width), "embed.norm": (width,), "embed.norm.b": (width,), "final.norm": (width,),
+              "final.norm.b": (width,), "head": (vocab, width)}
+    entries = []
+    qd, kd = heads * dim, kv_heads * dim
+    for i, kind in enumerate(FITEVIK_MIXERS):
+        l, m, p = "l%d." % i, "l%d.mix." % i, "l%d.mlp." % i
+        mixer = {"heads": heads, "dim": dim, "vdim": dim}
+        shapes.update({l + n: (width,) for n in ("norm1", "norm1.b", "norm2", "norm2.b")})
+        shapes.update({m + "q": (qd, width), m + "o": (width, qd)})
+        if kind == "hgrn2":
+            shapes.update({m + "f": (qd, width), m + "f.b": (qd,), m + "lower": (qd,), m + "v": (qd, width), m + "norm": (dim,)})
+        else:
+            mixer.update(kv_heads=kv_heads, scale=dim ** -0.5, mask={"size": window})
+            shapes.update({m + "q.norm": (qd,), m + "talk": (heads, heads), m + "sink": (heads,)})
+            if i > 0:
+                mixer["kv_from"] = 0
+            else:
+                shapes.update({m + "k": (kd, width), m + "v": (kd, width), m + "k.norm": (kd,)})
+        if i in (0, 3):
+            mlp = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+            shapes.update({p + "router": (experts, width), p + "router.b": (experts,)})
+            for e in range(experts):
+                shapes.update({p + "e%d.up" % e: (ff, width), p + "e%d.down" % e: (width, ff)})
+        else:
+            mlp = {"kind": "dense", "ff": top * ff}
+            shapes.update({p + "up": (top * ff, width), p + "up.b": (top * ff,), p + "down": (width, top * ff), p + "down.b": (width,)})
+        entries.append({"type": kind, "mixer": mixer, "mlp": mlp})
+    cfg = {"architecture": "Fitevik", "layers": entries, "norm": {"eps": 1e-5}, "logit_scale": 1.0, "max_positions": positions, "vocab": vocab, "width": width}
+
+    def fill(name, shape):
+        if name.endswith("talk"):
+            return 0.8 * np.eye(heads) + 0.2 / heads
+        if name.endswith("lower"):
+            return (0.5, 0.05)
+        return (1.0, 0.05) if name.endswith(("norm", "norm1", "norm2")) else (0.0, 0.02)
+
+    write_folder(folder, cfg, shapes, fill)
+
+
+def fitevik_report(be, only=None, use_graph=True):
+    """Decode and prefill rates of Fitevik layers at real sizes (random weights) beside Kitodra layers of the same width and heads, the
+    closest model: attention over a window of the same size and linear attention in turn, experts. Runs as for --lozedra-report."""
+    rng = np.random.default_rng(2)
+    for name, c in FITEVIK_SHAPES.items():
+        if only not in (None, name):
+            continue
+        n = len(FITEVIK_MIXERS)
+        print("layers of width %s, %d of each model" % (name, n), flush=True)
+        kit = dict(KITODRA_SHAPES[name], mixers=("attention_2", "lightning") * 2)
+        for label, write in (("Fitevik bf16", lambda f: write_fitevik(f, **c)), ("Kitodra bf16", lambda f: write_kitodra(f, **kit))):
+            mr = load_written(be, write, **MIX_SIZES)
+            fill_contexts(mr, LOZEDRA_VOCAB, rng)
+            layer_rates(be, label, mr, list(range(MIX_SEQS)), n, LOZEDRA_VOCAB, MIX_CTX, 32, MIX_PORTIONS, use_graph, rng)
+            mr.close()
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -1074,6 +1141,9 @@ def main():
     ap.add_argument("--kitodra-report", nargs="?", const="all", choices=["all"] + list(KITODRA_SHAPES),
                     help="decode and prefill rates of Kitodra layers (one of each mixer) at real sizes beside Lozedra layers of the "
                          "same sizes, then exit")
+    ap.add_argument("--fitevik-report", nargs="?", const="all", choices=["all"] + list(FITEVIK_SHAPES),
+                    help="decode and prefill rates of Fitevik layers (both mixers twice) at real sizes beside Kitodra layers of the "
+                         "same sizes, then exit")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU: this build has no multi-GPU path (run with --gpus 1)", file=sys.stderr)
@@ -1103,6 +1173,9 @@ def main():
         return
     if args.kitodra_report:
         kitodra_report(be, None if args.kitodra_report == "all" else args.kitodra_report, use_graph=not args.no_graph)
+        return
+    if args.fitevik_report:
+        fitevik_report(be, None if args.fitevik_report == "all" else args.fitevik_report, use_graph=not args.no_graph)
         return
     ctx = ragged_contexts(n=args.seqs) if args.seqs != BATCH else ragged_contexts()
     nseq = len(ctx)
