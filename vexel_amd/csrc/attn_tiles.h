@@ -61,6 +61,19 @@ template <bool NT> __device__ __forceinline__ bf16x8 ld8(const bf16 *p) {
     return NT ? __builtin_nontemporal_load((const bf16x8 *)p) : *(const bf16x8 *)p;
 }
 
+// The largest of the four lanes with the same lane % 16. (The copies are opaque: of two equal operands the compiler takes both results for
+// equal as well.)
+__device__ __forceinline__ float max_of_quarters(float v) {
+    typedef unsigned u32x2 __attribute__((ext_vector_type(2)));
+    unsigned a = __builtin_bit_cast(unsigned, v), b = a;
+    asm("" : "+v"(b));
+    u32x2 p = __builtin_bit_cast(u32x2, __builtin_amdgcn_permlane16_swap(a, b, false, false));  // lanes 16 apart
+    a = b = __builtin_bit_cast(unsigned, fmaxf(__builtin_bit_cast(float, (unsigned)p[0]), __builtin_bit_cast(float, (unsigned)p[1])));
+    asm("" : "+v"(b));
+    p = __builtin_bit_cast(u32x2, __builtin_amdgcn_permlane32_swap(a, b, false, false));        // lanes 32 apart
+    return fmaxf(__builtin_bit_cast(float, (unsigned)p[0]), __builtin_bit_cast(float, (unsigned)p[1]));
+}
+
 // The keys of one group of 32 for a wave: K (of every map) as two 16 x (32 KD) operands, V^T as VD 16 x 32 operands.
 template <int KD, int VD, int MAPS, bool NT> struct Keys {
     bf16x8 k[MAPS][2][KD];
@@ -129,9 +142,9 @@ template <int KD, int VD, int QT> struct Queries {
         }
         const float factor = a.p.softcap > 0.f ? 1.0f : qs[t];
         if (a.p.slopes) {
-            const float n0 = (float)(pos[t] - key);
+            const float b0 = far[t] * (float)(key - pos[t]);
 #pragma unroll
-            for (int j = 0; j < 8; j++) s[j] = fmaf((j < 4 ? st0[j & 3] : st1[j & 3]), factor, far[t] * ((float)j - n0));
+            for (int j = 0; j < 8; j++) s[j] = fmaf((j < 4 ? st0[j & 3] : st1[j & 3]), factor, fmaf(far[t], (float)j, b0));
         } else if (distant || !a.p.bias) {
 #pragma unroll
             for (int j = 0; j < 8; j++) s[j] = fmaf((j < 4 ? st0[j & 3] : st1[j & 3]), factor, far[t]);
@@ -152,8 +165,7 @@ template <int KD, int VD, int QT> struct Queries {
         float mx = s[0];
 #pragma unroll
         for (int j = 1; j < 8; j++) mx = fmaxf(mx, s[j]);
-        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        mx = max_of_quarters(mx);
         const float mn = fmaxf(m[t], mx);
         if (__any(mn > m[t])) {
             const float al = mn > -INFINITY ? __builtin_amdgcn_exp2f(m[t] - mn) : 1.0f;

@@ -33,13 +33,15 @@ struct ForgetArgs {
     char *ws;         // per chunk and head: see Chunk
 };
 
-// What prepare_kernel leaves for a chunk of one head.
+// What prepare_kernel leaves for a chunk of one head, in tiles of 16 x 32 in the order in which a wave's lanes hold an operand: element (r,
+// c) of a tile at lane r + 16 (c / 8), place c % 8.
 template <int DIM> struct Chunk {
-    bf16 q_hi[CH][DIM], q_lo[CH][DIM];   // decayed queries
-    bf16 k_hi[DIM][CH], k_lo[DIM][CH];   // decayed keys, transposed
-    bf16 a_hi[CH][CH], a_lo[CH][CH];     // scores [row][key]; blocks above the diagonal's pairs of blocks are not written
+    bf16 q_hi[NB][DIM / 32][512], q_lo[NB][DIM / 32][512];         // decayed queries: rows x channels
+    bf16 k_hi[DIM / 16][CH / 32][512], k_lo[DIM / 16][CH / 32][512];  // decayed keys: channels x rows
+    bf16 a_hi[NB][CH / 32][512], a_lo[NB][CH / 32][512];           // scores: rows x keys; tiles above the diagonal are not written
     float decay[DIM];
 };
+__device__ __forceinline__ int in_tile(int r, int c) { return ((r & 15) + ((c & 31) >> 3) * 16) * 8 + (c & 7); }
 
 // ---------------------------------------------------------------- few rows
 // Thread: columns 4 (tid % 8) .. of the workgroup's 32, state rows tid / 8 + 32 i.
@@ -127,88 +129,133 @@ __device__ __forceinline__ bf16x8 scaled_hi(bf16x8 hi, bf16x8 lo, const float *m
     return h;
 }
 
+// A thread works out the decays of one channel in one block, in registers; then the workgroup's waves share the scores. The scores inside
+// blocks read the chunk's queries and gates from LDS, those between blocks the decayed queries and keys, in the same place.
 template <int DIM>
-__global__ void __launch_bounds__(512) prepare_kernel(ForgetArgs a) {
-    constexpr int LD = DIM + 8, LG = DIM + 4, DS = DIM / 16;
+__global__ void __launch_bounds__(NB * DIM) prepare_kernel(ForgetArgs a) {
+    constexpr int LD = DIM + 8, LG = DIM + 4, DS = DIM / 16, WAVES = NB * DIM / 64;
     extern __shared__ float s_dyn[];
-    float *s_g = s_dyn, *s_e = s_g + CH * LG;            // 1 - gates [CH][LG]; decays of whole blocks [NB][DIM]
-    float *s_m = s_e + NB * DIM;                         // of the blocks between a pair of blocks: (2, 0), (3, 1), (3, 0)
-    bf16 *s_qh = (bf16 *)(s_m + 3 * DIM), *s_ql = s_qh + CH * LD, *s_kh = s_ql + CH * LD, *s_kl = s_kh + CH * LD;
+    float *s_e = s_dyn, *s_m = s_e + NB * DIM;           // decays of whole blocks [NB][DIM]; of the blocks between a pair: (2, 0), (3, 1), (3, 0)
+    float *s_b = s_m + 3 * DIM;                          // of the blocks ahead of each [NB][DIM]
+    float *s_g = s_b + NB * DIM;                         // 1 - gates [CH][LG]
+    bf16 *s_q = (bf16 *)(s_g + CH * LG);                 // queries [CH][LD]
+    bf16 *s_qh = (bf16 *)s_g, *s_ql = s_qh + CH * LD, *s_kh = s_ql + CH * LD, *s_kl = s_kh + CH * LD;
     const vx_forget_args &p = a.p;
     const int tid = threadIdx.x, lane = tid & 63, wave = wave_id(), h = blockIdx.y, l16 = lane & 15, q4 = (lane >> 4) * 4, q8 = (lane >> 4) * 8;
     int seq, ci, chunks;
     if (!item_of_seq(a.cu, a.n_seqs, CH, FEW + 1, blockIdx.x, &seq, &ci, &chunks)) return;
     const int row0 = a.cu[seq] + ci * CH, len = min(CH, a.cu[seq + 1] - row0);
-    const bf16 *q = (const bf16 *)p.q + (size_t)row0 * p.ldq + h * DIM;
-    const float *g = p.g + (size_t)row0 * p.ldg + h * DIM;
     Chunk<DIM> &out = ((Chunk<DIM> *)a.ws)[(size_t)blockIdx.x * p.heads + h];
-    for (int i = tid; i < CH * DIM; i += 512) {  // (rows beyond the sequence: they keep everything and write nothing)
-        const int t = i / DIM, d = i % DIM;
-        s_g[t * LG + d] = t < len ? g[(size_t)t * p.ldg + d] : 0.f;
+    const int d = tid % DIM, b = tid / DIM;
+    bf16 q[SB];
+    float g[SB];
+#pragma unroll
+    for (int j = 0; j < SB; j++) {  // (rows beyond the sequence: they keep everything and write nothing)
+        const int t = b * SB + j, row = row0 + min(t, len - 1);
+        q[j] = ((const bf16 *)p.q)[(size_t)row * p.ldq + h * DIM + d];
+        g[j] = p.g[(size_t)row * p.ldg + h * DIM + d];
     }
+    float keep = 1.f, left = 1.f, qd[SB], kd[SB];
+#pragma unroll
+    for (int j = 0; j < SB; j++) {
+        const int t = b * SB + j;
+        if (t >= len) q[j] = (bf16)0.f, g[j] = 0.f;
+        s_q[t * LD + d] = q[j], s_g[t * LG + d] = g[j];
+        keep *= 1.0f - g[j];
+        qd[j] = (float)q[j] * keep;
+    }
+#pragma unroll
+    for (int j = SB - 1; j >= 0; j--) {
+        kd[j] = g[j] * left;
+        left *= 1.0f - g[j];
+    }
+    s_e[b * DIM + d] = keep;
     __syncthreads();
-    // a thread: one channel of one block
-    for (int i = tid; i < NB * DIM; i += 512) {
-        const int d = i % DIM, b = i / DIM;
-        float keep = 1.f;
-        for (int t = b * SB; t < (b + 1) * SB; t++) {
-            keep *= 1.0f - s_g[t * LG + d];
-            const float v = t < len ? (float)q[(size_t)t * p.ldq + d] * keep : 0.f;
-            bf16 x, y;
-            split(v, &x, &y);
-            s_qh[t * LD + d] = x, s_ql[t * LD + d] = y;
-        }
-        s_e[b * DIM + d] = keep;
-        float left = 1.f;
-        for (int t = (b + 1) * SB - 1; t >= b * SB; t--) {
-            const float v = s_g[t * LG + d];
-            bf16 x, y;
-            split(v * left, &x, &y);
-            s_kh[t * LD + d] = x, s_kl[t * LD + d] = y;
-            left *= 1.0f - v;
-        }
-    }
-    __syncthreads();
-    for (int d = tid; d < DIM; d += 512) {
-        const float e1 = s_e[DIM + d], e2 = s_e[2 * DIM + d];
-        s_m[d] = e1, s_m[DIM + d] = e2, s_m[2 * DIM + d] = e1 * e2;
-        out.decay[d] = s_e[d] * e1 * e2 * s_e[3 * DIM + d];
-    }
-    for (int i = tid; i < NB * DIM; i += 512) {
-        const int d = i % DIM, b = i / DIM;
+    {
         float before = 1.f, after = 1.f;
-        for (int k = 0; k < b; k++) before *= s_e[k * DIM + d];
-        for (int k = b + 1; k < NB; k++) after *= s_e[k * DIM + d];
+#pragma unroll
+        for (int k = 0; k < NB; k++) {
+            const float e = s_e[k * DIM + d];
+            if (k < b) before *= e;
+            if (k > b) after *= e;
+        }
+        if (b == 0) {
+            const float e1 = s_e[DIM + d], e2 = s_e[2 * DIM + d];
+            s_m[d] = e1, s_m[DIM + d] = e2, s_m[2 * DIM + d] = e1 * e2;
+            out.decay[d] = keep * after;
+        }
+        s_b[b * DIM + d] = before;
         bf16x8 kh[2], kl[2];
 #pragma unroll
         for (int j = 0; j < SB; j++) {
-            const int t = b * SB + j;
             bf16 x, y;
-            split(((float)s_qh[t * LD + d] + (float)s_ql[t * LD + d]) * before, &x, &y);
-            out.q_hi[t][d] = x, out.q_lo[t][d] = y;
-            split(((float)s_kh[t * LD + d] + (float)s_kl[t * LD + d]) * after, &x, &y);
+            split(kd[j] * after, &x, &y);
             kh[j >> 3][j & 7] = x, kl[j >> 3][j & 7] = y;
         }
 #pragma unroll
         for (int x = 0; x < 2; x++) {
-            *(bf16x8 *)&out.k_hi[d][b * SB + x * 8] = kh[x];
-            *(bf16x8 *)&out.k_lo[d][b * SB + x * 8] = kl[x];
+            const int at = in_tile(d, b * SB + x * 8);
+            *(bf16x8 *)&out.k_hi[d >> 4][b >> 1][at] = kh[x];
+            *(bf16x8 *)&out.k_lo[d >> 4][b >> 1][at] = kl[x];
         }
+    }
+    // scores inside blocks: 16 lanes take one key, DS channels each, through the block's rows from the key's own on; a wave takes four
+    // neighbouring keys
+    for (int u = wave; u < NB * SB / 4; u += WAVES) {
+        const int blk = u >> 2, s = (u & 3) * 4 + (lane >> 4), slice = l16 * DS, first = (u & 3) * 4;
+        const float *gp = s_g + blk * SB * LG + slice;
+        const bf16 *qp = s_q + blk * SB * LD + slice;
+        float w[DS], own = 0.f;
+#pragma unroll
+        for (int e = 0; e < DS; e++) w[e] = gp[s * LG + e];
+        for (int t = first; t < SB; t++) {
+            float dot = 0.f;
+#pragma unroll
+            for (int e = 0; e < DS; e++) {
+                const float gt = t > s ? gp[t * LG + e] : 0.f;
+                w[e] = fmaf(-gt, w[e], w[e]);
+                dot = fmaf((float)qp[t * LD + e], w[e], dot);
+            }
+            dot = sum16(dot);
+            if (l16 == t && t >= s) own = dot;
+        }
+        bf16 x, y;
+        split(own, &x, &y);
+        const int at = in_tile(l16, blk * SB + s);
+        out.a_hi[blk][blk >> 1][at] = x, out.a_lo[blk][blk >> 1][at] = y;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int j = 0; j < SB; j++) {
+        const int t = b * SB + j;
+        bf16 x, y;
+        split(qd[j], &x, &y);
+        s_qh[t * LD + d] = x, s_ql[t * LD + d] = y;
+        split(kd[j], &x, &y);
+        s_kh[t * LD + d] = x, s_kl[t * LD + d] = y;
     }
     __syncthreads();
     // scores between blocks: a wave takes queries of block bi and keys of block bj
-    if (wave < 6) {
-        const int bi = wave < 1 ? 1 : wave < 3 ? 2 : 3, bj = wave < 1 ? 0 : wave < 3 ? wave - 1 : wave - 3;
+    for (int u = wave; u < 8; u += WAVES) {
+        if (u >= 6) {  // above the diagonal, where a pair of blocks is read together
+            const int bi = (u - 6) * 2;
+            const bf16x4 zero = bf16x4{(bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f};
+            const int at = in_tile(l16, (bi + 1) * SB + q4);
+            *(bf16x4 *)&out.a_hi[bi][bi >> 1][at] = zero;
+            *(bf16x4 *)&out.a_lo[bi][bi >> 1][at] = zero;
+            continue;
+        }
+        const int bi = u < 1 ? 1 : u < 3 ? 2 : 3, bj = u < 1 ? 0 : u < 3 ? u - 1 : u - 3;
         const float *m = bi - bj < 2 ? nullptr : s_m + (bi - bj == 3 ? 2 : bj) * DIM;
         f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int d = 0; d < DIM; d += 32) {
-            const int at_q = (bi * SB + l16) * LD + d + q8, at_k = (bj * SB + l16) * LD + d + q8;
+        for (int c = 0; c < DIM; c += 32) {
+            const int at_q = (bi * SB + l16) * LD + c + q8, at_k = (bj * SB + l16) * LD + c + q8;
             bf16x8 qh = *(const bf16x8 *)(s_qh + at_q), ql = *(const bf16x8 *)(s_ql + at_q);
             const bf16x8 kh = *(const bf16x8 *)(s_kh + at_k), kl = *(const bf16x8 *)(s_kl + at_k);
             if (m) {
                 bf16x8 low;
-                qh = scaled_hi(qh, ql, m + d + q8, &low);
+                qh = scaled_hi(qh, ql, m + c + q8, &low);
                 ql = low;
             }
             acc = mma(kl, qh, acc);
@@ -222,53 +269,30 @@ __global__ void __launch_bounds__(512) prepare_kernel(ForgetArgs a) {
             split(acc[r], &x, &y);
             hi[r] = x, lo[r] = y;
         }
-        *(bf16x4 *)&out.a_hi[bi * SB + l16][bj * SB + q4] = hi;
-        *(bf16x4 *)&out.a_lo[bi * SB + l16][bj * SB + q4] = lo;
-    } else {  // above the diagonal, where a pair of blocks is read together
-        const int bi = (wave - 6) * 2;
-        const bf16x4 zero = bf16x4{(bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f};
-        *(bf16x4 *)&out.a_hi[bi * SB + l16][(bi + 1) * SB + q4] = zero;
-        *(bf16x4 *)&out.a_lo[bi * SB + l16][(bi + 1) * SB + q4] = zero;
+        const int at = in_tile(l16, bj * SB + q4);
+        *(bf16x4 *)&out.a_hi[bi][bj >> 1][at] = hi;
+        *(bf16x4 *)&out.a_lo[bi][bj >> 1][at] = lo;
     }
-    // scores inside blocks: 16 lanes take one key, DS channels each, through the block's rows from the key's own on
-#pragma unroll 1
-    for (int half = 0; half < 2; half++) {
-        const int task = half * 512 + tid, b = task >> 8, s = (task >> 4) & 15, slice = tid & 15;
-        float w[DS], own = 0.f;
-#pragma unroll
-        for (int e = 0; e < DS; e++) w[e] = s_g[(b * SB + s) * LG + slice * DS + e];
-        for (int t = s & ~3; t < SB; t++) {  // (a wave's four keys start together)
-            const int row = b * SB + t;
-            float dot = 0.f;
-            if (t >= s) {
-#pragma unroll
-                for (int e = 0; e < DS; e++) {
-                    const float gt = s_g[row * LG + slice * DS + e];
-                    if (t > s) w[e] = fmaf(-gt, w[e], w[e]);
-                    dot = fmaf(row < len ? (float)q[(size_t)row * p.ldq + slice * DS + e] : 0.f, w[e], dot);
-                }
-            }
-            dot = sum16(dot);
-            if (slice == t) own = dot;  // (0 in rows ahead of the key)
-        }
-        bf16 x, y;
-        split(own, &x, &y);
-        out.a_hi[b * SB + slice][b * SB + s] = x, out.a_lo[b * SB + slice][b * SB + s] = y;
+    // the queries, decayed from the chunk's start on: a wave writes whole tiles
+    for (int u = wave; u < NB * DIM / 32; u += WAVES) {
+        const int blk = u / (DIM / 32), c = u % (DIM / 32) * 32 + q8, at = (blk * SB + l16) * LD + c;
+        bf16x8 lo;
+        const bf16x8 hi = scaled_hi(*(const bf16x8 *)(s_qh + at), *(const bf16x8 *)(s_ql + at), s_b + blk * DIM + c, &lo);
+        *(bf16x8 *)&out.q_hi[blk][c >> 5][lane * 8] = hi;
+        *(bf16x8 *)&out.q_lo[blk][c >> 5][lane * 8] = lo;
     }
 }
 
-// What a chunk's step of the walk reads, a chunk ahead.
-template <int DT, int TP> struct Operands {
-    bf16x8 qh[DT], ql[DT], ah[2], al[2], kh[TP][2], kl[TP][2], v;
-    f32x4 f[TP];
-};
+// Waves 0 .. 3: the outputs of a block of rows each. Waves 4 .. 7: the state, every fourth tile of 16 channels. The state before a chunk
+// and the chunk's values pass through LDS, in two buffers that take turns; what comes from memory is read AHEAD chunks ahead.
+constexpr int AHEAD = 3;
 
 template <int DT>
-__global__ void __launch_bounds__(256) walk_kernel(ForgetArgs a) {
+__global__ void __launch_bounds__(512) walk_kernel(ForgetArgs a) {
     constexpr int DIM = DT * 32, LD = DIM + 8, LV = VC + 8, TILES = DIM / 16, TP = (TILES + 3) / 4, NV = VC / 16;
     __shared__ bf16 s_h[2][VC * LD], s_l[2][VC * LD], s_v[2][CH * LV];
     const vx_forget_args &p = a.p;
-    const int tid = threadIdx.x, lane = tid & 63, wave = wave_id(), h = blockIdx.y, v0 = blockIdx.z * VC;
+    const int tid = threadIdx.x & 255, lane = tid & 63, wave = wave_id() & 3, h = blockIdx.y, v0 = blockIdx.z * VC;
     const int l16 = lane & 15, q4 = (lane >> 4) * 4, q8 = (lane >> 4) * 8, seq = blockIdx.x;
     const int row0 = a.cu[seq], rows = a.cu[seq + 1] - row0, chunks = (rows + CH - 1) / CH;
     if (rows <= FEW) return;
@@ -279,8 +303,65 @@ __global__ void __launch_bounds__(256) walk_kernel(ForgetArgs a) {
     }
     const Chunk<DIM> *chunk = (const Chunk<DIM> *)a.ws + (size_t)first * p.heads + h;
     const int cols = min(VC, p.vdim - v0);
+    if (wave_id() < 4) {
+        struct {
+            bf16x8 qh[DT], ql[DT], ah[2], al[2];
+        } op[AHEAD];
+        const auto fetch = [&](int c, auto &o) {
+            const Chunk<DIM> &k = chunk[(size_t)min(c, chunks - 1) * p.heads];
+#pragma unroll
+            for (int i = 0; i < DT; i++) {
+                o.qh[i] = *(const bf16x8 *)&k.q_hi[wave][i][lane * 8];
+                o.ql[i] = *(const bf16x8 *)&k.q_lo[wave][i][lane * 8];
+            }
+#pragma unroll
+            for (int i = 0; i < 2; i++) {
+                if (i * 2 > wave) break;
+                o.ah[i] = *(const bf16x8 *)&k.a_hi[wave][i][lane * 8];
+                o.al[i] = *(const bf16x8 *)&k.a_lo[wave][i][lane * 8];
+            }
+        };
+        const auto step = [&](int c, auto &o) {
+            const bf16 *sh = s_h[c & 1], *sl = s_l[c & 1], *sv = s_v[c & 1];
+            __syncthreads();
+            f32x4 acc[NV];
+#pragma unroll
+            for (int n = 0; n < NV; n++) {
+                acc[n] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int k = 0; k < DT; k++) {
+                    const int at = (n * 16 + l16) * LD + k * 32 + q8;
+                    const bf16x8 hi = *(const bf16x8 *)(sh + at), lo = *(const bf16x8 *)(sl + at);
+                    acc[n] = mma(lo, o.qh[k], acc[n]);
+                    acc[n] = mma(hi, o.ql[k], acc[n]);
+                    acc[n] = mma(hi, o.qh[k], acc[n]);
+                }
+#pragma unroll
+                for (int k = 0; k < 2; k++) {
+                    if (k * 2 > wave) break;
+                    const bf16x8 vt = column8(sv, LV, k * 32, n * 16, lane);
+                    acc[n] = mma(vt, o.al[k], acc[n]);
+                    acc[n] = mma(vt, o.ah[k], acc[n]);
+                }
+            }
+            if (c + AHEAD < chunks) fetch(c + AHEAD, o);
+            const int t = c * CH + wave * 16 + l16;
+            if (t >= rows) return;
+            float *out = p.out + (size_t)(row0 + t) * p.ldo + h * p.vdim + v0 + q4;
+#pragma unroll
+            for (int n = 0; n < NV; n++)
+                if (n * 16 < cols) *(f32x4 *)(out + n * 16) = acc[n];
+        };
+#pragma unroll
+        for (int i = 0; i < AHEAD; i++) fetch(i, op[i]);
+        for (int c = 0; c < chunks; c += AHEAD)
+#pragma unroll
+            for (int i = 0; i < AHEAD; i++)
+                if (c + i < chunks) step(c + i, op[i]);
+        return;
+    }
     float *state = p.state + ((size_t)a.slots[seq] * p.heads + h) * DIM * p.vdim + v0;
-    // this wave's channel tiles wave + 4 x: rows 16 tile + 4 (lane / 16) .., columns 16 n + lane % 16
+    // channels 16 tile + 4 (lane / 16) .. of tile wave + 4 x, columns 16 n + lane % 16
     f32x4 S[TP][NV];
     const bool old = a.pos[row0] > 0;
 #pragma unroll
@@ -293,37 +374,28 @@ __global__ void __launch_bounds__(256) walk_kernel(ForgetArgs a) {
                 S[x][n][r] = old && d < DIM && c < cols ? state[(size_t)d * p.vdim + c] : 0.f;
             }
     const bf16 *vp = (const bf16 *)p.v + (size_t)row0 * p.ldv + h * p.vdim + v0;
-    Operands<DT, TP> next;
-    const auto fetch = [&](int c) {
-        const Chunk<DIM> &o = chunk[(size_t)c * p.heads];
+    struct {
+        bf16x8 kh[TP][2], kl[TP][2], v;
+        f32x4 f[TP];
+    } op[AHEAD];
+    const auto fetch = [&](int c, auto &o) {
+        const Chunk<DIM> &k = chunk[(size_t)min(c, chunks - 1) * p.heads];
+        const int t = c * CH + (tid >> 2), col = (tid & 3) * 8;
 #pragma unroll
-        for (int k = 0; k < DT; k++) {
-            next.qh[k] = *(const bf16x8 *)&o.q_hi[wave * 16 + l16][k * 32 + q8];
-            next.ql[k] = *(const bf16x8 *)&o.q_lo[wave * 16 + l16][k * 32 + q8];
-        }
-#pragma unroll
-        for (int k = 0; k < 2; k++) {
-            if (k * 2 > wave) break;
-            next.ah[k] = *(const bf16x8 *)&o.a_hi[wave * 16 + l16][k * 32 + q8];
-            next.al[k] = *(const bf16x8 *)&o.a_lo[wave * 16 + l16][k * 32 + q8];
-        }
+        for (int e = 0; e < 8; e++) o.v[e] = (bf16)0.f;
+        if (t < rows && col < cols) o.v = *(const bf16x8 *)(vp + (size_t)t * p.ldv + col);
 #pragma unroll
         for (int x = 0; x < TP; x++) {
             const int tile = min(wave + 4 * x, TILES - 1);
 #pragma unroll
-            for (int k = 0; k < 2; k++) {
-                next.kh[x][k] = *(const bf16x8 *)&o.k_hi[tile * 16 + l16][k * 32 + q8];
-                next.kl[x][k] = *(const bf16x8 *)&o.k_lo[tile * 16 + l16][k * 32 + q8];
+            for (int i = 0; i < 2; i++) {
+                o.kh[x][i] = *(const bf16x8 *)&k.k_hi[tile][i][lane * 8];
+                o.kl[x][i] = *(const bf16x8 *)&k.k_lo[tile][i][lane * 8];
             }
-            next.f[x] = *(const f32x4 *)&o.decay[tile * 16 + q4];
+            o.f[x] = *(const f32x4 *)&k.decay[tile * 16 + q4];
         }
-        const int t = c * CH + (tid >> 2), col = (tid & 3) * 8;
-#pragma unroll
-        for (int e = 0; e < 8; e++) next.v[e] = (bf16)0.f;
-        if (t < rows && col < cols) next.v = *(const bf16x8 *)(vp + (size_t)t * p.ldv + col);
     };
-    fetch(0);
-    for (int c = 0; c < chunks; c++) {
+    const auto step = [&](int c, auto &o) {
         bf16 *sh = s_h[c & 1], *sl = s_l[c & 1], *sv = s_v[c & 1];
 #pragma unroll
         for (int x = 0; x < TP; x++) {
@@ -342,52 +414,32 @@ __global__ void __launch_bounds__(256) walk_kernel(ForgetArgs a) {
                 *(bf16x4 *)(sl + at) = lo;
             }
         }
-        *(bf16x8 *)(sv + (tid >> 2) * LV + (tid & 3) * 8) = next.v;
-        const Operands<DT, TP> cur = next;
+        *(bf16x8 *)(sv + (tid >> 2) * LV + (tid & 3) * 8) = o.v;
         __syncthreads();  // (the buffers written now were last read two chunks ago, before the barrier of the chunk between)
-        if (c + 1 < chunks) fetch(c + 1);
         bf16x8 vt[2][NV];
 #pragma unroll
         for (int k = 0; k < 2; k++)
 #pragma unroll
             for (int n = 0; n < NV; n++) vt[k][n] = column8(sv, LV, k * 32, n * 16, lane);
-        f32x4 acc[NV];
-#pragma unroll
-        for (int n = 0; n < NV; n++) {
-            acc[n] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-            for (int k = 0; k < DT; k++) {
-                const bf16x8 hi = *(const bf16x8 *)(sh + (n * 16 + l16) * LD + k * 32 + q8), lo = *(const bf16x8 *)(sl + (n * 16 + l16) * LD + k * 32 + q8);
-                acc[n] = mma(lo, cur.qh[k], acc[n]);
-                acc[n] = mma(hi, cur.ql[k], acc[n]);
-                acc[n] = mma(hi, cur.qh[k], acc[n]);
-            }
-#pragma unroll
-            for (int k = 0; k < 2; k++) {
-                if (k * 2 > wave) break;
-                acc[n] = mma(vt[k][n], cur.al[k], acc[n]);
-                acc[n] = mma(vt[k][n], cur.ah[k], acc[n]);
-            }
-        }
-        const int t = c * CH + wave * 16 + l16;
-        if (t < rows) {
-            float *out = p.out + (size_t)(row0 + t) * p.ldo + h * p.vdim + v0 + q4;
-#pragma unroll
-            for (int n = 0; n < NV; n++)
-                if (n * 16 < cols) *(f32x4 *)(out + n * 16) = acc[n];
-        }
 #pragma unroll
         for (int x = 0; x < TP; x++)
 #pragma unroll
             for (int n = 0; n < NV; n++) {
-                S[x][n] *= cur.f[x];
+                S[x][n] *= o.f[x];
 #pragma unroll
                 for (int k = 0; k < 2; k++) {
-                    S[x][n] = mma(cur.kl[x][k], vt[k][n], S[x][n]);
-                    S[x][n] = mma(cur.kh[x][k], vt[k][n], S[x][n]);
+                    S[x][n] = mma(o.kl[x][k], vt[k][n], S[x][n]);
+                    S[x][n] = mma(o.kh[x][k], vt[k][n], S[x][n]);
                 }
             }
-    }
+        if (c + AHEAD < chunks) fetch(c + AHEAD, o);
+    };
+#pragma unroll
+    for (int i = 0; i < AHEAD; i++) fetch(i, op[i]);
+    for (int c = 0; c < chunks; c += AHEAD)
+#pragma unroll
+        for (int i = 0; i < AHEAD; i++)
+            if (c + i < chunks) step(c + i, op[i]);
 #pragma unroll
     for (int x = 0; x < TP; x++)
 #pragma unroll
@@ -419,7 +471,8 @@ void launch_step(vx_backend *be, const ForgetArgs &a) {
 template <int DT>
 int launch_chunks(vx_backend *be, ForgetArgs a, int chunks) {
     constexpr int DIM = DT * 32;
-    constexpr size_t lds = (size_t)(CH * (DIM + 4) + (NB + 3) * DIM) * 4 + (size_t)4 * CH * (DIM + 8) * 2;
+    constexpr size_t inside = (size_t)CH * (DIM + 4) * 4 + (size_t)CH * (DIM + 8) * 2, between = (size_t)4 * CH * (DIM + 8) * 2;
+    constexpr size_t lds = (size_t)(2 * NB + 3) * DIM * 4 + (inside > between ? inside : between);
     const int rc = ensure_ws(be, &be->scan_ws, &be->scan_ws_bytes, (size_t)chunks * a.p.heads * sizeof(Chunk<DIM>), "scan");
     if (rc) return rc;
     a.ws = (char *)be->scan_ws;
@@ -428,9 +481,9 @@ int launch_chunks(vx_backend *be, ForgetArgs a, int chunks) {
         (void)hipFuncSetAttribute((const void *)prepare_kernel<DIM>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         allowed = true;
     }
-    prepare_kernel<DIM><<<dim3(chunks, a.p.heads), 512, lds, be->stream>>>(a);
+    prepare_kernel<DIM><<<dim3(chunks, a.p.heads), NB * DIM, lds, be->stream>>>(a);
     VX_CHECK_LAUNCH();
-    walk_kernel<DT><<<dim3(a.n_seqs, a.p.heads, ceil_div(a.p.vdim, VC)), 256, 0, be->stream>>>(a);
+    walk_kernel<DT><<<dim3(a.n_seqs, a.p.heads, ceil_div(a.p.vdim, VC)), 512, 0, be->stream>>>(a);
     VX_CHECK_LAUNCH();
     return VX_OK;
 }
