@@ -68,15 +68,15 @@ __global__ void __launch_bounds__(64 * MAX_WAVES) talk_kernel(TalkArgs t) {
     }
     const int tc = talk_cols(a.p.heads), m_tiles = (a.p.heads + 15) / 16, k_steps = (a.p.heads + 31) / 32;
     bf16 *s_talk = (bf16 *)(s_dyn + 2 * t.buf);
-    for (int i = tid; i < m_tiles * 16 * tc; i += blockDim.x) {
-        const int h = i / tc, g = i % tc;
-        s_talk[i] = h < a.p.heads && g < a.p.heads ? ((const bf16 *)a.p.talk)[h * a.p.heads + g] : (bf16)0.f;
-    }
-    for (int i = tid; i < 2 * t.buf; i += blockDim.x) s_dyn[i] = 0.f;  // (heads that pad a row stay zero)
-    __syncthreads();
-
     // this wave's tiles
     const int first_tile = wave * TPW, wave_tiles = min(TPW, t.tiles - first_tile);  // none or fewer for the last waves
+    const int32_t *bt = a.tables + (size_t)a.rows[seq] * a.max_blocks;
+    Keys<KD, VD, 1, false> ks;
+    ks.init(a, min(first_tile, t.tiles - 1) / t.per_kv, lane);
+    const auto block = [&](int b) { return bt[min(b, last_blk)]; };
+    int b0 = block(2 * g_first), b1 = block(2 * g_first + 1), n0 = block(2 * g_first + 2), n1 = block(2 * g_first + 3);
+    int f0 = block(2 * g_first + 4), f1 = block(2 * g_first + 5);  // (read from the table a group before their keys are)
+    if (SHARE && wave_tiles > 0) ks.load_k(b0, b1);
     // queries: in registers, in LDS where registers are short, or (four tiles) read again for every group
     constexpr bool LDS_Q = queries_in_lds(KD, TPW, SHARE), KEEP_Q = TPW <= 2 && !LDS_Q;
     bf16x8 *s_q = (bf16x8 *)(s_talk + m_tiles * 16 * tc) + wave * TPW * KD * 64 + lane;
@@ -108,10 +108,6 @@ __global__ void __launch_bounds__(64 * MAX_WAVES) talk_kernel(TalkArgs t) {
             if constexpr (LDS_Q) s_q[(i * KD + kk) * 64] = load_q(qp[i], kk * 32 + q8, a.p.k_dim, a.vec_q);  // (this wave alone reads it)
         }
     }
-    const int32_t *bt = a.tables + (size_t)a.rows[seq] * a.max_blocks;
-    Keys<KD, VD, 1, false> ks;
-    ks.init(a, tile_of(0) / t.per_kv, lane);
-    const auto block = [&](int b) { return bt[min(b, last_blk)]; };
     // this wave's products with the keys of a group to a buffer; the keys of tiles that share them are there already
     const int my_key = (l16 >> 2) * 8 + (l16 & 3);  // of the first 16 columns; of the others it is four further on
     const auto scores = [&](float *buf, int b0, int b1) {
@@ -183,16 +179,21 @@ __global__ void __launch_bounds__(64 * MAX_WAVES) talk_kernel(TalkArgs t) {
             }
         }
     };
-    int b0 = block(2 * g_first), b1 = block(2 * g_first + 1), n0 = block(2 * g_first + 2), n1 = block(2 * g_first + 3);
+    for (int i = tid; i < m_tiles * 16 * tc; i += blockDim.x) {
+        const int h = i / tc, g = i % tc;
+        s_talk[i] = h < a.p.heads && g < a.p.heads ? ((const bf16 *)a.p.talk)[h * a.p.heads + g] : (bf16)0.f;
+    }
+    if (t.h8 > a.p.heads)
+        for (int i = tid; i < 2 * t.buf; i += blockDim.x) s_dyn[i] = 0.f;  // (heads that pad a row stay zero)
+    __syncthreads();
     if (wave_tiles > 0) {
-        if (SHARE) ks.load_k(b0, b1);
         scores(s_dyn, b0, b1);
         if (SHARE) ks.load_k(n0, n1);  // (behind the last group: its own last block again)
     }
     for (int gi = g_first; gi < g_end; gi++) {
         float *buf = s_dyn + ((gi - g_first) & 1) * t.buf, *other = s_dyn + ((gi - g_first + 1) & 1) * t.buf;
         const int k0 = gi * 32;
-        const int f0 = block(2 * gi + 4), f1 = block(2 * gi + 5);
+        const int e0 = block(2 * gi + 6), e1 = block(2 * gi + 7);
         __syncthreads();
         mix(buf);
         if (gi + 1 < g_end && wave_tiles > 0) scores(other, n0, n1);  // (that buffer's scores were read before the barrier)
@@ -211,7 +212,7 @@ __global__ void __launch_bounds__(64 * MAX_WAVES) talk_kernel(TalkArgs t) {
             for (int j = 0; j < 8; j++) st[j >> 2][j & 3] = buf[key_at(t, q8 + j) + from[i]];
             qs.template step<1, false>(a, ks, st[0], st[1], i, k0, lane, whole, true, nullptr);
         }
-        b0 = n0, b1 = n1, n0 = f0, n1 = f1;
+        b0 = n0, b1 = n1, n0 = f0, n1 = f1, f0 = e0, f1 = e1;
     }
 #pragma unroll
     for (int i = 0; i < TPW; i++) {
@@ -393,6 +394,8 @@ int attn_talk(vx_backend *be, AttnArgs a, const vx_ragged *b) {
         int tpw = std::max(2, least_tpw(t)), lr = 0;
         while ((2 << lr) <= MAX_ROWS && plan(&t, lr + 1, tpw)) lr++;
         plan(&t, lr, tpw);
+        // (fewer where that leaves much of the chip without work)
+        while (lr > 0 && t.tiles > MAX_WAVES && count_items(b, 1 << lr, t.a.min_rows) < 64) plan(&t, --lr, tpw);
         if (t.tiles <= MAX_WAVES) tpw = 1;
         const int units = count_items(b, 1 << lr, t.a.min_rows), n = span(1 << lr);
         const int want = units >= 192 ? 1 : ceil_div(256, units);  // (a workgroup fills a compute unit)
